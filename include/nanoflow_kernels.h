@@ -291,6 +291,140 @@ NF_API int nf_keep_token_f16(const uint16_t* in, uint16_t* out, const int32_t* i
 NF_API int nf_argmax_f16(const uint16_t* logits, uint16_t* max_vals, int32_t* argmax, int rows, int cols,
                   nf_stream_t stream);
 
+/* ---- operators of the layer-stack pipeline: decoders that are a list of layers, each with its own
+ * mixer (attention over a window, linear recurrences) and feed-forward.  No counterpart in the
+ * reference, whose pipelines run one Llama layer.
+ *
+ * Activations and weights are bf16 or fp32 (`dtype`); the residual stream, norm weights, position
+ * tables, recurrent state and whatever enters a recurrence besides projections are fp32.  Rows are
+ * padded to `ld` elements (a multiple of 8); the columns past the true width are zero and stay zero. */
+enum nf_dtype { NF_F32 = 0, NF_BF16 = 1 };
+enum nf_activation { NF_ACT_NONE = 0, NF_ACT_SQUARED_RELU = 1 };
+
+/* D [M,N] = act(A [M,K] . B^T), B [N,K] (k contiguous).  bf16: K % 8 == 0, N % 8 == 0, fp32 sums,
+ * launches of at most 320 rows may be split over K through `workspace`
+ * (nf_gemm_nk_workspace_bytes_upto(max_M, N, K) bytes; null: never split).  fp32: every product and sum
+ * in 32-bit, K % 4 == 0. */
+NF_API size_t nf_gemm_nk_workspace_bytes_upto(int max_M, int N, int K);
+NF_API int nf_gemm_nk_bf16(const uint16_t* A, const uint16_t* B, uint16_t* D, int M, int N, int K, void* workspace,
+                           size_t workspace_bytes, nf_stream_t stream);
+NF_API int nf_gemm_nk_relu2_bf16(const uint16_t* A, const uint16_t* B, uint16_t* D, int M, int N, int K,
+                                 void* workspace, size_t workspace_bytes, nf_stream_t stream);
+NF_API int nf_gemm_nk_f32(const float* A, const float* B, float* D, int M, int N, int K, int act, nf_stream_t stream);
+/* The same product left as fp32 sums: P [shares][M][N], shares = nf_gemm_nk_sums_shares(M, N, K,
+ * max_shares) (1 unless the output tiles alone leave most of the chip idle), for a consumer that adds
+ * the shares itself.  nf_gemm_nk_sums_bytes_upto: the room that 1..max_M rows may take. */
+NF_API int nf_gemm_nk_sums_shares(int M, int N, int K, int max_shares);
+NF_API size_t nf_gemm_nk_sums_bytes_upto(int max_M, int N, int K, int max_shares);
+NF_API int nf_gemm_nk_sums_bf16(const uint16_t* A, const uint16_t* B, float* P, size_t p_bytes, int M, int N, int K,
+                                int max_shares, nf_stream_t stream);
+
+/* x [rows, ld] fp32 = embed[tokens[t]] + pos[positions[t]] (pos may be null); act = x in `dtype` (null: not
+ * written).  Tables have `ld` columns in `dtype`. */
+NF_API int nf_embed_rows(int dtype, const int32_t* tokens, const int32_t* positions, const void* embed, const void* pos,
+                         float* x, void* act, int rows, int ld, nf_stream_t stream);
+/* A sublayer's output normed and added to the residual stream: with y the sum of `shares` fp32 [rows, ld]
+ * slices (y_dtype NF_F32) or one bf16 [rows, ld] (NF_BF16, shares 1),
+ *   x += y / sqrt(mean(y^2) + eps) * weight    (mean over `width` columns),   act = x in `dtype` (may be null). */
+NF_API int nf_norm_add_rows(int y_dtype, const void* y, int shares, const float* weight, float* x, int dtype, void* act,
+                            int rows, int width, int ld, float eps, nf_stream_t stream);
+/* out [n, ld] in `dtype` = RMS norm of the n rows of x that row_index names. */
+NF_API int nf_gather_norm_rows(int dtype, const float* x, const int32_t* row_index, const float* weight, void* out, int n,
+                               int width, int ld, float eps, nf_stream_t stream);
+/* Token shift: with p the row before a row of x in its request (the request's slot of shift_state
+ * [slots, ld] for the first row of a portion, zeros at position 0),
+ *   out[s][t] = x[t] + (p - x[t]) * mu[s],  s < n_mix; out [n_mix][rows][ld] in `dtype`, mu [n_mix][ld]. */
+NF_API int nf_token_shift(int dtype, const float* x, const float* shift_state, const float* mu, void* out, int n_mix,
+                          const int32_t* input_indptr, const int32_t* rev_input_indptr, const int32_t* positions,
+                          const int32_t* state_slots, int rows, int ld, nf_stream_t stream);
+/* out [rows, cols] in `dtype` = tanh of the sum of `shares` fp32 [rows, cols] slices; cols % 4 == 0. */
+NF_API int nf_tanh_rows(int dtype, const float* sums, int shares, void* out, int rows, int cols, nf_stream_t stream);
+/* Row argmax over fp32 logits (row stride ld); equal maxima: the smallest column. */
+NF_API int nf_argmax_f32(const float* logits, int32_t* argmax, int rows, int cols, int ld, nf_stream_t stream);
+
+/* Rotary position tables: float pairs (cos, sin) [positions][dims / 2]; interleaved: dimension 2i is
+ * paired with 2i + 1, else i with i + dims / 2.  dims == 0: no rotation. */
+typedef struct nf_rotation {
+  const float* table;
+  int dims;
+  int interleaved;
+} nf_rotation;
+
+/* Paged KV cache of one attention layer: page p of the pool holds `page` positions as
+ *   K [kv_heads][page][k_pad]  then  V [kv_heads][v_pad][page]    (V transposed: a value column's
+ * positions are contiguous), elements of `dtype`; k_pad = dim rounded up to 32, v_pad = vdim to 16, both
+ * zero padded. */
+typedef struct nf_kv_layout {
+  int dtype, heads, kv_heads, dim, vdim, k_pad, v_pad, page;
+} nf_kv_layout;
+NF_API size_t nf_kv_page_elements(const nf_kv_layout* kv);
+
+/* Projected rows (q | k | v at the given columns of `proj`, row stride ld) -> per-head RMS norm of q and k
+ * (weights may be null), rotation, q scaled by nothing -> q_out [rows][heads][k_pad]; k and v appended to the
+ * cache at the row's position. */
+NF_API int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, int k_col, int v_col,
+                         const float* q_norm, const float* k_norm, float eps, const nf_rotation* rot, void* q_out,
+                         void* kv_data, const int32_t* kv_indptr, const int32_t* kv_indices,
+                         const int32_t* rev_input_indptr, const int32_t* positions, int rows, nf_stream_t stream);
+
+/* Attention over the cache.  A row at position p sees position j iff j <= p and (p - j < window or
+ * j < keep_first); window <= 0: all of j <= p.  Scores are q.k * scale; sink (may be null): exp(sink[h]) is
+ * added to the denominator.  Output: heads concatenated at column out_col of out (row stride out_ld),
+ * multiplied by out_scale.  Rows of requests [req_begin, req_begin + req_num) of the batch are computed;
+ * max_rows bounds their number of rows.  decode != 0: every one of those requests has exactly one row. */
+typedef struct nf_window_attention_args {
+  nf_kv_layout kv;
+  int window, keep_first;
+  float scale, out_scale;
+  const float* sink;
+  const void* q;
+  void* out;
+  int out_ld, out_col;
+  const void* kv_data;
+  const int32_t *input_indptr, *kv_indptr, *kv_indices, *rev_input_indptr, *positions;
+  int req_begin, req_num, row_begin, max_rows, decode;
+} nf_window_attention_args;
+NF_API int nf_window_attention(const nf_window_attention_args* args, nf_stream_t stream);
+
+/* Linear recurrences over a state S [dim][vdim] per head (fp32, [slots][heads][dim_pad][vdim_pad], pads =
+ * multiples of 16), per request carried in its slot and taken as zero at position 0:
+ *   NF_RECURRENCE_FIXED_DECAY:  S <- 2^log2_decay[h] S + k (x) v, read after the update: o = q . S.  q and k are
+ *     rotated and k is multiplied by k_scale first.
+ *   NF_RECURRENCE_TOKEN_DECAY:  read before the update, o = q . S + (q . (u * k)) v;  then row c of S is
+ *     multiplied by a factor of the token's own, exp(-exp(z[c] + w0[c])), and k (x) v is added.  z is the sum of
+ *     `z_shares` fp32 slices [rows, z_ld].
+ * A head's o is divided by its root mean square, multiplied by norm_weight (may be null) and silu(g), scaled by
+ * out_scale and written at column out_col of out.  With shift_x not null the last row of every request is kept
+ * in shift_state [slots, shift_ld] as well (the token shift of the next portion). */
+enum nf_recurrence_kind { NF_RECURRENCE_FIXED_DECAY = 0, NF_RECURRENCE_TOKEN_DECAY = 1 };
+typedef struct nf_recurrence_args {
+  int dtype, kind, heads, dim, vdim;
+  const void *q, *k, *v, *g; /* [rows][*_ld], a head's columns contiguous */
+  int q_ld, k_ld, v_ld, g_ld;
+  nf_rotation rot;
+  float k_scale;
+  const float* log2_decay; /* [heads], FIXED_DECAY */
+  const float* z;          /* TOKEN_DECAY from here */
+  int z_ld, z_shares;
+  const float *w0, *u;
+  const float* norm_weight;
+  float eps, out_scale;
+  float* state;
+  void* out;
+  int out_ld, out_col;
+  const float* shift_x;
+  float* shift_state;
+  int shift_ld;
+  const int32_t *input_indptr, *positions, *state_slots;
+  int req_begin, req_num, row_begin, rows; /* the requests computed, their first row and number of rows */
+  int total_rows;                          /* rows of the batch (the distance of two slices of z) */
+  void* workspace;
+  size_t workspace_bytes;
+} nf_recurrence_args;
+NF_API size_t nf_recurrence_state_elements(int dim, int vdim); /* per slot and head */
+NF_API size_t nf_recurrence_workspace_bytes(int heads, int dim, int vdim, int max_rows, int max_requests);
+NF_API int nf_linear_recurrence(const nf_recurrence_args* args, nf_stream_t stream);
+
 /* Calibration micro-benchmarks: ceilings measured on the device the library runs on, beside which
  * the kernels' rates are reported.  Each call launches, waits for and times its own kernels (HIP
  * events on `stream`); `scratch` is at least 8192 bytes of device memory the kernels may write.

@@ -50,7 +50,8 @@ enum nf_pipeline_type {
   NF_PIPE_NANOBATCH_KQVBIAS = 6,
   NF_PIPE_LOCAL = 7,             /* two nano-batches, GEMM and attention streams overlapped */
   NF_PIPE_NON_OVERLAP_LOCAL = 8, /* sequential baseline */
-  NF_PIPE_NANOBATCH_LOCAL = 9    /* nano-batched, single stream */
+  NF_PIPE_NANOBATCH_LOCAL = 9,   /* nano-batched, single stream */
+  NF_PIPE_LAYER_STACK = 10       /* a layer-stack model (pllm_stack_*); not in the reference */
 };
 
 /* vortexWeight (vortexData.cuh:7-12) */
@@ -311,6 +312,67 @@ NF_PLLM_API int pllm_reset_timings(void);
  *          inputs and outputs: "ln_attn" (QKV input), "kqv", "attn_out" (O input), "o_out",
  *          "ln_ffn" (gate/up input), "act" (down input). */
 NF_PLLM_API int pllm_debug_buffer(const char* name, uint16_t** ptr, int* rows, int* cols);
+
+/* ---- layer-stack models: decoders described by a list of layers, each with its own mixer (attention over
+ * a window, recurrences with a state per head, both side by side) and feed-forward.  No counterpart in
+ * the reference.  The model is described by its config.json, whose `architecture` selects the parser
+ * (the registry of csrc/host/stackModel.h); its weights come from a safetensors file or named host
+ * tensors.  A pipeline file can name such a model too: its "model" block is then that configuration (or
+ * {"path": DIR}) and "model_configs" may hold dtype, kv_pages and state_slots (pllm_set_model_config).
+ *
+ * Sequence: pllm_stack_set_config (or pllm_set_model_config), pllm_stack_init*, then pllm_update_stack /
+ * pllm_run* / pllm_serve as for the other pipelines, or a replay; pllm_finalize. */
+NF_PLLM_API int pllm_stack_set_config(const char* config_json, const char* dtype, int max_batch, int kv_pages,
+                                      int state_slots);
+/* 0 when the configured model is not a layer-stack model. */
+NF_PLLM_API int pllm_stack_state_slots(void);
+enum nf_host_tensor_type { NF_TENSOR_BF16 = 0, NF_TENSOR_F32 = 1, NF_TENSOR_I32 = 2 };
+typedef struct nf_host_tensor {
+  const char* name;
+  int type;
+  int ndim;
+  const int64_t* shape;
+  const void* data;
+} nf_host_tensor;
+/* Upload the weights (DIR/model.safetensors, or host tensors that are read before the call returns), allocate
+ * caches, states and buffers for batches of global_batch rows, start the pipeline. */
+NF_PLLM_API int pllm_stack_init(const char* model_dir, int global_batch);
+NF_PLLM_API int pllm_stack_init_tensors(const nf_host_tensor* tensors, int count, int global_batch);
+/* pllm_update with what a layer-stack model takes besides: the state slot of every request (required when the
+ * model has recurrent state), given tokens for the decode rows instead of the last samples (may be null), the rows
+ * whose logits are computed and sampled (null: the last row of every request). */
+typedef struct nf_stack_update {
+  const int32_t* state_slots;
+  const int32_t* decode_tokens;
+  const int32_t* logit_rows;
+  int logit_rows_num;
+} nf_stack_update;
+NF_PLLM_API int pllm_update_stack(const nf_vortex_update_data* update, const nf_stack_update* stack);
+/* fp32 logits of the last iteration, [*rows][*vocab], copied to `out` (at most cap_rows rows; out may be null to ask
+ * for the sizes). */
+NF_PLLM_API int pllm_get_logits(float* out, int cap_rows, int* rows, int* vocab);
+/* Keep the residual stream after every layer (before pllm_stack_init; iterations are then never replayed from
+ * graphs); copies the rows of one layer, [*rows][*width], `out` may be null. */
+NF_PLLM_API int pllm_stack_keep_layers(int on);
+NF_PLLM_API int pllm_stack_layer_output(int layer, float* out, int* rows, int* width);
+
+/* Replay of given tokens (what bin/trace_run does): every step is one iteration of the serving schedule, over
+ * pages and slots of its own pool.  Entry i has n_tokens[i] tokens (concatenated in `tokens`) and n_want[i] places
+ * among them whose logits are wanted (concatenated in `want`); out receives [sum of n_want][vocab].  A failed
+ * step ends the replay. */
+typedef struct nf_replay nf_replay;
+NF_PLLM_API nf_replay* pllm_replay_create(int kv_pages, int state_slots);
+NF_PLLM_API void pllm_replay_destroy(nf_replay* r);
+NF_PLLM_API int pllm_replay_step(nf_replay* r, int n, const char* const* ids, const int32_t* n_tokens, const int32_t* tokens,
+                                 const int32_t* n_want, const int32_t* want, float* out);
+NF_PLLM_API int pllm_replay_end(nf_replay* r, const char* id);
+/* counts = {live requests, free pages, free slots} */
+NF_PLLM_API int pllm_replay_state(nf_replay* r, int counts[3]);
+
+/* The batch former with recurrent state: a request holds one of `slots` slots from admission to retirement
+ * (before the first request; 0: none).  pllm_sched_state_slots: the slots of the last formed batch's requests. */
+NF_PLLM_API int pllm_sched_set_state_slots(nf_batch_former* f, int slots);
+NF_PLLM_API int pllm_sched_state_slots(nf_batch_former* f, const int32_t** slots, int* count);
 
 #ifdef __cplusplus
 }

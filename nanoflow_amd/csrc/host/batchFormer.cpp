@@ -20,6 +20,13 @@ int KVPool::alloc_page() {
 
 void KVPool::free_page(int idx) { free_.push_back(idx); }
 
+int StatePool::alloc() {
+  if (free_.empty()) throw std::runtime_error("StatePool: no free slot");
+  const int slot = free_.back();
+  free_.pop_back();
+  return slot;
+}
+
 // pages appended = (num_tokens + last_page_offset - 1) / page_size, where an empty cache
 // counts as a full last page (kv_cache.py:87-98).
 void KVCache::allocate_tokens(int num_tokens) {
@@ -36,6 +43,8 @@ void KVCache::release() {
   seqlen_ = 0;
   for (int idx : indices_) pool_->free_page(idx);
   indices_.clear();
+  if (states_ && slot_ >= 0) states_->release(slot_);
+  slot_ = -1;
 }
 
 BatchFormer::BatchFormer(int kv_capacity_pages, int page_size, int global_bsz, int nanobatch1, int kqv1,
@@ -85,11 +94,11 @@ void BatchFormer::schedule() {
   const int max_seq_len = avg_decode_ + avg_prefill_ + 2;
 
   while (prefill_idle_tokens > 0 && decode_idle_tokens > 0 && !queue_.empty() &&
-         new_min_avail_pages > (avg_prefill_ + avg_decode_ + P) / P) {
+         new_min_avail_pages > (avg_prefill_ + avg_decode_ + P) / P && (!has_states_ || states_.num_free() > 0)) {
     SchedRequest nr = std::move(queue_.front());
     queue_.pop_front();
     auto prompt = std::make_shared<const std::vector<int32_t>>(std::move(nr.prompt));
-    auto kv = std::make_shared<KVCache>(&pool_);
+    auto kv = std::make_shared<KVCache>(&pool_, has_states_ ? &states_ : nullptr);
     const int plen = (int)prompt->size();
     auto make = [&](int from, int to, bool chunked) {
       auto f = std::make_shared<FlyRequest>();
@@ -136,6 +145,30 @@ void BatchFormer::schedule() {
   }
 }
 
+void assembleBatch(const std::vector<BatchEntry>& decode, const std::vector<BatchEntry>& prefill, FormedBatch& out) {
+  for (auto* v : {&out.input_indptr, &out.kv_indptr, &out.kv_indices, &out.kv_last_page_len, &out.rev_input_indptr,
+                  &out.per_token_offset, &out.state_slots})
+    v->clear();
+  out.input_indptr.push_back(0);
+  out.kv_indptr.push_back(0);
+  int32_t req = 0;
+  for (const auto* set : {&decode, &prefill})
+    for (const BatchEntry& e : *set) {
+      const KVCache& kv = *e.cache;
+      const int first = kv.seqlen() - e.tokens;  // position of the entry's first token
+      for (int j = 0; j < e.tokens; ++j) {
+        out.rev_input_indptr.push_back(req);
+        out.per_token_offset.push_back(first + j);
+      }
+      out.input_indptr.push_back(out.input_indptr.back() + e.tokens);
+      out.kv_indices.insert(out.kv_indices.end(), kv.indices().begin(), kv.indices().end());
+      out.kv_last_page_len.push_back(kv.last_page_offset());
+      out.kv_indptr.push_back(out.kv_indptr.back() + (int)kv.indices().size());
+      if (kv.state_slot() >= 0) out.state_slots.push_back(kv.state_slot());
+      ++req;
+    }
+}
+
 void BatchFormer::form(FormedBatch& out) {
   out = FormedBatch();
   for (const auto& r : prefill_) out.input_tokens.insert(out.input_tokens.end(), r->input.begin(), r->input.end());
@@ -152,29 +185,10 @@ void BatchFormer::form(FormedBatch& out) {
   out.gemv_batch_size[3] = dpb - out.gemv_batch_size[0] - out.gemv_batch_size[1] - out.gemv_batch_size[2];
   for (int i = 0; i < 4; ++i) out.gemv_num_blocks[i] = num_blocks_[i];
 
-  std::vector<int> prev_len;
-  out.input_indptr.push_back(0);
-  out.kv_indptr.push_back(0);
-  auto add_kv = [&](const KVCache& kv) {
-    out.kv_indices.insert(out.kv_indices.end(), kv.indices().begin(), kv.indices().end());
-    out.kv_last_page_len.push_back(kv.last_page_offset());
-    out.kv_indptr.push_back(out.kv_indptr.back() + (int)kv.indices().size());
-  };
-  for (const auto& r : decode_) {
-    out.input_indptr.push_back(out.input_indptr.back() + (int)r->input.size());
-    prev_len.push_back(r->kv_cache->seqlen() - 1);  // the new token's slot is already counted
-    add_kv(*r->kv_cache);
-  }
-  for (const auto& r : prefill_) {
-    out.input_indptr.push_back(out.input_indptr.back() + (int)r->input.size());
-    prev_len.push_back(r->kv_cache->seqlen() - (int)r->input.size());
-    add_kv(*r->kv_cache);
-  }
-  for (size_t i = 0; i + 1 < out.input_indptr.size(); ++i)
-    for (int j = out.input_indptr[i]; j < out.input_indptr[i + 1]; ++j) {
-      out.rev_input_indptr.push_back((int32_t)i);
-      out.per_token_offset.push_back(j - out.input_indptr[i] + prev_len[i]);
-    }
+  std::vector<BatchEntry> decode, prefill;
+  for (const auto& r : decode_) decode.push_back({(int)r->input.size(), r->kv_cache.get()});
+  for (const auto& r : prefill_) prefill.push_back({(int)r->input.size(), r->kv_cache.get()});
+  assembleBatch(decode, prefill, out);
   out.keep_token_list = keep_list_;
   out.keepTokenListLength = old_token_length_;
 }

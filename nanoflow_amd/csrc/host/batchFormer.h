@@ -44,9 +44,28 @@ private:
   std::vector<int> free_;  // stack; back() is handed out next
 };
 
+// Slots of recurrent state (layer-stack models): one per admitted request, from admission to
+// retirement.  Most recently freed first, as the pages.
+class StatePool {
+public:
+  explicit StatePool(int capacity = 0) {
+    for (int i = capacity - 1; i >= 0; --i) free_.push_back(i);
+  }
+  int num_free() const { return (int)free_.size(); }
+  int alloc();  // throws std::runtime_error when empty
+  void release(int slot) { free_.push_back(slot); }
+
+private:
+  std::vector<int> free_;
+};
+
+// What one request holds: its pages and, for models with recurrent state, its slot.
 class KVCache {
 public:
-  explicit KVCache(KVPool* pool) : pool_(pool) {}
+  explicit KVCache(KVPool* pool, StatePool* states = nullptr) : pool_(pool), states_(states) {
+    if (states_) slot_ = states_->alloc();
+  }
+  int state_slot() const { return slot_; }  // -1: none
   int seqlen() const { return seqlen_; }
   const std::vector<int32_t>& indices() const { return indices_; }
   int last_page_offset() const { return (seqlen_ - 1 + pool_->page_size()) % pool_->page_size() + 1; }
@@ -55,8 +74,10 @@ public:
 
 private:
   KVPool* pool_;
+  StatePool* states_;
   std::vector<int32_t> indices_;
   int seqlen_ = 0;
+  int slot_ = -1;
 };
 
 struct FlyRequest {  // FlyRequestInfo (pipeline/utils/request_info.py:33-57)
@@ -79,14 +100,31 @@ struct FormedBatch {
   std::vector<int32_t> input_indptr, rev_input_indptr, per_token_offset;
   std::vector<int32_t> kv_indptr, kv_indices, kv_last_page_len;
   std::vector<int32_t> keep_token_list;  // over the PREVIOUS iteration's requests
+  std::vector<int32_t> state_slots;      // [req], empty for models without recurrent state
   int32_t gemv_batch_size[4] = {0, 0, 0, 0};
   int32_t gemv_num_blocks[4] = {0, 0, 0, 0};
 };
+
+// One request of a batch: what it contributes and what it holds (the tokens' slots counted already).
+struct BatchEntry {
+  int tokens;
+  const KVCache* cache;
+};
+// The metadata of a batch of one-row decode requests followed by prompt portions: indptr arrays, page
+// lists, positions, state slots.  Everything else in `out` is left alone.
+void assembleBatch(const std::vector<BatchEntry>& decode, const std::vector<BatchEntry>& prefill, FormedBatch& out);
 
 class BatchFormer {
 public:
   BatchFormer(int kv_capacity_pages, int page_size, int global_bsz, int nanobatch1, int kqv1, int kqv3,
               int average_prefill_length, int average_decode_length);
+
+  // Models with recurrent state: a request is admitted only while one of `slots` is free.  Before the first
+  // request.
+  void set_state_slots(int slots) {
+    states_ = StatePool(slots);
+    has_states_ = slots > 0;
+  }
 
   void add_request(SchedRequest r) { queue_.push_back(std::move(r)); }
   size_t queued() const { return queue_.size(); }
@@ -116,6 +154,8 @@ public:
 
 private:
   KVPool pool_;
+  StatePool states_;
+  bool has_states_ = false;
   std::deque<SchedRequest> queue_;
   int global_bsz_, nano1_, kqv1_, kqv3_, avg_prefill_, avg_decode_;
   std::vector<FlyPtr> decode_, prefill_, new_decode_, new_prefill_, old_decode_, old_prefill_;

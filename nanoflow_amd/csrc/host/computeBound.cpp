@@ -3,12 +3,21 @@
 #include <pthread.h>
 #include <sched.h>
 
+#include "pipelineFactory.h"
+#include "stackModel.h"
+
+#include <algorithm>
 #include <cstring>
 #include <iostream>
 
 std::vector<std::unique_ptr<Worker>> workers;
 std::vector<vortexOutputData> outputs;
 std::vector<int> aggregated_output;
+
+std::map<Worker::PipelineType, PipelineFactory>& pipelineFactories() {
+  static std::map<Worker::PipelineType, PipelineFactory> m;
+  return m;
+}
 
 struct SharedState {
   WorkerOp op = WorkerOp::STOP;
@@ -18,7 +27,7 @@ struct SharedState {
 static SharedState shared_state;
 static std::unique_ptr<SimpleThreadSync> global_sync;  // workers + the caller's thread
 static vortexInitData* persistant_input = nullptr;
-static std::vector<int> complete_input_tokens;
+static std::vector<int> complete_input_tokens, last_rows;
 static int g_profiling = 0;
 static WeightFormat g_weight_format = WeightFormat::F16;
 void setWeightFormat(WeightFormat format) { g_weight_format = format; }
@@ -101,8 +110,10 @@ void update(int nranks, std::vector<vortexUpdateData>& updateData) {
   int kept = 0;
   for (int i = 0; i < update_d.keepTokenListLength; ++i) kept += update_d.keep_token_list[i] == 1;
   const bool first = aggregated_output.empty();
+  const bool given = update_d.decode_tokens != nullptr;  // the decode rows' tokens come with the update
+  if (given) kept = update_d.decodePrefillBorder;
   if (kept != update_d.decodePrefillBorder || update_d.prefillTokensNum < 0 ||
-      (!first && update_d.keepTokenListLength > (int)aggregated_output.size())) {
+      (!first && !given && update_d.keepTokenListLength > (int)aggregated_output.size())) {
     std::fprintf(stderr,
                  "update: keep list of %d entries keeps %d slots, the batch has %d decode rows and the previous "
                  "iteration produced %zu outputs\n",
@@ -110,9 +121,21 @@ void update(int nranks, std::vector<vortexUpdateData>& updateData) {
     std::exit(EXIT_FAILURE);
   }
   complete_input_tokens.resize((size_t)kept + update_d.prefillTokensNum + 1);
-  buildInputTokens(aggregated_output.data(), (int)aggregated_output.size(), update_d.keep_token_list,
-                   update_d.keepTokenListLength, update_d.input_tokens, update_d.prefillTokensNum,
-                   complete_input_tokens.data());
+  if (given) {
+    std::copy_n(update_d.decode_tokens, kept, complete_input_tokens.begin());
+    std::copy_n(update_d.input_tokens, update_d.prefillTokensNum, complete_input_tokens.begin() + kept);
+  } else {
+    buildInputTokens(aggregated_output.data(), (int)aggregated_output.size(), update_d.keep_token_list,
+                     update_d.keepTokenListLength, update_d.input_tokens, update_d.prefillTokensNum,
+                     complete_input_tokens.data());
+  }
+  if (ActiveStackModel && !update_d.logit_rows) {  // the last row of every request is sampled
+    const int req = update_d.decodePrefillBorder + update_d.prefillNum;
+    last_rows.resize((size_t)req);
+    for (int i = 0; i < req; ++i) last_rows[i] = update_d.input_indptr[i + 1] - 1;
+    update_d.logit_rows = last_rows.data();
+    update_d.logit_rows_num = req;
+  }
   for (int i = 0; i < nranks; ++i) updateData[i].input_tokens = complete_input_tokens.data();
   shared_state.op = WorkerOp::UPDATE;
   shared_state.updates_ptr = &updateData;
@@ -167,18 +190,9 @@ void Worker::init() {
   HIP_CHECK(hipSetDevice(rank));
   // Type -> schedule as the reference maps them (pipeline/src/computeBound.cu:234-247): the five
   // types of its main Pipeline run the four-way nano-batch schedule, without their exchange steps.
-  const bool bias = hasKQVBias(PipeTy);
-  if (isFourWay(PipeTy))
-    pipeline = std::make_unique<Pipeline>(input, rank, nranks, vnranks, PipeTy == PipelineType::PLLMOFFLOAD,
-                                          PipeTy == PipelineType::NANOBATCH || PipeTy == PipelineType::NANOBATCH_KQVBIAS,
-                                          bias);
-  else if (PipeTy == PipelineType::NONOVERLAP || PipeTy == PipelineType::NONOVERLAP_KQVBIAS ||
-           PipeTy == PipelineType::NON_OVERLAP_LOCAL)
-    pipeline = std::make_unique<NonOverlapLocalPipeline>(input, rank, nranks, vnranks, bias);
-  else if (PipeTy == PipelineType::LOCAL || PipeTy == PipelineType::NANOBATCH_LOCAL)
-    pipeline = std::make_unique<LocalPipeline>(input, rank, nranks, vnranks, PipeTy == PipelineType::NANOBATCH_LOCAL);
-  else
-    NF_LOG_ERROR("Unknown pipeline type %d", static_cast<int>(PipeTy));
+  auto it = pipelineFactories().find(PipeTy);
+  if (it != pipelineFactories().end()) pipeline = it->second(input, rank, nranks, vnranks);
+  else NF_LOG_ERROR("Pipeline type %d is not part of this program", static_cast<int>(PipeTy));
   if (pipeline && g_profiling) pipeline->setProfiling(g_profiling);
   if (pipeline && g_graph_mode) pipeline->setGraphMode(true);
 }

@@ -57,13 +57,14 @@ public:
     LOCAL,
     NON_OVERLAP_LOCAL,
     NANOBATCH_LOCAL,
+    LAYER_STACK,  // models described by a list of layers (pipeline_stack.h); not in the reference
   };
   static PipelineType PipeTy;
   // Every type runs on the one rank of this build.  PLLM, NANOBATCH, PLLMOFFLOAD and the two
   // nano-batched bias types are the reference's main Pipeline (four QKV / attention nano-batches)
   // without its exchange steps, NONOVERLAP its sequential schedule, so that the reference's multi-GPU
   // pipeline files serve here once their gpu_num is 1.
-  static bool isSupported(PipelineType t) { return static_cast<int>(t) >= 0 && static_cast<int>(t) <= 9; }
+  static bool isSupported(PipelineType t) { return static_cast<int>(t) >= 0 && static_cast<int>(t) <= 10; }
   // the QKV GEMMs add vortexLayerWeight::B_KQV
   static bool hasKQVBias(PipelineType t) {
     return t == PipelineType::KQVBIAS || t == PipelineType::NONOVERLAP_KQVBIAS ||
@@ -76,7 +77,7 @@ public:
   }
   static bool isSequential(PipelineType t) {
     return t == PipelineType::NON_OVERLAP_LOCAL || t == PipelineType::NONOVERLAP_KQVBIAS ||
-           t == PipelineType::NONOVERLAP;
+           t == PipelineType::NONOVERLAP || t == PipelineType::LAYER_STACK;
   }
 
 private:

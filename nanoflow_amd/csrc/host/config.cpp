@@ -7,6 +7,7 @@
 
 #include "helper.h"
 #include "mini_json.h"
+#include "stackModel.h"
 
 vortexModelConfig ModelConfig;
 
@@ -49,6 +50,44 @@ void vortexModelConfig::printConfig() const {
             << "\nSMOOTH_A: " << smooth_a << "\nSMOOTH_B: " << smooth_b << std::endl;
 }
 
+// A relative model path is taken from the pipeline file's own directory.
+static std::string modelDirectory(const std::string& pipeline_file, const std::string& path) {
+  if (!path.empty() && path[0] == '/') return path;
+  const size_t slash = pipeline_file.rfind('/');
+  return slash == std::string::npos ? path : pipeline_file.substr(0, slash + 1) + path;
+}
+
+bool setStackModelConfig(const mini_json::Value& model, const std::string& dtype, int max_batch, int kv_pages, int state_slots,
+                         std::string* error) {
+  try {
+    auto s = std::make_shared<StackModelConfig>();
+    s->spec = parseStackModel(model);
+    if (dtype == "bfloat16") s->dtype = NF_BF16;
+    else if (dtype == "float32") s->dtype = NF_F32;
+    else throw std::runtime_error("dtype \"" + dtype + "\": bfloat16 or float32");
+    if (max_batch < 1 || kv_pages < 1 || state_slots < 1)
+      throw std::runtime_error("max_batch_size, the KV pages and the state slots must be at least 1");
+    s->kv_pages = kv_pages;
+    s->state_slots = state_slots;
+    vortexModelConfig c;
+    c.model_layer = c.run_layer = (int)s->spec.layers.size();
+    c.model_hidden_dim = s->spec.width;
+    c.vocab_size = (size_t)s->spec.vocab;
+    c.rms_norm_eps = (float)s->spec.eps;
+    c.max_batch_size = max_batch;
+    c.frame_page_size = 16;
+    c.calculateConfig();
+    c.max_page_num = (size_t)kv_pages;
+    c.k_temp_size = 0;  // the tmp buffer is sized by the schedule's own plan
+    ModelConfig = c;
+    ActiveStackModel = s;
+    return true;
+  } catch (const std::exception& e) {
+    if (error) *error = e.what();
+    return false;
+  }
+}
+
 bool updateVortexModelConfig(const std::string& filename) {
   mini_json::Value j;
   try {
@@ -59,6 +98,18 @@ bool updateVortexModelConfig(const std::string& filename) {
   }
   try {
     const auto& model = j.at("model");
+    if (model.contains("architecture") || model.contains("path")) {
+      // a layer-stack model: its own configuration in place of the Llama sizes, or the directory it is in
+      const mini_json::Value own =
+          model.contains("path") ? mini_json::parse_file(modelDirectory(filename, model.at("path").str) + "/config.json") : model;
+      const auto& mc = j.at("model_configs");
+      std::string error;
+      if (!setStackModelConfig(own, mc.contains("dtype") ? mc.at("dtype").str : "bfloat16", mc.value<int>("max_batch_size", 2048),
+                               mc.value<int>("kv_pages", 1024 * mc.value<int>("allocate_kv_data_batch", 400) / 16),
+                               mc.value<int>("state_slots", 256), &error))
+        throw std::runtime_error(error);
+      return true;
+    }
     vortexModelConfig c;
     c.model_hidden_dim = (int)model.at("hidden_size").number();
     c.model_qo_heads = (int)model.at("num_attention_heads").number();
@@ -94,6 +145,7 @@ bool updateVortexModelConfig(const std::string& filename) {
     c.model_gqa = c.model_qo_heads / c.model_kv_heads;
     c.calculateConfig();
     ModelConfig = c;
+    ActiveStackModel.reset();
   } catch (const std::exception& e) {
     std::cerr << "config " << filename << ": " << e.what() << std::endl;
     return false;

@@ -90,3 +90,12 @@ extern vortexModelConfig ModelConfig;
 // Reads the "model" and "model_configs" blocks of a pipeline JSON into ModelConfig.
 // Returns false (and leaves ModelConfig untouched) when the file cannot be read or parsed.
 bool updateVortexModelConfig(const std::string& filename);
+
+// The same for a layer-stack model (stackModel.h): `model` is its own configuration (config.json).  Sets
+// ActiveStackModel and the limits in ModelConfig; dtype "bfloat16" or "float32".  On failure both are
+// left untouched and *error holds the reason.
+namespace mini_json {
+struct Value;
+}
+bool setStackModelConfig(const mini_json::Value& model, const std::string& dtype, int max_batch, int kv_pages, int state_slots,
+                         std::string* error);

@@ -16,7 +16,18 @@
 #include <numeric>
 
 #include "pipeline.h"
+#include "pipelineFactory.h"
 #include "tensorManager.h"
+
+template <bool kOffload, bool kSingleStream, bool kBias>
+static std::unique_ptr<PipelineBase> make(vortexInitData* in, int rank, int nranks, int vnranks) {
+  return std::unique_ptr<PipelineBase>(new Pipeline(in, rank, nranks, vnranks, kOffload, kSingleStream, kBias));
+}
+static const RegisterPipeline registered[] = {{Worker::PipelineType::PLLM, make<false, false, false>},
+                                              {Worker::PipelineType::NANOBATCH, make<false, true, false>},
+                                              {Worker::PipelineType::PLLMOFFLOAD, make<true, false, false>},
+                                              {Worker::PipelineType::KQVBIAS, make<false, false, true>},
+                                              {Worker::PipelineType::NANOBATCH_KQVBIAS, make<false, true, true>}};
 
 Pipeline::Pipeline(vortexInitData* input_data, int nrank, int nranks, int vnranks, bool enable_offload_,
                    bool nanobatch_only_, bool kqv_bias_)

@@ -5,6 +5,16 @@
 // pipeline/src/pipeline_nonoverlap_local.cu:25-62, wiring :245-304, update :108-126,327-385.
 #include "pipeline.h"
 
+#include "pipelineFactory.h"
+
+template <bool kBias>
+static std::unique_ptr<PipelineBase> make(vortexInitData* in, int rank, int nranks, int vnranks) {
+  return std::unique_ptr<PipelineBase>(new NonOverlapLocalPipeline(in, rank, nranks, vnranks, kBias));
+}
+static const RegisterPipeline registered[] = {{Worker::PipelineType::NON_OVERLAP_LOCAL, make<false>},
+                                              {Worker::PipelineType::NONOVERLAP, make<false>},
+                                              {Worker::PipelineType::NONOVERLAP_KQVBIAS, make<true>}};
+
 NonOverlapLocalPipeline::NonOverlapLocalPipeline(vortexInitData* input_data, int nrank, int nranks,
                                                  int vnranks, bool kqv_bias_)
     : PipelineBase(input_data, nrank, nranks, vnranks) {

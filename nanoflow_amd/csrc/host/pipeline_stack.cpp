@@ -1,0 +1,399 @@
+#include "pipeline_stack.h"
+
+#include <algorithm>
+
+#include "pipelineFactory.h"
+
+namespace {
+
+// Above this many rows a projection back to the residual width has tiles enough without a split over
+// K, and its output is rounded before the norm reads it; below, the norm adds the fp32 shares itself.
+constexpr int kSumsMaxRows = 512;
+constexpr int kSumsMaxShares = 16;
+
+const RegisterPipeline registered(Worker::PipelineType::LAYER_STACK, [](vortexInitData* input, int rank, int nranks, int vnranks) {
+  return std::unique_ptr<PipelineBase>(new LayerStackPipeline(input, rank, nranks, vnranks));
+});
+
+}  // namespace
+
+LayerStackPipeline::LayerStackPipeline(vortexInitData* input_data, int nrank, int nranks, int vnranks)
+    : PipelineBase(input_data, nrank, nranks, vnranks), model(input_data->stack.get()) {
+  stream_all = createPipelineStream(0, 0);
+  stream_side = createPipelineStream(0, 0);
+  HIP_CHECK(hipEventCreateWithFlags(&fork, hipEventDisableTiming));
+  HIP_CHECK(hipEventCreateWithFlags(&join, hipEventDisableTiming));
+}
+
+LayerStackPipeline::~LayerStackPipeline() {
+  clearGraphs();
+  delete[] output_data.sampled_token_array;
+  if (layer_outputs) (void)hipFree(layer_outputs);
+  if (fork) (void)hipEventDestroy(fork);
+  if (join) (void)hipEventDestroy(join);
+  if (stream_side) (void)hipStreamDestroy(stream_side);
+  if (stream_all) (void)hipStreamDestroy(stream_all);
+}
+
+int LayerStackPipeline::maxLogitRows(const StackModelSpec& spec, int max_rows) {
+  const size_t fit = ((size_t)1 << 30) / (4 * (size_t)((spec.vocab + 7) / 8 * 8));  // 1 GiB of logits
+  return (int)std::min<size_t>((size_t)max_rows, std::max<size_t>(fit, 1));
+}
+
+LayerStackPipeline::Buffers LayerStackPipeline::plan(const StackModel& m, int T, AllocationManager<half>& arena) {
+  const StackModelSpec& spec = m.spec;
+  const size_t es = m.elementBytes(), ld = (size_t)spec.ld();
+  const bool bf16 = m.dtype == NF_BF16;
+  Buffers b;
+  size_t attn_proj = 0, q = 0, mix = 0, rk = 0, vg = 0, w1 = 0, z = 0, heads = 0, ff = 0, ws = 0, ws_side = 0, recur = 0;
+  auto few = [&](const DeviceMatrix& w) { return bf16 ? nf_gemm_nk_workspace_bytes_upto(T, w.N, w.K) : 0; };
+  auto sums = [&](int rows, const DeviceMatrix& w, int shares) {
+    return bf16 ? nf_gemm_nk_sums_bytes_upto(rows, w.N, w.K, shares) : (size_t)rows * w.N * 4;
+  };
+  const int sum_rows = bf16 ? std::min(T, kSumsMaxRows) : T;
+  for (size_t i = 0; i < spec.layers.size(); ++i) {
+    const LayerSpec& s = spec.layers[i];
+    const LayerWeights& w = m.weights.layers[i];
+    if (s.attention) {
+      attn_proj = std::max(attn_proj, (size_t)w.attention.qkv.N);
+      q = std::max(q, (size_t)s.attention->heads * m.kvLayout((int)i).k_pad);
+      ws_side = std::max(ws_side, few(w.attention.qkv));
+    }
+    if (s.recurrence) {
+      const RecurrenceSpec& r = *s.recurrence;
+      recur = std::max(recur, nf_recurrence_workspace_bytes(r.heads, r.dim, r.vdim, T, T));
+      if (r.kind == NF_RECURRENCE_FIXED_DECAY) {
+        mix = std::max(mix, (size_t)w.recurrence.qkvg.N);
+        ws = std::max(ws, few(w.recurrence.qkvg));
+      } else {
+        mix = std::max(mix, 5 * ld);
+        rk = std::max(rk, (size_t)w.recurrence.r.N);
+        vg = std::max(vg, (size_t)w.recurrence.v.N);
+        w1 = std::max(w1, (size_t)w.recurrence.w1.N);
+        z = std::max(z, (size_t)w.recurrence.w2.N);
+        b.w1_sums_bytes = std::max(b.w1_sums_bytes, sums(T, w.recurrence.w1, kSumsMaxShares));
+        b.z_bytes = std::max(b.z_bytes, sums(T, w.recurrence.w2, 1));
+        ws = std::max({ws, few(w.recurrence.r), few(w.recurrence.v)});
+      }
+    }
+    heads = std::max(heads, (size_t)w.out.K);
+    b.y_sums_bytes = std::max(b.y_sums_bytes, sums(sum_rows, w.out, kSumsMaxShares));
+    if (s.mlp) {
+      ff = std::max(ff, (size_t)w.up.N);
+      ws = std::max(ws, few(w.up));
+      b.y_sums_bytes = std::max(b.y_sums_bytes, sums(sum_rows, w.down, kSumsMaxShares));
+    }
+  }
+  const int L = maxLogitRows(spec, T);
+  b.logits_bytes = sums(L, m.weights.head, 1);
+  b.gemm_ws_bytes = std::max(ws, ws_side);
+  b.recur_ws_bytes = recur;
+  b.x = (float*)arena.allocBytes(T * ld * 4);
+  b.act = bf16 ? arena.allocBytes(T * ld * es) : b.x;
+  b.attn_proj = arena.allocBytes(T * attn_proj * es);
+  b.q = arena.allocBytes(T * q * es);
+  b.mix = arena.allocBytes(T * mix * es);
+  for (int i = 0; i < 4; ++i) b.rkvg[i] = arena.allocBytes(T * (i < 2 ? rk : vg) * es);
+  b.w1_sums = (float*)arena.allocBytes(b.w1_sums_bytes);
+  b.w1_act = arena.allocBytes(T * w1 * es);
+  b.z = (float*)arena.allocBytes(std::max(b.z_bytes, T * z * 4));
+  b.heads = arena.allocBytes(T * heads * es);
+  b.y = bf16 && T > kSumsMaxRows ? arena.allocBytes(T * ld * es) : nullptr;
+  b.y_sums = (float*)arena.allocBytes(b.y_sums_bytes);
+  b.ff = arena.allocBytes(T * ff * es);
+  b.head_in = arena.allocBytes(L * ld * es);
+  b.logits = (float*)arena.allocBytes(b.logits_bytes);
+  b.argmax = (int32_t*)arena.allocBytes((size_t)L * 4);
+  b.gemm_ws = arena.allocBytes(b.gemm_ws_bytes);
+  b.gemm_ws_side = arena.allocBytes(b.gemm_ws_bytes);
+  b.recur_ws = arena.allocBytes(recur);
+  return b;
+}
+
+size_t LayerStackPipeline::tmpBytes(const StackModel& m, int max_rows) {
+  AllocationManager<half> count((half*)nullptr, (size_t)1 << 46);  // addresses only
+  (void)plan(m, max_rows, count);
+  return count.getAllocation() * sizeof(half);
+}
+
+void LayerStackPipeline::config(vortexConfigData* config_data_) {
+  clearGraphs();
+  config_error.clear();
+  this->config_data = *config_data_;
+  const int T = config_data.global_batch_size;
+  if (T <= 0 || T > ModelConfig.max_batch_size) {
+    configFail("LayerStackPipeline::config: global batch %d not in (0, %d]", T, ModelConfig.max_batch_size);
+    return;
+  }
+  AllocationManager<half> arena(input_data->tmp_buffer, input_data->tmp_buffer_size);
+  buf = plan(*model, T, arena);
+  // columns past a row's true width are never written and must read as zero
+  HIP_CHECK(hipMemset(input_data->tmp_buffer, 0, arena.getAllocation() * sizeof(half)));
+  if (layer_outputs) (void)hipFree(layer_outputs);
+  layer_outputs = nullptr;
+  const StackModelSpec& spec = model->spec;
+  const int ld = spec.ld();
+  if (keep_layers) HIP_CHECK(hipMalloc(&layer_outputs, spec.layers.size() * (size_t)T * ld * sizeof(float)));
+
+  for (StackOperator* op : std::initializer_list<StackOperator*>{&embedding, &linear, &normAdd, &tokenShift, &tanhRows, &qkvAppend,
+                                                                 &attention, &recurrence, &gatherNorm, &sampler}) {
+    op->setStream(stream_all);
+    op->batch = &batch;
+    op->dtype = model->dtype;
+  }
+  linear_side.setStream(stream_side);
+  linear_side.batch = &batch;
+  linear_side.dtype = model->dtype;
+  linear.workspace = buf.gemm_ws;
+  linear_side.workspace = buf.gemm_ws_side;
+  linear.workspace_bytes = linear_side.workspace_bytes = buf.gemm_ws_bytes;
+  void* act = model->dtype == NF_BF16 ? buf.act : nullptr;  // in fp32 the residual stream is the activation
+  embedding.w = &model->weights;
+  embedding.x = buf.x;
+  embedding.act = act;
+  embedding.ld = ld;
+  normAdd.x = buf.x;
+  normAdd.act = act;
+  normAdd.width = gatherNorm.width = spec.width;
+  normAdd.ld = gatherNorm.ld = tokenShift.ld = ld;
+  normAdd.eps = gatherNorm.eps = qkvAppend.eps = (float)spec.eps;
+  tokenShift.x = buf.x;
+  tokenShift.out = buf.mix;
+  gatherNorm.x = buf.x;
+  gatherNorm.weight = model->weights.final_norm;
+  gatherNorm.out = buf.head_in;
+  sampler.logits = buf.logits;
+  sampler.argmax = buf.argmax;
+  sampler.cols = spec.vocab;
+  sampler.ld = model->weights.head.N;
+  setName();
+
+  delete[] output_data.sampled_token_array;
+  output_data = vortexOutputData();
+  output_data.sampled_token_array = new int[T]();
+  output_data.global_batch_size = T;
+  if (profiling) setProfiling(profilingLevel());
+}
+
+void LayerStackPipeline::setName() {
+  SET_NAME_REF(embedding);
+  SET_NAME_REF(linear);
+  SET_NAME_REF(linear_side);
+  SET_NAME_REF(normAdd);
+  SET_NAME_REF(tokenShift);
+  SET_NAME_REF(tanhRows);
+  SET_NAME_REF(qkvAppend);
+  SET_NAME_REF(attention);
+  SET_NAME_REF(recurrence);
+  SET_NAME_REF(gatherNorm);
+  SET_NAME_REF(sampler);
+}
+
+void LayerStackPipeline::setProfiling(int level) {
+  profiling = level > 0;
+  profile_gemms = level > 1;
+  const unsigned stride = profileStride();
+  timings.layer_stride = (int)stride;
+  const size_t n = model->spec.layers.size();
+  attention.enableProfiling(profiling ? n : 0, stride);
+  linear.enableProfiling(profile_gemms ? 8 * n + 1 : 0, 1);
+  linear_side.enableProfiling(profile_gemms ? n : 0, 1);
+}
+
+void LayerStackPipeline::update(vortexUpdateData* u) {
+  this->update_data = *u;
+  batch.decode = u->decodePrefillBorder;
+  batch.prefill = u->prefillNum;
+  batch.rows = u->decodePrefillBorder + u->prefillTokensNum;
+  batch.logit_rows = u->logit_rows_num;
+  batch.tokens = u->input_tokens;
+  batch.positions = u->per_token_offset;
+  batch.input_indptr = u->input_indptr;
+  batch.rev_input_indptr = u->rev_input_indptr;
+  batch.kv_indptr = u->kv_indptr;
+  batch.kv_indices = u->kv_indices;
+  batch.state_slots = u->state_slots;
+  batch.logit_row_index = u->logit_rows;
+  output_data.sampled_tokens = batch.logit_rows;
+}
+
+// Projection back to the residual width, norm, residual add.
+void LayerStackPipeline::sublayerOut(const void* a, const DeviceMatrix& w, const float* norm) {
+  if (model->dtype == NF_BF16 && batch.rows > kSumsMaxRows) {
+    linear.set(a, w, buf.y, batch.rows).run();
+    normAdd.y = buf.y;
+    normAdd.y_dtype = NF_BF16;
+    normAdd.shares = 1;
+  } else {
+    linear.setSums(a, w, buf.y_sums, buf.y_sums_bytes, batch.rows, kSumsMaxShares).run();
+    normAdd.y = buf.y_sums;
+    normAdd.y_dtype = NF_F32;
+    normAdd.shares = linear.shares();
+  }
+  normAdd.weight = norm;
+  normAdd.run();
+}
+
+void LayerStackPipeline::attentionBranch(int layer, hipStream_t s) {
+  const AttentionSpec& a = *model->spec.layers[layer].attention;
+  const LayerWeights& w = model->weights.layers[layer];
+  linear_side.setStream(s);
+  qkvAppend.setStream(s);
+  attention.setStream(s);
+  linear_side.set(buf.act, w.attention.qkv, buf.attn_proj, batch.rows).run();
+  qkvAppend.kv = model->kvLayout(layer);
+  qkvAppend.proj = buf.attn_proj;
+  qkvAppend.ld = w.attention.qkv.N;
+  qkvAppend.w = &w.attention;
+  qkvAppend.q_out = buf.q;
+  qkvAppend.kv_data = model->kv_data[layer];
+  qkvAppend.run();
+  nf_window_attention_args& g = attention.args;
+  g.kv = qkvAppend.kv;
+  g.window = a.window;
+  g.keep_first = a.keep_first;
+  g.scale = (float)a.scale;
+  g.out_scale = (float)a.out_scale;
+  g.sink = w.attention.sink;
+  g.q = buf.q;
+  g.out = buf.heads;
+  g.out_ld = w.out.K;
+  g.out_col = 0;
+  g.kv_data = model->kv_data[layer];
+  attention.run();
+}
+
+void LayerStackPipeline::recurrenceBranch(int layer) {
+  const LayerSpec& spec = model->spec.layers[layer];
+  const RecurrenceSpec& r = *spec.recurrence;
+  const LayerWeights& lw = model->weights.layers[layer];
+  const RecurrenceWeights& w = lw.recurrence;
+  const int T = batch.rows;
+  const size_t es = model->elementBytes();
+  auto at = [&](const void* p, int col) { return (const void*)((const uint8_t*)p + (size_t)col * es); };
+  nf_recurrence_args& a = recurrence.args;
+  a = nf_recurrence_args{};
+  a.dtype = model->dtype;
+  a.kind = r.kind;
+  a.heads = r.heads;
+  a.dim = r.dim;
+  a.vdim = r.vdim;
+  if (r.kind == NF_RECURRENCE_FIXED_DECAY) {
+    linear.set(buf.act, w.qkvg, buf.mix, T).run();
+    a.q = at(buf.mix, w.q_col);
+    a.k = at(buf.mix, w.k_col);
+    a.v = at(buf.mix, w.v_col);
+    a.g = at(buf.mix, w.g_col);
+    a.q_ld = a.k_ld = a.v_ld = a.g_ld = w.qkvg.N;
+    a.rot = w.rot;
+    a.k_scale = (float)r.k_scale;
+    a.log2_decay = w.log2_decay;
+  } else {
+    tokenShift.shift_state = model->shift_state[layer];
+    tokenShift.mu = w.mu;
+    tokenShift.run();
+    auto mixed = [&](int s) { return (const void*)((const uint8_t*)buf.mix + (size_t)s * T * tokenShift.ld * es); };
+    const DeviceMatrix* in[4] = {&w.r, &w.k, &w.v, &w.g};
+    for (int i = 0; i < 4; ++i) linear.set(mixed(i), *in[i], buf.rkvg[i], T).run();
+    linear.setSums(mixed(4), w.w1, buf.w1_sums, buf.w1_sums_bytes, T, kSumsMaxShares).run();
+    tanhRows.sums = buf.w1_sums;
+    tanhRows.shares = linear.shares();
+    tanhRows.cols = w.w1.N;
+    tanhRows.out = buf.w1_act;
+    tanhRows.run();
+    linear.setSums(buf.w1_act, w.w2, buf.z, buf.z_bytes, T, 1).run();
+    a.q = buf.rkvg[0];
+    a.k = buf.rkvg[1];
+    a.v = buf.rkvg[2];
+    a.g = buf.rkvg[3];
+    a.q_ld = w.r.N;
+    a.k_ld = w.k.N;
+    a.v_ld = w.v.N;
+    a.g_ld = w.g.N;
+    a.z = buf.z;
+    a.z_ld = w.w2.N;
+    a.z_shares = 1;
+    a.w0 = w.w0;
+    a.u = w.u;
+    a.norm_weight = w.norm;
+    a.shift_x = buf.x;
+    a.shift_state = model->shift_state[layer];
+    a.shift_ld = tokenShift.ld;
+  }
+  a.eps = (float)model->spec.eps;
+  a.out_scale = (float)r.out_scale;
+  a.state = model->state[layer];
+  a.out = buf.heads;
+  a.out_ld = lw.out.K;
+  a.out_col = spec.attention ? spec.attention->heads * spec.attention->vdim : 0;
+  a.workspace = buf.recur_ws;
+  a.workspace_bytes = buf.recur_ws_bytes;
+  recurrence.run();
+}
+
+void LayerStackPipeline::enqueueMixer(int layer) {
+  const LayerSpec& s = model->spec.layers[layer];
+  const bool both = s.attention && s.recurrence;
+  if (both) {  // two mixers that read the same rows and write different columns
+    HIP_CHECK(hipEventRecord(fork, stream_all));
+    HIP_CHECK(hipStreamWaitEvent(stream_side, fork, 0));
+    attentionBranch(layer, stream_side);
+    HIP_CHECK(hipEventRecord(join, stream_side));
+  } else if (s.attention) {
+    attentionBranch(layer, stream_all);
+  }
+  if (s.recurrence) recurrenceBranch(layer);
+  if (both) HIP_CHECK(hipStreamWaitEvent(stream_all, join, 0));
+  sublayerOut(buf.heads, model->weights.layers[layer].out, model->weights.layers[layer].norm1);
+}
+
+void LayerStackPipeline::enqueueIteration() {
+  const StackModelSpec& spec = model->spec;
+  embedding.run();
+  for (int i = 0; i < (int)spec.layers.size(); ++i) {
+    enqueueMixer(i);
+    const LayerWeights& w = model->weights.layers[i];
+    if (spec.layers[i].mlp) {
+      linear.set(buf.act, w.up, buf.ff, batch.rows, spec.layers[i].mlp->act).run();
+      sublayerOut(buf.ff, w.down, w.norm2);
+    }
+    if (layer_outputs)
+      HIP_CHECK(hipMemcpyAsync(layer_outputs + (size_t)i * config_data.global_batch_size * spec.ld(), buf.x,
+                               (size_t)batch.rows * spec.ld() * sizeof(float), hipMemcpyDeviceToDevice, stream_all));
+  }
+  if (batch.logit_rows == 0) return;
+  gatherNorm.run();
+  linear.setSums(buf.head_in, model->weights.head, buf.logits, buf.logits_bytes, batch.logit_rows, 1).run();
+  sampler.run();
+}
+
+vortexOutputData LayerStackPipeline::run() {
+  HIP_CHECK(hipEventRecord(events[EventManager::GEMM_TIMING_START], stream_all));
+  std::vector<int> sig = baseSignature();
+  sig.push_back(batch.logit_rows);
+  if (layer_outputs) {
+    ++graph_eager;
+    enqueueIteration();
+  } else {
+    runIteration(stream_all, sig, [this] { enqueueIteration(); });
+  }
+  HIP_CHECK(hipEventRecord(events[EventManager::GEMM_TIMING_END], stream_all));
+  if (batch.logit_rows > 0)
+    HIP_CHECK(hipMemcpyAsync(output_data.sampled_token_array, buf.argmax, batch.logit_rows * sizeof(int), hipMemcpyDeviceToHost,
+                             stream_all));
+  HIP_CHECK(hipStreamSynchronize(stream_all));
+  float ms = 0;
+  HIP_CHECK(hipEventElapsedTime(&ms, events[EventManager::GEMM_TIMING_START], events[EventManager::GEMM_TIMING_END]));
+  timings.iter_ms = ms;
+  if (profiling) {
+    // one attention operator launches for the decode rows and for the prompts
+    double& t = batch.decode > 0 ? timings.decode_attn_ms : timings.prefill_attn_ms;
+    long& n = batch.decode > 0 ? timings.decode_attn_launches : timings.prefill_attn_launches;
+    attention.collectProfile(t, n);
+  }
+  if (profile_gemms) {
+    linear.collectProfile(timings.gemm_ms, timings.gemm_launches);
+    linear_side.collectProfile(timings.gemm_ms, timings.gemm_launches);
+  }
+  return output_data;
+}

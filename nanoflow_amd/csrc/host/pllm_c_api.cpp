@@ -5,6 +5,9 @@
 #include <cstring>
 
 #include "computeBound.h"
+#include "mini_json.h"
+#include "pipeline_stack.h"
+#include "stackServe.h"
 
 static thread_local char g_err[512] = "";
 static int fail(int code, const char* fmt, ...) {
@@ -58,6 +61,10 @@ int pllm_set_model_config(const char* json_path) {
   if (g_inited) return fail(NF_PLLM_ERR_STATE, "pllm_set_model_config: pipeline already initialised");
   if (!updateVortexModelConfig(json_path))
     return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_set_model_config: cannot load %s", json_path);
+  if (ActiveStackModel) {
+    g_config_loaded = true;
+    return NF_PLLM_OK;
+  }
   const auto& c = ModelConfig;
   if (c.gpu_num != 1)
     return fail(NF_PLLM_ERR_UNSUPPORTED, "model_configs.gpu_num=%d: this build runs one GPU", c.gpu_num);
@@ -90,6 +97,8 @@ int pllm_init(const nf_vortex_init_data* input, int pipeline_type) {
     return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_init: null pointer in init data");
   if (pipeline_type < 0 || pipeline_type > NF_PIPE_NANOBATCH_LOCAL)
     return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_init: unknown pipeline type %d", pipeline_type);
+  if (ActiveStackModel)
+    return fail(NF_PLLM_ERR_STATE, "pllm_init: the configured model is a layer-stack model; call pllm_stack_init");
   auto ty = static_cast<Worker::PipelineType>(pipeline_type);
   if (!Worker::isSupported(ty)) return fail(NF_PLLM_ERR_UNSUPPORTED, "pllm_init: unknown pipeline type %d", pipeline_type);
   if (getWeightFormat() == WeightFormat::E4M3 && Worker::hasKQVBias(ty))
@@ -290,7 +299,9 @@ int pllm_config(const nf_vortex_config_data* c) {
   return NF_PLLM_OK;
 }
 
-int pllm_update(const nf_vortex_update_data* u) {
+int pllm_update(const nf_vortex_update_data* u) { return pllm_update_stack(u, nullptr); }
+
+int pllm_update_stack(const nf_vortex_update_data* u, const nf_stack_update* x) {
   if (!g_configured) return fail(NF_PLLM_ERR_STATE, "pllm_update: call pllm_config first");
   if (g_running) return fail(NF_PLLM_ERR_STATE, "pllm_update: a run is in flight; call pllm_run_async_wait");
   if (!u || !u->input_indptr || !u->rev_input_indptr || !u->kv_indptr || !u->kv_indices ||
@@ -328,6 +339,39 @@ int pllm_update(const nf_vortex_update_data* u) {
   d.per_token_offset = u->per_token_offset;
   d.gemv_batch_size = u->gemv_batch_size;
   d.gemv_num_blocks = u->gemv_num_blocks;
+  if (ActiveStackModel) {
+    const StackModelConfig& m = *ActiveStackModel;
+    if (m.spec.hasState() && (!x || !x->state_slots))
+      return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_update: the model has recurrent state and the update names no slots");
+    if (x && x->state_slots) {
+      for (int i = 0; i < req; ++i)
+        if (x->state_slots[i] < 0 || x->state_slots[i] >= m.state_slots)
+          return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_update: request %d has state slot %d of %d", i, x->state_slots[i], m.state_slots);
+      d.state_slots = const_cast<int32_t*>(x->state_slots);
+    }
+    for (int i = 0; i < tok; ++i)
+      if (u->per_token_offset[i] < 0 || u->per_token_offset[i] >= m.spec.max_positions)
+        return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_update: row %d is at position %d of %d", i, u->per_token_offset[i], m.spec.max_positions);
+    const int cap = LayerStackPipeline::maxLogitRows(m.spec, T);
+    if (x && x->logit_rows) {
+      if (x->logit_rows_num < 0 || x->logit_rows_num > cap)
+        return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_update: the logits of %d rows (at most %d)", x->logit_rows_num, cap);
+      for (int i = 0; i < x->logit_rows_num; ++i)
+        if (x->logit_rows[i] < 0 || x->logit_rows[i] >= tok)
+          return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_update: logits of row %d of %d", x->logit_rows[i], tok);
+      d.logit_rows = const_cast<int32_t*>(x->logit_rows);
+      d.logit_rows_num = x->logit_rows_num;
+    } else if (req > cap) {
+      return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_update: the logits of %d requests (at most %d)", req, cap);
+    }
+    if (x && x->decode_tokens) {
+      d.decode_tokens = x->decode_tokens;
+      g_upd[0] = d;
+      update(g_nranks, g_upd);
+      g_updated = true;
+      return NF_PLLM_OK;
+    }
+  }
   // kept slots + prefill tokens must add up to the batch rows
   int kept = 0;
   for (int i = 0; i < u->keepTokenListLength; ++i) kept += u->keep_token_list[i] == 1;
@@ -511,6 +555,10 @@ int pllm_debug_buffer(const char* name, uint16_t** ptr, int* rows, int* cols) {
 // ---------------------------------------------------------------- batch former / serve loop
 #include "batchFormer.h"
 
+struct nf_replay {
+  StackReplay replay;
+};
+
 struct nf_batch_former {
   BatchFormer former;
   FormedBatch batch;
@@ -665,6 +713,157 @@ int pllm_serve(nf_batch_former* f, int skip_cycles, int warmup_cycles, int run_c
   stats->gpu_iter_ms = s.gpu_iter_ms;
   stats->tokens_processed = s.tokens_processed;
   g_updated = false;
+  return NF_PLLM_OK;
+}
+
+int pllm_stack_set_config(const char* config_json, const char* dtype, int max_batch, int kv_pages, int state_slots) {
+  if (!config_json || !dtype) return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_stack_set_config: null pointer");
+  if (g_inited) return fail(NF_PLLM_ERR_STATE, "pllm_stack_set_config: pipeline already initialised");
+  std::string error;
+  try {
+    if (!setStackModelConfig(mini_json::parse_file(config_json), dtype, max_batch, kv_pages, state_slots, &error))
+      return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_stack_set_config: %s", error.c_str());
+  } catch (const std::exception& e) {
+    return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_stack_set_config: %s", e.what());
+  }
+  g_config_loaded = true;
+  return NF_PLLM_OK;
+}
+
+int pllm_stack_state_slots(void) { return ActiveStackModel ? ActiveStackModel->state_slots : 0; }
+
+static int stack_start(const char* who, const HostTensors& tensors, int global_batch) {
+  if (!ActiveStackModel) return fail(NF_PLLM_ERR_STATE, "%s: configure a layer-stack model first", who);
+  if (g_inited) return fail(NF_PLLM_ERR_STATE, "%s: already initialised", who);
+  if (global_batch < 1 || global_batch > ModelConfig.max_batch_size)
+    return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "%s: global batch %d not in (0, %d]", who, global_batch, ModelConfig.max_batch_size);
+  startStackPipeline(tensors, global_batch);
+  g_cfg[0] = vortexConfigData();
+  g_cfg[0].global_batch_size = global_batch;
+  g_inited = g_configured = true;
+  g_updated = g_running = false;
+  return NF_PLLM_OK;
+}
+
+int pllm_stack_init(const char* model_dir, int global_batch) {
+  if (!model_dir) return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_stack_init: null pointer");
+  try {
+    const SafetensorsFile file(std::string(model_dir) + "/model.safetensors");
+    return stack_start("pllm_stack_init", file.tensors(), global_batch);
+  } catch (const std::exception& e) {
+    return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_stack_init: %s", e.what());
+  }
+}
+
+int pllm_stack_init_tensors(const nf_host_tensor* t, int count, int global_batch) {
+  if (!t || count < 1) return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_stack_init_tensors: no tensors");
+  try {
+    HostTensors m;
+    for (int i = 0; i < count; ++i) {
+      if (!t[i].name || !t[i].data || (t[i].ndim > 0 && !t[i].shape) || t[i].type < NF_TENSOR_BF16 || t[i].type > NF_TENSOR_I32)
+        return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_stack_init_tensors: tensor %d", i);
+      HostTensor h;
+      h.type = static_cast<HostTensor::Type>(t[i].type);
+      h.shape.assign(t[i].shape, t[i].shape + t[i].ndim);
+      h.data = t[i].data;
+      m[t[i].name] = h;
+    }
+    return stack_start("pllm_stack_init_tensors", m, global_batch);
+  } catch (const std::exception& e) {
+    return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_stack_init_tensors: %s", e.what());
+  }
+}
+
+static LayerStackPipeline* stack_pipeline() { return dynamic_cast<LayerStackPipeline*>(currentPipeline()); }
+
+int pllm_get_logits(float* out, int cap_rows, int* rows, int* vocab) {
+  LayerStackPipeline* p = stack_pipeline();
+  if (!p || g_running || !rows || !vocab) return fail(NF_PLLM_ERR_STATE, "pllm_get_logits: no finished iteration of a layer-stack model");
+  *rows = p->logitRows();
+  *vocab = p->vocab();
+  const int n = std::min(cap_rows, *rows);
+  if (out && n > 0)
+    HIP_CHECK(hipMemcpy2D(out, (size_t)*vocab * 4, p->logits(), (size_t)p->logitLd() * 4, (size_t)*vocab * 4, (size_t)n, hipMemcpyDeviceToHost));
+  return NF_PLLM_OK;
+}
+
+int pllm_stack_keep_layers(int on) {
+  if (g_inited) return fail(NF_PLLM_ERR_STATE, "pllm_stack_keep_layers: call it before pllm_stack_init");
+  LayerStackPipeline::keep_layers = on != 0;
+  return NF_PLLM_OK;
+}
+
+int pllm_stack_layer_output(int layer, float* out, int* rows, int* width) {
+  LayerStackPipeline* p = stack_pipeline();
+  if (!p || g_running || !rows || !width || !p->layerOutputs())
+    return fail(NF_PLLM_ERR_STATE, "pllm_stack_layer_output: no kept layers");
+  const StackModelSpec& s = ActiveStackModel->spec;
+  if (layer < 0 || layer >= (int)s.layers.size()) return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_stack_layer_output: layer %d", layer);
+  *rows = p->rows();
+  *width = s.width;
+  if (out && *rows > 0)
+    HIP_CHECK(hipMemcpy2D(out, (size_t)s.width * 4, p->layerOutputs() + (size_t)layer * p->maxRows() * s.ld(), (size_t)s.ld() * 4,
+                          (size_t)s.width * 4, (size_t)*rows, hipMemcpyDeviceToHost));
+  return NF_PLLM_OK;
+}
+
+nf_replay* pllm_replay_create(int kv_pages, int state_slots) {
+  if (!ActiveStackModel || !g_configured || kv_pages < 1 || kv_pages > ActiveStackModel->kv_pages || state_slots < 1 ||
+      state_slots > ActiveStackModel->state_slots) {
+    fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_replay_create: %d pages and %d slots of a running layer-stack pipeline", kv_pages, state_slots);
+    return nullptr;
+  }
+  return new nf_replay{StackReplay(kv_pages, ModelConfig.frame_page_size, state_slots)};
+}
+
+void pllm_replay_destroy(nf_replay* r) { delete r; }
+
+int pllm_replay_step(nf_replay* r, int n, const char* const* ids, const int32_t* n_tokens, const int32_t* tokens,
+                     const int32_t* n_want, const int32_t* want, float* out) {
+  if (!r || n < 0 || (n > 0 && (!ids || !n_tokens || !tokens || !n_want)))
+    return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_replay_step: null pointer");
+  if (!g_configured || g_running) return fail(NF_PLLM_ERR_STATE, "pllm_replay_step: no idle pipeline");
+  try {
+    std::vector<StackReplay::Entry> entries((size_t)n);
+    for (int i = 0; i < n; ++i) {
+      entries[i].id = ids[i];
+      entries[i].tokens.assign(tokens, tokens + n_tokens[i]);
+      tokens += n_tokens[i];
+      if (n_want[i] > 0) entries[i].want.assign(want, want + n_want[i]), want += n_want[i];
+    }
+    const std::vector<float> logits = r->replay.step(entries);
+    if (!logits.empty() && out) std::memcpy(out, logits.data(), logits.size() * sizeof(float));
+  } catch (const std::exception& e) {
+    return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_replay_step: %s", e.what());
+  }
+  return NF_PLLM_OK;
+}
+
+int pllm_replay_end(nf_replay* r, const char* id) {
+  if (!r || !id) return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_replay_end: null pointer");
+  r->replay.end(id);
+  return NF_PLLM_OK;
+}
+
+int pllm_replay_state(nf_replay* r, int counts[3]) {
+  if (!r || !counts) return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_replay_state: null pointer");
+  counts[0] = r->replay.live();
+  counts[1] = r->replay.free_pages();
+  counts[2] = r->replay.free_slots();
+  return NF_PLLM_OK;
+}
+
+int pllm_sched_set_state_slots(nf_batch_former* f, int slots) {
+  if (!f || slots < 0 || f->former.queued() + f->former.decoding() + f->former.prefilling() > 0)
+    return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_sched_set_state_slots: %d slots, before the first request", slots);
+  f->former.set_state_slots(slots);
+  return NF_PLLM_OK;
+}
+
+int pllm_sched_state_slots(nf_batch_former* f, const int32_t** slots, int* count) {
+  if (!f || !slots || !count) return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_sched_state_slots: null");
+  *slots = f->batch.state_slots.data();
+  *count = (int)f->batch.state_slots.size();
   return NF_PLLM_OK;
 }
 

@@ -22,6 +22,7 @@ static void to_update(FormedBatch& b, vortexUpdateData& u) {
   u.per_token_offset = b.per_token_offset.data();
   u.gemv_batch_size = b.gemv_batch_size;
   u.gemv_num_blocks = b.gemv_num_blocks;
+  u.state_slots = b.state_slots.empty() ? nullptr : b.state_slots.data();
 }
 
 ServeStats serveLoop(BatchFormer& former, int skip_cycles, int warmup_cycles, int run_cycles,

@@ -1,0 +1,181 @@
+// Layer-stack models: decoders described by a list of layers, each with its own mixer and
+// feed-forward.  A design registers a parser under its name (the `architecture` of its config.json)
+// that turns the configuration into the mechanisms below; the pipeline, the cache and state managers and
+// the loader work from that description and know no design by name.
+#pragma once
+#include <cstddef>
+#include <cstdint>
+#include <functional>
+#include <map>
+#include <memory>
+#include <optional>
+#include <string>
+#include <vector>
+
+#include "mini_json.h"
+#include "nanoflow_kernels.h"
+
+struct RotationSpec {
+  int dims = 0;
+  double base = 1e4;
+  bool interleaved = false;
+};
+
+// Softmax attention over a window with kept first positions.
+struct AttentionSpec {
+  std::string prefix;  // of its tensors
+  int heads = 0, kv_heads = 0, dim = 0, vdim = 0;
+  double scale = 1;
+  int window = 0, keep_first = 0;  // window 0: everything before
+  bool qk_norm = false, sink = false;
+  RotationSpec rot;
+  double out_scale = 1;
+};
+
+// Linear recurrence with a state per head (nf_recurrence_kind).
+struct RecurrenceSpec {
+  std::string prefix;
+  nf_recurrence_kind kind = NF_RECURRENCE_FIXED_DECAY;
+  int heads = 0, dim = 0, vdim = 0;
+  std::vector<double> decay;  // FIXED_DECAY
+  RotationSpec rot;           // FIXED_DECAY
+  double k_scale = 1;         // FIXED_DECAY
+  double out_scale = 1;
+};
+
+// A layer's mixer: attention, a recurrence, or both side by side on the same input.
+struct MlpSpec {
+  int ff = 0;
+  nf_activation act = NF_ACT_SQUARED_RELU;
+};
+struct LayerSpec {
+  std::optional<AttentionSpec> attention;
+  std::optional<RecurrenceSpec> recurrence;
+  std::optional<MlpSpec> mlp;
+};
+
+struct StackModelSpec {
+  std::string architecture;
+  int width = 0, vocab = 0, max_positions = 0;
+  double eps = 1e-5;
+  bool learned_positions = false;
+  std::vector<LayerSpec> layers;
+  int ld() const { return (width + 7) / 8 * 8; }
+  bool hasAttention() const {
+    for (const auto& l : layers)
+      if (l.attention) return true;
+    return false;
+  }
+  bool hasState() const {
+    for (const auto& l : layers)
+      if (l.recurrence) return true;
+    return false;
+  }
+};
+
+// ---- model registry
+using StackParser = std::function<StackModelSpec(const mini_json::Value& config)>;
+std::map<std::string, StackParser>& stackArchitectures();
+struct RegisterStackArchitecture {
+  RegisterStackArchitecture(const std::string& name, StackParser parser) { stackArchitectures()[name] = std::move(parser); }
+};
+// The description of a model configuration (its config.json); throws std::runtime_error with the reason when
+// the architecture is unknown or the configuration is not complete.
+StackModelSpec parseStackModel(const mini_json::Value& config);
+
+// ---- named host tensors, and the safetensors file they come from
+struct HostTensor {
+  enum Type { BF16, F32, I32 } type = BF16;
+  std::vector<int64_t> shape;
+  const void* data = nullptr;
+  size_t elements() const {
+    size_t n = 1;
+    for (int64_t d : shape) n *= (size_t)d;
+    return n;
+  }
+};
+using HostTensors = std::map<std::string, HostTensor>;
+
+class SafetensorsFile {  // a read-only mapping; the tensors point into it
+public:
+  explicit SafetensorsFile(const std::string& path);
+  ~SafetensorsFile();
+  SafetensorsFile(const SafetensorsFile&) = delete;
+  SafetensorsFile& operator=(const SafetensorsFile&) = delete;
+  const HostTensors& tensors() const { return tensors_; }
+
+private:
+  void* map_ = nullptr;
+  size_t bytes_ = 0;
+  HostTensors tensors_;
+};
+
+// ---- device weights, in the form the operators take: projections that read the same input fused into
+// one [N][K] matrix, N and K padded to 8 with zeros, vectors in fp32
+struct DeviceMatrix {
+  void* ptr = nullptr;
+  int N = 0, K = 0;
+};
+struct AttentionWeights {
+  DeviceMatrix qkv;
+  int q_col = 0, k_col = 0, v_col = 0;
+  float *q_norm = nullptr, *k_norm = nullptr, *sink = nullptr;
+  nf_rotation rot{};
+};
+struct RecurrenceWeights {
+  DeviceMatrix qkvg;                   // FIXED_DECAY
+  int q_col = 0, k_col = 0, v_col = 0, g_col = 0;
+  float* log2_decay = nullptr;
+  nf_rotation rot{};
+  DeviceMatrix r, k, v, g, w1, w2;     // TOKEN_DECAY
+  float *mu = nullptr, *w0 = nullptr, *u = nullptr, *norm = nullptr;  // mu [5][ld] in the order r k v g w
+};
+struct LayerWeights {
+  AttentionWeights attention;
+  RecurrenceWeights recurrence;
+  DeviceMatrix out;                    // over the attention heads, then the recurrence's
+  DeviceMatrix up, down;
+  float *norm1 = nullptr, *norm2 = nullptr;
+};
+struct StackWeights {
+  DeviceMatrix embed, pos, head;
+  float* final_norm = nullptr;
+  std::vector<LayerWeights> layers;
+};
+
+// What one pipeline serves: description, weights, caches and recurrent state, all on the device.
+class StackModel {
+public:
+  // Uploads; throws std::runtime_error when a tensor is missing or has the wrong shape.
+  StackModel(const StackModelSpec& spec, const HostTensors& tensors, nf_dtype dtype, int kv_pages, int page_size,
+             int state_slots);
+  ~StackModel();
+  StackModel(const StackModel&) = delete;
+  StackModel& operator=(const StackModel&) = delete;
+
+  const StackModelSpec spec;
+  const nf_dtype dtype;
+  const int kv_pages, page_size, state_slots;
+  StackWeights weights;
+  // per layer; null where the layer has none
+  std::vector<void*> kv_data;       // kv_pages pages (nf_kv_layout)
+  std::vector<float*> state;        // [state_slots][heads][dim_pad][vdim_pad]
+  std::vector<float*> shift_state;  // [state_slots][ld]
+  nf_kv_layout kvLayout(int layer) const;
+  size_t elementBytes() const { return dtype == NF_BF16 ? 2 : 4; }
+
+private:
+  struct Loader;
+  std::vector<void*> owned_;
+  std::map<std::pair<int, double>, float*> rotation_tables_;
+  void* allocate(size_t bytes);  // zeroed device memory that lives as long as the model
+  nf_rotation rotation(const RotationSpec& r);
+};
+
+// The model the current configuration names, and how it is to be held (set with the configuration).
+struct StackModelConfig {
+  StackModelSpec spec;
+  nf_dtype dtype = NF_BF16;
+  int kv_pages = 0, state_slots = 0;
+};
+extern std::shared_ptr<StackModelConfig> ActiveStackModel;  // null: a Llama-type model

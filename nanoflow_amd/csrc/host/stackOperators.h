@@ -1,0 +1,193 @@
+// Operators of the layer-stack pipeline over the kernel layer's C ABI (nf_embed_rows ... nf_argmax_f32),
+// in the vocabulary of OperatorWrapper: a stream, run(), per-launch timing.
+#pragma once
+#include "operatorWrapper.h"
+#include "stackModel.h"
+
+// The iteration's device arrays (TensorManager's mirrors) and the integers that shape its launches.
+struct StackBatch {
+  int rows = 0;         // tokens
+  int decode = 0;       // requests [0, decode) have one row each, rows [0, decode)
+  int prefill = 0;      // requests [decode, decode + prefill): portions of prompts
+  int logit_rows = 0;   // rows the head computes
+  const int32_t *tokens = nullptr, *positions = nullptr, *input_indptr = nullptr, *rev_input_indptr = nullptr;
+  const int32_t *kv_indptr = nullptr, *kv_indices = nullptr, *state_slots = nullptr, *logit_row_index = nullptr;
+};
+
+struct StackOperator : public OperatorWrapper {
+  const StackBatch* batch = nullptr;
+  nf_dtype dtype = NF_BF16;
+  StackOperator() : OperatorWrapper(false, false) {}
+};
+
+// D = act(A . W^T).  The output is rounded to the activations' type, or left as fp32 sums in shares of K
+// for an operator that adds them (sums()).
+struct StackLinear : public StackOperator {
+  const void* a = nullptr;
+  void* d = nullptr;
+  DeviceMatrix w;
+  nf_activation act = NF_ACT_NONE;
+  int rows = 0;
+  bool as_sums = false;
+  int max_shares = 1;
+  size_t d_bytes = 0;  // of a sums buffer
+  void* workspace = nullptr;
+  size_t workspace_bytes = 0;
+
+  StackLinear& set(const void* a_, const DeviceMatrix& w_, void* d_, int rows_, nf_activation act_ = NF_ACT_NONE) {
+    a = a_;
+    w = w_;
+    d = d_;
+    rows = rows_;
+    act = act_;
+    as_sums = false;
+    return *this;
+  }
+  StackLinear& setSums(const void* a_, const DeviceMatrix& w_, void* d_, size_t bytes, int rows_, int max_shares_) {
+    set(a_, w_, d_, rows_);
+    as_sums = true;
+    d_bytes = bytes;
+    max_shares = max_shares_;
+    return *this;
+  }
+  int shares() const {
+    return as_sums && dtype == NF_BF16 ? nf_gemm_nk_sums_shares(rows, w.N, w.K, max_shares) : 1;
+  }
+  double totalCompute() const { return 2.0 * rows * (double)w.N * w.K; }
+  void work() override {
+    if (dtype == NF_F32) {
+      NF_KERNEL_CHECK(nf_gemm_nk_f32((const float*)a, (const float*)w.ptr, (float*)d, rows, w.N, w.K, act, stream));
+    } else if (as_sums) {
+      NF_KERNEL_CHECK(nf_gemm_nk_sums_bf16((const uint16_t*)a, (const uint16_t*)w.ptr, (float*)d, d_bytes, rows, w.N, w.K,
+                                           max_shares, stream));
+    } else {
+      auto f = act == NF_ACT_SQUARED_RELU ? nf_gemm_nk_relu2_bf16 : nf_gemm_nk_bf16;
+      NF_KERNEL_CHECK(f((const uint16_t*)a, (const uint16_t*)w.ptr, (uint16_t*)d, rows, w.N, w.K, workspace, workspace_bytes,
+                        stream));
+    }
+  }
+};
+
+struct StackEmbedding : public StackOperator {
+  const StackWeights* w = nullptr;
+  float* x = nullptr;
+  void* act = nullptr;
+  int ld = 0;
+  void work() override {
+    NF_KERNEL_CHECK(nf_embed_rows(dtype, batch->tokens, batch->positions, w->embed.ptr, w->pos.ptr, x, act, batch->rows, ld, stream));
+  }
+};
+
+// A sublayer's output, normed, added to the residual stream.
+struct StackNormAdd : public StackOperator {
+  const void* y = nullptr;
+  nf_dtype y_dtype = NF_F32;
+  int shares = 1;
+  const float* weight = nullptr;
+  float* x = nullptr;
+  void* act = nullptr;
+  int width = 0, ld = 0;
+  float eps = 0;
+  void work() override {
+    NF_KERNEL_CHECK(nf_norm_add_rows(y_dtype, y, shares, weight, x, dtype, act, batch->rows, width, ld, eps, stream));
+  }
+};
+
+struct StackTokenShift : public StackOperator {
+  const float *x = nullptr, *shift_state = nullptr, *mu = nullptr;
+  void* out = nullptr;
+  int n_mix = 5, ld = 0;
+  void work() override {
+    NF_KERNEL_CHECK(nf_token_shift(dtype, x, shift_state, mu, out, n_mix, batch->input_indptr, batch->rev_input_indptr,
+                                   batch->positions, batch->state_slots, batch->rows, ld, stream));
+  }
+};
+
+struct StackTanh : public StackOperator {
+  const float* sums = nullptr;
+  int shares = 1, cols = 0;
+  void* out = nullptr;
+  void work() override { NF_KERNEL_CHECK(nf_tanh_rows(dtype, sums, shares, out, batch->rows, cols, stream)); }
+};
+
+// Per-head norm and rotation of projected rows, append to the paged cache (the counterpart of RoPEAppend).
+struct StackQKVAppend : public StackOperator {
+  nf_kv_layout kv{};
+  const void* proj = nullptr;
+  int ld = 0;
+  const AttentionWeights* w = nullptr;
+  float eps = 0;
+  void *q_out = nullptr, *kv_data = nullptr;
+  void work() override {
+    NF_KERNEL_CHECK(nf_qkv_append(&kv, proj, ld, w->q_col, w->k_col, w->v_col, w->q_norm, w->k_norm, eps, &w->rot, q_out,
+                                  kv_data, batch->kv_indptr, batch->kv_indices, batch->rev_input_indptr, batch->positions,
+                                  batch->rows, stream));
+  }
+};
+
+// Attention of the decode rows, then of the prompts' portions.
+struct StackAttention : public StackOperator {
+  nf_window_attention_args args{};
+  void work() override {
+    nf_window_attention_args a = args;
+    a.input_indptr = batch->input_indptr;
+    a.kv_indptr = batch->kv_indptr;
+    a.kv_indices = batch->kv_indices;
+    a.rev_input_indptr = batch->rev_input_indptr;
+    a.positions = batch->positions;
+    if (batch->decode > 0) {
+      a.req_begin = 0;
+      a.req_num = a.max_rows = batch->decode;
+      a.row_begin = 0;
+      a.decode = 1;
+      NF_KERNEL_CHECK(nf_window_attention(&a, stream));
+    }
+    if (batch->prefill > 0) {
+      a.req_begin = a.row_begin = batch->decode;
+      a.req_num = batch->prefill;
+      a.max_rows = batch->rows - batch->decode;
+      a.decode = 0;
+      NF_KERNEL_CHECK(nf_window_attention(&a, stream));
+    }
+  }
+};
+
+struct StackRecurrence : public StackOperator {
+  nf_recurrence_args args{};
+  void work() override {
+    nf_recurrence_args a = args;
+    a.input_indptr = batch->input_indptr;
+    a.positions = batch->positions;
+    a.state_slots = batch->state_slots;
+    a.total_rows = batch->rows;
+    if (batch->decode > 0) {
+      a.req_begin = a.row_begin = 0;
+      a.req_num = a.rows = batch->decode;
+      NF_KERNEL_CHECK(nf_linear_recurrence(&a, stream));
+    }
+    if (batch->prefill > 0) {
+      a.req_begin = a.row_begin = batch->decode;
+      a.req_num = batch->prefill;
+      a.rows = batch->rows - batch->decode;
+      NF_KERNEL_CHECK(nf_linear_recurrence(&a, stream));
+    }
+  }
+};
+
+// The rows whose logits are wanted, through the model's norm.
+struct StackGatherNorm : public StackOperator {
+  const float *x = nullptr, *weight = nullptr;
+  void* out = nullptr;
+  int width = 0, ld = 0;
+  float eps = 0;
+  void work() override {
+    NF_KERNEL_CHECK(nf_gather_norm_rows(dtype, x, batch->logit_row_index, weight, out, batch->logit_rows, width, ld, eps, stream));
+  }
+};
+
+struct StackArgmax : public StackOperator {
+  const float* logits = nullptr;
+  int32_t* argmax = nullptr;
+  int cols = 0, ld = 0;
+  void work() override { NF_KERNEL_CHECK(nf_argmax_f32(logits, argmax, batch->logit_rows, cols, ld, stream)); }
+};

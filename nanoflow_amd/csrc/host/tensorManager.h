@@ -47,9 +47,9 @@ public:
       auto& g = gpu_update_datas[i];
       auto& h = host_update_datas[i];
       int32_t* dev[] = {g.input_tokens, g.input_indptr, g.kv_indptr, g.kv_indices, g.kv_last_page_len,
-                        g.per_token_offset, g.rev_input_indptr, g.keep_token_list};
+                        g.per_token_offset, g.rev_input_indptr, g.keep_token_list, g.state_slots, g.logit_rows};
       int32_t* hst[] = {h.input_tokens, h.input_indptr, h.kv_indptr, h.kv_indices, h.kv_last_page_len,
-                        h.per_token_offset, h.rev_input_indptr, h.keep_token_list};
+                        h.per_token_offset, h.rev_input_indptr, h.keep_token_list, h.state_slots, h.logit_rows};
       for (auto p : dev) (void)hipFree(p);
       for (auto p : hst) (void)hipHostFree(p);
       delete[] g.gemv_batch_size;
@@ -84,6 +84,8 @@ public:
       alloc_pair(g.per_token_offset, h.per_token_offset, mb);
       alloc_pair(g.rev_input_indptr, h.rev_input_indptr, mb);
       alloc_pair(g.keep_token_list, h.keep_token_list, mb);
+      alloc_pair(g.state_slots, h.state_slots, mb);
+      alloc_pair(g.logit_rows, h.logit_rows, mb);
       g.gemv_batch_size = new int32_t[4];
       g.gemv_num_blocks = new int32_t[4];
       h.gemv_batch_size = g.gemv_batch_size;
@@ -102,7 +104,7 @@ public:
     const int used_pages = u.kv_indptr[total_batch];
     if (total_batch > ModelConfig.max_batch_size || total_token > ModelConfig.max_batch_size ||
         (size_t)used_pages > ModelConfig.max_page_num ||
-        u.keepTokenListLength > ModelConfig.max_batch_size ||
+        u.keepTokenListLength > ModelConfig.max_batch_size || u.logit_rows_num > ModelConfig.max_batch_size ||
         total_token != u.decodePrefillBorder + u.prefillTokensNum) {
       NF_LOG_ERROR("update data does not fit: requests %d tokens %d (max %d), pages %d (max %zu), "
                    "border %d + prefill tokens %d",
@@ -124,6 +126,9 @@ public:
     stage(h.per_token_offset, g.per_token_offset, u.per_token_offset, total_token, s);
     stage(h.rev_input_indptr, g.rev_input_indptr, u.rev_input_indptr, total_token, s);
     stage(h.keep_token_list, g.keep_token_list, u.keep_token_list, u.keepTokenListLength, s);
+    if (u.state_slots) stage(h.state_slots, g.state_slots, u.state_slots, total_batch, s);
+    g.logit_rows_num = h.logit_rows_num = u.logit_rows_num;
+    stage(h.logit_rows, g.logit_rows, u.logit_rows, u.logit_rows_num, s);
     return &g;
   }
 

@@ -3,10 +3,13 @@
 #pragma once
 #include <cstddef>
 #include <cstdint>
+#include <memory>
 #include <string>
 #include <vector>
 
 #include "tensor.h"
+
+class StackModel;  // stackModel.h
 
 struct vortexWeight {
   half* ptr = nullptr;
@@ -47,6 +50,8 @@ struct vortexInitData {
   size_t weight_size = 0;
   half* tmp_buffer = nullptr;  // device
   size_t tmp_buffer_size = 0;  // in halves
+  // a layer-stack model instead of kv_data and weight (not in the reference's struct)
+  std::shared_ptr<StackModel> stack;
 };
 
 struct vortexUpdateData {
@@ -64,6 +69,11 @@ struct vortexUpdateData {
   int32_t* per_token_offset = nullptr;  // [tokens] position of each token in its request
   int32_t* gemv_batch_size = nullptr;   // host, [4]
   int32_t* gemv_num_blocks = nullptr;   // host, [4]
+  // Not in the reference's struct: what layer-stack models and replays of given tokens need besides.
+  int32_t* state_slots = nullptr;       // [req] slot of the recurrent state (null: the model has none)
+  int32_t* logit_rows = nullptr;        // [logit_rows_num] rows of the dense batch whose logits are wanted
+  int logit_rows_num = 0;
+  const int32_t* decode_tokens = nullptr;  // host, [decodePrefillBorder]: fed to the decode rows instead of the last samples
 };
 
 struct vortexOutputData {

@@ -1,0 +1,94 @@
+// k-contiguous bf16 GEMMs: rounded to bf16, or as fp32 sums (whole or in shares of K) for a consumer
+// that adds them itself.
+#include "gemm_nk_impl.h"
+
+namespace {
+
+// Tile of a launch that stores fp32 sums, and its split over K: as splitk_plan, but from 257 rows on
+// (where a split does not pay) the largest tile that still gives every CU work.
+struct SumPlan {
+  int tile;  // 0: 64x256, 1: 128x128, 2: 256x256
+  int shares, k_per;
+};
+
+SumPlan sum_plan(int M, int N, int K, int max_shares) {
+  SumPlan p{M <= 64 ? 0 : 1, 1, (K + BK - 1) / BK * BK};
+  const long long t256 = (long long)((M + 255) / 256) * ((N + 255) / 256);
+  if (M > 256 && t256 >= cu_count() / 2) p.tile = 2;
+  if (max_shares < 2 || M > 256 || K < 256) return p;
+  const int bm = p.tile == 0 ? 64 : 128, bn = p.tile == 0 ? 256 : 128;
+  const int tiles = ((M + bm - 1) / bm) * ((N + bn - 1) / bn);
+  const int want = std::min(std::min(cu_count() / tiles, K / 128), std::min(max_shares, kMaxShares));
+  if (want < 2) return p;
+  p.k_per = ((K + want - 1) / want + BK - 1) / BK * BK;
+  p.shares = (K + p.k_per - 1) / p.k_per;
+  return p;
+}
+
+template <int BM, int BN, int WM, int WN>
+int launch_sums(const uint16_t* A, const uint16_t* B, float* P, int M, int N, int K, const SumPlan& p, hipStream_t s) {
+  using SM = GemmSmem<BM, BN, 1>;
+  auto kern = gemm_f16_splitk_kernel<BF16, BM, BN, WM, WN, false, true>;
+  static bool attr_set = false;  // benign race: the call is idempotent
+  if (!attr_set) {
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kern),
+                                             hipFuncAttributeMaxDynamicSharedMemorySize, (int)SM::bytes);
+    if (e != hipSuccess) {
+      set_error("gemm: cannot reserve %zu bytes of LDS: %s", SM::bytes, hipGetErrorString(e));
+      return NF_ERR_RUNTIME;
+    }
+    attr_set = true;
+  }
+  const int tiles_m = (M + BM - 1) / BM, tiles_n = (N + BN - 1) / BN;
+  const int grid = ((tiles_m * tiles_n * p.shares + 7) / 8) * 8;
+  kern<<<grid, WM * WN * 64, SM::bytes, s>>>(A, B, nullptr, P, nullptr, M, N, K, p.shares, p.k_per, tiles_m, tiles_n);
+  return check_launch("gemm (fp32 sums) launch");
+}
+
+}  // namespace
+
+extern "C" {
+
+size_t nf_gemm_nk_workspace_bytes_upto(int max_M, int N, int K) {
+  size_t need = 0;
+  for (int m = 1; m <= max_M && m <= kTallRows; ++m) {
+    int k_per = 0;
+    const int shares = splitk_plan(m, N, K, &k_per);
+    if (shares > 1) need = std::max(need, (size_t)shares * m * N * sizeof(float));
+  }
+  return need;
+}
+
+int nf_gemm_nk_bf16(const uint16_t* A, const uint16_t* B, uint16_t* D, int M, int N, int K, void* workspace,
+                    size_t workspace_bytes, nf_stream_t stream) {
+  return gemm_nk_entry<BF16>("nf_gemm_nk_bf16", A, B, D, M, N, K, workspace, workspace_bytes, stream);
+}
+
+int nf_gemm_nk_sums_shares(int M, int N, int K, int max_shares) {
+  return M > 0 && N > 0 && K > 0 ? sum_plan(M, N, K, max_shares).shares : 1;
+}
+
+size_t nf_gemm_nk_sums_bytes_upto(int max_M, int N, int K, int max_shares) {
+  size_t need = 0;
+  for (int m = 1; m <= max_M; m = m < 257 ? m + 1 : m + 64)
+    need = std::max(need, (size_t)nf_gemm_nk_sums_shares(m, N, K, max_shares) * m * N * sizeof(float));
+  return std::max(need, (size_t)nf_gemm_nk_sums_shares(max_M, N, K, max_shares) * max_M * N * sizeof(float));
+}
+
+int nf_gemm_nk_sums_bf16(const uint16_t* A, const uint16_t* B, float* P, size_t p_bytes, int M, int N, int K,
+                         int max_shares, nf_stream_t stream) {
+  const char* who = "nf_gemm_nk_sums_bf16";
+  int rc = check_gemm_args(who, A, B, P, M, N, K);
+  if (rc) return rc;
+  if (M == 0) return NF_OK;
+  const SumPlan p = sum_plan(M, N, K, max_shares);
+  NF_REQUIRE(p_bytes >= (size_t)p.shares * M * N * sizeof(float), "%s: %d shares of %d x %d do not fit %zu bytes", who,
+             p.shares, M, N, p_bytes);
+  NF_REQUIRE((size_t)32 * N * 4 < 0x7fffffffull, "%s: N=%d", who, N);
+  hipStream_t s = (hipStream_t)stream;
+  if (p.tile == 0) return launch_sums<64, 256, 1, 4>(A, B, P, M, N, K, p, s);
+  if (p.tile == 1) return launch_sums<128, 128, 2, 2>(A, B, P, M, N, K, p, s);
+  return launch_sums<256, 256, 2, 2>(A, B, P, M, N, K, p, s);
+}
+
+}  // extern "C"

@@ -1,0 +1,23 @@
+#pragma once
+// bf16 GEMMs on k-contiguous weights ([N][K], the orientation a checkpoint holds), with an optional
+// activation in the epilogue: what the layer-stack pipeline's projections run on.  Same tiles, split-K
+// plans and kernels as the fp16 entries.
+#include "gemm_impl.h"
+
+template <class E>
+static int gemm_nk_entry(const char* who, const uint16_t* A, const uint16_t* B, uint16_t* D, int M, int N, int K,
+                         void* workspace, size_t workspace_bytes, nf_stream_t stream) {
+  int rc = check_gemm_args(who, A, B, D, M, N, K);
+  if (rc) return rc;
+  if (M == 0) return NF_OK;
+  hipStream_t s = (hipStream_t)stream;
+  int k_per = 0;
+  const int shares = M <= kTallRows ? splitk_plan(M, N, K, &k_per) : 1;
+  if (shares < 2 || !workspace || workspace_bytes < (size_t)shares * M * N * sizeof(float))
+    return dispatch_plain<E, true>(A, B, nullptr, D, M, N, K, 1.f, 0.f, N, s);
+  NF_REQUIRE((uintptr_t)workspace % 16 == 0, "%s: the workspace must be 16-byte aligned", who);
+  float* P = static_cast<float*>(workspace);
+  if (M <= 64) return launch_splitk<E, 64, 256, 1, 4, true>(A, B, nullptr, D, M, N, K, 1.f, 0.f, N, shares, k_per, P, s);
+  if (M > 256) return launch_splitk<E, 320, 128, 2, 2, true>(A, B, nullptr, D, M, N, K, 1.f, 0.f, N, shares, k_per, P, s);
+  return launch_splitk<E, 128, 128, 2, 2, true>(A, B, nullptr, D, M, N, K, 1.f, 0.f, N, shares, k_per, P, s);
+}

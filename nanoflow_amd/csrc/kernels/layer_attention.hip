@@ -1,0 +1,538 @@
+// Attention of the layer-stack pipeline: per-head norm + rotation + append to the paged cache, and
+// attention over a window with kept first positions and a sink in the softmax, for any head sizes.
+//
+// bf16 (attn_window_kernel, v_mfma_f32_16x16x32_bf16): S^T = K . Q^T, then O^T = V^T . P^T, per
+// (request, kv head, up to 16 of its query heads).  The 16 MFMA columns carry (token, head) pairs.
+//   * The rows of the two 16-key score tiles of a 32-key step are assigned so that a lane ends up with
+//     8 CONSECUTIVE keys of its column -- row 4g + r of tile b is key 8g + 4b + r -- which is the
+//     second product's operand without a permute; V is cached transposed (a value column's 16 positions
+//     of a page are contiguous), so its operand is one 16-byte load as well.  Neither goes through LDS.
+//   * Softmax weights keep 32 bits: P is multiplied as two bf16 terms, P = hi + lo.
+//   * Only the 32-key steps that hold a visible key are visited: those of the kept first positions,
+//     then those of the window.
+//   * decode: one token per request, the wavefronts of a workgroup take every n-th step and merge
+//     (m, l, O) through LDS.  prefill: every wavefront has NB column blocks of its own and walks their
+//     keys; the keys of the next step are requested while the current one is computed.
+// fp32 (attn_rows_kernel): one wavefront per (row, head), every product in 32-bit.
+#include <algorithm>
+#include <cmath>
+
+#include "layer_common.h"
+
+namespace nf {
+
+constexpr int kPage = 16;
+constexpr int kMaxHeadDim = 256;
+
+__host__ __device__ inline size_t kv_page_elements(const nf_kv_layout& kv) {
+  return (size_t)kv.kv_heads * kv.page * (kv.k_pad + kv.v_pad);
+}
+
+// ---------------------------------------------------------------- norm, rotation, append
+// One wavefront per (row, head): query heads, then key heads, then value heads.
+template <class T>
+__global__ __launch_bounds__(256) void qkv_append_kernel(nf_kv_layout kv, const T* __restrict__ proj, int ld, int q_col,
+                                                         int k_col, int v_col, const float* __restrict__ q_norm,
+                                                         const float* __restrict__ k_norm, float eps, nf_rotation rot,
+                                                         T* __restrict__ q_out, T* __restrict__ kv_data,
+                                                         const int32_t* __restrict__ kv_indptr,
+                                                         const int32_t* __restrict__ kv_indices,
+                                                         const int32_t* __restrict__ rev_input_indptr,
+                                                         const int32_t* __restrict__ positions) {
+  __shared__ float row_buf[4][kMaxHeadDim];
+  const int t = blockIdx.x, lane = threadIdx.x & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int job = blockIdx.y * 4 + wave;
+  const int H = kv.heads, G = kv.kv_heads;
+  const int pos = positions[t], req = rev_input_indptr[t];
+  T* page = nullptr;
+  int entry = 0;
+  if (job >= H && job < H + 2 * G) {
+    page = kv_data + (size_t)kv_indices[kv_indptr[req] + pos / kPage] * kv_page_elements(kv);
+    entry = pos % kPage;
+  }
+  const bool is_qk = job < H + G;
+  if (is_qk) {
+    const bool is_q = job < H;
+    const int head = is_q ? job : job - H;
+    const T* src = proj + (size_t)t * ld + (is_q ? q_col : k_col) + (size_t)head * kv.dim;
+    const float* w = is_q ? q_norm : k_norm;
+    float v[kMaxHeadDim / 64];
+    float sq = 0.f;
+#pragma unroll
+    for (int i = 0; i < kMaxHeadDim / 64; ++i) {
+      const int c = i * 64 + lane;
+      v[i] = c < kv.dim ? Act<T>::load(src + c) : 0.f;
+      sq += v[i] * v[i];
+    }
+    if (w) {
+      const float inv = 1.f / sqrtf(wave_sum(sq) / (float)kv.dim + eps);
+#pragma unroll
+      for (int i = 0; i < kMaxHeadDim / 64; ++i) {
+        const int c = i * 64 + lane;
+        if (c < kv.dim) v[i] = v[i] * inv * w[c];
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < kMaxHeadDim / 64; ++i) row_buf[wave][i * 64 + lane] = v[i];
+  }
+  __syncthreads();  // a lane's rotation partner is another lane's element
+  if (is_qk) {
+    const bool is_q = job < H;
+    const int head = is_q ? job : job - H;
+    T* dst = is_q ? q_out + ((size_t)t * H + head) * kv.k_pad : page + ((size_t)head * kPage + entry) * kv.k_pad;
+    const int half = rot.dims / 2;
+#pragma unroll
+    for (int i = 0; i < kMaxHeadDim / 64; ++i) {
+      const int c = i * 64 + lane;
+      if (c >= kv.k_pad) continue;
+      float y = row_buf[wave][c];  // zero past dim
+      if (c < 2 * half) {
+        const int f = rot.interleaved ? c >> 1 : (c < half ? c : c - half);
+        const bool first = rot.interleaved ? !(c & 1) : c < half;
+        const float other = row_buf[wave][rot.interleaved ? c ^ 1 : (first ? c + half : c - half)];
+        const float cs = rot.table[((size_t)pos * half + f) * 2], sn = rot.table[((size_t)pos * half + f) * 2 + 1];
+        y = first ? y * cs - other * sn : y * cs + other * sn;
+      }
+      Act<T>::store(dst + c, y);
+    }
+  } else if (job < H + 2 * G) {
+    const int head = job - H - G;
+    const T* src = proj + (size_t)t * ld + v_col + (size_t)head * kv.vdim;
+    T* dst = page + (size_t)G * kPage * kv.k_pad + (size_t)head * kv.v_pad * kPage + entry;
+    for (int c = lane; c < kv.v_pad; c += 64) Act<T>::store(dst + (size_t)c * kPage, c < kv.vdim ? Act<T>::load(src + c) : 0.f);
+  }
+}
+
+// ---------------------------------------------------------------- which 32-key (or 64-key) steps are visited
+struct StepRange {
+  int head, skip_to, total;  // steps [0, head), then [skip_to, ...): `total` of both
+  __device__ __forceinline__ int at(int i) const { return i < head ? i : skip_to + i - head; }
+};
+// The steps of `width` keys in which a token at a position in [p0, p1] sees a key.
+__device__ __forceinline__ StepRange visible_steps(int p0, int p1, int window, int keep_first, int width) {
+  const int end = p1 / width + 1;
+  if (window <= 0) return {0, 0, end};
+  const int kept = keep_first > p1 + 1 ? p1 + 1 : keep_first;
+  const int head = (kept + width - 1) / width;
+  const int lo = p0 - window + 1;
+  int skip_to = lo > 0 ? lo / width : 0;
+  if (skip_to < head) skip_to = head;
+  return {head, skip_to, head + (end > skip_to ? end - skip_to : 0)};
+}
+
+__device__ __forceinline__ bool sees(int p, int j, int window, int keep_first) {
+  return j <= p && (window <= 0 || p - j < window || j < keep_first);
+}
+
+// ---------------------------------------------------------------- fp32
+template <class T>
+__global__ __launch_bounds__(64) void attn_rows_kernel(nf_window_attention_args a) {
+  __shared__ __attribute__((aligned(16))) float sq[kMaxHeadDim];
+  __shared__ float sp[64];
+  const nf_kv_layout kv = a.kv;
+  const int lane = threadIdx.x, t = a.row_begin + blockIdx.x, h = blockIdx.y;
+  const int req = a.rev_input_indptr[t], p = a.positions[t];
+  const int g = h / (kv.heads / kv.kv_heads);
+  const T* q = (const T*)a.q + ((size_t)t * kv.heads + h) * kv.k_pad;
+  for (int c = lane; c < kv.k_pad; c += 64) sq[c] = Act<T>::load(q + c);
+  __syncthreads();
+  const T* pool = (const T*)a.kv_data;
+  const size_t page_elems = kv_page_elements(kv);
+  const int32_t* pages = a.kv_indices + a.kv_indptr[req];
+  float m = a.sink ? a.sink[h] : -1e30f;
+  float l = 0.f;  // this lane's part of the denominator
+  float o[kMaxHeadDim / 64] = {};
+  const StepRange steps = visible_steps(p, p, a.window, a.keep_first, 64);
+  for (int i = 0; i < steps.total; ++i) {
+    const int base = steps.at(i) * 64, j = base + lane;
+    const bool see = sees(p, j, a.window, a.keep_first);
+    float s = -INFINITY;
+    if (see) {
+      const T* k = pool + (size_t)pages[j / kPage] * page_elems + ((size_t)g * kPage + j % kPage) * kv.k_pad;
+      float dot = 0.f;
+      for (int c = 0; c < kv.k_pad; c += 4) {
+        const float4_t kk = Act<T>::load4(k + c), qq = *reinterpret_cast<const float4_t*>(sq + c);
+        dot += kk[0] * qq[0] + kk[1] * qq[1] + kk[2] * qq[2] + kk[3] * qq[3];
+      }
+      s = dot * a.scale;
+    }
+    float mx = s;
+#pragma unroll
+    for (int d = 32; d > 0; d >>= 1) mx = fmaxf(mx, __shfl_xor(mx, d, 64));
+    const float m_new = fmaxf(m, mx), alpha = expf(m - m_new);
+    const float w = see ? expf(s - m_new) : 0.f;
+    m = m_new;
+    l = l * alpha + w;
+    __syncthreads();
+    sp[lane] = w;
+    __syncthreads();
+#pragma unroll
+    for (int e = 0; e < kMaxHeadDim / 64; ++e) o[e] *= alpha;
+    const int n_pages = min(4, (p - base) / kPage + 1);
+    for (int b = 0; b < n_pages; ++b) {
+      const T* v = pool + (size_t)pages[base / kPage + b] * page_elems + (size_t)kv.kv_heads * kPage * kv.k_pad +
+                   (size_t)g * kv.v_pad * kPage;
+#pragma unroll
+      for (int e = 0; e < kMaxHeadDim / 64; ++e) {
+        const int c = e * 64 + lane;
+        if (c >= kv.v_pad) break;
+#pragma unroll
+        for (int r = 0; r < kPage; r += 4) {
+          const float4_t vv = Act<T>::load4(v + (size_t)c * kPage + r);
+#pragma unroll
+          for (int x = 0; x < 4; ++x) {
+            const float wt = sp[b * kPage + r + x];
+            if (wt != 0.f) o[e] += wt * vv[x];  // an entry past the sequence may hold anything
+          }
+        }
+      }
+    }
+  }
+  l = wave_sum(l);
+  if (a.sink) l += expf(a.sink[h] - m);
+  const float inv = a.out_scale / l;
+  T* out = (T*)a.out + (size_t)t * a.out_ld + a.out_col + (size_t)h * kv.vdim;
+#pragma unroll
+  for (int e = 0; e < kMaxHeadDim / 64; ++e) {
+    const int c = e * 64 + lane;
+    if (c < kv.vdim) Act<T>::store(out + c, o[e] * inv);
+  }
+}
+
+// ---------------------------------------------------------------- bf16
+typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
+union B8 {
+  u32x4 u;
+  bf16x8_t b;
+  uint32_t w[4];
+};
+
+template <bool kStream>
+__device__ __forceinline__ u32x4 load_cache(const bf16_t* p) {
+  typedef uint32_t v4 __attribute__((ext_vector_type(4)));
+  if constexpr (kStream) {  // decode reads every cached byte once
+    const v4 x = __builtin_nontemporal_load(reinterpret_cast<const v4*>(p));
+    return u32x4{x.x, x.y, x.z, x.w};
+  } else {
+    return *reinterpret_cast<const u32x4*>(p);
+  }
+}
+
+// KD: 32-wide pieces of k_pad, VD: 16-wide pieces of v_pad (both upper bounds), NB: column blocks per
+// wavefront.  gs: query heads of a kv head in one workgroup (at most 16).
+template <int KD, int VD, int NB, bool kDecode>
+__global__ __launch_bounds__(512) void attn_window_kernel(nf_window_attention_args a, int gs, int chunks, int tile_tokens) {
+  extern __shared__ __attribute__((aligned(16))) float merge_lds[];
+  const nf_kv_layout kv = a.kv;
+  const int lane = threadIdx.x & 63, l16 = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int waves = blockDim.x >> 6;
+  const int group = kv.heads / kv.kv_heads;
+  const int kvh = blockIdx.y / chunks, h0 = (blockIdx.y % chunks) * gs;  // this workgroup's heads: kvh * group + h0 ...
+  const int heads = min(gs, group - h0);
+  const int tpb = 16 / gs;  // tokens per column block
+
+  int req, row0, tok0, len;  // request, its first row, this wavefront's first token in it, its rows
+  if constexpr (kDecode) {
+    req = a.req_begin + blockIdx.x;
+    row0 = a.input_indptr[req];
+    tok0 = 0;
+    len = 1;
+  } else {
+    int tile = blockIdx.x;
+    req = -1;
+    for (int r = a.req_begin; r < a.req_begin + a.req_num; ++r) {
+      const int n = (a.input_indptr[r + 1] - a.input_indptr[r] + tile_tokens - 1) / tile_tokens;
+      if (tile < n) {
+        req = r;
+        tile = n - 1 - tile;  // the tiles that see most keys start first
+        break;
+      }
+      tile -= n;
+    }
+    if (req < 0) return;
+    row0 = a.input_indptr[req];
+    len = a.input_indptr[req + 1] - row0;
+    tok0 = tile * tile_tokens + wave * NB * tpb;
+    if (tok0 >= len) return;
+  }
+
+  int pos[NB], row[NB];
+  bool live[NB];
+  B8 qf[NB][KD];
+  const int kd = kv.k_pad / 32, vd = kv.v_pad / 16;
+#pragma unroll
+  for (int n = 0; n < NB; ++n) {
+    const int tok = kDecode ? 0 : tok0 + n * tpb + l16 / gs, hc = l16 % gs;
+    live[n] = (kDecode ? l16 < heads : l16 < tpb * gs && tok < len && hc < heads);
+    row[n] = row0 + (live[n] ? tok : (kDecode ? 0 : tok0));
+    pos[n] = a.positions[row[n]];
+    const bf16_t* q = (const bf16_t*)a.q + ((size_t)row[n] * kv.heads + kvh * group + h0 + (live[n] ? hc : 0)) * kv.k_pad + g * 8;
+#pragma unroll
+    for (int j = 0; j < KD; ++j) qf[n][j].u = live[n] && j < kd ? *reinterpret_cast<const u32x4*>(q + j * 32) : u32x4{0, 0, 0, 0};
+  }
+  const int p0 = a.positions[row0 + tok0];
+  const int p1 = kDecode ? p0 : p0 + min(NB * tpb, len - tok0) - 1;
+  const StepRange steps = visible_steps(p0, p1, a.window, a.keep_first, 32);
+
+  const size_t page_elems = kv_page_elements(kv);
+  const int32_t* pages = a.kv_indices + a.kv_indptr[req];
+  const int last_page = p1 / kPage;
+  const bf16_t* pool = (const bf16_t*)a.kv_data;
+  // this lane's pieces inside a page: K rows of tile b (b = 0, 1), V column piece
+  const int key = 8 * (l16 >> 2) + (l16 & 3);  // of tile 0 in the step; tile 1: + 4
+  const int kpg = key >> 4;                    // its page of the step's two (tile 1's is the same)
+  const size_t k_off0 = ((size_t)kvh * kPage + (key & 15)) * kv.k_pad + g * 8;
+  const size_t k_off1 = k_off0 + (size_t)4 * kv.k_pad;
+  const size_t v_off = (size_t)kv.kv_heads * kPage * kv.k_pad + ((size_t)kvh * kv.v_pad + l16) * kPage + (g & 1) * 8;
+  const int vpg = g >> 1;
+
+  float4_t o[NB][VD];
+  float m[NB], l[NB];
+#pragma unroll
+  for (int n = 0; n < NB; ++n) {
+    m[n] = -1e30f;
+    l[n] = 0.f;
+#pragma unroll
+    for (int i = 0; i < VD; ++i) o[n][i] = float4_t{0.f, 0.f, 0.f, 0.f};
+  }
+  const float scale2 = a.scale * 1.44269504088896340736f;
+
+  auto page_ptr = [&](int step, int which) {
+    int idx = step * 2 + which;
+    if (idx > last_page) idx = last_page;  // its keys are past every token of the tile: read something mapped
+    return pool + (size_t)pages[idx] * page_elems;
+  };
+  B8 kf[2][KD];
+  auto load_k = [&](int step) {
+    const bf16_t* k = page_ptr(step, kpg);
+#pragma unroll
+    for (int j = 0; j < KD; ++j)
+      if (j < kd) {
+        kf[0][j].u = load_cache<kDecode>(k + k_off0 + j * 32);
+        kf[1][j].u = load_cache<kDecode>(k + k_off1 + j * 32);
+      }
+  };
+  const int first = kDecode ? wave : 0, stride = kDecode ? waves : 1;
+  if (first < steps.total) load_k(steps.at(first));
+  for (int it = first; it < steps.total; it += stride) {
+    const int step = steps.at(it), base = step * 32;
+    // V of this step, then (after the scores) K of the next: in flight while the softmax runs
+    B8 vf[VD];
+    const bf16_t* v = page_ptr(step, vpg) + v_off;
+#pragma unroll
+    for (int i = 0; i < VD; ++i)
+      if (i < vd) vf[i].u = load_cache<kDecode>(v + (size_t)i * 16 * kPage);
+    float4_t s[NB][2];
+#pragma unroll
+    for (int n = 0; n < NB; ++n)
+#pragma unroll
+      for (int b = 0; b < 2; ++b) {
+        s[n][b] = float4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int j = 0; j < KD; ++j)
+          if (j < kd) s[n][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[b][j].b, qf[n][j].b, s[n][b], 0, 0, 0);
+      }
+    if (it + stride < steps.total) load_k(steps.at(it + stride));
+    const bool whole = base + 31 <= p0 && (a.window <= 0 || p1 - base < a.window || base + 31 < a.keep_first);
+#pragma unroll
+    for (int n = 0; n < NB; ++n) {
+      const int j0 = base + 8 * g;
+      float mx = -1e30f;
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          s[n][b][r] *= scale2;
+          if (!whole && !sees(pos[n], j0 + 4 * b + r, a.window, a.keep_first)) s[n][b][r] = -INFINITY;
+          mx = fmaxf(mx, s[n][b][r]);
+        }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      if (__any(mx > m[n])) {
+        const float m_new = fmaxf(m[n], mx), alpha = __builtin_amdgcn_exp2f(m[n] - m_new);
+        m[n] = m_new;
+        l[n] *= alpha;
+#pragma unroll
+        for (int i = 0; i < VD; ++i) o[n][i] *= alpha;
+      }
+      B8 hi, lo;
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int r = 0; r < 4; r += 2) {
+          const float w0 = __builtin_amdgcn_exp2f(s[n][b][r] - m[n]), w1 = __builtin_amdgcn_exp2f(s[n][b][r + 1] - m[n]);
+          l[n] += w0 + w1;
+          const uint32_t h2 = f32_to_bf16_pair(w0, w1);
+          hi.w[b * 2 + r / 2] = h2;
+          lo.w[b * 2 + r / 2] = f32_to_bf16_pair(w0 - __uint_as_float(h2 << 16), w1 - __uint_as_float(h2 & 0xffff0000u));
+        }
+#pragma unroll
+      for (int i = 0; i < VD; ++i)
+        if (i < vd) {
+          o[n][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[i].b, hi.b, o[n][i], 0, 0, 0);
+          o[n][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[i].b, lo.b, o[n][i], 0, 0, 0);
+        }
+    }
+  }
+
+  bf16_t* out = (bf16_t*)a.out;
+#pragma unroll
+  for (int n = 0; n < NB; ++n) {
+    l[n] += __shfl_xor(l[n], 16, 64);
+    l[n] += __shfl_xor(l[n], 32, 64);
+  }
+  if constexpr (kDecode) {
+    // merge the wavefronts: m and l of [wave][16 columns], O of [wave][heads][v_pad]
+    float* sm = merge_lds;
+    float* sl = sm + waves * 16;
+    float* so = sl + waves * 16;
+    if (g == 0) {
+      sm[wave * 16 + l16] = m[0];
+      sl[wave * 16 + l16] = l[0];
+    }
+    if (l16 < heads)
+#pragma unroll
+      for (int i = 0; i < VD; ++i)
+        if (i < vd) *reinterpret_cast<float4_t*>(so + ((size_t)wave * gs + l16) * kv.v_pad + i * 16 + g * 4) = o[0][i];
+    __syncthreads();
+    for (int e = threadIdx.x; e < heads * kv.vdim; e += blockDim.x) {
+      const int hc = e / kv.vdim, c = e % kv.vdim;
+      const int h = kvh * group + h0 + hc;
+      const float snk = a.sink ? a.sink[h] * 1.44269504088896340736f : -1e30f;
+      float mm = snk;
+      for (int w = 0; w < waves; ++w) mm = fmaxf(mm, sm[w * 16 + hc]);
+      float den = a.sink ? __builtin_amdgcn_exp2f(snk - mm) : 0.f, acc = 0.f;
+      for (int w = 0; w < waves; ++w) {
+        const float f = __builtin_amdgcn_exp2f(sm[w * 16 + hc] - mm);
+        den += sl[w * 16 + hc] * f;
+        acc += so[((size_t)w * gs + hc) * kv.v_pad + c] * f;
+      }
+      Act<bf16_t>::store(out + (size_t)row0 * a.out_ld + a.out_col + (size_t)h * kv.vdim + c, acc * (a.out_scale / den));
+    }
+  } else {
+#pragma unroll
+    for (int n = 0; n < NB; ++n) {
+      if (!live[n]) continue;
+      const int h = kvh * group + h0 + l16 % gs;
+      float den = l[n], f = 1.f;
+      if (a.sink) {
+        const float snk = a.sink[h] * 1.44269504088896340736f, mm = fmaxf(m[n], snk);
+        f = __builtin_amdgcn_exp2f(m[n] - mm);
+        den = den * f + __builtin_amdgcn_exp2f(snk - mm);
+      }
+      const float inv = f * a.out_scale / den;
+      bf16_t* dst = out + (size_t)row[n] * a.out_ld + a.out_col + (size_t)h * kv.vdim;
+      const bool vec = (kv.vdim | a.out_ld | a.out_col) % 4 == 0;
+#pragma unroll
+      for (int i = 0; i < VD; ++i) {
+        const int c = i * 16 + g * 4;
+        if (i >= vd || c >= kv.vdim) continue;
+        if (vec) {
+          Act<bf16_t>::store4(dst + c, o[n][i] * inv);
+        } else {
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            if (c + r < kv.vdim) Act<bf16_t>::store(dst + c + r, o[n][i][r] * inv);
+        }
+      }
+    }
+  }
+}
+
+template <int KD, int VD>
+static int launch_window(const nf_window_attention_args& a, hipStream_t s) {
+  const int group = a.kv.heads / a.kv.kv_heads;
+  // a kv head's query heads in chunks of at most 16, as equal as possible
+  const int chunks = (group + 15) / 16, gs = (group + chunks - 1) / chunks;
+  const unsigned gy = (unsigned)(a.kv.kv_heads * chunks);
+  if (a.decode) {
+    auto lds_of = [&](int w) { return (size_t)w * (32 + (size_t)gs * a.kv.v_pad) * sizeof(float); };
+    int waves = (long long)a.req_num * gy >= 512 ? 4 : 8;
+    while (waves > 1 && lds_of(waves) > 64 * 1024) waves /= 2;
+    attn_window_kernel<KD, VD, 1, true><<<dim3((unsigned)a.req_num, gy), waves * 64, lds_of(waves), s>>>(a, gs, chunks, 0);
+    return check_launch("nf_window_attention (decode)");
+  }
+  constexpr int NB = KD <= 4 ? 2 : 1;
+  const int tile_tokens = 4 * NB * (16 / gs);
+  const unsigned tiles = (unsigned)(a.max_rows / tile_tokens + a.req_num);
+  attn_window_kernel<KD, VD, NB, false><<<dim3(tiles, gy), 256, 0, s>>>(a, gs, chunks, tile_tokens);
+  return check_launch("nf_window_attention (prefill)");
+}
+
+}  // namespace nf
+
+using namespace nf;
+
+static int check_layout(const char* who, const nf_kv_layout& kv) {
+  NF_REQUIRE(kv.dtype == NF_F32 || kv.dtype == NF_BF16, "%s: unknown dtype %d", who, kv.dtype);
+  NF_REQUIRE(kv.heads > 0 && kv.kv_heads > 0 && kv.heads % kv.kv_heads == 0, "%s: %d query heads over %d kv heads", who,
+             kv.heads, kv.kv_heads);
+  NF_REQUIRE(kv.page == kPage && kv.dim > 0 && kv.vdim > 0 && kv.dim <= kMaxHeadDim && kv.vdim <= kMaxHeadDim &&
+                 kv.k_pad == (kv.dim + 31) / 32 * 32 && kv.v_pad == (kv.vdim + 15) / 16 * 16,
+             "%s: page %d, dim %d (pad %d), vdim %d (pad %d): pages of 16, head sizes up to %d", who, kv.page, kv.dim,
+             kv.k_pad, kv.vdim, kv.v_pad, kMaxHeadDim);
+  return NF_OK;
+}
+
+extern "C" {
+
+size_t nf_kv_page_elements(const nf_kv_layout* kv) { return kv ? kv_page_elements(*kv) : 0; }
+
+int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, int k_col, int v_col, const float* q_norm,
+                  const float* k_norm, float eps, const nf_rotation* rot, void* q_out, void* kv_data,
+                  const int32_t* kv_indptr, const int32_t* kv_indices, const int32_t* rev_input_indptr,
+                  const int32_t* positions, int rows, nf_stream_t stream) {
+  const char* who = "nf_qkv_append";
+  NF_REQUIRE(kv && rot, "%s: null pointer", who);
+  int rc = check_layout(who, *kv);
+  if (rc) return rc;
+  NF_REQUIRE(rot->dims >= 0 && rot->dims % 2 == 0 && rot->dims <= kv->dim && (rot->dims == 0 || rot->table),
+             "%s: %d of %d dimensions rotated", who, rot->dims, kv->dim);
+  NF_REQUIRE(rows >= 0 && q_col >= 0 && k_col >= 0 && v_col >= 0 && q_col + kv->heads * kv->dim <= ld &&
+                 k_col + kv->kv_heads * kv->dim <= ld && v_col + kv->kv_heads * kv->vdim <= ld,
+             "%s: columns %d %d %d do not fit rows of %d", who, q_col, k_col, v_col, ld);
+  if (rows == 0) return NF_OK;
+  NF_REQUIRE(proj && q_out && kv_data && kv_indptr && kv_indices && rev_input_indptr && positions, "%s: null pointer", who);
+  const dim3 grid((unsigned)rows, (unsigned)((kv->heads + 2 * kv->kv_heads + 3) / 4));
+  hipStream_t s = (hipStream_t)stream;
+  if (kv->dtype == NF_BF16)
+    qkv_append_kernel<bf16_t><<<grid, 256, 0, s>>>(*kv, (const bf16_t*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot,
+                                                   (bf16_t*)q_out, (bf16_t*)kv_data, kv_indptr, kv_indices, rev_input_indptr,
+                                                   positions);
+  else
+    qkv_append_kernel<float><<<grid, 256, 0, s>>>(*kv, (const float*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot,
+                                                  (float*)q_out, (float*)kv_data, kv_indptr, kv_indices, rev_input_indptr,
+                                                  positions);
+  return check_launch(who);
+}
+
+int nf_window_attention(const nf_window_attention_args* args, nf_stream_t stream) {
+  const char* who = "nf_window_attention";
+  NF_REQUIRE(args, "%s: null pointer", who);
+  const nf_window_attention_args& a = *args;
+  int rc = check_layout(who, a.kv);
+  if (rc) return rc;
+  NF_REQUIRE(a.req_num >= 0 && a.req_begin >= 0 && a.max_rows >= 0 && a.row_begin >= 0 && a.keep_first >= 0,
+             "%s: requests %d + %d, rows %d + %d, keep_first %d", who, a.req_begin, a.req_num, a.row_begin, a.max_rows,
+             a.keep_first);
+  NF_REQUIRE(a.out_col >= 0 && a.out_col + a.kv.heads * a.kv.vdim <= a.out_ld, "%s: output columns %d + %d of %d", who,
+             a.out_col, a.kv.heads * a.kv.vdim, a.out_ld);
+  NF_REQUIRE(!a.decode || a.max_rows == a.req_num, "%s: %d decode requests with %d rows", who, a.req_num, a.max_rows);
+  if (a.req_num == 0 || a.max_rows == 0) return NF_OK;
+  NF_REQUIRE(a.q && a.out && a.kv_data && a.input_indptr && a.kv_indptr && a.kv_indices && a.rev_input_indptr && a.positions,
+             "%s: null pointer", who);
+  hipStream_t s = (hipStream_t)stream;
+  if (a.kv.dtype == NF_F32) {
+    NF_REQUIRE(a.kv.heads <= 65535, "%s: %d heads exceed the grid", who, a.kv.heads);
+    attn_rows_kernel<float><<<dim3((unsigned)a.max_rows, (unsigned)a.kv.heads), 64, 0, s>>>(a);
+    return check_launch(who);
+  }
+  const int kd = a.kv.k_pad / 32, vd = a.kv.v_pad / 16;
+  if (kd <= 2 && vd <= 4) return launch_window<2, 4>(a, s);
+  if (kd <= 4 && vd <= 8) return launch_window<4, 8>(a, s);
+  return launch_window<8, 16>(a, s);
+}
+
+}  // extern "C"

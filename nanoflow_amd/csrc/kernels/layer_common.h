@@ -1,0 +1,57 @@
+#pragma once
+// Helpers of the layer-stack operators: activations in fp32 or bf16, arithmetic in fp32.
+#include "common.h"
+
+namespace nf {
+
+struct bf16_t {
+  uint16_t bits;
+};
+
+__device__ __forceinline__ float bf16_bits_to_f32(uint32_t b) { return __uint_as_float(b << 16); }
+__device__ __forceinline__ uint32_t f32_to_bf16_pair(float lo, float hi) {  // round to nearest even
+  typedef float f32x2_t __attribute__((ext_vector_type(2)));
+  typedef __bf16 bf16x2_t __attribute__((ext_vector_type(2)));
+  return __builtin_bit_cast(uint32_t, __builtin_convertvector(f32x2_t{lo, hi}, bf16x2_t));
+}
+
+template <class T>
+struct Act;
+template <>
+struct Act<float> {
+  static constexpr int dtype = NF_F32;
+  static __device__ __forceinline__ float load(const float* p) { return *p; }
+  static __device__ __forceinline__ void store(float* p, float v) { *p = v; }
+  static __device__ __forceinline__ float4_t load4(const float* p) { return *reinterpret_cast<const float4_t*>(p); }
+  static __device__ __forceinline__ void store4(float* p, float4_t v) { *reinterpret_cast<float4_t*>(p) = v; }
+};
+template <>
+struct Act<bf16_t> {
+  static constexpr int dtype = NF_BF16;
+  static __device__ __forceinline__ float load(const bf16_t* p) { return bf16_bits_to_f32(p->bits); }
+  static __device__ __forceinline__ void store(bf16_t* p, float v) { p->bits = (uint16_t)(f32_to_bf16_pair(v, 0.f) & 0xffffu); }
+  static __device__ __forceinline__ float4_t load4(const bf16_t* p) {
+    const u32x2 w = *reinterpret_cast<const u32x2*>(p);
+    return float4_t{bf16_bits_to_f32(w.x & 0xffffu), __uint_as_float(w.x & 0xffff0000u), bf16_bits_to_f32(w.y & 0xffffu),
+                    __uint_as_float(w.y & 0xffff0000u)};
+  }
+  static __device__ __forceinline__ void store4(bf16_t* p, float4_t v) {
+    *reinterpret_cast<u32x2*>(p) = u32x2{f32_to_bf16_pair(v[0], v[1]), f32_to_bf16_pair(v[2], v[3])};
+  }
+};
+
+__device__ __forceinline__ float silu_f32(float g) { return g / (1.f + expf(-g)); }
+
+// Sum over a workgroup of up to 1024 threads; every thread gets it.  `scratch`: 16 floats of LDS that
+// no one else touches between the caller's last barrier and its next one.
+__device__ __forceinline__ float block_sum(float v, float* scratch) {
+  v = wave_sum(v);
+  const int waves = (blockDim.x + 63) >> 6;
+  if ((threadIdx.x & 63) == 0) scratch[threadIdx.x >> 6] = v;
+  __syncthreads();
+  float s = 0.f;
+  for (int w = 0; w < waves; ++w) s += scratch[w];
+  return s;
+}
+
+}  // namespace nf

@@ -8,15 +8,6 @@
 
 namespace nf {
 
-static thread_local char g_err[512] = "";
-
-void set_error(const char* fmt, ...) {
-  va_list ap;
-  va_start(ap, fmt);
-  vsnprintf(g_err, sizeof(g_err), fmt, ap);
-  va_end(ap);
-}
-
 // ---------------------------------------------------------------- row gathers
 
 // out[r,:] = src[row_of(r),:]; one workgroup per output row.
@@ -380,8 +371,6 @@ using namespace nf;
 
 extern "C" {
 
-int nf_abi_version(void) { return 1; }
-const char* nf_last_error(void) { return nf::g_err; }
 
 int nf_embedding_f16(const int32_t* tokens, const uint16_t* table, uint16_t* out, int n_tokens,
                      int hidden, nf_stream_t stream) {

@@ -1,0 +1,176 @@
+"""Plain, slow float64 restatement of the layer-stack designs (decoders put together from a list of
+layers: retention, windowed attention with kept first tokens and a sink, a token-shift recurrence with
+data-dependent decay, two mixers side by side).  Test infrastructure only: one function per mechanism,
+whole sequences at once, nothing shared with the product path.
+
+A model is (config, tensors): the parsed config.json and a dict name -> numpy array (any float type).
+Nothing is cached between calls and every token sees the whole sequence before it, so this says what
+the logits are whatever way a serving engine cuts the tokens up.
+"""
+from __future__ import annotations
+
+import numpy as np
+
+
+def f64(a):
+    return np.asarray(a, dtype=np.float64)
+
+
+def rms_norm(x, eps, w=None):
+    y = x / np.sqrt((x * x).mean(axis=-1, keepdims=True) + eps)
+    return y if w is None else y * f64(w)
+
+
+def sigmoid(z):
+    return 0.5 * (1.0 + np.tanh(0.5 * z))
+
+
+def silu(z):
+    return z * sigmoid(z)
+
+
+def squared_relu(z):
+    return np.maximum(z, 0.0) ** 2
+
+
+def rotate(x, positions, dims, base, interleaved):
+    """x [T, heads, d]; the first `dims` of d are turned by position * base^(-2i/dims), in pairs
+    (i, i + dims/2), or (2i, 2i + 1) when interleaved."""
+    if dims == 0:
+        return x.copy()
+    half = dims // 2
+    i = np.arange(half, dtype=np.float64)
+    angle = f64(positions)[:, None] * f64(base) ** (-2.0 * i / dims)       # [T, half]
+    c, s = np.cos(angle)[:, None, :], np.sin(angle)[:, None, :]
+    first, second = (2 * np.arange(half), 2 * np.arange(half) + 1) if interleaved else \
+        (np.arange(half), np.arange(half) + half)
+    u, v = x[..., first], x[..., second]
+    out = x.copy()
+    out[..., first] = u * c - v * s
+    out[..., second] = v * c + u * s
+    return out
+
+
+def window_mask(T, size, keep_first):
+    """[T, T] bool: does position i see position j."""
+    i, j = np.arange(T)[:, None], np.arange(T)[None, :]
+    return (j <= i) & ((i - j < size) | (j < keep_first))
+
+
+def sink_attention(q, k, v, mask, scale, sink):
+    """q [T, H, d], k [T, G, d], v [T, G, e], sink [H] (or None): softmax whose denominator also
+    holds exp(sink)."""
+    T, H, _ = q.shape
+    per = H // k.shape[1]
+    out = np.empty((T, H, v.shape[-1]))
+    for h in range(H):
+        s = np.where(mask, (q[:, h] @ k[:, h // per].T) * scale, -np.inf)
+        m = s.max(axis=1, keepdims=True)
+        if sink is not None:
+            m = np.maximum(m, f64(sink)[h])
+        p = np.exp(s - m)
+        den = p.sum(axis=1, keepdims=True)
+        if sink is not None:
+            den = den + np.exp(f64(sink)[h] - m)
+        out[:, h] = (p / den) @ v[:, h // per]
+    return out
+
+
+def fixed_decay_recurrence(q, k, v, decay):
+    """Per head: the state fades by a constant, takes in key (x) value, and is then read by the query."""
+    T, H, d = q.shape
+    S = np.zeros((H, d, v.shape[-1]))
+    out = np.empty((T, H, v.shape[-1]))
+    g = f64(decay)[:, None, None]
+    for t in range(T):
+        S = g * S + k[t][:, :, None] * v[t][:, None, :]
+        out[t] = np.einsum("hkv,hk->hv", S, q[t])
+    return out
+
+
+def bonus_recurrence(r, k, v, w, u):
+    """Per head: the state is read first, with the current key weighted by u; then each of its rows fades
+    by the token's own factor and takes in key (x) value."""
+    T, H, d = r.shape
+    S = np.zeros((H, d, v.shape[-1]))
+    out = np.empty((T, H, v.shape[-1]))
+    for t in range(T):
+        kv = k[t][:, :, None] * v[t][:, None, :]
+        out[t] = np.einsum("hkv,hk->hv", S + f64(u)[:, :, None] * kv, r[t])
+        S = w[t][:, :, None] * S + kv
+    return out
+
+
+def previous_token(h):
+    return np.concatenate([np.zeros_like(h[:1]), h[:-1]], axis=0)
+
+
+def linear(t, name, x):
+    return x @ f64(t[name]).T
+
+
+def retention_mixer(t, pre, m, eps, h, positions):
+    T, H = h.shape[0], m["heads"]
+    q = linear(t, pre + "q", h).reshape(T, H, m["dim"])
+    k = linear(t, pre + "k", h).reshape(T, H, m["dim"])
+    v = linear(t, pre + "v", h).reshape(T, H, m["vdim"])
+    rot = m["rot"]
+    q = rotate(q, positions, rot["dims"], rot["base"], False)
+    k = rotate(k, positions, rot["dims"], rot["base"], False) * m["dim"] ** -0.5
+    o = rms_norm(fixed_decay_recurrence(q, k, v, m["decay"]), eps).reshape(T, -1)
+    return linear(t, pre + "o", o * silu(linear(t, pre + "g", h)))
+
+
+def window_attention_mixer(t, pre, m, eps, h, positions):
+    T, H, G = h.shape[0], m["heads"], m["kv_heads"]
+    q = linear(t, pre + "q", h).reshape(T, H, m["dim"])
+    k = linear(t, pre + "k", h).reshape(T, G, m["dim"])
+    v = linear(t, pre + "v", h).reshape(T, G, m["vdim"])
+    rot = m["rot"]
+    q = rotate(rms_norm(q, eps, t[pre + "q.norm"]), positions, rot["dims"], rot["base"], True)
+    k = rotate(rms_norm(k, eps, t[pre + "k.norm"]), positions, rot["dims"], rot["base"], True)
+    mask = window_mask(T, m["mask"]["size"], m["mask"]["keep_first"])
+    o = sink_attention(q, k, v, mask, m["scale"], t[pre + "sink"])
+    return linear(t, pre + "o", o.reshape(T, -1))
+
+
+def token_shift_mixer(t, pre, m, eps, h):
+    T, H, d = h.shape[0], m["heads"], m["dim"]
+    prev = previous_token(h)
+    mix = {s: h + (prev - h) * f64(t[pre + "mu." + s]) for s in "rkvgw"}
+    r, k, v = (linear(t, pre + s, mix[s]).reshape(T, H, d) for s in "rkv")
+    gate = silu(linear(t, pre + "g", mix["g"]))
+    z = linear(t, pre + "w2", np.tanh(linear(t, pre + "w1", mix["w"]))) + f64(t[pre + "w0"])
+    w = np.exp(-np.exp(z)).reshape(T, H, d)
+    o = rms_norm(bonus_recurrence(r, k, v, w, t[pre + "u"]), eps).reshape(T, -1)
+    return linear(t, pre + "o", o * f64(t[pre + "norm"]) * gate)
+
+
+def mixer(t, pre, kind, m, eps, h, positions):
+    if kind == "retention":
+        return retention_mixer(t, pre, m, eps, h, positions)
+    assert kind == "parallel", kind
+    return (m["left_scale"] * window_attention_mixer(t, pre + "left.", m["left"], eps, h, positions)
+            + m["right_scale"] * token_shift_mixer(t, pre + "right.", m["right"], eps, h))
+
+
+def feed_forward(t, pre, m, h):
+    assert m["kind"] == "dense", m
+    return linear(t, pre + "down", squared_relu(linear(t, pre + "up", h)))
+
+
+def forward(cfg, t, tokens, want_layers=False):
+    """Logits [T, vocab] of a whole sequence (and the residual stream after every layer)."""
+    tokens = np.asarray(tokens)
+    positions = np.arange(len(tokens))
+    eps = cfg["norm"]["eps"]
+    x = f64(t["embed"])[tokens] + f64(t["pos"])[positions]
+    layers = []
+    for i, layer in enumerate(cfg["layers"]):
+        pre = f"l{i}."
+        x = x + rms_norm(mixer(t, pre + "mix.", layer["type"], layer["mixer"], eps, x, positions), eps, t[pre + "norm1"])
+        if layer.get("mlp"):
+            x = x + rms_norm(feed_forward(t, pre + "mlp.", layer["mlp"], x), eps, t[pre + "norm2"])
+        layers.append(x)
+    logits = linear(t, "head", rms_norm(x, eps, t["final.norm"]))
+    return (logits, np.stack(layers)) if want_layers else logits

@@ -293,3 +293,77 @@ class Engine:
 
     def __exit__(self, *exc):
         self.close()
+
+
+class StackEngine:
+    """One layer-stack pipeline on cuda:0 (nanoflow_pllm.h, pllm_stack_*).  ``model``: a configuration (dict,
+    config.json, or a directory with one); ``weights``: a directory with model.safetensors, a dict of host arrays, or
+    None for random ones.  The caches, states and buffers are the library's own."""
+
+    def __init__(self, model, *, dtype="bfloat16", global_batch=2048, kv_pages=1024, state_slots=64, weights=None, seed=0,
+                 keep_layers=False, rank=16):
+        from . import stack_models
+        self.cfg = stack_models.load_config(model)
+        self.dtype, self.T, self.kv_pages, self.state_slots = dtype, global_batch, kv_pages, state_slots
+        self._open = False
+        fd, path = tempfile.mkstemp(suffix=".json", prefix="nanoflow_stack_")
+        with os.fdopen(fd, "w") as f:
+            json.dump(self.cfg, f)
+        try:
+            P.setRank(1, 1)
+            P.stackSetConfig(path, dtype, global_batch, kv_pages, state_slots)
+        finally:
+            os.unlink(path)
+        P.stackKeepLayers(keep_layers)
+        if isinstance(weights, str):
+            P.stackInit(weights, global_batch)
+        else:
+            P.stackInitTensors(stack_models.random_tensors(self.cfg, seed, rank) if weights is None else weights, global_batch)
+        self._open = True
+
+    @property
+    def vocab(self) -> int:
+        return self.cfg["vocab"]
+
+    def replay(self, kv_pages=None, state_slots=None) -> P.Replay:
+        return P.Replay(kv_pages or self.kv_pages, state_slots or self.state_slots)
+
+    def former(self, avg_prefill: int, avg_decode: int) -> P.BatchFormer:
+        """A batch former over this engine's pages and state slots."""
+        f = P.BatchFormer(self.kv_pages, 16, self.T, self.T, self.T, 0, avg_prefill, avg_decode)
+        f.set_state_slots(self.state_slots)
+        return f
+
+    def update(self, b: synth.Batch, state_slots, keep_token_list=None, decode_tokens=None, logit_rows=None):
+        """Stages one iteration (as Engine.update), with the requests' state slots."""
+        nd = b.decodePrefillBorder
+        arrs = {k: np.ascontiguousarray(v, dtype=np.int32) for k, v in {
+            "tokens": b.input_tokens[nd:], "indptr": b.input_indptr, "rev": b.rev_input_indptr, "off": b.per_token_offset,
+            "kvp": b.kv_indptr, "kvi": b.kv_indices, "kvl": b.kv_last_page_len,
+            "keep": np.ones(nd, np.int32) if keep_token_list is None else keep_token_list}.items()}
+        u = P.VortexUpdateData()
+        u.decodePrefillBorder, u.prefillNum, u.prefillTokensNum = nd, b.prefillNum, b.prefillTokensNum
+        u.keepTokenListLength = len(arrs["keep"])
+        for setter, key in ((u.setInputEmbedding, "tokens"), (u.setInputIndptr, "indptr"), (u.setRevInputIndptr, "rev"),
+                            (u.setPerTokenOffset, "off"), (u.setKVIndptr, "kvp"), (u.setKVIndices, "kvi"),
+                            (u.setKVLastPageLen, "kvl"), (u.setKeepTokenList, "keep")):
+            setter(arrs[key].ctypes.data)
+        u.setGemvBatchSize([nd, 0, 0, 0])
+        u.setGemvNumBlocks([0, 0, 0, 0])
+        self._hold = (arrs, u)
+        P.updateStack(u, state_slots=state_slots, decode_tokens=decode_tokens, logit_rows=logit_rows)
+
+    def run(self) -> np.ndarray:
+        P.run()
+        return P.getPipelineOutput()
+
+    def close(self):
+        if self._open:
+            P.finalize()
+            self._open = False
+
+    def __enter__(self):
+        return self
+
+    def __exit__(self, *exc):
+        self.close()

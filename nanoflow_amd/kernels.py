@@ -29,7 +29,40 @@ SYMBOLS = [
     "nf_split_kqv_f16", "nf_extract_rank_columns_f16", "nf_silu_mul_f16", "nf_transpose_f16", "nf_sleep_us",
     "nf_gemm_tile_menu", "nf_gemm_tiled_workspace_bytes", "nf_gemm_f16_tiled",
     "nf_rmsnorm_quantize_e4m3", "nf_gemm_f8q_f16", "nf_dual_swiglu_f8q_f16",
+    "nf_gemm_nk_workspace_bytes_upto", "nf_gemm_nk_bf16", "nf_gemm_nk_relu2_bf16", "nf_gemm_nk_f32",
+    "nf_gemm_nk_sums_shares", "nf_gemm_nk_sums_bytes_upto", "nf_gemm_nk_sums_bf16", "nf_embed_rows", "nf_norm_add_rows",
+    "nf_gather_norm_rows", "nf_token_shift", "nf_tanh_rows", "nf_argmax_f32", "nf_kv_page_elements", "nf_qkv_append",
+    "nf_window_attention", "nf_recurrence_state_elements", "nf_recurrence_workspace_bytes", "nf_linear_recurrence",
 ]
+
+
+# structs of the layer-stack operators (nf_rotation, nf_kv_layout, ...)
+class Rotation(C.Structure):
+    _fields_ = [("table", C.c_void_p), ("dims", C.c_int), ("interleaved", C.c_int)]
+
+
+class KVLayout(C.Structure):
+    _fields_ = [(n, C.c_int) for n in ("dtype", "heads", "kv_heads", "dim", "vdim", "k_pad", "v_pad", "page")]
+
+
+class WindowAttentionArgs(C.Structure):
+    _fields_ = [("kv", KVLayout), ("window", C.c_int), ("keep_first", C.c_int), ("scale", C.c_float),
+                ("out_scale", C.c_float), ("sink", C.c_void_p), ("q", C.c_void_p), ("out", C.c_void_p),
+                ("out_ld", C.c_int), ("out_col", C.c_int), ("kv_data", C.c_void_p)] + \
+        [(n, C.c_void_p) for n in ("input_indptr", "kv_indptr", "kv_indices", "rev_input_indptr", "positions")] + \
+        [(n, C.c_int) for n in ("req_begin", "req_num", "row_begin", "max_rows", "decode")]
+
+
+class RecurrenceArgs(C.Structure):
+    _fields_ = [(n, C.c_int) for n in ("dtype", "kind", "heads", "dim", "vdim")] + \
+        [(n, C.c_void_p) for n in ("q", "k", "v", "g")] + [(n, C.c_int) for n in ("q_ld", "k_ld", "v_ld", "g_ld")] + \
+        [("rot", Rotation), ("k_scale", C.c_float), ("log2_decay", C.c_void_p), ("z", C.c_void_p), ("z_ld", C.c_int),
+         ("z_shares", C.c_int), ("w0", C.c_void_p), ("u", C.c_void_p), ("norm_weight", C.c_void_p), ("eps", C.c_float),
+         ("out_scale", C.c_float), ("state", C.c_void_p), ("out", C.c_void_p), ("out_ld", C.c_int), ("out_col", C.c_int),
+         ("shift_x", C.c_void_p), ("shift_state", C.c_void_p), ("shift_ld", C.c_int), ("input_indptr", C.c_void_p),
+         ("positions", C.c_void_p), ("state_slots", C.c_void_p)] + \
+        [(n, C.c_int) for n in ("req_begin", "req_num", "row_begin", "rows", "total_rows")] + \
+        [("workspace", C.c_void_p), ("workspace_bytes", C.c_size_t)]
 
 
 class NanoflowKernelError(RuntimeError):
@@ -108,8 +141,28 @@ def lib() -> C.CDLL:
         l.nf_attention_paged_f16.argtypes = [vp] * 7 + [i32] * 8 + [vp, sz, vp]
         l.nf_keep_token_f16.argtypes = [vp, vp, vp, i32, i32, vp]
         l.nf_argmax_f16.argtypes = [vp, vp, vp, i32, i32, vp]
+        l.nf_gemm_nk_bf16.argtypes = l.nf_gemm_nk_relu2_bf16.argtypes = [vp, vp, vp, i32, i32, i32, vp, sz, vp]
+        l.nf_gemm_nk_f32.argtypes = [vp, vp, vp, i32, i32, i32, i32, vp]
+        l.nf_gemm_nk_sums_shares.argtypes = [i32] * 4
+        l.nf_gemm_nk_sums_bf16.argtypes = [vp, vp, vp, sz, i32, i32, i32, i32, vp]
+        l.nf_embed_rows.argtypes = [i32, vp, vp, vp, vp, vp, vp, i32, i32, vp]
+        l.nf_norm_add_rows.argtypes = [i32, vp, i32, vp, vp, i32, vp, i32, i32, i32, f32, vp]
+        l.nf_gather_norm_rows.argtypes = [i32, vp, vp, vp, vp, i32, i32, i32, f32, vp]
+        l.nf_token_shift.argtypes = [i32, vp, vp, vp, vp, i32, vp, vp, vp, vp, i32, i32, vp]
+        l.nf_tanh_rows.argtypes = [i32, vp, i32, vp, i32, i32, vp]
+        l.nf_argmax_f32.argtypes = [vp, vp, i32, i32, i32, vp]
+        l.nf_qkv_append.argtypes = [C.POINTER(KVLayout), vp, i32, i32, i32, i32, vp, vp, f32, C.POINTER(Rotation), vp, vp, vp,
+                                    vp, vp, vp, i32, vp]
+        l.nf_window_attention.argtypes = [C.POINTER(WindowAttentionArgs), vp]
+        l.nf_linear_recurrence.argtypes = [C.POINTER(RecurrenceArgs), vp]
+        size_calls = {"nf_kv_page_elements": [C.POINTER(KVLayout)], "nf_recurrence_state_elements": [i32, i32],
+                      "nf_recurrence_workspace_bytes": [i32] * 5, "nf_gemm_nk_workspace_bytes_upto": [i32] * 3,
+                      "nf_gemm_nk_sums_bytes_upto": [i32] * 4}
+        for name, types in size_calls.items():
+            getattr(l, name).restype = sz
+            getattr(l, name).argtypes = types
         for name in SYMBOLS:
-            if name not in ("nf_last_error", "nf_attention_workspace_bytes", "nf_gemm_workspace_bytes",
+            if name not in size_calls and name not in ("nf_last_error", "nf_attention_workspace_bytes", "nf_gemm_workspace_bytes",
                             "nf_gemm_workspace_bytes_upto", "nf_gemm_f8w_workspace_bytes", "nf_gemm_tiled_workspace_bytes",
                             "nf_dual_swiglu_workspace_bytes", "nf_dual_swiglu_workspace_bytes_upto",
                             "nf_gemm_f8w_split_workspace_bytes", "nf_gemm_f8w_split_workspace_bytes_upto",
@@ -544,3 +597,151 @@ def calibrate_paged_read(pool, kv_indptr, kv_indices, kv_last_page_len, batch: i
                                          kv_last_page_len.data_ptr(), batch, num_kv_heads, kv_bytes, reps,
                                          scratch.data_ptr(), scratch.numel(), C.byref(g), _stream()), "nf_calibrate_paged_read")
     return g.value
+
+
+# ---------------------------------------------------------------- layer-stack operators
+# Activations are float32 or bfloat16 tensors (the operators' dtype follows them); see the C header for
+# the layouts.
+
+F32, BF16 = 0, 1
+FIXED_DECAY, TOKEN_DECAY = 0, 1
+
+
+def _dt(t):
+    return {torch.float32: F32, torch.bfloat16: BF16}[t.dtype]
+
+
+def _call(name, *args):
+    _check(getattr(lib(), name)(*args), name)
+
+
+def gemm_nk(a, b, squared_relu=False, workspace=None):
+    """act(a . b^T), b [N, K], in the type of a."""
+    M, K = a.shape
+    N = b.shape[0]
+    d = torch.empty((M, N), dtype=a.dtype, device=a.device)
+    if a.dtype == torch.float32:
+        _call("nf_gemm_nk_f32", _p(a), _p(b), _p(d), M, N, K, int(squared_relu), _stream())
+    else:
+        ws_bytes = workspace.numel() * workspace.element_size() if workspace is not None else 0
+        _call("nf_gemm_nk_relu2_bf16" if squared_relu else "nf_gemm_nk_bf16", _p(a), _p(b), _p(d), M, N, K, _p(workspace),
+              ws_bytes, _stream())
+    return d
+
+
+def gemm_nk_sums(a, b, max_shares=1):
+    """fp32 sums [shares, M, N] of a . b^T (bf16 operands)."""
+    M, K = a.shape
+    N = b.shape[0]
+    shares = lib().nf_gemm_nk_sums_shares(M, N, K, max_shares)
+    p = torch.empty((shares, M, N), dtype=torch.float32, device=a.device)
+    _call("nf_gemm_nk_sums_bf16", _p(a), _p(b), _p(p), p.numel() * 4, M, N, K, max_shares, _stream())
+    return p
+
+
+def embed_rows(tokens, positions, embed, pos):
+    """(fp32 rows, rows in the tables' type)"""
+    T, ld = tokens.numel(), embed.shape[1]
+    x = torch.empty((T, ld), dtype=torch.float32, device=embed.device)
+    act = torch.empty((T, ld), dtype=embed.dtype, device=embed.device)
+    _call("nf_embed_rows", _dt(embed), _p(tokens), _p(positions), _p(embed), _p(pos), _p(x), _p(act), T, ld, _stream())
+    return x, act
+
+
+def norm_add_rows(y, weight, x, act, width, eps):
+    """x += norm(y) * weight in place; y [shares, T, ld] fp32 or [T, ld] bf16; act receives x in its type."""
+    shares = y.shape[0] if y.dim() == 3 else 1
+    T, ld = x.shape
+    _call("nf_norm_add_rows", _dt(y), _p(y), shares, _p(weight), _p(x), _dt(act), _p(act), T, width, ld, eps, _stream())
+
+
+def gather_norm_rows(x, index, weight, width, eps, dtype):
+    out = torch.empty((index.numel(), x.shape[1]), dtype=dtype, device=x.device)
+    _call("nf_gather_norm_rows", _dt(out), _p(x), _p(index), _p(weight), _p(out), index.numel(), width, x.shape[1], eps, _stream())
+    return out
+
+
+def token_shift(x, shift_state, mu, input_indptr, rev_input_indptr, positions, state_slots, dtype):
+    T, ld = x.shape
+    out = torch.empty((mu.shape[0], T, ld), dtype=dtype, device=x.device)
+    _call("nf_token_shift", _dt(out), _p(x), _p(shift_state), _p(mu), _p(out), mu.shape[0], _p(input_indptr),
+          _p(rev_input_indptr), _p(positions), _p(state_slots), T, ld, _stream())
+    return out
+
+
+def tanh_rows(sums, dtype):
+    out = torch.empty(sums.shape[1:], dtype=dtype, device=sums.device)
+    _call("nf_tanh_rows", _dt(out), _p(sums), sums.shape[0], _p(out), sums.shape[1], sums.shape[2], _stream())
+    return out
+
+
+def argmax_f32(logits, cols=None):
+    out = torch.empty((logits.shape[0],), dtype=torch.int32, device=logits.device)
+    _call("nf_argmax_f32", _p(logits), _p(out), logits.shape[0], cols or logits.shape[1], logits.shape[1], _stream())
+    return out
+
+
+def kv_layout(dtype, heads, kv_heads, dim, vdim) -> KVLayout:
+    return KVLayout(BF16 if dtype == torch.bfloat16 else F32, heads, kv_heads, dim, vdim, (dim + 31) // 32 * 32,
+                    (vdim + 15) // 16 * 16, 16)
+
+
+def kv_pool(layout: KVLayout, pages, device="cuda"):
+    n = lib().nf_kv_page_elements(C.byref(layout))
+    return torch.zeros((pages, n), dtype=torch.bfloat16 if layout.dtype == BF16 else torch.float32, device=device)
+
+
+def rotation(table=None, dims=0, interleaved=False) -> Rotation:
+    """table: fp32 [positions, dims / 2, 2] of (cos, sin)."""
+    return Rotation(_p(table) if table is not None else None, dims, int(interleaved))
+
+
+def qkv_append(layout, proj, cols, q_norm, k_norm, eps, rot, pool, kv_indptr, kv_indices, rev_input_indptr, positions):
+    """Returns the normed, rotated queries [T, heads, k_pad]; keys and values go to the pool's pages."""
+    T = proj.shape[0]
+    q = torch.empty((T, layout.heads, layout.k_pad), dtype=proj.dtype, device=proj.device)
+    _call("nf_qkv_append", C.byref(layout), _p(proj), proj.shape[1], *cols, _p(q_norm), _p(k_norm), eps, C.byref(rot), _p(q),
+          _p(pool), _p(kv_indptr), _p(kv_indices), _p(rev_input_indptr), _p(positions), T, _stream())
+    return q
+
+
+def window_attention(layout, q, pool, batch, *, window, keep_first, scale, sink=None, out_scale=1.0, decode=0):
+    """batch: dict of device arrays input_indptr, kv_indptr, kv_indices, rev_input_indptr, positions; the first
+    `decode` requests have one row each.  Returns [T, heads * vdim]."""
+    T = q.shape[0]
+    out = torch.zeros((T, layout.heads * layout.vdim), dtype=q.dtype, device=q.device)
+    n_req = batch["input_indptr"].numel() - 1
+    a = WindowAttentionArgs(kv=layout, window=window, keep_first=keep_first, scale=scale, out_scale=out_scale, sink=_p(sink),
+                            q=_p(q), out=_p(out), out_ld=out.shape[1], out_col=0, kv_data=_p(pool))
+    for n in ("input_indptr", "kv_indptr", "kv_indices", "rev_input_indptr", "positions"):
+        setattr(a, n, _p(batch[n]))
+    for first, n, rows, dec in ((0, decode, decode, 1), (decode, n_req - decode, T - decode, 0)):
+        if n:
+            a.req_begin, a.req_num, a.row_begin, a.max_rows, a.decode = first, n, first, rows, dec
+            _call("nf_window_attention", C.byref(a), _stream())
+    return out
+
+
+def linear_recurrence(kind, q, k, v, g, heads, dim, vdim, state, batch, *, eps, decode=0, rot=None, k_scale=1.0,
+                      log2_decay=None, z=None, w0=None, u=None, norm_weight=None, out_scale=1.0, shift_x=None,
+                      shift_state=None):
+    """q, k, v, g: 2-d tensors of rows; batch: device arrays input_indptr, positions, state_slots.  Returns
+    [T, heads * vdim]; the state is updated in place."""
+    T = q.shape[0]
+    out = torch.zeros((T, heads * vdim), dtype=q.dtype, device=q.device)
+    n_req = batch["input_indptr"].numel() - 1
+    ws = torch.empty((max(lib().nf_recurrence_workspace_bytes(heads, dim, vdim, T, n_req), 16),), dtype=torch.uint8, device=q.device)
+    a = RecurrenceArgs(dtype=_dt(q), kind=kind, heads=heads, dim=dim, vdim=vdim, q=_p(q), k=_p(k), v=_p(v), g=_p(g),
+                       q_ld=q.shape[1], k_ld=k.shape[1], v_ld=v.shape[1], g_ld=g.shape[1], rot=rot or Rotation(),
+                       k_scale=k_scale, log2_decay=_p(log2_decay), z=_p(z), z_ld=z.shape[1] if z is not None else 0,
+                       z_shares=1, w0=_p(w0), u=_p(u), norm_weight=_p(norm_weight), eps=eps, out_scale=out_scale,
+                       state=_p(state), out=_p(out), out_ld=out.shape[1], out_col=0, shift_x=_p(shift_x),
+                       shift_state=_p(shift_state), shift_ld=shift_x.shape[1] if shift_x is not None else 0, total_rows=T,
+                       workspace=_p(ws), workspace_bytes=ws.numel())
+    for n in ("input_indptr", "positions", "state_slots"):
+        setattr(a, n, _p(batch[n]))
+    for first, n, rows in ((0, decode, decode), (decode, n_req - decode, T - decode)):
+        if n:
+            a.req_begin, a.req_num, a.row_begin, a.rows = first, n, first, rows
+            _call("nf_linear_recurrence", C.byref(a), _stream())
+    return out

@@ -39,6 +39,7 @@ class PipelineType(enum.IntEnum):
     LOCAL = 7
     NON_OVERLAP_LOCAL = 8
     NANOBATCH_LOCAL = 9
+    LAYER_STACK = 10
 
     @property
     def has_kqv_bias(self) -> bool:
@@ -48,7 +49,8 @@ class PipelineType(enum.IntEnum):
     @property
     def is_sequential(self) -> bool:
         """One stream, no nano-batch split: four GEMM tags, one decode-attention group."""
-        return self in (PipelineType.NON_OVERLAP_LOCAL, PipelineType.NONOVERLAP_KQVBIAS, PipelineType.NONOVERLAP)
+        return self in (PipelineType.NON_OVERLAP_LOCAL, PipelineType.NONOVERLAP_KQVBIAS, PipelineType.NONOVERLAP,
+                        PipelineType.LAYER_STACK)
 
     @property
     def is_four_way(self) -> bool:
@@ -76,6 +78,7 @@ pipeline_map = {
     "KQVBIAS": PipelineType.KQVBIAS,
     "NANOBATCH_KQVBIAS": PipelineType.NANOBATCH_KQVBIAS,
     "NONOVERLAP_KQVBIAS": PipelineType.NONOVERLAP_KQVBIAS,
+    "LAYER_STACK": PipelineType.LAYER_STACK,   # models described by a list of layers; not in the reference
 }
 
 
@@ -488,6 +491,8 @@ def _sched_lib():
                                               C.POINTER(C.c_int), C.POINTER(C.c_double * 4)]
         l.pllm_sched_future_page_usage.argtypes = [C.c_void_p, C.POINTER(C.c_int64), C.c_int]
         l.pllm_serve.argtypes = [C.c_void_p, C.c_int, C.c_int, C.c_int, C.POINTER(ServeStats)]
+        l.pllm_sched_set_state_slots.argtypes = [C.c_void_p, C.c_int]
+        l.pllm_sched_state_slots.argtypes = [C.c_void_p, C.POINTER(_i32p), C.POINTER(C.c_int)]
         l._sched_declared = True
     return l
 
@@ -546,6 +551,16 @@ class BatchFormer:
         a = np.ascontiguousarray(ids, dtype=np.int32)
         _check(self._l.pllm_sched_harvest(self._h, a.ctypes.data_as(_i32p), len(a)), "sched_harvest")
 
+    def set_state_slots(self, slots: int):
+        """Models with recurrent state: at most `slots` requests are admitted at a time (before the first)."""
+        _check(self._l.pllm_sched_set_state_slots(self._h, slots), "sched_set_state_slots")
+
+    def state_slots(self) -> np.ndarray:
+        """The slots of the last formed batch's requests."""
+        p, n = _i32p(), C.c_int()
+        _check(self._l.pllm_sched_state_slots(self._h, C.byref(p), C.byref(n)), "sched_state_slots")
+        return np.ctypeslib.as_array(p, shape=(n.value,)).copy() if n.value else np.zeros(0, np.int32)
+
     def advance(self, now=0.0, placeholder_zero=False) -> int:
         n = C.c_int()
         _check(self._l.pllm_sched_advance(self._h, now, int(placeholder_zero), C.byref(n)), "sched_advance")
@@ -581,3 +596,131 @@ class BatchFormer:
         st = ServeStats()
         _check(self._l.pllm_serve(self._h, skip_cycles, warmup_cycles, run_cycles, C.byref(st)), "serve")
         return st
+
+
+# ---------------------------------------------------------------- layer-stack models
+
+class _CHostTensor(C.Structure):
+    _fields_ = [("name", C.c_char_p), ("type", C.c_int), ("ndim", C.c_int), ("shape", C.POINTER(C.c_int64)), ("data", C.c_void_p)]
+
+
+class _CStackUpdate(C.Structure):
+    _fields_ = [("state_slots", C.c_void_p), ("decode_tokens", C.c_void_p), ("logit_rows", C.c_void_p), ("logit_rows_num", C.c_int)]
+
+
+def _stack_lib():
+    l = lib()
+    if not getattr(l, "_stack_declared", False):
+        ip = C.POINTER(C.c_int)
+        l.pllm_stack_set_config.argtypes = [C.c_char_p, C.c_char_p, C.c_int, C.c_int, C.c_int]
+        l.pllm_stack_init.argtypes = [C.c_char_p, C.c_int]
+        l.pllm_stack_init_tensors.argtypes = [C.POINTER(_CHostTensor), C.c_int, C.c_int]
+        l.pllm_update_stack.argtypes = [C.POINTER(_CUpdateData), C.POINTER(_CStackUpdate)]
+        l.pllm_get_logits.argtypes = [C.c_void_p, C.c_int, ip, ip]
+        l.pllm_stack_keep_layers.argtypes = [C.c_int]
+        l.pllm_stack_layer_output.argtypes = [C.c_int, C.c_void_p, ip, ip]
+        l.pllm_replay_create.restype = C.c_void_p
+        l.pllm_replay_create.argtypes = [C.c_int, C.c_int]
+        l.pllm_replay_destroy.restype = None
+        l.pllm_replay_destroy.argtypes = [C.c_void_p]
+        l.pllm_replay_step.argtypes = [C.c_void_p, C.c_int, C.POINTER(C.c_char_p)] + [C.c_void_p] * 5
+        l.pllm_replay_end.argtypes = [C.c_void_p, C.c_char_p]
+        l.pllm_replay_state.argtypes = [C.c_void_p, C.POINTER(C.c_int * 3)]
+        l._stack_declared = True
+    return l
+
+
+def stackSetConfig(config_json: str, dtype: str, max_batch: int, kv_pages: int, state_slots: int):
+    """The model of a config.json whose ``architecture`` is registered; dtype "bfloat16" or "float32"."""
+    _check(_stack_lib().pllm_stack_set_config(config_json.encode(), dtype.encode(), max_batch, kv_pages, state_slots), "stackSetConfig")
+
+
+def stackStateSlots() -> int:
+    return _stack_lib().pllm_stack_state_slots()
+
+
+def stackInit(model_dir: str, global_batch: int):
+    """Weights from model_dir/model.safetensors; starts the pipeline."""
+    _check(_stack_lib().pllm_stack_init(model_dir.encode(), global_batch), "stackInit")
+
+
+def stackInitTensors(tensors: dict, global_batch: int):
+    """Weights from host arrays: float32, int32, or uint16 (bfloat16 bit patterns)."""
+    kinds = {np.dtype(np.uint16): 0, np.dtype(np.float32): 1, np.dtype(np.int32): 2}
+    keep, c = [], (_CHostTensor * len(tensors))()
+    for i, (name, a) in enumerate(tensors.items()):
+        a = np.ascontiguousarray(a)
+        shape = (C.c_int64 * max(a.ndim, 1))(*a.shape)
+        keep.extend([a, shape])
+        c[i] = _CHostTensor(name.encode(), kinds[a.dtype], a.ndim, shape, a.ctypes.data)
+    _check(_stack_lib().pllm_stack_init_tensors(c, len(tensors), global_batch), "stackInitTensors")
+
+
+def updateStack(update: VortexUpdateData, state_slots=None, decode_tokens=None, logit_rows=None):
+    arrs = [None if a is None else np.ascontiguousarray(a, dtype=np.int32) for a in (state_slots, decode_tokens, logit_rows)]
+    ptr = lambda a: None if a is None else (a if a.size else np.zeros(1, np.int32)).ctypes.data
+    x = _CStackUpdate(*(ptr(a) for a in arrs), 0 if arrs[2] is None else arrs[2].size)
+    cu = update._to_c()
+    _check(_stack_lib().pllm_update_stack(C.byref(cu), C.byref(x)), "updateStack")
+
+
+def getLogits() -> np.ndarray:
+    """fp32 logits of the last iteration [rows, vocab]."""
+    rows, vocab = C.c_int(), C.c_int()
+    l = _stack_lib()
+    _check(l.pllm_get_logits(None, 0, C.byref(rows), C.byref(vocab)), "getLogits")
+    out = np.empty((rows.value, vocab.value), np.float32)
+    _check(l.pllm_get_logits(out.ctypes.data, rows.value, C.byref(rows), C.byref(vocab)), "getLogits")
+    return out
+
+
+def stackKeepLayers(on: bool):
+    _check(_stack_lib().pllm_stack_keep_layers(int(on)), "stackKeepLayers")
+
+
+def stackLayerOutput(layer: int) -> np.ndarray:
+    """The residual stream after a layer in the last iteration [rows, width] (stackKeepLayers)."""
+    rows, width = C.c_int(), C.c_int()
+    l = _stack_lib()
+    _check(l.pllm_stack_layer_output(layer, None, C.byref(rows), C.byref(width)), "stackLayerOutput")
+    out = np.empty((rows.value, width.value), np.float32)
+    _check(l.pllm_stack_layer_output(layer, out.ctypes.data, C.byref(rows), C.byref(width)), "stackLayerOutput")
+    return out
+
+
+class Replay:
+    """Given tokens through the running layer-stack pipeline, step by step (StackReplay)."""
+
+    def __init__(self, kv_pages: int, state_slots: int):
+        self._l = _stack_lib()
+        self._h = self._l.pllm_replay_create(kv_pages, state_slots)
+        if not self._h:
+            raise NanoflowPipelineError(self._l.pllm_last_error().decode())
+
+    def step(self, entries, vocab: int):
+        """entries: [(id, tokens, want)]; returns {id: logits [len(want), vocab]}."""
+        ids = (C.c_char_p * max(len(entries), 1))(*[str(e[0]).encode() for e in entries])
+        cat = lambda parts: np.concatenate([np.asarray(p, np.int32).ravel() for p in parts] + [np.zeros(1, np.int32)])
+        n_tok, n_want = cat([[len(e[1])] for e in entries]), cat([[len(e[2])] for e in entries])
+        tok, want = cat([e[1] for e in entries]), cat([e[2] for e in entries])
+        out = np.empty((int(n_want.sum()), vocab), np.float32)
+        _check(self._l.pllm_replay_step(self._h, len(entries), ids, n_tok.ctypes.data, tok.ctypes.data, n_want.ctypes.data,
+                                        want.ctypes.data, out.ctypes.data), "replay step")
+        res, at = {}, 0
+        for e in entries:
+            res[e[0]] = out[at:at + len(e[2])]
+            at += len(e[2])
+        return res
+
+    def end(self, id):
+        _check(self._l.pllm_replay_end(self._h, str(id).encode()), "replay end")
+
+    def state(self) -> dict:
+        c = (C.c_int * 3)()
+        _check(self._l.pllm_replay_state(self._h, C.byref(c)), "replay state")
+        return dict(live=c[0], free_pages=c[1], free_slots=c[2])
+
+    def close(self):
+        if self._h:
+            self._l.pllm_replay_destroy(self._h)
+            self._h = None

@@ -25,6 +25,10 @@ reference's pipeline/utils/serve_8B.py:
 * ``serve_configs.weight_format`` (optional, not in the reference's schema): "f16" (default) or "e4m3" --
   the five GEMM weights of every layer are quantised on the device as they are loaded or made
   (per-output-channel scales) and served from the fp8 form.
+* A model described by a list of layers (``model`` = its own configuration with ``architecture``, or ``{"path": DIR}``
+  of a directory with config.json; ``serve_configs.pipeline_type`` "LAYER_STACK"): ``weight_path`` (or the path) holds
+  model.safetensors, ``model_configs.dtype`` is "bfloat16" (default) or "float32", ``model_configs.state_slots`` the number
+  of requests that may hold recurrent state at a time (default 256), ``model_configs.kv_pages`` overrides the pool.
 * KV pool = ``1024 * allocate_kv_data_batch // 16`` pages per layer (serve_8B.py:643).
 * writes PREFIX.stat, PREFIX.stat.csv (same columns as serve_8B.py:792-793), PREFIX.req_time,
   PREFIX.req_tokens (prompt + generated ids of every retired request, one Python list per line,
@@ -92,11 +96,35 @@ def read_trace(path, tokenizer=None):
     return reqs
 
 
+def is_stack(cfg) -> bool:
+    """The file names a model described by a list of layers instead of Llama sizes."""
+    return "architecture" in cfg["model"] or "path" in cfg["model"]
+
+
+def stack_engine(cfg, config_path, empty_weight):
+    """The engine of a pipeline file that names a layer-stack model, and its KV pages."""
+    from nanoflow_amd import engine, stack_models
+    m, mc, pc, sc = cfg["model"], cfg["model_configs"], cfg["pipeline_configs"], cfg["serve_configs"]
+    if sc.get("pipeline_type", "LAYER_STACK") != "LAYER_STACK":
+        raise SystemExit(f"serve_configs.pipeline_type {sc['pipeline_type']!r}: a layer-stack model runs as LAYER_STACK")
+    path = os.path.join(os.path.dirname(os.path.abspath(config_path)), m["path"]) if "path" in m else None
+    model = stack_models.load_config(path or m)
+    pages = mc.get("kv_pages") or 1024 * mc["allocate_kv_data_batch"] // 16
+    wdir = sc.get("weight_path") or path
+    if not empty_weight and not (wdir and os.path.isfile(os.path.join(wdir, "model.safetensors"))):
+        raise SystemExit("serve_configs.weight_path holds no model.safetensors (or pass --empty_weight True)")
+    eng = engine.StackEngine(model, dtype=mc.get("dtype", "bfloat16"), global_batch=pc["global_batch_size"], kv_pages=pages,
+                             state_slots=mc.get("state_slots", 256), weights=None if empty_weight else wdir)
+    return eng, pages
+
+
 def parse_config(cfg):
     """(model shape, pipeline type, (global batch, nano-batch 1, kqv1, kqv3), KV pages per layer) of a
     pipeline JSON in the reference's schema."""
     from nanoflow_amd import synth, pllm_python as P
     m, mc, pc, sc = cfg["model"], cfg["model_configs"], cfg["pipeline_configs"], cfg["serve_configs"]
+    if is_stack(cfg):
+        raise SystemExit("a layer-stack model is served through stack_engine()")
     if mc.get("gpu_num", 1) != 1 or sc.get("actual_gpu_num", 1) != 1:
         raise SystemExit("this build serves on one GPU (gpu_num and actual_gpu_num must be 1)")
     shape = synth.ModelShape(hidden=m["hidden_size"], Hq=m["num_attention_heads"], Hkv=m["num_key_value_heads"],
@@ -131,14 +159,20 @@ def main():
     assert torch.cuda.is_available(), "needs the MI355X"
     cfg = json.load(open(a.config_path))
     mc, sc = cfg["model_configs"], cfg["serve_configs"]
-    shape, pt, (T, nano1, kqv1, kqv3), pages = parse_config(cfg)
+    stack = is_stack(cfg)
+    if stack:
+        eng, pages = stack_engine(cfg, a.config_path, empty_weight)
+        vocab, longest = eng.vocab, eng.cfg["max_positions"]
+    else:
+        shape, pt, (T, nano1, kqv1, kqv3), pages = parse_config(cfg)
+        vocab, longest = shape.vocab, None
     # the file's GEMM tags (their B layout decides the orientation the weights are handed over in);
     # a list written for another schedule's GEMM count falls back to the default tags
     tags = cfg["pipeline_configs"].get("gemm_op_tag") or []
-    tags = list(tags) if len(tags) == pt.gemm_tags else None
+    tags = list(tags) if not stack and len(tags) == pt.gemm_tags else None
 
     weights = None
-    if not empty_weight:
+    if not empty_weight and not stack:
         from nanoflow_amd import weights as W
         wdir = sc.get("weight_path")
         if not wdir:
@@ -157,15 +191,21 @@ def main():
 
     tokenizer = load_tokenizer(sc)
     reqs = read_trace(a.trace_path, tokenizer)
-    too_big = [r[0] for r in reqs if len(r[1]) and int(r[1].max()) >= shape.vocab]
+    too_big = [r[0] for r in reqs if len(r[1]) and int(r[1].max()) >= vocab]
     if too_big:
-        raise SystemExit(f"{a.trace_path}: request {too_big[0]} has a token id beyond the model's vocabulary of {shape.vocab}")
+        raise SystemExit(f"{a.trace_path}: request {too_big[0]} has a token id beyond the model's vocabulary of {vocab}")
+    too_long = [r[0] for r in reqs if longest and len(r[1]) + r[2] > longest]
+    if too_long:
+        raise SystemExit(f"{a.trace_path}: request {too_long[0]} is longer than the model's {longest} positions")
     avg_in = sum(len(r[1]) for r in reqs) // len(reqs)
     avg_out = sum(r[2] for r in reqs) // len(reqs)
-    eng = engine.Engine(shape, pt, global_batch=T, nano1=nano1, kqv1=kqv1, kqv3=kqv3, kv_pages=pages,
-                        run_layer=mc.get("run_layer", shape.layers), kv_fill="zeros", weights=weights,
-                        weight_format=sc.get("weight_format", "f16"), gemm_tags=tags)
-    former = P.BatchFormer(pages, shape.page_size, T, nano1, kqv1, kqv3, avg_in, avg_out)
+    if stack:
+        former = eng.former(avg_in, avg_out)
+    else:
+        eng = engine.Engine(shape, pt, global_batch=T, nano1=nano1, kqv1=kqv1, kqv3=kqv3, kv_pages=pages,
+                            run_layer=mc.get("run_layer", shape.layers), kv_fill="zeros", weights=weights,
+                            weight_format=sc.get("weight_format", "f16"), gemm_tags=tags)
+        former = P.BatchFormer(pages, shape.page_size, T, nano1, kqv1, kqv3, avg_in, avg_out)
 
     pending = list(reqs)                  # not yet released, in arrival order
     passed = 0.0
@@ -226,7 +266,10 @@ def main():
                                 per_token_offset=b["per_token_offset"], kv_indptr=b["kv_indptr"],
                                 kv_indices=b["kv_indices"], kv_last_page_len=b["kv_last_page_len"],
                                 kv_len=np.zeros(0, np.int32), num_pages=pages)
-            eng.update(batch, keep_token_list=b["keep_token_list"])
+            if stack:
+                eng.update(batch, former.state_slots(), keep_token_list=b["keep_token_list"])
+            else:
+                eng.update(batch, keep_token_list=b["keep_token_list"])
             P.run_async()
             in_flight = True
             if prev_ids is not None:

@@ -1,0 +1,109 @@
+"""Layer-stack designs seen from Python: the tensors a configuration asks for, and random weights of
+those shapes (benchmarks, tests, serving without a checkpoint).  What a design computes is known to the
+C++ registry (csrc/host/stackModel.h) alone."""
+from __future__ import annotations
+
+import json
+import os
+
+import numpy as np
+
+
+def load_config(model) -> dict:
+    """A configuration: a dict, a config.json, or the directory that holds one."""
+    if isinstance(model, dict):
+        return model
+    path = os.path.join(model, "config.json") if os.path.isdir(model) else model
+    with open(path) as f:
+        return json.load(f)
+
+
+def _zovovik_shapes(cfg: dict, rank: int) -> dict:
+    W = cfg["width"]
+    out = {"embed": (cfg["vocab"], W), "pos": (cfg["max_positions"], W), "head": (cfg["vocab"], W), "final.norm": (W,)}
+    for i, layer in enumerate(cfg["layers"]):
+        l, m = f"l{i}.", layer["mixer"]
+        out[l + "norm1"] = (W,)
+        if layer["type"] == "retention":
+            qk, vg = m["heads"] * m["dim"], m["heads"] * m["vdim"]
+            out.update({l + "mix.q": (qk, W), l + "mix.k": (qk, W), l + "mix.v": (vg, W), l + "mix.g": (vg, W), l + "mix.o": (W, vg)})
+        else:
+            a, r = m["left"], m["right"]
+            p, q = l + "mix.left.", l + "mix.right."
+            out.update({p + "q": (a["heads"] * a["dim"], W), p + "k": (a["kv_heads"] * a["dim"], W),
+                        p + "v": (a["kv_heads"] * a["vdim"], W), p + "q.norm": (a["dim"],), p + "k.norm": (a["dim"],),
+                        p + "sink": (a["heads"],), p + "o": (W, a["heads"] * a["vdim"])})
+            n = r["heads"] * r["dim"]
+            out.update({q + "mu." + s: (W,) for s in "rkvgw"})
+            out.update({q + s: (n, W) for s in "rkvg"})
+            out.update({q + "w1": (rank, W), q + "w2": (n, rank), q + "w0": (n,), q + "u": (r["heads"], r["dim"]),
+                        q + "norm": (n,), q + "o": (W, n)})
+        if layer.get("mlp"):
+            out.update({l + "norm2": (W,), l + "mlp.up": (layer["mlp"]["ff"], W), l + "mlp.down": (W, layer["mlp"]["ff"])})
+    return out
+
+
+ARCHITECTURES = {"Zovovik": _zovovik_shapes}
+
+
+def tensor_shapes(cfg: dict, rank: int = 16) -> dict:
+    """name -> shape; `rank` is the inner size of the token decay's two-step projection (a tensor's own size, not in
+    the configuration)."""
+    if cfg.get("architecture") not in ARCHITECTURES:
+        raise ValueError(f"unknown architecture {cfg.get('architecture')!r}: one of {', '.join(ARCHITECTURES)}")
+    return ARCHITECTURES[cfg["architecture"]](cfg, rank)
+
+
+def bf16_bits(a) -> np.ndarray:
+    """float array -> bfloat16 bit patterns (uint16), round to nearest even."""
+    u = np.ascontiguousarray(a, dtype=np.float32).view(np.uint32)
+    return ((u + np.uint32(0x7fff) + ((u >> np.uint32(16)) & np.uint32(1))) >> np.uint32(16)).astype(np.uint16)
+
+
+def bits_to_f32(b) -> np.ndarray:
+    return (b.astype(np.uint32) << np.uint32(16)).view(np.float32)
+
+
+def random_tensors(cfg: dict, seed: int = 0, rank: int = 16) -> dict:
+    """name -> bfloat16 bit patterns: projections N(0, 1 / inputs), norms around 1, shifts in [0, 1], token decays
+    that keep a state for a few to a few thousand tokens."""
+    rng = np.random.default_rng(seed)
+    out = {}
+    for name, shape in tensor_shapes(cfg, rank).items():
+        leaf = name.split(".")[-1]
+        big = int(np.prod(shape)) > 1 << 22     # large matrices: one block of normals, repeated
+        n = min(int(np.prod(shape)), 1 << 22)
+        x = rng.standard_normal(n, dtype=np.float32)
+        if "norm" in leaf:
+            x = 1.0 + 0.1 * x
+        elif ".mu." in name:
+            x = rng.random(n, dtype=np.float32)
+        elif leaf == "w0":
+            x = -4.0 + 1.5 * x
+        elif leaf in ("u", "sink"):
+            x = 0.5 * x
+        elif name in ("embed", "pos"):
+            pass
+        else:
+            x *= shape[-1] ** -0.5
+        b = bf16_bits(x)
+        out[name] = (np.resize(b, shape) if big else b.reshape(shape))
+    return out
+
+
+def save_model(directory: str, cfg: dict, tensors: dict):
+    """config.json and model.safetensors of `tensors` (bfloat16 bit patterns, float32 or int32 arrays)."""
+    os.makedirs(directory, exist_ok=True)
+    with open(os.path.join(directory, "config.json"), "w") as f:
+        json.dump(cfg, f, indent=1)
+    kinds = {np.dtype(np.uint16): "BF16", np.dtype(np.float32): "F32", np.dtype(np.int32): "I32"}
+    header, at = {}, 0
+    for name, a in tensors.items():
+        header[name] = {"dtype": kinds[a.dtype], "shape": list(a.shape), "data_offsets": [at, at + a.nbytes]}
+        at += a.nbytes
+    h = json.dumps(header).encode()
+    h += b" " * (-len(h) % 8)
+    with open(os.path.join(directory, "model.safetensors"), "wb") as f:
+        f.write(len(h).to_bytes(8, "little") + h)
+        for a in tensors.values():
+            f.write(np.ascontiguousarray(a).tobytes())

@@ -6,8 +6,9 @@
 
 namespace {
 
-// Above this many rows a projection back to the residual width has tiles enough without a split over
-// K, and its output is rounded before the norm reads it; below, the norm adds the fp32 shares itself.
+// A projection back to the residual width that is not split over K is rounded before the norm reads it
+// when it has more than this many rows (fp32 rows would cost more than they are worth there); otherwise the
+// norm adds the fp32 shares itself.
 constexpr int kSumsMaxRows = 512;
 constexpr int kSumsMaxShares = 16;
 
@@ -50,7 +51,6 @@ LayerStackPipeline::Buffers LayerStackPipeline::plan(const StackModel& m, int T,
   auto sums = [&](int rows, const DeviceMatrix& w, int shares) {
     return bf16 ? nf_gemm_nk_sums_bytes_upto(rows, w.N, w.K, shares) : (size_t)rows * w.N * 4;
   };
-  const int sum_rows = bf16 ? std::min(T, kSumsMaxRows) : T;
   for (size_t i = 0; i < spec.layers.size(); ++i) {
     const LayerSpec& s = spec.layers[i];
     const LayerWeights& w = m.weights.layers[i];
@@ -77,11 +77,11 @@ LayerStackPipeline::Buffers LayerStackPipeline::plan(const StackModel& m, int T,
       }
     }
     heads = std::max(heads, (size_t)w.out.K);
-    b.y_sums_bytes = std::max(b.y_sums_bytes, sums(sum_rows, w.out, kSumsMaxShares));
+    b.y_sums_bytes = std::max(b.y_sums_bytes, sums(T, w.out, kSumsMaxShares));
     if (s.mlp) {
       ff = std::max(ff, (size_t)w.up.N);
       ws = std::max(ws, few(w.up));
-      b.y_sums_bytes = std::max(b.y_sums_bytes, sums(sum_rows, w.down, kSumsMaxShares));
+      b.y_sums_bytes = std::max(b.y_sums_bytes, sums(T, w.down, kSumsMaxShares));
     }
   }
   const int L = maxLogitRows(spec, T);
@@ -219,7 +219,8 @@ void LayerStackPipeline::update(vortexUpdateData* u) {
 
 // Projection back to the residual width, norm, residual add.
 void LayerStackPipeline::sublayerOut(const void* a, const DeviceMatrix& w, const float* norm) {
-  if (model->dtype == NF_BF16 && batch.rows > kSumsMaxRows) {
+  if (model->dtype == NF_BF16 && batch.rows > kSumsMaxRows &&
+      nf_gemm_nk_sums_shares(batch.rows, w.N, w.K, kSumsMaxShares) < 2) {
     linear.set(a, w, buf.y, batch.rows).run();
     normAdd.y = buf.y;
     normAdd.y_dtype = NF_BF16;

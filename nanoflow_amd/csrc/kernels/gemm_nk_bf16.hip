@@ -4,8 +4,9 @@
 
 namespace {
 
-// Tile of a launch that stores fp32 sums, and its split over K: as splitk_plan, but from 257 rows on
-// (where a split does not pay) the largest tile that still gives every CU work.
+// Tile of a launch that stores fp32 sums, and its split over K: enough shares of at least 128 to give
+// every CU a tile while the sums stay within 64 MiB; two shares of 256 x 256 tiles where dense_split_plan
+// says so; else, from 257 rows on, the largest tile that still gives every CU work.
 struct SumPlan {
   int tile;  // 0: 64x256, 1: 128x128, 2: 256x256
   int shares, k_per;
@@ -15,10 +16,14 @@ SumPlan sum_plan(int M, int N, int K, int max_shares) {
   SumPlan p{M <= 64 ? 0 : 1, 1, (K + BK - 1) / BK * BK};
   const long long t256 = (long long)((M + 255) / 256) * ((N + 255) / 256);
   if (M > 256 && t256 >= cu_count() / 2) p.tile = 2;
-  if (max_shares < 2 || M > 256 || K < 256) return p;
+  if (max_shares < 2 || K < 256) return p;
+  int k_dense = 0;
+  if (dense_split_plan(M, N, K, &k_dense) > 1) return SumPlan{2, 2, k_dense};
+  if (p.tile == 2) return p;
   const int bm = p.tile == 0 ? 64 : 128, bn = p.tile == 0 ? 256 : 128;
   const int tiles = ((M + bm - 1) / bm) * ((N + bn - 1) / bn);
-  const int want = std::min(std::min(cu_count() / tiles, K / 128), std::min(max_shares, kMaxShares));
+  const int fit = (int)std::min<size_t>(((size_t)64 << 20) / ((size_t)M * N * 4), 64);
+  const int want = std::min(std::min(std::min(cu_count() / tiles, K / 128), std::min(max_shares, kMaxShares)), fit);
   if (want < 2) return p;
   p.k_per = ((K + want - 1) / want + BK - 1) / BK * BK;
   p.shares = (K + p.k_per - 1) / p.k_per;
@@ -70,7 +75,7 @@ int nf_gemm_nk_sums_shares(int M, int N, int K, int max_shares) {
 
 size_t nf_gemm_nk_sums_bytes_upto(int max_M, int N, int K, int max_shares) {
   size_t need = 0;
-  for (int m = 1; m <= max_M; m = m < 257 ? m + 1 : m + 64)
+  for (int m = 1; m <= max_M; ++m)
     need = std::max(need, (size_t)nf_gemm_nk_sums_shares(m, N, K, max_shares) * m * N * sizeof(float));
   return std::max(need, (size_t)nf_gemm_nk_sums_shares(max_M, N, K, max_shares) * max_M * N * sizeof(float));
 }

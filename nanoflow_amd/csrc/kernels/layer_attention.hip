@@ -104,6 +104,120 @@ __global__ __launch_bounds__(256) void qkv_append_kernel(nf_kv_layout kv, const 
   }
 }
 
+// The same for sizes and columns that are multiples of four, which is what models have: a (row, query or key head) is
+// 16 lanes with 16-byte groups; values are turned through LDS, 16 rows of a head at a time, so that the
+// transposed cache is written four positions at once where four rows are an aligned run of one page.
+template <class T>
+__global__ __launch_bounds__(256) void qkv_append4_kernel(nf_kv_layout kv, const T* __restrict__ proj, int ld, int q_col,
+                                                          int k_col, int v_col, const float* __restrict__ q_norm,
+                                                          const float* __restrict__ k_norm, float eps, nf_rotation rot,
+                                                          T* __restrict__ q_out, T* __restrict__ kv_data,
+                                                          const int32_t* __restrict__ kv_indptr,
+                                                          const int32_t* __restrict__ kv_indices,
+                                                          const int32_t* __restrict__ rev_input_indptr,
+                                                          const int32_t* __restrict__ positions, int rows, int qk_blocks) {
+  __shared__ __attribute__((aligned(16))) float buf[kMaxHeadDim * 17];
+  __shared__ long long row_page[16];  // element offset of the row's page, and its entry
+  __shared__ int row_entry[16];
+  const int H = kv.heads, G = kv.kv_heads, tid = threadIdx.x;
+  if ((int)blockIdx.x < qk_blocks) {
+    constexpr int kVec = kMaxHeadDim / 64;
+    const int job = blockIdx.x * 16 + (tid >> 4), l = tid & 15;
+    const bool live = job < rows * (H + G);
+    const int t = live ? job / (H + G) : 0, head = live ? job % (H + G) : 0;
+    const bool is_q = head < H;
+    const T* src = proj + (size_t)t * ld + (is_q ? q_col + head * kv.dim : k_col + (head - H) * kv.dim);
+    const float* w = is_q ? q_norm : k_norm;
+    float* mine = buf + (tid >> 4) * kMaxHeadDim;
+    const int pos = positions[t], half = rot.dims / 2;
+    T* dst;
+    if (is_q) {
+      dst = q_out + ((size_t)t * H + head) * kv.k_pad;
+    } else {
+      const int page = kv_indices[kv_indptr[rev_input_indptr[t]] + pos / kPage];
+      dst = kv_data + (size_t)page * kv_page_elements(kv) + ((size_t)(head - H) * kPage + pos % kPage) * kv.k_pad;
+    }
+    float4_t v[kVec];
+    float sq = 0.f;
+#pragma unroll
+    for (int i = 0; i < kVec; ++i) {
+      const int c = (i * 16 + l) * 4;
+      v[i] = float4_t{0.f, 0.f, 0.f, 0.f};
+      if (c < kv.dim) v[i] = Act<T>::load4(src + c);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) sq += v[i][e] * v[i][e];
+    }
+    if (w) {
+#pragma unroll
+      for (int m = 8; m > 0; m >>= 1) sq += __shfl_xor(sq, m, 64);
+      const float inv = 1.f / sqrtf(sq / (float)kv.dim + eps);
+#pragma unroll
+      for (int i = 0; i < kVec; ++i) {
+        const int c = (i * 16 + l) * 4;
+        if (c < kv.dim) v[i] = v[i] * inv * *reinterpret_cast<const float4_t*>(w + c);
+      }
+    }
+    if (!rot.interleaved)
+#pragma unroll
+      for (int i = 0; i < kVec; ++i) {
+        const int c = (i * 16 + l) * 4;
+        if (c < 2 * half) *reinterpret_cast<float4_t*>(mine + c) = v[i];
+      }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < kVec; ++i) {
+      const int c = (i * 16 + l) * 4;
+      if (c >= kv.k_pad || !live) continue;
+      float4_t y = v[i];
+      if (c < 2 * half) {
+        const float* tab = rot.table + (size_t)pos * half * 2;
+        if (rot.interleaved) {
+          const float4_t cs = *reinterpret_cast<const float4_t*>(tab + c);  // cos, sin of pair c / 2, then of the next
+          y = float4_t{v[i][0] * cs[0] - v[i][1] * cs[1], v[i][1] * cs[0] + v[i][0] * cs[1], v[i][2] * cs[2] - v[i][3] * cs[3],
+                       v[i][3] * cs[2] + v[i][2] * cs[3]};
+        } else {
+          const bool first = c < half;
+          const int f = first ? c : c - half;
+          const float4_t other = *reinterpret_cast<const float4_t*>(mine + (first ? c + half : f));
+          const float4_t t0 = *reinterpret_cast<const float4_t*>(tab + 2 * f), t1 = *reinterpret_cast<const float4_t*>(tab + 2 * f + 4);
+          const float4_t cs{t0[0], t0[2], t1[0], t1[2]}, sn{t0[1], t0[3], t1[1], t1[3]};
+          y = first ? v[i] * cs - other * sn : v[i] * cs + other * sn;
+        }
+      }
+      Act<T>::store4(dst + c, y);
+    }
+    return;
+  }
+  const int block = blockIdx.x - qk_blocks, head = block % G, row0 = block / G * 16;
+  if (tid < 16) {
+    const int t = min(row0 + tid, rows - 1), pos = positions[t];
+    row_page[tid] = (long long)kv_indices[kv_indptr[rev_input_indptr[t]] + pos / kPage] * (long long)kv_page_elements(kv);
+    row_entry[tid] = row0 + tid < rows ? pos % kPage : -1;
+  }
+  const int r = tid >> 4;
+  const T* src = proj + (size_t)min(row0 + r, rows - 1) * ld + v_col + head * kv.vdim;
+  for (int c = (tid & 15) * 4; c < kv.v_pad; c += 64) {
+    float4_t v{0.f, 0.f, 0.f, 0.f};
+    if (c < kv.vdim) v = Act<T>::load4(src + c);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) buf[(c + e) * 17 + r] = v[e];
+  }
+  __syncthreads();
+  T* base = kv_data + (size_t)G * kPage * kv.k_pad + (size_t)head * kv.v_pad * kPage;
+  for (int e = tid; e < kv.v_pad * 4; e += 256) {
+    const int c = e >> 2, r0 = (e & 3) * 4, en = row_entry[r0];
+    const float* v = buf + c * 17 + r0;
+    if (en >= 0 && en % 4 == 0 && row_entry[r0 + 3] == en + 3 && row_page[r0] == row_page[r0 + 3]) {
+      // rows of one request are consecutive positions, so the two in between belong to the run as well
+      Act<T>::store4(base + row_page[r0] + (size_t)c * kPage + en, float4_t{v[0], v[1], v[2], v[3]});
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (row_entry[r0 + i] >= 0) Act<T>::store(base + row_page[r0 + i] + (size_t)c * kPage + row_entry[r0 + i], v[i]);
+    }
+  }
+}
+
 // ---------------------------------------------------------------- which 32-key (or 64-key) steps are visited
 struct StepRange {
   int head, skip_to, total;  // steps [0, head), then [skip_to, ...): `total` of both
@@ -299,14 +413,14 @@ __global__ __launch_bounds__(512) void attn_window_kernel(nf_window_attention_ar
   }
   const float scale2 = a.scale * 1.44269504088896340736f;
 
-  auto page_ptr = [&](int step, int which) {
-    int idx = step * 2 + which;
-    if (idx > last_page) idx = last_page;  // its keys are past every token of the tile: read something mapped
-    return pool + (size_t)pages[idx] * page_elems;
+  // page ids are read a step before the loads that need them
+  auto page_id = [&](int it, int which) {
+    const int idx = steps.at(it) * 2 + which;
+    return pages[idx < last_page ? idx : last_page];  // past the last page the keys are no one's: read something mapped
   };
   B8 kf[2][KD];
-  auto load_k = [&](int step) {
-    const bf16_t* k = page_ptr(step, kpg);
+  auto load_k = [&](int id) {
+    const bf16_t* k = pool + (size_t)id * page_elems;
 #pragma unroll
     for (int j = 0; j < KD; ++j)
       if (j < kd) {
@@ -315,15 +429,21 @@ __global__ __launch_bounds__(512) void attn_window_kernel(nf_window_attention_ar
       }
   };
   const int first = kDecode ? wave : 0, stride = kDecode ? waves : 1;
-  if (first < steps.total) load_k(steps.at(first));
+  if (first >= steps.total && !kDecode) return;
+  const int final_it = steps.total - 1;
+  int k_id = page_id(min(first, final_it), kpg), v_id = page_id(min(first, final_it), vpg);
+  load_k(k_id);
+  k_id = page_id(min(first + stride, final_it), kpg);
   for (int it = first; it < steps.total; it += stride) {
     const int step = steps.at(it), base = step * 32;
     // V of this step, then (after the scores) K of the next: in flight while the softmax runs
     B8 vf[VD];
-    const bf16_t* v = page_ptr(step, vpg) + v_off;
+    const bf16_t* v = pool + (size_t)v_id * page_elems + v_off;
 #pragma unroll
     for (int i = 0; i < VD; ++i)
       if (i < vd) vf[i].u = load_cache<kDecode>(v + (size_t)i * 16 * kPage);
+    const int next_k_id = page_id(min(it + 2 * stride, final_it), kpg);
+    v_id = page_id(min(it + stride, final_it), vpg);
     float4_t s[NB][2];
 #pragma unroll
     for (int n = 0; n < NB; ++n)
@@ -334,7 +454,8 @@ __global__ __launch_bounds__(512) void attn_window_kernel(nf_window_attention_ar
         for (int j = 0; j < KD; ++j)
           if (j < kd) s[n][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[b][j].b, qf[n][j].b, s[n][b], 0, 0, 0);
       }
-    if (it + stride < steps.total) load_k(steps.at(it + stride));
+    if (it + stride < steps.total) load_k(k_id);
+    k_id = next_k_id;
     const bool whole = base + 31 <= p0 && (a.window <= 0 || p1 - base < a.window || base + 31 < a.keep_first);
 #pragma unroll
     for (int n = 0; n < NB; ++n) {
@@ -344,10 +465,10 @@ __global__ __launch_bounds__(512) void attn_window_kernel(nf_window_attention_ar
       for (int b = 0; b < 2; ++b)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          s[n][b][r] *= scale2;
           if (!whole && !sees(pos[n], j0 + 4 * b + r, a.window, a.keep_first)) s[n][b][r] = -INFINITY;
           mx = fmaxf(mx, s[n][b][r]);
         }
+      mx = mx > -1e30f ? mx * scale2 : mx;
       mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
       if (__any(mx > m[n])) {
@@ -362,7 +483,8 @@ __global__ __launch_bounds__(512) void attn_window_kernel(nf_window_attention_ar
       for (int b = 0; b < 2; ++b)
 #pragma unroll
         for (int r = 0; r < 4; r += 2) {
-          const float w0 = __builtin_amdgcn_exp2f(s[n][b][r] - m[n]), w1 = __builtin_amdgcn_exp2f(s[n][b][r + 1] - m[n]);
+          const float w0 = __builtin_amdgcn_exp2f(fmaf(s[n][b][r], scale2, -m[n]));
+          const float w1 = __builtin_amdgcn_exp2f(fmaf(s[n][b][r + 1], scale2, -m[n]));
           l[n] += w0 + w1;
           const uint32_t h2 = f32_to_bf16_pair(w0, w1);
           hi.w[b * 2 + r / 2] = h2;
@@ -495,8 +617,22 @@ int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, i
              "%s: columns %d %d %d do not fit rows of %d", who, q_col, k_col, v_col, ld);
   if (rows == 0) return NF_OK;
   NF_REQUIRE(proj && q_out && kv_data && kv_indptr && kv_indices && rev_input_indptr && positions, "%s: null pointer", who);
-  const dim3 grid((unsigned)rows, (unsigned)((kv->heads + 2 * kv->kv_heads + 3) / 4));
   hipStream_t s = (hipStream_t)stream;
+  const size_t four = 4 * (kv->dtype == NF_BF16 ? 2 : 4);
+  if ((kv->dim | kv->vdim | ld | q_col | k_col | v_col) % 4 == 0 && (uintptr_t)proj % four == 0 &&
+      rot->dims % (rot->interleaved ? 4 : 8) == 0 && (long long)rows * (kv->heads + kv->kv_heads) < (1ll << 31)) {
+    const int qk_blocks = (rows * (kv->heads + kv->kv_heads) + 15) / 16, blocks = qk_blocks + (rows + 15) / 16 * kv->kv_heads;
+    if (kv->dtype == NF_BF16)
+      qkv_append4_kernel<bf16_t><<<blocks, 256, 0, s>>>(*kv, (const bf16_t*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps,
+                                                        *rot, (bf16_t*)q_out, (bf16_t*)kv_data, kv_indptr, kv_indices,
+                                                        rev_input_indptr, positions, rows, qk_blocks);
+    else
+      qkv_append4_kernel<float><<<blocks, 256, 0, s>>>(*kv, (const float*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps,
+                                                       *rot, (float*)q_out, (float*)kv_data, kv_indptr, kv_indices,
+                                                       rev_input_indptr, positions, rows, qk_blocks);
+    return check_launch(who);
+  }
+  const dim3 grid((unsigned)rows, (unsigned)((kv->heads + 2 * kv->kv_heads + 3) / 4));
   if (kv->dtype == NF_BF16)
     qkv_append_kernel<bf16_t><<<grid, 256, 0, s>>>(*kv, (const bf16_t*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot,
                                                    (bf16_t*)q_out, (bf16_t*)kv_data, kv_indptr, kv_indices, rev_input_indptr,
@@ -524,9 +660,13 @@ int nf_window_attention(const nf_window_attention_args* args, nf_stream_t stream
   NF_REQUIRE(a.q && a.out && a.kv_data && a.input_indptr && a.kv_indptr && a.kv_indices && a.rev_input_indptr && a.positions,
              "%s: null pointer", who);
   hipStream_t s = (hipStream_t)stream;
+  NF_REQUIRE(a.kv.heads <= 65535, "%s: %d heads exceed the grid", who, a.kv.heads);
   if (a.kv.dtype == NF_F32) {
-    NF_REQUIRE(a.kv.heads <= 65535, "%s: %d heads exceed the grid", who, a.kv.heads);
     attn_rows_kernel<float><<<dim3((unsigned)a.max_rows, (unsigned)a.kv.heads), 64, 0, s>>>(a);
+    return check_launch(who);
+  }
+  if (!(a.scale > 0.f)) {  // the matrix kernel takes the maximum before it scales
+    attn_rows_kernel<bf16_t><<<dim3((unsigned)a.max_rows, (unsigned)a.kv.heads), 64, 0, s>>>(a);
     return check_launch(who);
   }
   const int kd = a.kv.k_pad / 32, vd = a.kv.v_pad / 16;

@@ -40,7 +40,12 @@ struct Act<bf16_t> {
   }
 };
 
-__device__ __forceinline__ float silu_f32(float g) { return g / (1.f + expf(-g)); }
+// silu in fp32; where the result is rounded to bf16 the hardware's reciprocal and exponential do
+template <class T>
+__device__ __forceinline__ float silu(float g) {
+  if constexpr (std::is_same_v<T, float>) return g / (1.f + expf(-g));
+  else return g * __builtin_amdgcn_rcpf(1.f + __expf(-g));
+}
 
 // Sum over a workgroup of up to 1024 threads; every thread gets it.  `scratch`: 16 floats of LDS that
 // no one else touches between the caller's last barrier and its next one.

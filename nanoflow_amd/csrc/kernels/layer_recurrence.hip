@@ -9,6 +9,19 @@
 // recur_seq_kernel: one workgroup per (request, head) holds the head's state in registers and walks
 // the request's rows, a few at a time through LDS.  Decode (one row): the state is streamed in, used,
 // and streamed out once.
+//
+// Portions of prompts are cut into chunks that are computed side by side, in three launches:
+//   recur_chunk_state_kernel  what every chunk adds to a state that enters it as zero, and the factor the
+//                             entering state is multiplied by;
+//   recur_chunk_scan_kernel   the state that enters each chunk (one pass over the chunks per element), and
+//                             the state the request leaves behind;
+//   recur_chunk_out_kernel    every chunk's outputs from its entering state.
+// Inside a chunk the state lives in MFMA accumulators (v_mfma_f32_16x16x4_f32: products and sums in fp32)
+// and 16 tokens are taken at a time:  o = (decayed q) S + A v,  S <- decays * S + (decayed k)^T v,  A[i][j] =
+// q_i . k_j times the decay between the two.  An accumulator's rows 4g + r are the k index g of the r-th
+// MFMA that multiplies by it, so S and A are operands where they lie.  A token's own decays enter as
+// q 2^(L before i) and k 2^-(L through j), L counted from the start of the 16 tokens; where some L is
+// below -100 fewer tokens are taken at a time.
 #include <algorithm>
 #include <cmath>
 
@@ -146,7 +159,7 @@ __global__ __launch_bounds__(1024) void recur_seq_kernel(nf_recurrence_args a, i
         const int c = e * 64 + lane;
         if (c >= a.vdim) continue;
         const int hc = h * a.vdim + c;
-        float y = o[e] * inv * silu_f32(Act<T>::load((const T*)a.g + (size_t)row * a.g_ld + hc));
+        float y = o[e] * inv * silu<T>(Act<T>::load((const T*)a.g + (size_t)row * a.g_ld + hc));
         if (a.norm_weight) y *= a.norm_weight[hc];
         Act<T>::store((T*)a.out + (size_t)row * a.out_ld + a.out_col + hc, y);
       }
@@ -186,6 +199,548 @@ static int launch_seq(const nf_recurrence_args& a, hipStream_t s) {
   return go(ic<16>{});
 }
 
+// ---------------------------------------------------------------- chunks of a prompt's portion
+constexpr int kStep = 16;           // tokens per step inside a chunk
+constexpr float kMinStepLog2 = -100.f;
+
+struct ChunkSpan {
+  int req, row0, n, slot;  // request, first row, rows (0: no such chunk), index of its chunk in the workspace
+};
+// Chunk `slot` of the launch: chunks of `len` rows, request after request.
+__device__ __forceinline__ ChunkSpan find_chunk(const nf_recurrence_args& a, int slot, int len) {
+  int c = slot;
+  for (int r = a.req_begin; r < a.req_begin + a.req_num; ++r) {
+    const int row0 = a.input_indptr[r], rows = a.input_indptr[r + 1] - row0, n = (rows + len - 1) / len;
+    if (c < n) return {r, row0 + c * len, min(len, rows - c * len), slot};
+    c -= n;
+  }
+  return {-1, 0, 0, slot};
+}
+
+template <int KIND, int NKT, int NVT>
+struct ChunkShape {
+  static constexpr int KP = NKT * 16, VP = 4 * NVT * 16;
+  static constexpr int kPitch = KP + 4, vPitch = VP + 4;
+  static constexpr int kGroups = (kStep * KP / 4 + 255) / 256;  // four-element groups per thread of a staged q or k
+  static constexpr int vGroups = kStep * VP / 4 / 256;
+  static constexpr int kPairs = (kStep * KP / 2 + 255) / 256;   // rotation pairs per thread
+  static constexpr int kParts = 256 / KP, kPartTok = kStep / kParts;  // TOKEN_DECAY: thread = (channel, part of the tokens)
+};
+
+template <int KIND, int NKT, int NVT, bool kQ>
+struct ChunkLds {
+  using C = ChunkShape<KIND, NKT, NVT>;
+  static constexpr bool kToken = KIND == NF_RECURRENCE_TOKEN_DECAY;
+  __attribute__((aligned(16))) float q[kQ ? kStep * C::kPitch : 4];            // raw, or times 2^(L before the token)
+  __attribute__((aligned(16))) float k[kStep * C::kPitch];                     // raw, or times 2^(decay to the end of the step)
+  __attribute__((aligned(16))) float kb[kQ && kToken ? kStep * C::kPitch : 4];  // k 2^-(L through it)
+  __attribute__((aligned(16))) float v[kStep * C::vPitch];
+  __attribute__((aligned(16))) float o[kQ ? kStep * C::vPitch : 4];
+  __attribute__((aligned(16))) float keep[C::KP];                              // TOKEN_DECAY: factor of a state row over the step
+  float part[kToken ? C::kParts : 1][C::KP];
+  float bonus[kStep];
+  __attribute__((aligned(16))) float ss[kStep][4];
+};
+
+// A step's rows in registers: requested one step ahead, so that their latency passes under the step before.
+// Loads are never branched around: rows and columns past the end read a valid place and are masked when they are
+// written to LDS.
+template <class T, int KIND, int NKT, int NVT, bool kQ>
+struct StepLoads {
+  using C = ChunkShape<KIND, NKT, NVT>;
+  float4_t q[kQ ? C::kGroups : 1], k[C::kGroups], v[C::vGroups], g[kQ ? C::vGroups : 1];
+  float cs[KIND == NF_RECURRENCE_FIXED_DECAY ? C::kPairs : 1], sn[KIND == NF_RECURRENCE_FIXED_DECAY ? C::kPairs : 1];
+  float z[KIND == NF_RECURRENCE_TOKEN_DECAY ? C::kPartTok : 1];
+
+  // rows [row, last] exist
+  __device__ __forceinline__ void request(const nf_recurrence_args& a, int h, int row, int last) {
+    const int tid = threadIdx.x;
+#pragma unroll
+    for (int i = 0; i < C::kGroups; ++i) {
+      const int e = i * 256 + tid, t = e / (C::KP / 4), c = e % (C::KP / 4) * 4;
+      const size_t r = (size_t)min(row + t, last);
+      const int cc = c < a.dim ? c : 0;
+      if constexpr (kQ) q[i] = Act<T>::load4((const T*)a.q + r * a.q_ld + h * a.dim + cc);
+      k[i] = Act<T>::load4((const T*)a.k + r * a.k_ld + h * a.dim + cc);
+    }
+#pragma unroll
+    for (int i = 0; i < C::vGroups; ++i) {
+      const int e = i * 256 + tid, t = e / (C::VP / 4), c = e % (C::VP / 4) * 4;
+      const size_t r = (size_t)min(row + t, last);
+      const int cc = c < a.vdim ? c : 0;
+      v[i] = Act<T>::load4((const T*)a.v + r * a.v_ld + h * a.vdim + cc);
+      if constexpr (kQ) g[i] = Act<T>::load4((const T*)a.g + r * a.g_ld + h * a.vdim + cc);
+    }
+    if constexpr (KIND == NF_RECURRENCE_FIXED_DECAY) {
+      const int half = a.rot.dims / 2;
+      if (half > 0) {
+#pragma unroll
+        for (int i = 0; i < C::kPairs; ++i) {
+          const int e = i * 256 + tid, t = e / (C::KP / 2), f = min(e % (C::KP / 2), half - 1);
+          const float* tab = a.rot.table + ((size_t)a.positions[min(row + t, last)] * half + f) * 2;
+          cs[i] = tab[0];
+          sn[i] = tab[1];
+        }
+      }
+    } else {
+      const int c = tid % C::KP, part = tid / C::KP;
+#pragma unroll
+      for (int i = 0; i < C::kPartTok; ++i) {
+        const size_t r = (size_t)min(row + part * C::kPartTok + i, last);
+        const int cc = h * a.dim + (c < a.dim ? c : 0);
+        z[i] = a.z[r * a.z_ld + cc];
+        for (int s = 1; s < a.z_shares; ++s) z[i] += a.z[((size_t)s * a.total_rows + r) * a.z_ld + cc];
+      }
+    }
+  }
+
+  // The first n rows to LDS, the others as zeros.
+  __device__ __forceinline__ void store(const nf_recurrence_args& a, ChunkLds<KIND, NKT, NVT, kQ>& s, int n) const {
+    const float4_t zero{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < C::kGroups; ++i) {
+      const int e = i * 256 + (int)threadIdx.x, t = e / (C::KP / 4), c = e % (C::KP / 4) * 4;
+      if (C::KP < 64 && t >= kStep) continue;
+      const bool live = t < n && c < a.dim;
+      if constexpr (kQ) *reinterpret_cast<float4_t*>(s.q + t * C::kPitch + c) = live ? q[i] : zero;
+      *reinterpret_cast<float4_t*>(s.k + t * C::kPitch + c) = live ? k[i] * a.k_scale : zero;
+    }
+#pragma unroll
+    for (int i = 0; i < C::vGroups; ++i) {
+      const int e = i * 256 + (int)threadIdx.x, t = e / (C::VP / 4), c = e % (C::VP / 4) * 4;
+      *reinterpret_cast<float4_t*>(s.v + t * C::vPitch + c) = t < n && c < a.vdim ? v[i] : zero;
+    }
+  }
+
+  // FIXED_DECAY, after store() and a barrier: q and k rotated where they lie.
+  __device__ __forceinline__ void rotate(const nf_recurrence_args& a, ChunkLds<KIND, NKT, NVT, kQ>& s) const {
+    const int half = a.rot.dims / 2;
+#pragma unroll
+    for (int i = 0; i < C::kPairs; ++i) {
+      const int e = i * 256 + (int)threadIdx.x, t = e / (C::KP / 2), f = e % (C::KP / 2);
+      if (f >= half || t >= kStep) continue;
+      const int c1 = t * C::kPitch + (a.rot.interleaved ? 2 * f : f), c2 = c1 + (a.rot.interleaved ? 1 : half);
+      const float k1 = s.k[c1], k2 = s.k[c2];
+      s.k[c1] = k1 * cs[i] - k2 * sn[i];
+      s.k[c2] = k2 * cs[i] + k1 * sn[i];
+      if constexpr (kQ) {
+        const float q1 = s.q[c1], q2 = s.q[c2];
+        s.q[c1] = q1 * cs[i] - q2 * sn[i];
+        s.q[c2] = q2 * cs[i] + q1 * sn[i];
+      }
+    }
+  }
+};
+
+// What a thread of a TOKEN_DECAY chunk keeps of its key channel.
+struct ChannelDecay {
+  float w0, lw[kStep], before, total;
+};
+
+// TOKEN_DECAY, between two barriers after store(): the log2 decays of this thread's tokens, their sum to LDS, and the
+// tokens' bonus terms from raw q and k.
+template <class T, int NKT, int NVT, bool kQ>
+__device__ __forceinline__ void decay_sums(const nf_recurrence_args& a, ChunkLds<NF_RECURRENCE_TOKEN_DECAY, NKT, NVT, kQ>& s,
+                                           const StepLoads<T, NF_RECURRENCE_TOKEN_DECAY, NKT, NVT, kQ>& ld, ChannelDecay& d, int h,
+                                           int n) {
+  using C = ChunkShape<NF_RECURRENCE_TOKEN_DECAY, NKT, NVT>;
+  const int c = threadIdx.x % C::KP, part = threadIdx.x / C::KP;
+  float sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < C::kPartTok; ++i) {
+    const float l = fmaxf(-expf(ld.z[i] + d.w0) * 1.44269504088896340736f, -126.f);
+    d.lw[i] = part * C::kPartTok + i < n && c < a.dim ? l : 0.f;
+    sum += d.lw[i];
+  }
+  s.part[part][c] = sum;
+  if constexpr (kQ) {
+    const int t = threadIdx.x >> 4, l = threadIdx.x & 15;
+    float b = 0.f;
+    for (int e = l; e < a.dim; e += 16) b += s.q[t * C::kPitch + e] * s.k[t * C::kPitch + e] * a.u[(size_t)h * a.dim + e];
+#pragma unroll
+    for (int m = 8; m > 0; m >>= 1) b += __shfl_xor(b, m, 64);
+    if (l == 0) s.bonus[t] = b;
+  }
+}
+
+// The channel's decay before this thread's tokens and over the step; whether it stays above kMinStepLog2.
+template <int NKT, int NVT, bool kQ>
+__device__ __forceinline__ bool decay_totals(ChunkLds<NF_RECURRENCE_TOKEN_DECAY, NKT, NVT, kQ>& s, ChannelDecay& d) {
+  using C = ChunkShape<NF_RECURRENCE_TOKEN_DECAY, NKT, NVT>;
+  const int c = threadIdx.x % C::KP, part = threadIdx.x / C::KP;
+  d.before = d.total = 0.f;
+#pragma unroll
+  for (int p = 0; p < C::kParts; ++p) {
+    const float x = s.part[p][c];
+    if (p < part) d.before += x;
+    d.total += x;
+  }
+  return d.total >= kMinStepLog2;
+}
+
+// q, k and k's quotient form from raw q and k.
+template <int NKT, int NVT, bool kQ>
+__device__ __forceinline__ void decay_apply(ChunkLds<NF_RECURRENCE_TOKEN_DECAY, NKT, NVT, kQ>& s, const ChannelDecay& d) {
+  using C = ChunkShape<NF_RECURRENCE_TOKEN_DECAY, NKT, NVT>;
+  const int c = threadIdx.x % C::KP, part = threadIdx.x / C::KP;
+  float after = 0.f;  // sums of later tokens only: no difference of large sums
+#pragma unroll
+  for (int p = C::kParts - 1; p > 0; --p)
+    if (p > part) after += s.part[p][c];
+  float before = d.before;
+#pragma unroll
+  for (int i = 0; i < C::kPartTok; ++i) {
+    float own_after = after;
+#pragma unroll
+    for (int j = C::kPartTok - 1; j > 0; --j)
+      if (j > i) own_after += d.lw[j];
+    const int at = (part * C::kPartTok + i) * C::kPitch + c;
+    const float k = s.k[at];
+    s.k[at] = k * __builtin_amdgcn_exp2f(own_after);
+    if constexpr (kQ) {
+      s.q[at] *= __builtin_amdgcn_exp2f(before);
+      before += d.lw[i];
+      s.kb[at] = k * __builtin_amdgcn_exp2f(-before);
+    }
+  }
+  if (part == 0) s.keep[c] = __builtin_amdgcn_exp2f(d.total);
+}
+
+// S <- keep * S + k^T v over the step; the wavefront's NVT column tiles.
+template <int KIND, int NKT, int NVT, bool kQ>
+__device__ __forceinline__ void update_state(float4_t (&S)[NKT][NVT], const ChunkLds<KIND, NKT, NVT, kQ>& s, int n, float ld2,
+                                             const float (&vr)[NVT][4]) {
+  using C = ChunkShape<KIND, NKT, NVT>;
+  const int lane = threadIdx.x & 63, l16 = lane & 15, g = lane >> 4;
+  float kf[4];  // FIXED_DECAY: decay from the token to the end of the step
+  float keep_all = 1.f;
+  if constexpr (KIND == NF_RECURRENCE_FIXED_DECAY) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) kf[r] = 4 * g + r < n ? __builtin_amdgcn_exp2f((float)(n - 1 - 4 * g - r) * ld2) : 0.f;
+    keep_all = __builtin_amdgcn_exp2f((float)n * ld2);
+  }
+#pragma unroll
+  for (int kt = 0; kt < NKT; ++kt) {
+    float4_t keep{keep_all, keep_all, keep_all, keep_all};
+    if constexpr (KIND == NF_RECURRENCE_TOKEN_DECAY) keep = *reinterpret_cast<const float4_t*>(s.keep + kt * 16 + 4 * g);
+    float k[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      k[r] = s.k[(4 * g + r) * C::kPitch + kt * 16 + l16];
+      if constexpr (KIND == NF_RECURRENCE_FIXED_DECAY) k[r] *= kf[r];
+    }
+#pragma unroll
+    for (int vt = 0; vt < NVT; ++vt) {
+      S[kt][vt] *= keep;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) S[kt][vt] = __builtin_amdgcn_mfma_f32_16x16x4f32(k[r], vr[vt][r], S[kt][vt], 0, 0, 0);
+    }
+  }
+}
+
+// Workspace: [chunks][heads] states in fragment order -- tile (kt, vt) of 16 x 16, lane, four rows -- then
+// (TOKEN_DECAY) [chunks][heads][kp] factors.
+__device__ __forceinline__ float* chunk_states(const nf_recurrence_args& a, const RecurrenceDims& pd, int slot, int h) {
+  return (float*)a.workspace + ((size_t)slot * a.heads + h) * pd.kp * pd.vp;
+}
+__device__ __forceinline__ float* chunk_factors(const nf_recurrence_args& a, const RecurrenceDims& pd, int max_chunks, int slot, int h) {
+  return (float*)a.workspace + (size_t)max_chunks * a.heads * pd.kp * pd.vp + ((size_t)slot * a.heads + h) * pd.kp;
+}
+
+template <class T, int KIND, int NKT, int NVT>
+__global__ __launch_bounds__(256) void recur_chunk_state_kernel(nf_recurrence_args a, int len, int max_chunks) {
+  using C = ChunkShape<KIND, NKT, NVT>;
+  constexpr bool kToken = KIND == NF_RECURRENCE_TOKEN_DECAY;
+  __shared__ ChunkLds<KIND, NKT, NVT, false> s;
+  const RecurrenceDims pd = padded(a.dim, a.vdim);
+  const int h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, g = lane >> 4;
+  const ChunkSpan ch = find_chunk(a, blockIdx.x, len);
+  if (ch.n == 0) return;
+  const float ld2 = kToken ? 0.f : a.log2_decay[h];
+  const int last = ch.row0 + ch.n - 1;
+  StepLoads<T, KIND, NKT, NVT, false> ld;
+  ld.request(a, h, ch.row0, last);
+  ChannelDecay d;
+  const int channel = threadIdx.x % C::KP;
+  if constexpr (kToken) d.w0 = a.w0[h * a.dim + (channel < a.dim ? channel : 0)];
+  float log2_all = 0.f;
+  float4_t S[NKT][NVT];
+#pragma unroll
+  for (int kt = 0; kt < NKT; ++kt)
+#pragma unroll
+    for (int vt = 0; vt < NVT; ++vt) S[kt][vt] = float4_t{0.f, 0.f, 0.f, 0.f};
+  for (int t0 = 0; t0 < ch.n; t0 += kStep) {
+    const int n = min(kStep, ch.n - t0);
+    __syncthreads();
+    ld.store(a, s, n);
+    if constexpr (kToken) {
+      decay_sums<T, NKT, NVT, false>(a, s, ld, d, h, n);
+      __syncthreads();
+      decay_totals<NKT, NVT, false>(s, d);  // every factor formed here is at most 1, whatever the logs
+      log2_all += d.total;
+      decay_apply<NKT, NVT, false>(s, d);
+    } else {
+      __syncthreads();
+      ld.rotate(a, s);
+    }
+    if (t0 + kStep < ch.n) ld.request(a, h, ch.row0 + t0 + kStep, last);
+    __syncthreads();
+    float vr[NVT][4];
+#pragma unroll
+    for (int vt = 0; vt < NVT; ++vt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) vr[vt][r] = s.v[(4 * g + r) * C::vPitch + (wave * NVT + vt) * 16 + l16];
+    update_state<KIND, NKT, NVT, false>(S, s, n, ld2, vr);
+  }
+  float* dst = chunk_states(a, pd, ch.slot, h);
+  const int v_tiles = pd.vp / 16;
+#pragma unroll
+  for (int kt = 0; kt < NKT; ++kt)
+#pragma unroll
+    for (int vt = 0; vt < NVT; ++vt) {
+      const int tile = wave * NVT + vt;
+      if (kt * 16 < pd.kp && tile < v_tiles) *reinterpret_cast<float4_t*>(dst + ((size_t)(kt * v_tiles + tile) * 64 + lane) * 4) = S[kt][vt];
+    }
+  if constexpr (kToken)
+    if ((int)threadIdx.x < pd.kp) chunk_factors(a, pd, max_chunks, ch.slot, h)[threadIdx.x] = exp2f(log2_all);
+}
+
+template <int KIND>
+__global__ __launch_bounds__(256) void recur_chunk_scan_kernel(nf_recurrence_args a, int len, int max_chunks) {
+  const RecurrenceDims pd = padded(a.dim, a.vdim);
+  const int req = a.req_begin + blockIdx.x, h = blockIdx.y;
+  const int row0 = a.input_indptr[req], rows = a.input_indptr[req + 1] - row0;
+  if (rows <= 0) return;
+  int slot0 = 0;
+  for (int r = a.req_begin; r < req; ++r) slot0 += (a.input_indptr[r + 1] - a.input_indptr[r] + len - 1) / len;
+  const int chunks = (rows + len - 1) / len, state_slot = a.state_slots[req];
+  const int f4 = blockIdx.z * 256 + threadIdx.x, e = f4 * 4;  // four rows of a column, in fragment order
+  if (e < pd.kp * pd.vp) {
+    const int v_tiles = pd.vp / 16, lane = f4 & 63, tile = f4 >> 6;
+    const int k = tile / v_tiles * 16 + (lane >> 4) * 4, c = tile % v_tiles * 16 + (lane & 15);
+    float* state = a.state + ((size_t)state_slot * a.heads + h) * pd.kp * pd.vp + (size_t)k * pd.vp + c;
+    const float ld2 = KIND == NF_RECURRENCE_FIXED_DECAY ? a.log2_decay[h] : 0.f;
+    float4_t cur{0.f, 0.f, 0.f, 0.f};
+    if (a.positions[row0] != 0)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) cur[r] = state[(size_t)r * pd.vp];
+    constexpr int kAhead = 4;  // loads do not depend on the running state
+    for (int c0 = 0; c0 < chunks; c0 += kAhead) {
+      float4_t add[kAhead], f[kAhead];
+#pragma unroll
+      for (int i = 0; i < kAhead; ++i) {
+        const int ci = min(c0 + i, chunks - 1);
+        add[i] = *reinterpret_cast<const float4_t*>(chunk_states(a, pd, slot0 + ci, h) + e);
+        if constexpr (KIND == NF_RECURRENCE_TOKEN_DECAY) {
+          f[i] = *reinterpret_cast<const float4_t*>(chunk_factors(a, pd, max_chunks, slot0 + ci, h) + k);
+        } else {
+          const float x = exp2f((float)min(len, rows - ci * len) * ld2);
+          f[i] = float4_t{x, x, x, x};
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < kAhead; ++i) {
+        if (c0 + i >= chunks) continue;
+        *reinterpret_cast<float4_t*>(chunk_states(a, pd, slot0 + c0 + i, h) + e) = cur;
+        cur = cur * f[i] + add[i];
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) state[(size_t)r * pd.vp] = cur[r];
+  }
+  if (a.shift_x && h == 0 && blockIdx.z == 0)
+    for (int c = threadIdx.x * 4; c < a.shift_ld; c += 1024)
+      *reinterpret_cast<float4_t*>(a.shift_state + (size_t)state_slot * a.shift_ld + c) =
+          *reinterpret_cast<const float4_t*>(a.shift_x + (size_t)(row0 + rows - 1) * a.shift_ld + c);
+}
+
+template <class T, int KIND, int NKT, int NVT>
+__global__ __launch_bounds__(256) void recur_chunk_out_kernel(nf_recurrence_args a, int len) {
+  using C = ChunkShape<KIND, NKT, NVT>;
+  constexpr bool kToken = KIND == NF_RECURRENCE_TOKEN_DECAY;
+  __shared__ ChunkLds<KIND, NKT, NVT, true> s;
+  const RecurrenceDims pd = padded(a.dim, a.vdim);
+  const int h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, g = lane >> 4;
+  const ChunkSpan ch = find_chunk(a, blockIdx.x, len);
+  if (ch.n == 0) return;
+  const float ld2 = kToken ? 0.f : a.log2_decay[h];
+  const int last = ch.row0 + ch.n - 1;
+  StepLoads<T, KIND, NKT, NVT, true> ld;
+  ld.request(a, h, ch.row0, last);
+  ChannelDecay d;
+  const int channel = threadIdx.x % C::KP;
+  if constexpr (kToken) d.w0 = a.w0[h * a.dim + (channel < a.dim ? channel : 0)];
+  float4_t S[NKT][NVT];
+  const float* src = chunk_states(a, pd, ch.slot, h);
+  const int v_tiles = pd.vp / 16;
+#pragma unroll
+  for (int kt = 0; kt < NKT; ++kt)
+#pragma unroll
+    for (int vt = 0; vt < NVT; ++vt) {
+      const int tile = wave * NVT + vt;
+      const bool in = kt * 16 < pd.kp && tile < v_tiles;
+      S[kt][vt] = *reinterpret_cast<const float4_t*>(src + ((size_t)(in ? kt * v_tiles + tile : 0) * 64 + lane) * 4);
+      if (!in) S[kt][vt] = float4_t{0.f, 0.f, 0.f, 0.f};
+    }
+  float4_t norm_w[C::vGroups];
+#pragma unroll
+  for (int i = 0; i < C::vGroups; ++i) {
+    const int c = (i * 256 + (int)threadIdx.x) % (C::VP / 4) * 4;
+    norm_w[i] = float4_t{1.f, 1.f, 1.f, 1.f};
+    if (a.norm_weight && c < a.vdim) norm_w[i] = *reinterpret_cast<const float4_t*>(a.norm_weight + h * a.vdim + c);
+  }
+  int n;
+  for (int t0 = 0; t0 < ch.n; t0 += n) {
+    n = min(kStep, ch.n - t0);
+    const int row = ch.row0 + t0;
+    for (;;) {
+      __syncthreads();
+      ld.store(a, s, n);
+      __syncthreads();
+      if constexpr (kToken) {
+        decay_sums<T, NKT, NVT, true>(a, s, ld, d, h, n);
+        __syncthreads();
+        const bool ok = decay_totals<NKT, NVT, true>(s, d);
+        if (__syncthreads_or(!ok) && n > 1) {
+          n = n > 4 ? 4 : 1;
+          continue;
+        }
+        decay_apply<NKT, NVT, true>(s, d);
+      } else {
+        ld.rotate(a, s);
+      }
+      break;
+    }
+    float4_t gate[C::vGroups];
+#pragma unroll
+    for (int i = 0; i < C::vGroups; ++i) gate[i] = ld.g[i];
+    if (t0 + n < ch.n) ld.request(a, h, row + n, last);
+    __syncthreads();
+    // A^T[j][i] in fragment form: lane holds j = 4g + r of i = l16; and the part of o that the entering state gives
+    float4_t at{0.f, 0.f, 0.f, 0.f}, o[NVT];
+#pragma unroll
+    for (int vt = 0; vt < NVT; ++vt) o[vt] = float4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int kt = 0; kt < NKT; ++kt) {
+      const float4_t q = *reinterpret_cast<const float4_t*>(s.q + l16 * C::kPitch + kt * 16 + 4 * g);
+      const float4_t k = *reinterpret_cast<const float4_t*>((kToken ? s.kb : s.k) + l16 * C::kPitch + kt * 16 + 4 * g);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        at = __builtin_amdgcn_mfma_f32_16x16x4f32(k[r], q[r], at, 0, 0, 0);
+#pragma unroll
+        for (int vt = 0; vt < NVT; ++vt) o[vt] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[r], S[kt][vt][r], o[vt], 0, 0, 0);
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int j = 4 * g + r, i = l16;
+      if constexpr (!kToken) {
+        at[r] = j <= i ? at[r] * __builtin_amdgcn_exp2f((float)(i - j) * ld2) : 0.f;
+      } else {
+        at[r] = j < i ? at[r] : 0.f;
+        if (j == i) at[r] = s.bonus[i];
+      }
+      if (j >= n || i >= n) at[r] = 0.f;
+    }
+    if constexpr (!kToken) {  // row i = 4g + r of o: the entering state has decayed i + 1 times
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float f = __builtin_amdgcn_exp2f((float)(4 * g + r + 1) * ld2);
+#pragma unroll
+        for (int vt = 0; vt < NVT; ++vt) o[vt][r] *= f;
+      }
+    }
+    float vr[NVT][4];
+#pragma unroll
+    for (int vt = 0; vt < NVT; ++vt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        vr[vt][r] = s.v[(4 * g + r) * C::vPitch + (wave * NVT + vt) * 16 + l16];
+        o[vt] = __builtin_amdgcn_mfma_f32_16x16x4f32(at[r], vr[vt][r], o[vt], 0, 0, 0);
+      }
+    update_state<KIND, NKT, NVT, true>(S, s, n, ld2, vr);
+
+    // per-head norm over all columns, gate; through LDS, so that rows are written in whole runs
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      float ss = 0.f;
+#pragma unroll
+      for (int vt = 0; vt < NVT; ++vt) {
+        ss += o[vt][r] * o[vt][r];
+        s.o[(4 * g + r) * C::vPitch + (wave * NVT + vt) * 16 + l16] = o[vt][r];
+      }
+#pragma unroll
+      for (int m = 8; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
+      if (l16 == 0) s.ss[4 * g + r][wave] = ss;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < C::vGroups; ++i) {
+      const int e = i * 256 + (int)threadIdx.x, t = e / (C::VP / 4), c = e % (C::VP / 4) * 4;
+      const float4_t part = *reinterpret_cast<const float4_t*>(s.ss[t]);
+      const float inv = a.out_scale / sqrtf((part[0] + part[1] + part[2] + part[3]) / (float)a.vdim + a.eps);
+      float4_t y = *reinterpret_cast<const float4_t*>(s.o + t * C::vPitch + c) * inv * norm_w[i];
+#pragma unroll
+      for (int x = 0; x < 4; ++x) y[x] *= silu<T>(gate[i][x]);
+      if (t < n && c < a.vdim)
+        Act<T>::store4((T*)a.out + (size_t)(row + t) * a.out_ld + a.out_col + (size_t)h * a.vdim + c, y);
+    }
+  }
+}
+
+// Chunk length and count of a launch, or 0 chunks where the sequential kernel is the better one (few rows per request,
+// states beyond the tiles) or the workspace is too small.
+struct ChunkPlan {
+  int len, chunks;
+};
+static size_t chunk_bytes(int heads, int dim, int vdim) {
+  const RecurrenceDims pd = padded(dim, vdim);
+  return (size_t)heads * (pd.kp * pd.vp + pd.kp) * sizeof(float);
+}
+constexpr int kMinChunk = 64, kMaxChunkRequests = 64;
+static ChunkPlan chunk_plan(const nf_recurrence_args& a) {
+  const RecurrenceDims pd = padded(a.dim, a.vdim);
+  if (pd.kp > 128 || pd.vp > 128 || (long long)a.rows < 24ll * a.req_num || !a.workspace) return {0, 0};
+  // rows are read and written four elements at a time
+  const size_t four = 4 * (a.dtype == NF_BF16 ? 2 : 4);
+  const uintptr_t at = (uintptr_t)a.q | (uintptr_t)a.k | (uintptr_t)a.v | (uintptr_t)a.g | (uintptr_t)a.out;
+  if ((a.dim | a.vdim | a.q_ld | a.k_ld | a.v_ld | a.g_ld | a.out_ld | a.out_col) % 4 || at % four ||
+      (uintptr_t)a.norm_weight % 16)
+    return {0, 0};
+  int len = kMinChunk;
+  while (len < 256 && (long long)(a.rows / (2 * len)) * a.heads >= 512) len *= 2;
+  const int chunks = a.rows / len + a.req_num;
+  if ((size_t)chunks * chunk_bytes(a.heads, a.dim, a.vdim) > a.workspace_bytes) return {0, 0};
+  return {len, chunks};
+}
+
+template <class T, int KIND, int NKT, int NVT>
+static int launch_chunks(const nf_recurrence_args& a, const ChunkPlan& p, hipStream_t s) {
+  const RecurrenceDims pd = padded(a.dim, a.vdim);
+  const dim3 grid((unsigned)p.chunks, (unsigned)a.heads);
+  recur_chunk_state_kernel<T, KIND, NKT, NVT><<<grid, 256, 0, s>>>(a, p.len, p.chunks);
+  int rc = check_launch("nf_linear_recurrence (chunk states)");
+  if (rc) return rc;
+  const unsigned parts = (unsigned)((pd.kp * pd.vp / 4 + 255) / 256);
+  recur_chunk_scan_kernel<KIND><<<dim3((unsigned)a.req_num, (unsigned)a.heads, parts), 256, 0, s>>>(a, p.len, p.chunks);
+  rc = check_launch("nf_linear_recurrence (chunk scan)");
+  if (rc) return rc;
+  recur_chunk_out_kernel<T, KIND, NKT, NVT><<<grid, 256, 0, s>>>(a, p.len);
+  return check_launch("nf_linear_recurrence (chunk outputs)");
+}
+
+template <class T, int KIND>
+static int launch_recurrence(nf_recurrence_args a, hipStream_t s) {
+  if (KIND == NF_RECURRENCE_TOKEN_DECAY) a.k_scale = 1.f;
+  const ChunkPlan p = chunk_plan(a);
+  if (p.chunks == 0) return launch_seq<T, KIND>(a, s);
+  const RecurrenceDims pd = padded(a.dim, a.vdim);
+  const bool wide = pd.vp > 64;
+  if (pd.kp <= 32) return wide ? launch_chunks<T, KIND, 2, 2>(a, p, s) : launch_chunks<T, KIND, 2, 1>(a, p, s);
+  if (pd.kp <= 64) return wide ? launch_chunks<T, KIND, 4, 2>(a, p, s) : launch_chunks<T, KIND, 4, 1>(a, p, s);
+  return wide ? launch_chunks<T, KIND, 8, 2>(a, p, s) : launch_chunks<T, KIND, 8, 1>(a, p, s);
+}
+
 }  // namespace nf
 
 using namespace nf;
@@ -198,7 +753,11 @@ size_t nf_recurrence_state_elements(int dim, int vdim) {
   return (size_t)pd.kp * pd.vp;
 }
 
-size_t nf_recurrence_workspace_bytes(int heads, int dim, int vdim, int max_rows, int max_requests) { return 0; }
+size_t nf_recurrence_workspace_bytes(int heads, int dim, int vdim, int max_rows, int max_requests) {
+  if (heads <= 0 || dim <= 0 || vdim <= 0 || max_rows <= 0) return 0;
+  const size_t chunks = (size_t)max_rows / kMinChunk + std::min(max_requests, kMaxChunkRequests);
+  return chunks * chunk_bytes(heads, dim, vdim);
+}
 
 int nf_linear_recurrence(const nf_recurrence_args* args, nf_stream_t stream) {
   const char* who = "nf_linear_recurrence";
@@ -227,10 +786,10 @@ int nf_linear_recurrence(const nf_recurrence_args* args, nf_stream_t stream) {
   NF_REQUIRE(!a.shift_x || (a.shift_state && a.shift_ld > 0 && a.shift_ld % 4 == 0), "%s: shift state missing", who);
   hipStream_t s = (hipStream_t)stream;
   if (a.dtype == NF_BF16)
-    return a.kind == NF_RECURRENCE_FIXED_DECAY ? launch_seq<bf16_t, NF_RECURRENCE_FIXED_DECAY>(a, s)
-                                               : launch_seq<bf16_t, NF_RECURRENCE_TOKEN_DECAY>(a, s);
-  return a.kind == NF_RECURRENCE_FIXED_DECAY ? launch_seq<float, NF_RECURRENCE_FIXED_DECAY>(a, s)
-                                             : launch_seq<float, NF_RECURRENCE_TOKEN_DECAY>(a, s);
+    return a.kind == NF_RECURRENCE_FIXED_DECAY ? launch_recurrence<bf16_t, NF_RECURRENCE_FIXED_DECAY>(a, s)
+                                               : launch_recurrence<bf16_t, NF_RECURRENCE_TOKEN_DECAY>(a, s);
+  return a.kind == NF_RECURRENCE_FIXED_DECAY ? launch_recurrence<float, NF_RECURRENCE_FIXED_DECAY>(a, s)
+                                             : launch_recurrence<float, NF_RECURRENCE_TOKEN_DECAY>(a, s);
 }
 
 }  // extern "C"

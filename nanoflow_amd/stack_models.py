@@ -79,7 +79,7 @@ def random_tensors(cfg: dict, seed: int = 0, rank: int = 16) -> dict:
         elif ".mu." in name:
             x = rng.random(n, dtype=np.float32)
         elif leaf == "w0":
-            x = -4.0 + 1.5 * x
+            x = -7.0 + 6.0 * rng.random(n, dtype=np.float32)
         elif leaf in ("u", "sink"):
             x = 0.5 * x
         elif name in ("embed", "pos"):

@@ -129,7 +129,8 @@ void update(int nranks, std::vector<vortexUpdateData>& updateData) {
                      update_d.keepTokenListLength, update_d.input_tokens, update_d.prefillTokensNum,
                      complete_input_tokens.data());
   }
-  if (ActiveStackModel && !update_d.logit_rows) {  // the last row of every request is sampled
+  const bool default_rows = ActiveStackModel && !update_d.logit_rows;
+  if (default_rows) {  // the last row of every request is sampled
     const int req = update_d.decodePrefillBorder + update_d.prefillNum;
     last_rows.resize((size_t)req);
     for (int i = 0; i < req; ++i) last_rows[i] = update_d.input_indptr[i + 1] - 1;
@@ -141,6 +142,10 @@ void update(int nranks, std::vector<vortexUpdateData>& updateData) {
   shared_state.updates_ptr = &updateData;
   global_sync->barrier();
   global_sync->barrier();
+  if (default_rows) {  // the caller's struct may serve the next iteration as well
+    update_d.logit_rows = nullptr;
+    update_d.logit_rows_num = 0;
+  }
 }
 
 void config(int nranks, std::vector<vortexConfigData>& config) {

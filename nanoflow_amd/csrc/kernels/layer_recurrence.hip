@@ -74,7 +74,7 @@ __global__ __launch_bounds__(1024) void recur_seq_kernel(nf_recurrence_args a, i
   const int slice = tid >> 8, col = slice * 64 + (tid & 15) * 4, krow = (tid & 255) >> 4, swave = (tid & 255) >> 6;
   const int row0 = a.input_indptr[req], row1 = a.input_indptr[req + 1];
   if (row0 >= row1) return;
-  const int slot = a.state_slots[req];
+  const int slot = a.state_slots[req], np = pd.kp / 16;
   float* state = a.state + ((size_t)slot * a.heads + h) * pd.kp * pd.vp;
   const bool fresh = a.positions[row0] == 0;
   const float decay = KIND == NF_RECURRENCE_FIXED_DECAY ? exp2f(a.log2_decay[h]) : 1.f;
@@ -126,7 +126,8 @@ __global__ __launch_bounds__(1024) void recur_seq_kernel(nf_recurrence_args a, i
       float4_t o{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int i = 0; i < NP; ++i) {
-        const int k = min(krow + 16 * i, pd.kp - 1);  // rows past the state's last hold zeros of no effect
+        if (i >= np) continue;  // the state has np x 16 rows
+        const int k = krow + 16 * i;
         const float w = KIND == NF_RECURRENCE_TOKEN_DECAY ? sw[t * pd.kp + k] : decay;
         o += S[i] * sq[t * pd.kp + k];
         S[i] = S[i] * w + v * sk[t * pd.kp + k];

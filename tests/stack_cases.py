@@ -1,0 +1,62 @@
+"""Shared by the tests of layer-stack models: small configurations, batches over permuted pages."""
+import numpy as np
+
+from nanoflow_amd import stack_models, synth
+
+
+def retention(heads=3, dim=24, vdim=40, rot=16, base=500.0, decay=(0.5, 0.97, 1.0)):
+    return {"type": "retention", "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "decay": list(decay)[:heads],
+                                           "rot": {"dims": rot, "base": base}}}
+
+
+def parallel(heads=6, kv_heads=2, dim=32, vdim=48, window=21, keep=5, scale=0.2, rot=20, base=300.0, right_heads=3,
+             right_dim=20, left_scale=0.7, right_scale=1.6):
+    return {"type": "parallel", "mixer": {
+        "left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale,
+                 "mask": {"size": window, "keep_first": keep}, "rot": {"dims": rot, "base": base}},
+        "left_scale": left_scale, "right": {"heads": right_heads, "dim": right_dim}, "right_scale": right_scale}}
+
+
+def config(layers, width=104, vocab=211, ff=88, eps=1e-5, max_positions=600):
+    """layers: mixers, each with its feed-forward width (None: no feed-forward) or the default one."""
+    out = []
+    for entry in layers:
+        mixer, f = entry if isinstance(entry, tuple) else (entry, ff)
+        out.append({**mixer, "mlp": None if f is None else {"kind": "dense", "ff": f}})
+    return {"architecture": "Zovovik", "width": width, "vocab": vocab, "max_positions": max_positions, "norm": {"eps": eps}, "layers": out}
+
+
+# sizes that are not multiples of 8, equal and unequal head counts, no feed-forward, a window of one, windows without kept tokens
+CONFIGS = {
+    "mixed": config([retention(), parallel(), (retention(heads=1, dim=16, vdim=16, rot=16, decay=(0.9,)), None), parallel(
+        heads=4, kv_heads=4, dim=16, vdim=16, window=33, keep=0, rot=16, right_heads=1, right_dim=64)]),
+    "odd": config([parallel(heads=5, kv_heads=1, dim=18, vdim=10, window=7, keep=3, rot=6, right_heads=2, right_dim=10),
+                   retention(heads=2, dim=10, vdim=6, rot=4, decay=(0.8, 0.999))], width=52, vocab=97, ff=70, eps=1e-3),
+    "wide heads": config([parallel(heads=2, kv_heads=1, dim=160, vdim=144, window=64, keep=16, rot=64, right_heads=1, right_dim=128),
+                          retention(heads=1, dim=96, vdim=128, rot=96, decay=(0.99,))], width=128, ff=160),
+    "retention only": config([retention(heads=2, dim=64, vdim=64, rot=32, decay=(0.99, 0.9)), retention(heads=2, dim=32, vdim=96, rot=32)]),
+    "window of one": config([parallel(heads=20, kv_heads=1, dim=8, vdim=8, window=1, keep=0, rot=8, right_heads=2, right_dim=8)], width=64),
+}
+
+
+def tensors(cfg, seed=0, rank=12):
+    """(bfloat16 bit patterns, the same values as float arrays)"""
+    bits = stack_models.random_tensors(cfg, seed, rank)
+    return bits, {k: stack_models.bits_to_f32(v) for k, v in bits.items()}
+
+
+def batch(decode, portions, seed=0, extra_pages=5):
+    """A batch of decode requests (history lengths) and portions (history, tokens) over permuted pages."""
+    return synth.make_batch(decode, portions, vocab=10, seed=seed, extra_pages=extra_pages)
+
+
+def history_batch(b):
+    """The batch that brings every request of b to where b starts, over the same pages (None: all start at zero)."""
+    lens = np.diff(b.input_indptr)
+    prev = b.kv_len - lens
+    reqs = [i for i in range(len(prev)) if prev[i] > 0]
+    if not reqs:
+        return None, []
+    h = synth.make_batch([], [(0, int(prev[i])) for i in reqs], vocab=10, seed=1)
+    h.kv_indices = np.concatenate([b.kv_indices[b.kv_indptr[i]:b.kv_indptr[i] + (int(prev[i]) + 15) // 16] for i in reqs]).astype(np.int32)
+    return h, reqs

@@ -1,0 +1,190 @@
+"""Layer-stack models without a GPU: the plain implementation against other statements of the same mechanisms,
+configurations, state slots in the batch former."""
+import ctypes
+import json
+
+import numpy as np
+import pytest
+
+from nanoflow_amd import pllm_python as P, stack_models
+from oracle import stack_oracle as S
+
+import stack_cases as cases
+
+
+def test_fixed_decay_recurrence_is_a_decayed_sum():
+    rng = np.random.default_rng(0)
+    q, k, v = rng.standard_normal((9, 2, 5)), rng.standard_normal((9, 2, 5)), rng.standard_normal((9, 2, 3))
+    decay = [0.5, 0.9]
+    o = S.fixed_decay_recurrence(q, k, v, decay)
+    for t in range(9):
+        for h in range(2):
+            want = sum(decay[h] ** (t - j) * (q[t, h] @ k[j, h]) * v[j, h] for j in range(t + 1))
+            np.testing.assert_allclose(o[t, h], want, rtol=1e-12)
+
+
+def test_bonus_recurrence_is_a_decayed_sum():
+    rng = np.random.default_rng(1)
+    r, k, v = rng.standard_normal((8, 2, 4)), rng.standard_normal((8, 2, 4)), rng.standard_normal((8, 2, 3))
+    w, u = rng.random((8, 2, 4)), rng.standard_normal((2, 4))
+    o = S.bonus_recurrence(r, k, v, w, u)
+    for t in range(8):
+        for h in range(2):
+            want = (r[t, h] * u[h] * k[t, h]).sum() * v[t, h]
+            for j in range(t):
+                keep = np.prod(w[j + 1:t, h], axis=0)
+                want = want + (r[t, h] * keep * k[j, h]).sum() * v[j, h]
+            np.testing.assert_allclose(o[t, h], want, rtol=1e-12)
+
+
+@pytest.mark.parametrize("interleaved", [False, True])
+def test_rotation_depends_on_distance_only_and_leaves_the_rest(interleaved):
+    rng = np.random.default_rng(2)
+    a, b = rng.standard_normal((1, 1, 10)), rng.standard_normal((1, 1, 10))
+    dots = [(S.rotate(a, [p + 7], 6, 100.0, interleaved) * S.rotate(b, [p], 6, 100.0, interleaved))[..., :6].sum() for p in (0, 3, 50)]
+    np.testing.assert_allclose(dots, dots[0], rtol=1e-12)
+    np.testing.assert_array_equal(S.rotate(a, [9], 6, 100.0, interleaved)[..., 6:], a[..., 6:])
+    np.testing.assert_array_equal(S.rotate(a, [0], 6, 100.0, interleaved), a)
+
+
+def test_window_mask_edges():
+    m = S.window_mask(40, 8, 3)
+    assert m[30, 23] and not m[30, 22] and m[30, 2] and not m[30, 3] and not m[30, 31] and m[5, 0]
+
+
+def test_sink_takes_its_share():
+    q = np.zeros((1, 1, 4))
+    o = S.sink_attention(q, np.zeros((1, 1, 4)), np.ones((1, 1, 2)), np.ones((1, 1), bool), 1.0, [np.log(3.0)])
+    np.testing.assert_allclose(o, 0.25)
+    np.testing.assert_allclose(S.sink_attention(q, np.zeros((1, 1, 4)), np.ones((1, 1, 2)), np.ones((1, 1), bool), 1.0, None), 1.0)
+
+
+def test_a_prefix_does_not_see_what_follows():
+    cfg = cases.CONFIGS["mixed"]
+    _, t = cases.tensors(cfg)
+    tokens = np.random.default_rng(3).integers(0, cfg["vocab"], 50)
+    whole = S.forward(cfg, t, tokens)
+    np.testing.assert_allclose(S.forward(cfg, t, tokens[:31]), whole[:31], rtol=1e-9, atol=1e-9)
+
+
+def _set(tmp_path, cfg, dtype="bfloat16", pages=8, slots=2):
+    p = tmp_path / "config.json"
+    p.write_text(json.dumps(cfg))
+    P.stackSetConfig(str(p), dtype, 64, pages, slots)
+
+
+def test_configurations_are_checked(tmp_path):
+    try:
+        for name, cfg in cases.CONFIGS.items():
+            _set(tmp_path, cfg, slots=3)
+            assert P.stackStateSlots() == 3 and P.maxPageNum() == 8
+        good = cases.CONFIGS["mixed"]
+        bad = [({**good, "architecture": "Nosuch"}, "unknown architecture"), ({k: v for k, v in good.items() if k != "width"}, "width"),
+               ({**good, "layers": []}, "layers"), (cases.config([cases.parallel(heads=5, kv_heads=2)]), "multiple"),
+               (cases.config([cases.retention(heads=3, decay=(0.5, 0.5))]), "decay"),
+               (cases.config([cases.retention(rot=17)]), "rotated"), (cases.config([cases.parallel(window=0)]), "mask"),
+               (cases.config([cases.retention(dim=300)]), "head sizes"),
+               ({**good, "layers": [{**good["layers"][0], "type": "nosuch"}]}, "unknown mixer"),
+               ({**good, "layers": [{**good["layers"][0], "mlp": {"kind": "nosuch", "ff": 8}}]}, "feed-forward")]
+        for cfg, word in bad:
+            with pytest.raises(P.NanoflowPipelineError, match=word):
+                _set(tmp_path, cfg)
+        with pytest.raises(P.NanoflowPipelineError, match="dtype"):
+            _set(tmp_path, good, dtype="float16")
+    finally:
+        P.setModelConfig(_llama_config(tmp_path))       # the process's other tests configure Llama models
+    assert P.stackStateSlots() == 0
+
+
+def _llama_config(tmp_path):
+    import os
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    return os.path.join(root, "nanoflow_amd", "config_all", "llama3-8B.json")
+
+
+def test_pipeline_file_names_a_stack_model(tmp_path):
+    cfg = cases.CONFIGS["odd"]
+    stack_models.save_model(str(tmp_path / "m"), cfg, {"head": np.zeros((2, 2), np.float32)})
+    base = {"model_configs": {"max_batch_size": 32, "kv_pages": 12, "state_slots": 5, "dtype": "float32"}, "pipeline_configs": {}}
+    try:
+        for model in (cfg, {"path": "m"}, {"path": str(tmp_path / "m")}):
+            f = tmp_path / "pipeline.json"
+            f.write_text(json.dumps({"model": model, **base}))
+            P.setModelConfig(str(f))
+            assert P.stackStateSlots() == 5 and P.maxPageNum() == 12
+    finally:
+        P.setModelConfig(_llama_config(tmp_path))
+
+
+def test_safetensors_of_random_tensors_reads_back(tmp_path):
+    from safetensors import safe_open
+    cfg = cases.CONFIGS["mixed"]
+    bits, _ = cases.tensors(cfg)
+    stack_models.save_model(str(tmp_path), cfg, bits)
+    with safe_open(str(tmp_path / "model.safetensors"), "pt") as f:
+        assert set(f.keys()) == set(bits) == set(stack_models.tensor_shapes(cfg))
+        for k in ("embed", "l1.mix.left.sink", "l1.mix.right.u"):
+            np.testing.assert_array_equal(f.get_tensor(k).float().numpy(), stack_models.bits_to_f32(bits[k]))
+
+
+def _drive(former, cycles=400):
+    """Runs the scheduler without a GPU; yields the formed batches."""
+    for _ in range(cycles):
+        st = former.state()
+        if st["queued"] + st["decoding"] + st["prefilling"] == 0:
+            return
+        former.schedule()
+        b = former.form()
+        yield b, former.state_slots()
+        former.advance(0.0)
+
+
+def test_state_slots_limit_admission_and_are_used_again():
+    f = P.BatchFormer(64, 16, 40, 40, 40, 0, 20, 6)
+    f.set_state_slots(3)
+    rng = np.random.default_rng(0)
+    for i in range(11):
+        f.add_request(i, rng.integers(0, 9, int(rng.integers(1, 70))), int(rng.integers(2, 9)))
+    seen, most = set(), 0
+    for b, slots in _drive(f):
+        n = b["decodePrefillBorder"] + b["prefillNum"]
+        assert len(slots) == n and len(set(slots.tolist())) == n and set(slots.tolist()) <= {0, 1, 2}
+        seen |= set(slots.tolist())
+        most = max(most, n)
+    assert f.state()["retired"] == 11 and most == 3 and seen == {0, 1, 2}
+    f.close()
+
+
+def test_a_request_keeps_its_slot_and_pages_until_it_retires():
+    f = P.BatchFormer(64, 16, 24, 24, 24, 0, 30, 8)
+    f.set_state_slots(4)
+    for i, n in enumerate((50, 20, 33)):
+        f.add_request(i, np.zeros(n, np.int32), 5 + i)
+    owner = {}
+    for b, slots in _drive(f):
+        for r, s in enumerate(slots.tolist()):
+            first_page = int(b["kv_indices"][b["kv_indptr"][r]])
+            start = b["per_token_offset"][b["input_indptr"][r]] == 0
+            assert start or owner[s] == first_page          # the request in a slot is recognised by its first page
+            owner[s] = first_page
+    f.close()
+
+
+def test_without_slots_nothing_changes():
+    f = P.BatchFormer(64, 16, 40, 40, 40, 0, 20, 6)
+    f.add_request(0, np.zeros(10, np.int32), 3)
+    for b, slots in _drive(f):
+        assert len(slots) == 0
+    f.close()
+
+
+def test_argument_errors_without_a_gpu():
+    from nanoflow_amd import kernels as K
+    l = K.lib()
+    a = K.RecurrenceArgs(dtype=K.BF16, kind=7, heads=1, dim=8, vdim=8)
+    assert l.nf_linear_recurrence(ctypes.byref(a), None) == -1 and b"kind" in l.nf_last_error()
+    w = K.WindowAttentionArgs(kv=K.KVLayout(K.BF16, 4, 3, 8, 8, 32, 16, 16))
+    assert l.nf_window_attention(ctypes.byref(w), None) == -1 and b"kv heads" in l.nf_last_error()
+    assert l.nf_gemm_nk_bf16(None, None, None, 4, 12, 64, None, 0, None) == -1
+    assert l.nf_norm_add_rows(0, None, 17, None, None, 0, None, 4, 8, 8, 1e-5, None) == -1
+    assert l.nf_recurrence_state_elements(20, 40) == 32 * 48

@@ -24,14 +24,20 @@ struct Act<float> {
   static __device__ __forceinline__ void store(float* p, float v) { *p = v; }
   static __device__ __forceinline__ float4_t load4(const float* p) { return *reinterpret_cast<const float4_t*>(p); }
   static __device__ __forceinline__ void store4(float* p, float4_t v) { *reinterpret_cast<float4_t*>(p) = v; }
+  // four elements as they are stored, for loads that wait in registers
+  typedef float4_t raw4;
+  static __device__ __forceinline__ raw4 load_raw4(const float* p) { return *reinterpret_cast<const float4_t*>(p); }
+  static __device__ __forceinline__ float4_t widen4(raw4 w) { return w; }
 };
 template <>
 struct Act<bf16_t> {
   static constexpr int dtype = NF_BF16;
   static __device__ __forceinline__ float load(const bf16_t* p) { return bf16_bits_to_f32(p->bits); }
   static __device__ __forceinline__ void store(bf16_t* p, float v) { p->bits = (uint16_t)(f32_to_bf16_pair(v, 0.f) & 0xffffu); }
-  static __device__ __forceinline__ float4_t load4(const bf16_t* p) {
-    const u32x2 w = *reinterpret_cast<const u32x2*>(p);
+  typedef u32x2 raw4;
+  static __device__ __forceinline__ raw4 load_raw4(const bf16_t* p) { return *reinterpret_cast<const u32x2*>(p); }
+  static __device__ __forceinline__ float4_t load4(const bf16_t* p) { return widen4(load_raw4(p)); }
+  static __device__ __forceinline__ float4_t widen4(raw4 w) {
     return float4_t{bf16_bits_to_f32(w.x & 0xffffu), __uint_as_float(w.x & 0xffff0000u), bf16_bits_to_f32(w.y & 0xffffu),
                     __uint_as_float(w.y & 0xffff0000u)};
   }

@@ -249,7 +249,7 @@ struct ChunkLds {
 template <class T, int KIND, int NKT, int NVT, bool kQ>
 struct StepLoads {
   using C = ChunkShape<KIND, NKT, NVT>;
-  float4_t q[kQ ? C::kGroups : 1], k[C::kGroups], v[C::vGroups], g[kQ ? C::vGroups : 1];
+  typename Act<T>::raw4 q[kQ ? C::kGroups : 1], k[C::kGroups], v[C::vGroups], g[kQ ? C::vGroups : 1];
   float cs[KIND == NF_RECURRENCE_FIXED_DECAY ? C::kPairs : 1], sn[KIND == NF_RECURRENCE_FIXED_DECAY ? C::kPairs : 1];
   float z[KIND == NF_RECURRENCE_TOKEN_DECAY ? C::kPartTok : 1];
 
@@ -261,16 +261,16 @@ struct StepLoads {
       const int e = i * 256 + tid, t = e / (C::KP / 4), c = e % (C::KP / 4) * 4;
       const size_t r = (size_t)min(row + t, last);
       const int cc = c < a.dim ? c : 0;
-      if constexpr (kQ) q[i] = Act<T>::load4((const T*)a.q + r * a.q_ld + h * a.dim + cc);
-      k[i] = Act<T>::load4((const T*)a.k + r * a.k_ld + h * a.dim + cc);
+      if constexpr (kQ) q[i] = Act<T>::load_raw4((const T*)a.q + r * a.q_ld + h * a.dim + cc);
+      k[i] = Act<T>::load_raw4((const T*)a.k + r * a.k_ld + h * a.dim + cc);
     }
 #pragma unroll
     for (int i = 0; i < C::vGroups; ++i) {
       const int e = i * 256 + tid, t = e / (C::VP / 4), c = e % (C::VP / 4) * 4;
       const size_t r = (size_t)min(row + t, last);
       const int cc = c < a.vdim ? c : 0;
-      v[i] = Act<T>::load4((const T*)a.v + r * a.v_ld + h * a.vdim + cc);
-      if constexpr (kQ) g[i] = Act<T>::load4((const T*)a.g + r * a.g_ld + h * a.vdim + cc);
+      v[i] = Act<T>::load_raw4((const T*)a.v + r * a.v_ld + h * a.vdim + cc);
+      if constexpr (kQ) g[i] = Act<T>::load_raw4((const T*)a.g + r * a.g_ld + h * a.vdim + cc);
     }
     if constexpr (KIND == NF_RECURRENCE_FIXED_DECAY) {
       const int half = a.rot.dims / 2;
@@ -303,13 +303,13 @@ struct StepLoads {
       const int e = i * 256 + (int)threadIdx.x, t = e / (C::KP / 4), c = e % (C::KP / 4) * 4;
       if (C::KP < 64 && t >= kStep) continue;
       const bool live = t < n && c < a.dim;
-      if constexpr (kQ) *reinterpret_cast<float4_t*>(s.q + t * C::kPitch + c) = live ? q[i] : zero;
-      *reinterpret_cast<float4_t*>(s.k + t * C::kPitch + c) = live ? k[i] * a.k_scale : zero;
+      if constexpr (kQ) *reinterpret_cast<float4_t*>(s.q + t * C::kPitch + c) = live ? Act<T>::widen4(q[i]) : zero;
+      *reinterpret_cast<float4_t*>(s.k + t * C::kPitch + c) = live ? Act<T>::widen4(k[i]) * a.k_scale : zero;
     }
 #pragma unroll
     for (int i = 0; i < C::vGroups; ++i) {
       const int e = i * 256 + (int)threadIdx.x, t = e / (C::VP / 4), c = e % (C::VP / 4) * 4;
-      *reinterpret_cast<float4_t*>(s.v + t * C::vPitch + c) = t < n && c < a.vdim ? v[i] : zero;
+      *reinterpret_cast<float4_t*>(s.v + t * C::vPitch + c) = t < n && c < a.vdim ? Act<T>::widen4(v[i]) : zero;
     }
   }
 
@@ -448,8 +448,10 @@ __device__ __forceinline__ float* chunk_factors(const nf_recurrence_args& a, con
   return (float*)a.workspace + (size_t)max_chunks * a.heads * pd.kp * pd.vp + ((size_t)slot * a.heads + h) * pd.kp;
 }
 
+// The bound of two workgroups a CU keeps the state in VGPRs: with more room the compiler moves it to accumulation
+// registers, and every scaling of it through moves between the two files.
 template <class T, int KIND, int NKT, int NVT>
-__global__ __launch_bounds__(256) void recur_chunk_state_kernel(nf_recurrence_args a, int len, int max_chunks) {
+__global__ __launch_bounds__(256, 2) void recur_chunk_state_kernel(nf_recurrence_args a, int len, int max_chunks) {
   using C = ChunkShape<KIND, NKT, NVT>;
   constexpr bool kToken = KIND == NF_RECURRENCE_TOKEN_DECAY;
   __shared__ ChunkLds<KIND, NKT, NVT, false> s;
@@ -556,7 +558,7 @@ __global__ __launch_bounds__(256) void recur_chunk_scan_kernel(nf_recurrence_arg
 }
 
 template <class T, int KIND, int NKT, int NVT>
-__global__ __launch_bounds__(256) void recur_chunk_out_kernel(nf_recurrence_args a, int len) {
+__global__ __launch_bounds__(256, 2) void recur_chunk_out_kernel(nf_recurrence_args a, int len) {
   using C = ChunkShape<KIND, NKT, NVT>;
   constexpr bool kToken = KIND == NF_RECURRENCE_TOKEN_DECAY;
   __shared__ ChunkLds<KIND, NKT, NVT, true> s;
@@ -583,13 +585,6 @@ __global__ __launch_bounds__(256) void recur_chunk_out_kernel(nf_recurrence_args
       S[kt][vt] = *reinterpret_cast<const float4_t*>(src + ((size_t)(in ? kt * v_tiles + tile : 0) * 64 + lane) * 4);
       if (!in) S[kt][vt] = float4_t{0.f, 0.f, 0.f, 0.f};
     }
-  float4_t norm_w[C::vGroups];
-#pragma unroll
-  for (int i = 0; i < C::vGroups; ++i) {
-    const int c = (i * 256 + (int)threadIdx.x) % (C::VP / 4) * 4;
-    norm_w[i] = float4_t{1.f, 1.f, 1.f, 1.f};
-    if (a.norm_weight && c < a.vdim) norm_w[i] = *reinterpret_cast<const float4_t*>(a.norm_weight + h * a.vdim + c);
-  }
   int n;
   for (int t0 = 0; t0 < ch.n; t0 += n) {
     n = min(kStep, ch.n - t0);
@@ -612,7 +607,7 @@ __global__ __launch_bounds__(256) void recur_chunk_out_kernel(nf_recurrence_args
       }
       break;
     }
-    float4_t gate[C::vGroups];
+    typename Act<T>::raw4 gate[C::vGroups];
 #pragma unroll
     for (int i = 0; i < C::vGroups; ++i) gate[i] = ld.g[i];
     if (t0 + n < ch.n) ld.request(a, h, row + n, last);
@@ -680,9 +675,11 @@ __global__ __launch_bounds__(256) void recur_chunk_out_kernel(nf_recurrence_args
       const int e = i * 256 + (int)threadIdx.x, t = e / (C::VP / 4), c = e % (C::VP / 4) * 4;
       const float4_t part = *reinterpret_cast<const float4_t*>(s.ss[t]);
       const float inv = a.out_scale / sqrtf((part[0] + part[1] + part[2] + part[3]) / (float)a.vdim + a.eps);
-      float4_t y = *reinterpret_cast<const float4_t*>(s.o + t * C::vPitch + c) * inv * norm_w[i];
+      float4_t y = *reinterpret_cast<const float4_t*>(s.o + t * C::vPitch + c) * inv;
+      if (a.norm_weight && c < a.vdim) y *= *reinterpret_cast<const float4_t*>(a.norm_weight + h * a.vdim + c);
+      const float4_t g4 = Act<T>::widen4(gate[i]);
 #pragma unroll
-      for (int x = 0; x < 4; ++x) y[x] *= silu<T>(gate[i][x]);
+      for (int x = 0; x < 4; ++x) y[x] *= silu<T>(g4[x]);
       if (t < n && c < a.vdim)
         Act<T>::store4((T*)a.out + (size_t)(row + t) * a.out_ld + a.out_col + (size_t)h * a.vdim + c, y);
     }
@@ -709,7 +706,9 @@ static ChunkPlan chunk_plan(const nf_recurrence_args& a) {
       (uintptr_t)a.norm_weight % 16)
     return {0, 0};
   int len = kMinChunk;
-  while (len < 256 && (long long)(a.rows / (2 * len)) * a.heads >= 512) len *= 2;
+  // longer chunks, fewer states through memory, as long as every CU has the workgroups it can hold
+  const int enough = pd.kp * pd.vp > 64 * 64 ? 512 : 1024;
+  while (len < 256 && (long long)(a.rows / (2 * len)) * a.heads >= enough) len *= 2;
   const int chunks = a.rows / len + a.req_num;
   if ((size_t)chunks * chunk_bytes(a.heads, a.dim, a.vdim) > a.workspace_bytes) return {0, 0};
   return {len, chunks};

@@ -241,6 +241,14 @@ def test_a_key_at_the_windows_edge(dtype, query):
             close(got[-1], want[-1], dtype, f"key {key} decode {n_decode}")
 
 
+@pytest.mark.parametrize("scale", [0.0, -0.3])
+def test_scales_that_are_not_positive(scale):
+    b = cases.batch([40], [(0, 50)], seed=2)
+    for dtype in DTYPES:
+        got, want = attention_case(dtype, 4, 2, 32, 32, 20, 3, b, 1, seed=1, scale=scale)
+        close(got, want, dtype)
+
+
 def test_long_decode_context_and_many_requests():
     b = cases.batch(np.random.default_rng(0).integers(1, 700, 80).tolist(), [], seed=1)
     got, want = attention_case(BF16, 8, 2, 64, 64, 300, 20, b, 80, seed=2)

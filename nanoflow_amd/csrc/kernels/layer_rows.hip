@@ -1,6 +1,6 @@
 // Row operators of the layer-stack pipeline: embedding plus learned positions, norm of a sublayer's
 // output added to the residual stream, token shift, tanh, the gathered final norm, fp32 argmax.
-// HBM-bound; one workgroup per row, 16-byte accesses, the row kept in registers between the
+// HBM-bound; one workgroup per row (token shift: per 1024 columns of a row), 16-byte accesses, the row kept in registers between the
 // reduction and the write.  The residual stream is fp32.
 #include "layer_common.h"
 
@@ -91,7 +91,8 @@ __global__ __launch_bounds__(kRowThreads) void token_shift_kernel(
   const int t = blockIdx.x, req = rev_input_indptr[t];
   const float* prev = nullptr;  // the token before this one: a row of the batch, the state, or nothing
   if (positions[t] > 0) prev = t > input_indptr[req] ? x + (size_t)(t - 1) * ld : shift_state + (size_t)state_slots[req] * ld;
-  for (int c = threadIdx.x * 4; c < ld; c += kRowThreads * 4) {
+  const int c = (blockIdx.y * kRowThreads + threadIdx.x) * 4;
+  if (c < ld) {
     const float4_t h = *reinterpret_cast<const float4_t*>(x + (size_t)t * ld + c);
     const float4_t p = prev ? *reinterpret_cast<const float4_t*>(prev + c) : float4_t{0.f, 0.f, 0.f, 0.f};
     for (int s = 0; s < n_mix; ++s) {
@@ -238,11 +239,12 @@ int nf_token_shift(int dtype, const float* x, const float* shift_state, const fl
   NF_REQUIRE(x && shift_state && mu && out && input_indptr && rev_input_indptr && positions && state_slots,
              "nf_token_shift: null pointer");
   hipStream_t s = (hipStream_t)stream;
+  const dim3 grid((unsigned)rows, (unsigned)((ld / 4 + kRowThreads - 1) / kRowThreads));
   if (dtype == NF_BF16)
-    token_shift_kernel<bf16_t><<<rows, kRowThreads, 0, s>>>(x, shift_state, mu, (bf16_t*)out, n_mix, input_indptr,
+    token_shift_kernel<bf16_t><<<grid, kRowThreads, 0, s>>>(x, shift_state, mu, (bf16_t*)out, n_mix, input_indptr,
                                                             rev_input_indptr, positions, state_slots, rows, ld);
   else
-    token_shift_kernel<float><<<rows, kRowThreads, 0, s>>>(x, shift_state, mu, (float*)out, n_mix, input_indptr,
+    token_shift_kernel<float><<<grid, kRowThreads, 0, s>>>(x, shift_state, mu, (float*)out, n_mix, input_indptr,
                                                            rev_input_indptr, positions, state_slots, rows, ld);
   return check_launch("nf_token_shift");
 }

@@ -2,7 +2,9 @@
 layers).  Zovovik: retention, windowed attention with kept first tokens and a sink, a token-shift recurrence
 with data-dependent decay, two mixers side by side.  Fipuzen: attention with a unit sink, a query temperature
 and a gate per head, latent attention, lightning attention, a mixture of experts with identity experts, token
-inputs to every layer.  Test infrastructure only: one function per mechanism, whole sequences at once, nothing
+inputs to every layer.  Pudadra: differential attention over a window on convolved projections with capped
+scores, latent attention over a window, experts in groups of which some are left out, a gated shared
+expert.  Test infrastructure only: one function per mechanism, whole sequences at once, nothing
 shared with the product path.
 
 A model is (config, tensors): the parsed config.json and a dict name -> numpy array (any float type).
@@ -210,11 +212,11 @@ def lightning_mixer(t, pre, m, eps, h):
     return linear(t, pre + "o", rms_norm(o, eps, t[pre + "norm"]) * sigmoid(linear(t, pre + "g", h)))
 
 
-def latent_attention(q_plain, q_turned, latent, k_turned, w_uk, w_uv, scale):
+def latent_attention(q_plain, q_turned, latent, k_turned, w_uk, w_uv, scale, mask=None):
     """q_plain [T, H, d], q_turned [T, H, r], latent [T, c], k_turned [T, r], w_uk [H, d, c], w_uv [H, e, c]: keys and
     values of every head are written out and attended to one head at a time."""
     T, H, _ = q_plain.shape
-    mask = window_mask(T, T + 1, 0)
+    mask = window_mask(T, T + 1, 0) if mask is None else mask
     out = np.empty((T, H, w_uv.shape[1]))
     for h in range(H):
         k, v = latent @ w_uk[h].T, latent @ w_uv[h].T
@@ -287,10 +289,132 @@ def fipuzen_forward(cfg, t, tokens, want_layers=False):
     return (logits, np.stack(layers)) if want_layers else logits
 
 
+# ---------------------------------------------------------------- Pudadra
+
+def short_conv(u, w):
+    """u [T, C], w [C, taps]: every channel is mixed over time with the taps - 1 values before it, zeros before the first."""
+    T, taps = u.shape[0], w.shape[1]
+    padded = np.concatenate([np.zeros((taps - 1, u.shape[1])), u])
+    return sum(padded[j:j + T] * f64(w)[:, j] for j in range(taps))
+
+
+def stretched_frequencies(f, factor, low, high, original):
+    """Frequencies whose wavelength is short against `original` positions stay, long ones are divided by `factor`, and
+    in between one goes over into the other."""
+    turns = original * f / (2 * np.pi)          # original / wavelength
+    s = np.clip((turns - low) / (high - low), 0.0, 1.0)
+    return np.where(turns > high, f, np.where(turns < low, f / factor, (1 - s) * f / factor + s * f))
+
+
+def rotate_by(x, angles):
+    """x [T, heads, d], angles [T, n]: dimensions i and i + n are turned by angle i, those from 2n on stay."""
+    n = angles.shape[1]
+    c, s = np.cos(angles)[:, None, :], np.sin(angles)[:, None, :]
+    u, v = x[..., :n], x[..., n:2 * n]
+    return np.concatenate([u * c - v * s, v * c + u * s, x[..., 2 * n:]], axis=-1)
+
+
+def capped(s, cap):
+    return s if cap is None else cap * np.tanh(s / cap)
+
+
+def map_weight(lq1, lk1, lq2, lk2, diff):
+    return np.exp(f64(lq1) @ f64(lk1)) - np.exp(f64(lq2) @ f64(lk2)) + diff
+
+
+def differential_attention(q, k, v, mask, scale, cap, weight, diff, eps):
+    """q [T, H, 2, d], k [T, G, 2, d], v [T, G, e]: two attentions over the same values, the second taken off `weight`
+    times, and what is left normed per head."""
+    T, H = q.shape[:2]
+    per = H // k.shape[1]
+    out = np.empty((T, H, v.shape[-1]))
+    for h in range(H):
+        g = h // per
+        a = [softmax(np.where(mask, capped((q[:, h, x] @ k[:, g, x].T) * scale, cap), -np.inf)) @ v[:, g] for x in (0, 1)]
+        out[:, h] = rms_norm(a[0] - weight * a[1], eps) * (1.0 - diff)
+    return out
+
+
+def differential_attention_mixer(t, pre, m, eps, h, positions):
+    T, H, G, d = h.shape[0], m["heads"], m["kv_heads"], m["dim"]
+    q, k, v = (short_conv(linear(t, pre + s, h), t[pre + s + ".conv"]) for s in "qkv")
+    rot = m["rot"]
+    f = f64(rot["base"]) ** (-2.0 * np.arange(rot["dims"] // 2) / max(rot["dims"], 1))
+    if rot.get("scaling"):
+        f = stretched_frequencies(f, **rot["scaling"])
+    angles = f64(positions)[:, None] * f
+    turn = lambda x, n: rotate_by(x.reshape(T, n * 2, d), angles).reshape(T, n, 2, d)
+    weight = map_weight(*(t[pre + s] for s in ("lq1", "lk1", "lq2", "lk2")), m["diff"])
+    o = differential_attention(turn(q, H), turn(k, G), v.reshape(T, G, m["vdim"]), window_mask(T, m["mask"]["size"], 0), m["scale"],
+                               m.get("softcap"), weight, m["diff"], eps)
+    return linear(t, pre + "o", o.reshape(T, -1))
+
+
+def windowed_latent_attention_mixer(t, pre, m, eps, h, positions):
+    T, H, d, r, c = h.shape[0], m["heads"], m["dim"], m["rot_dim"], m["kv_rank"]
+    q = linear(t, pre + "q", h).reshape(T, H, d + r)
+    down = linear(t, pre + "dkv", h)
+    latent = rms_norm(down[:, :c], eps, t[pre + "dkv.norm"])
+    turn = lambda x: rotate(x, positions, r, m["rot"]["base"], True)
+    o = latent_attention(q[..., :d], turn(q[..., d:]), latent, turn(down[:, None, c:])[:, 0], f64(t[pre + "uk"]).reshape(H, d, c),
+                         f64(t[pre + "uv"]).reshape(H, -1, c), m["scale"], window_mask(T, m["mask"]["size"], 0))
+    return linear(t, pre + "o", o.reshape(T, -1))
+
+
+def grouped_choice(s, top, count, keep):
+    """The `top` largest of s [T, outputs] among the `keep` of `count` runs of neighbours whose largest entries are largest."""
+    T, n = s.shape
+    best = s.reshape(T, count, n // count).max(axis=-1)
+    kept = np.argsort(-best, axis=-1, kind="stable")[:, :keep]
+    open_ = np.zeros((T, count), bool)
+    np.put_along_axis(open_, kept, True, axis=1)
+    return np.argsort(np.where(np.repeat(open_, n // count, axis=1), -s, np.inf), axis=-1, kind="stable")[:, :top]
+
+
+def shared_expert(t, pre, h):
+    y = linear(t, pre + "down", squared_relu(linear(t, pre + "up", h)))
+    return sigmoid(linear(t, pre + "sg", h)) * y
+
+
+def grouped_mixture(t, pre, m, h):
+    r = m["router"]
+    s = softmax(linear(t, pre + "router", h))
+    g = r.get("groups") or {"count": 1, "keep": 1}
+    chosen = grouped_choice(s, r["top"], g["count"], g["keep"])
+    y = shared_expert(t, pre + "shared.", h) if m.get("shared") else np.zeros_like(h)
+    for token in range(h.shape[0]):
+        for e in chosen[token]:
+            y[token] += s[token, e] * linear(t, f"{pre}e{e}.down", squared_relu(linear(t, f"{pre}e{e}.up", h[token])))
+    return y
+
+
+def pudadra_forward(cfg, t, tokens, want_layers=False):
+    tokens = np.asarray(tokens)
+    positions, eps, mult = np.arange(len(tokens)), cfg["norm"]["eps"], cfg["residual_mult"]
+    norm = lambda x, name: rms_norm(x, eps, 1.0 + f64(t[name]))
+    x = f64(t["embed"])[tokens]
+    layers = []
+    for i, layer in enumerate(cfg["layers"]):
+        pre, m, f = f"l{i}.", layer["mixer"], layer.get("mlp")
+        mix = {"attention": differential_attention_mixer, "latent_attention": windowed_latent_attention_mixer}[layer["type"]]
+        x = x + mult * mix(t, pre + "mix.", m, eps, norm(x, pre + "norm1"), positions)
+        if f:
+            h = norm(x, pre + "norm2")
+            if f["kind"] == "dense":
+                x = x + mult * linear(t, pre + "mlp.down", gelu_erf(linear(t, pre + "mlp.up", h)))
+            else:
+                x = x + mult * grouped_mixture(t, pre + "mlp.", f, h)
+        layers.append(x)
+    logits = linear(t, "embed", norm(x, "final.norm")) * cfg["logit_scale"]
+    return (logits, np.stack(layers)) if want_layers else logits
+
+
 def forward(cfg, t, tokens, want_layers=False):
     """Logits [T, vocab] of a whole sequence (and the residual stream after every layer)."""
     if cfg["architecture"] == "Fipuzen":
         return fipuzen_forward(cfg, t, tokens, want_layers)
+    if cfg["architecture"] == "Pudadra":
+        return pudadra_forward(cfg, t, tokens, want_layers)
     tokens = np.asarray(tokens)
     positions = np.arange(len(tokens))
     eps = cfg["norm"]["eps"]

@@ -310,6 +310,8 @@ NF_API int nf_gemm_nk_bf16(const uint16_t* A, const uint16_t* B, uint16_t* D, in
                            size_t workspace_bytes, nf_stream_t stream);
 NF_API int nf_gemm_nk_relu2_bf16(const uint16_t* A, const uint16_t* B, uint16_t* D, int M, int N, int K,
                                  void* workspace, size_t workspace_bytes, nf_stream_t stream);
+NF_API int nf_gemm_nk_gelu_bf16(const uint16_t* A, const uint16_t* B, uint16_t* D, int M, int N, int K,
+                                 void* workspace, size_t workspace_bytes, nf_stream_t stream);
 NF_API int nf_gemm_nk_silu_bf16(const uint16_t* A, const uint16_t* B, uint16_t* D, int M, int N, int K,
                                 void* workspace, size_t workspace_bytes, nf_stream_t stream);
 NF_API int nf_gemm_nk_bias_bf16(const uint16_t* A, const uint16_t* B, const uint16_t* bias, uint16_t* D, int M, int N,
@@ -339,15 +341,24 @@ typedef struct nf_routing {
 } nf_routing;
 NF_API int nf_routing_max_tiles(int sorted_rows, int experts, int tile_rows);
 /* Scores s = softmax of the router's outputs (the sum of `shares` fp32 [rows, ld] slices, `outputs` of the columns);
- * the `top` largest of s + correction are chosen (the smaller index where two are equal), their weights are
- * s * scale.  Outputs from `experts` on are identity experts.  outputs <= 1024, top <= 64. */
-NF_API int nf_route(const float* z, int shares, int ld, int rows, int outputs, int experts, int top, const float* correction,
-                    float scale, const nf_routing* routing, nf_stream_t stream);
+ * the `top` largest of s + correction (null: none) are chosen (the smaller index where two are equal), their weights are
+ * s * scale.  Outputs from `experts` on are identity experts.  groups > 1: the outputs are that many equal runs of
+ * neighbours, of which only the keep_groups with the largest entries are open to choice.  always > 0: behind its
+ * choices every token has that many more experts, experts .. experts + always - 1 of the grouped product, each with weight
+ * sigmoid(z[outputs]).  A row of the routing's arrays is then top + always long and offsets one of experts + always.
+ * outputs <= 1024, experts + always <= 1024, top + always <= 64. */
+typedef struct nf_route_args {
+  const float* z;
+  int shares, ld, rows, outputs, experts, top, always, groups, keep_groups;
+  const float* correction;
+  float scale;
+} nf_route_args;
+NF_API int nf_route(const nf_route_args* args, const nf_routing* routing, nf_stream_t stream);
 
 /* Grouped product D_g = act(A_g . B_g^T), B [groups][N][K]; N, K and all strides multiples of 8.
  * routing.n_tiles null: every group has M rows, at a + g * a_group and d + g * d_group (elements).
  * Else the groups are the routing's experts: D holds sorted rows, A too, or (gather) the tokens themselves, M of
- * them; max_rows bounds the number of sorted rows.  act: NF_ACT_NONE or NF_ACT_GELU. */
+ * them; max_rows bounds the number of sorted rows.  act: NF_ACT_NONE, NF_ACT_GELU or NF_ACT_SQUARED_RELU. */
 typedef struct nf_grouped_gemm_args {
   int dtype, act, groups, M, N, K;
   const void* a;
@@ -374,7 +385,7 @@ typedef struct nf_norm {
 /* out [n, ld] in `dtype` = norm of rows row_index[i] of x (null: rows 0 .. n - 1). */
 NF_API int nf_norm_rows(int dtype, const float* x, const int32_t* row_index, const nf_norm* norm, void* out, int n, int width,
                         int ld, nf_stream_t stream);
-/* The end of a sublayer:  x += y_norm(y),  act = next(x) in `dtype` (null: not written).  y is the sum of `shares` fp32
+/* The end of a sublayer:  x += y_scale * y_norm(y),  act = next(x) in `dtype` (null: not written).  y is the sum of `shares` fp32
  * [rows, ld] slices (y_dtype NF_F32) or one bf16 [rows, ld]; or, with routing not null, a mixture's output: the weighted sum
  * over a token's `top` choices of sorted rows of y (row stride y_ld, `dtype`) and of `identity` [rows, ld] (`dtype`). */
 typedef struct nf_residual_args {
@@ -385,6 +396,7 @@ typedef struct nf_residual_args {
   int top, y_ld;
   const void* identity;
   nf_norm y_norm, next;
+  float y_scale;
   float* x;
   int dtype;
   void* act;
@@ -422,37 +434,54 @@ typedef struct nf_rotation {
 } nf_rotation;
 
 /* Paged KV cache of one attention layer: page p of the pool holds `page` positions as
- *   K [kv_heads][page][k_pad]  then  V [kv_heads][v_pad][page]    (V transposed: a value column's
+ *   K [kv_heads][maps][page][k_pad]  then  V [kv_heads][v_pad][page]    (V transposed: a value column's
  * positions are contiguous), elements of `dtype`; k_pad = dim rounded up to 32, v_pad = vdim to 16, both
- * zero padded. */
+ * zero padded.  maps: attentions of a head over the same values (1, or 2 whose difference is taken), each with `dim`
+ * columns of queries and keys of its own; heads come one after the other, a head's maps side by side. */
 typedef struct nf_kv_layout {
-  int dtype, heads, kv_heads, dim, vdim, k_pad, v_pad, page;
+  int dtype, heads, kv_heads, dim, vdim, k_pad, v_pad, page, maps;
 } nf_kv_layout;
 NF_API size_t nf_kv_page_elements(const nf_kv_layout* kv);
 
 /* Projected rows (q | k | v at the given columns of `proj`, row stride ld) -> per-head RMS norm of q and k
- * (weights may be null), rotation, q scaled by nothing -> q_out [rows][heads][k_pad]; k and v appended to the
+ * (weights may be null), rotation, q scaled by nothing -> q_out [rows][heads][maps][k_pad]; k and v appended to the
  * cache at the row's position.  q_temp (may be null): q of position p is multiplied by
  * 1 + coef * ln(floor((p + 1) / every) + 1) as well. */
 typedef struct nf_query_temperature {
   float coef;
   int every;
 } nf_query_temperature;
+/* Short causal convolution over time, each column of the projected rows by itself (conv null: none), ahead of norm and
+ * rotation:  y_t = sum_j weight[j] * proj_(t - taps + 1 + j), zeros before position 0.  weight [taps][ld] and state
+ * [slots][taps - 1][ld] have the rows' type and columns; position p lies in row p % (taps - 1) of its request's slot.
+ * nf_qkv_append keeps the state of requests that bring one row; nf_conv_state, after it, that of those among requests
+ * [req_begin, req_begin + req_num) that bring more. */
+typedef struct nf_short_conv {
+  int taps;
+  const void* weight;
+  void* state;
+  const int32_t *input_indptr, *state_slots;
+} nf_short_conv;
+NF_API int nf_conv_state(int dtype, const void* proj, int ld, const nf_short_conv* conv, const int32_t* positions, int req_begin,
+                         int req_num, nf_stream_t stream);
 NF_API int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, int k_col, int v_col,
                          const float* q_norm, const float* k_norm, float eps, const nf_rotation* rot,
-                         const nf_query_temperature* q_temp, void* q_out, void* kv_data, const int32_t* kv_indptr, const int32_t* kv_indices,
+                         const nf_query_temperature* q_temp, const nf_short_conv* conv, void* q_out, void* kv_data, const int32_t* kv_indptr, const int32_t* kv_indices,
                          const int32_t* rev_input_indptr, const int32_t* positions, int rows, nf_stream_t stream);
 
 /* Attention over the cache.  A row at position p sees position j iff j <= p and (p - j < window or
- * j < keep_first); window <= 0: all of j <= p.  Scores are q.k * scale; sink (may be null): exp(sink[h]) is
+ * j < keep_first); window <= 0: all of j <= p.  Scores are q.k * scale, brought within
+ * +-softcap by softcap * tanh(score / softcap) where softcap > 0; sink (may be null): exp(sink[h]) is
  * added to the denominator.  Output: heads concatenated at column out_col of out (row stride out_ld),
  * multiplied by out_scale and, with gate not null, by sigmoid(gate[row][head]) (row stride gate_ld, the layout's
- * type).  Rows of requests [req_begin, req_begin + req_num) of the batch are computed;
+ * type).  Two maps: a head's output is that of its first less map_weight times that of its second (no sinks).  head_norm
+ * != 0: divided by its root mean square (head_eps inside the root) ahead of out_scale.  Rows of requests [req_begin, req_begin + req_num) of the batch are computed;
  * max_rows bounds their number of rows.  decode != 0: every one of those requests has exactly one row. */
 typedef struct nf_window_attention_args {
   nf_kv_layout kv;
   int window, keep_first;
-  float scale, out_scale;
+  float scale, out_scale, softcap, map_weight, head_eps;
+  int head_norm;
   const float* sink;
   const void* gate;
   int gate_ld;
@@ -505,11 +534,12 @@ NF_API int nf_latent_gather(const nf_latent_expand_args* args, nf_stream_t strea
 NF_API int nf_latent_pack(const nf_latent_expand_args* args, nf_stream_t stream);
 NF_API int nf_latent_queries(const nf_kv_layout* kv, int dim_pad, const void* proj, int ld, int q_col, int rot_dim, const nf_rotation* rot,
                              const int32_t* positions, void* q, int row_begin, int rows, nf_stream_t stream);
-/* Causal softmax attention of q rows over the latents, scores q . row * scale, values the rows' latents:
+/* Causal softmax attention of q rows over the latents (window > 0: over the last `window` of them), scores q . row * scale, values the rows' latents:
  * out [rows][heads][rank_pad] in the layout's type.  Requests and rows as for nf_window_attention.  workspace
  * (nf_latent_workspace_bytes; may be null): few requests are split over their keys through it. */
 typedef struct nf_latent_attention_args {
   nf_latent_layout layout;
+  int window;
   float scale;
   const void* q;
   void* out;

@@ -60,7 +60,7 @@ LayerStackPipeline::Buffers LayerStackPipeline::plan(const StackModel& m, int T,
     const LayerWeights& w = m.weights.layers[i];
     if (s.attention) {
       attn_proj = std::max(attn_proj, (size_t)w.attention.qkv.N);
-      q = std::max(q, (size_t)s.attention->heads * m.kvLayout((int)i).k_pad);
+      q = std::max(q, (size_t)s.attention->heads * s.attention->maps() * m.kvLayout((int)i).k_pad);
       ws_side = std::max(ws_side, few(w.attention.qkv));
     }
     if (s.recurrence) {
@@ -101,10 +101,10 @@ LayerStackPipeline::Buffers LayerStackPipeline::plan(const StackModel& m, int T,
     }
     if (s.mixture) {
       const MixtureSpec& x = *s.mixture;
-      top = std::max(top, (size_t)x.top);
-      experts = std::max(experts, (size_t)x.experts);
-      expert_ff = std::max(expert_ff, (size_t)x.top * w.up.N);
-      tiles = std::max(tiles, (size_t)nf_routing_max_tiles(T * x.top, x.experts, 64));
+      top = std::max(top, (size_t)x.perToken());
+      experts = std::max(experts, (size_t)(x.experts + x.always()));
+      expert_ff = std::max(expert_ff, (size_t)x.perToken() * w.up.N);
+      tiles = std::max(tiles, (size_t)nf_routing_max_tiles(T * x.perToken(), x.experts + x.always(), 64));
       b.router_sums_bytes = std::max(b.router_sums_bytes, sums(T, w.router, kSumsMaxShares));
     }
     if (spec.token_side > 0) {
@@ -216,6 +216,7 @@ void LayerStackPipeline::config(vortexConfigData* config_data_) {
   firstNorm.norm = model->weights.layers[0].norm1;
   firstNorm.out = buf.act;
   residualAdd.args.x = buf.x;
+  residualAdd.args.y_scale = (float)spec.residual_scale;
   residualAdd.args.width = gatherNorm.width = firstNorm.width = spec.width;
   residualAdd.args.ld = gatherNorm.ld = tokenShift.ld = firstNorm.ld = ld;
   qkvAppend.eps = latentAppend.eps = gatedNorm.eps = (float)spec.eps;
@@ -336,29 +337,33 @@ void LayerStackPipeline::sublayerOut(const void* a, const DeviceMatrix& w, const
 void LayerStackPipeline::mixtureOut(int layer) {
   const MixtureSpec& s = *model->spec.layers[layer].mixture;
   const LayerWeights& w = model->weights.layers[layer];
-  const int T = batch.rows, slots = T * s.top, ld = model->spec.ld();
+  const int T = batch.rows, experts = s.experts + s.always(), slots = T * s.perToken(), ld = model->spec.ld();
   const void* h = sublayerInput();
   linear.setSums(h, w.router, buf.router_sums, buf.router_sums_bytes, T, kSumsMaxShares).run();
-  router.z = buf.router_sums;
-  router.shares = linear.shares();
-  router.ld = w.router.N;
-  router.outputs = s.experts + s.identity;
-  router.experts = s.experts;
-  router.top = s.top;
-  router.correction = w.correction;
-  router.scale = (float)s.scale;
+  nf_route_args& z = router.args;
+  z.z = buf.router_sums;
+  z.shares = linear.shares();
+  z.ld = w.router.N;
+  z.outputs = s.outputs();
+  z.experts = s.experts;
+  z.top = s.top;
+  z.always = s.always();
+  z.groups = s.groups;
+  z.keep_groups = s.keep_groups;
+  z.correction = w.correction;
+  z.scale = (float)s.scale;
   router.routing = buf.routing;
-  router.routing.tile_rows = nf_grouped_tile_rows(model->dtype, slots, s.experts);
+  router.routing.tile_rows = nf_grouped_tile_rows(model->dtype, slots, experts);
   router.run();
-  grouped.experts(h, ld, w.up, buf.expert_ff, w.up.N, s.experts, router.routing, true, slots, s.act);
+  grouped.experts(h, ld, w.up, buf.expert_ff, w.up.N, experts, router.routing, true, slots, s.act);
   grouped.run();
-  grouped.experts(buf.expert_ff, w.up.N, w.down, buf.expert_out, ld, s.experts, router.routing, false, slots, NF_ACT_NONE);
+  grouped.experts(buf.expert_ff, w.up.N, w.down, buf.expert_out, ld, experts, router.routing, false, slots, NF_ACT_NONE);
   grouped.run();
   nf_residual_args& r = residualAdd.args;
   r.routing = &router.routing;
   r.y = buf.expert_out;
   r.y_ld = ld;
-  r.top = s.top;
+  r.top = s.perToken();
   r.identity = h;
   r.y_norm = model->spec.pre_norm ? nf_norm{} : w.norm2;
   setNext(afterFeedForward(layer));
@@ -396,7 +401,8 @@ int LayerStackPipeline::expandPages(int layer) const {
   double pairs = 0;
   for (int r = first; r < end; ++r) {
     const double rows = in[r + 1] - in[r], context = (double)(kv[r + 1] - kv[r]) * model->page_size;
-    pairs += rows * std::max(context - rows / 2, rows / 2);
+    const double seen = std::max(context - rows / 2, rows / 2);
+    pairs += rows * (s.window > 0 ? std::min(seen, (double)s.window) : seen);
   }
   const double product = (double)l.rank_pad * (w.dim_pad + w.vdim_pad), tokens = (double)(kv[end] - kv[first]) * model->page_size;
   const double saved = pairs * (l.row_ld + l.rank_pad - (w.dim_pad + s.rot_dim + w.vdim_pad)) + (batch.rows - batch.decode) * product;
@@ -448,6 +454,7 @@ void LayerStackPipeline::latentBranch(int layer) {
     nf_window_attention_args& g = attention.args;
     g = nf_window_attention_args{};
     g.kv = x.kv;
+    g.window = s.window;
     g.scale = (float)s.scale;
     g.out_scale = 1.f;
     g.q = buf.latent_q;
@@ -466,6 +473,7 @@ void LayerStackPipeline::latentBranch(int layer) {
   grouped.run();
   nf_latent_attention_args& a = latentAttention.args;
   a.layout = l;
+  a.window = s.window;
   a.scale = (float)s.scale;
   a.q = buf.q;
   a.out = buf.latent;
@@ -491,6 +499,8 @@ void LayerStackPipeline::attentionBranch(int layer, hipStream_t s) {
   qkvAppend.w = &w.attention;
   qkvAppend.q_temp.reset();
   if (a.q_temp) qkvAppend.q_temp = nf_query_temperature{(float)a.q_temp->coef, a.q_temp->every};
+  qkvAppend.conv_taps = a.conv_taps;
+  qkvAppend.conv_state = model->conv_state[layer];
   qkvAppend.q_out = buf.q;
   qkvAppend.kv_data = model->kv_data[layer];
   qkvAppend.run();
@@ -500,6 +510,10 @@ void LayerStackPipeline::attentionBranch(int layer, hipStream_t s) {
   g.keep_first = a.keep_first;
   g.scale = (float)a.scale;
   g.out_scale = (float)a.out_scale;
+  g.softcap = (float)a.softcap;
+  g.map_weight = w.attention.map_weight;
+  g.head_norm = a.head_norm;
+  g.head_eps = (float)model->spec.eps;
   g.sink = w.attention.sink;
   g.gate = a.head_gate ? (const uint8_t*)buf.attn_proj + (size_t)w.attention.g_col * model->elementBytes() : nullptr;
   g.gate_ld = qkvAppend.ld;

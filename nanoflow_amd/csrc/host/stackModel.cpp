@@ -38,7 +38,11 @@ StackModelSpec parseStackModel(const mini_json::Value& config) {
     require(l.attention || l.recurrence || l.latent, at + "no mixer");
     require(!l.latent || (!l.attention && !l.recurrence), at + "latent attention beside another mixer");
     require(!l.mlp || !l.mixture, at + "two feed-forwards");
-    auto rotation = [&](const RotationSpec& r, int dim) { require(r.dims >= 0 && r.dims <= dim && r.dims % 2 == 0, at + "rotated dimensions"); };
+    auto rotation = [&](const RotationSpec& r, int dim) {
+      require(r.dims >= 0 && r.dims <= dim && r.dims % 2 == 0, at + "rotated dimensions");
+      require(!r.scaling || (r.scaling->factor > 0 && r.scaling->low > 0 && r.scaling->high > r.scaling->low && r.scaling->original > 0),
+              at + "scaling of the rotation");
+    };
     if (l.attention) {
       const auto& a = *l.attention;
       require(a.heads > 0 && a.kv_heads > 0 && a.heads % a.kv_heads == 0, at + "query heads must be a multiple of the kv heads");
@@ -47,11 +51,15 @@ StackModelSpec parseStackModel(const mini_json::Value& config) {
       require(a.window >= 0 && a.keep_first >= 0, at + "window");
       require(!a.q_temp || a.q_temp->every > 0, at + "query temperature");
       require(!a.sink || !a.unit_sink, at + "two sinks");
+      require(!a.difference || (!a.sink && !a.unit_sink), at + "a sink in a difference of attentions");
+      require(a.softcap >= 0, at + "bound of the scores");
+      require(a.conv_taps >= 0 && a.conv_taps <= 64, at + "a convolution has 1..64 taps");
     }
     if (l.latent) {
       const auto& a = *l.latent;
       require(a.heads > 0 && a.dim > 0 && a.vdim > 0 && a.rot_dim >= 0 && a.rot_dim <= 256 && a.kv_rank > 0 && a.kv_rank <= 2048,
               at + "latent attention sizes (a latent of 1..2048, a rotated part of 0..256)");
+      require(a.window >= 0, at + "window");
       rotation(a.rot, a.rot_dim);
     }
     if (l.recurrence) {
@@ -68,6 +76,10 @@ StackModelSpec parseStackModel(const mini_json::Value& config) {
       require(m.ff > 0, at + "feed-forward width");
       require(m.experts > 0 && m.identity >= 0 && m.experts + m.identity <= 1024, at + "1..1024 experts, the identity experts among them");
       require(m.top > 0 && m.top <= m.experts + m.identity && m.top <= 64, at + "a token uses 1..64 of the experts");
+      require(m.groups > 0 && m.outputs() % m.groups == 0 && m.keep_groups > 0 && m.keep_groups <= m.groups &&
+                  m.top <= m.outputs() / m.groups * m.keep_groups,
+              at + "equal groups of experts, the kept ones with room for the choice");
+      require(m.shared_ff >= 0 && (m.shared_ff == 0 || m.always() > 0), at + "a shared expert beside at most 63 chosen ones");
     }
   }
   return s;
@@ -238,9 +250,9 @@ struct StackModel::Loader {
     for (size_t i = 0; i < parts.size(); ++i) put_rows(get(parts[i].name, {parts[i].rows}), 1, parts[i].rows, 0, at[i], N);
     return finish(1, N).ptr;
   }
-  nf_norm norm(const std::string& name, nf_norm_kind kind) {
+  nf_norm norm(const std::string& name, nf_norm_kind kind, double scale = 1) {
     const int W = m.spec.width, ld = m.spec.ld();
-    return nf_norm{kind, vectors({name}, {W}, W, ld), kind == NF_NORM_LAYER ? vectors({name + ".b"}, {W}, W, ld) : nullptr, (float)m.spec.eps};
+    return nf_norm{kind, vectors({name}, {W}, W, ld, m.spec.norm_offset, scale), kind == NF_NORM_LAYER ? vectors({name + ".b"}, {W}, W, ld) : nullptr, (float)m.spec.eps};
   }
 
   void latent(const LatentAttentionSpec& a, const std::string& p, LayerWeights& lw) {
@@ -283,15 +295,41 @@ struct StackModel::Loader {
   }
 
   void mixture(const MixtureSpec& s, const std::string& p, LayerWeights& w) {
-    const int W = m.spec.width, ff = pad8(s.ff), K = pad8(W), outputs = s.experts + s.identity;
-    start((size_t)s.experts * ff, K);
+    const int W = m.spec.width, columns = s.expertFf(), ff = pad8(columns), K = pad8(W), all = s.experts + s.always();
+    auto share = [&](int j) { return std::max(0, std::min(columns, s.shared_ff - j * columns)); };  // of the shared expert's columns
+    start((size_t)all * ff, K);
     for (int e = 0; e < s.experts; ++e) put_rows(get(p + "e" + std::to_string(e) + ".up", {s.ff, W}), s.ff, W, e * ff, 0, K);
+    for (int j = 0; j < s.always(); ++j) put_block(get(p + "shared.up", {s.shared_ff, W}), W, j * columns, share(j), 0, W, (s.experts + j) * ff, 0, K);
     w.up = finish(ff, K);
-    start((size_t)s.experts * K, ff);
+    start((size_t)all * K, ff);
     for (int e = 0; e < s.experts; ++e) put_rows(get(p + "e" + std::to_string(e) + ".down", {W, s.ff}), W, s.ff, e * K, 0, ff);
+    for (int j = 0; j < s.always(); ++j)
+      put_block(get(p + "shared.down", {W, s.shared_ff}), s.shared_ff, 0, W, j * columns, share(j), (s.experts + j) * K, 0, ff);
     w.down = finish(K, ff);
-    w.router = matrix({{p + "router", outputs}}, W);
-    w.correction = vectors({p + "correction"}, {outputs}, outputs, outputs);
+    std::vector<Part> router{{p + "router", s.outputs()}};
+    if (s.always() > 0) router.push_back({p + "shared.sg", 1});
+    w.router = matrix(router, W);
+    if (s.correction) w.correction = vectors({p + "correction"}, {s.outputs()}, s.outputs(), s.outputs());
+  }
+  // weights [channels][taps] of convolutions on the columns from at[i] on -> [taps][N] in the activations' type
+  void* taps(const std::vector<Part>& parts, const std::vector<int>& at, int n, int N) {
+    start(n, N);
+    for (size_t i = 0; i < parts.size(); ++i) {
+      const HostTensor& t = get(parts[i].name, {parts[i].rows, n});
+      for (int c = 0; c < parts[i].rows; ++c)
+        for (int j = 0; j < n; ++j) put(staging.data() + ((size_t)j * N + at[i] + c) * m.elementBytes(), element(t, (size_t)c * n + j));
+    }
+    return finish(n, N).ptr;
+  }
+  // exp(lq1 . lk1) - exp(lq2 . lk2) + difference
+  float map_weight(const AttentionSpec& a, const std::string& p) {
+    auto dot = [&](const char* q, const char* k) {
+      const HostTensor &x = get(p + q, {a.dim}), &y = get(p + k, {a.dim});
+      double sum = 0;
+      for (int c = 0; c < a.dim; ++c) sum += (double)element(x, c) * element(y, c);
+      return sum;
+    };
+    return (float)(std::exp(dot("lq1", "lk1")) - std::exp(dot("lq2", "lk2")) + *a.difference);
   }
   float* upload(const std::vector<float>& v) {
     float* d = static_cast<float*>(m.allocate(v.size() * sizeof(float)));
@@ -299,11 +337,11 @@ struct StackModel::Loader {
     return d;
   }
   // vectors of `rows` x `cols`, each row padded to `ld`
-  float* vectors(const std::vector<std::string>& names, std::vector<int64_t> shape, int cols, int ld) {
+  float* vectors(const std::vector<std::string>& names, std::vector<int64_t> shape, int cols, int ld, double offset = 0, double scale = 1) {
     std::vector<float> v((size_t)names.size() * ld, 0.f);
     for (size_t s = 0; s < names.size(); ++s) {
       const HostTensor& t = get(names[s], shape);
-      for (int c = 0; c < cols; ++c) v[s * ld + c] = element(t, c);
+      for (int c = 0; c < cols; ++c) v[s * ld + c] = (float)((element(t, c) + offset) * scale);
     }
     return upload(v);
   }
@@ -318,17 +356,29 @@ void* StackModel::allocate(size_t bytes) {
   return p;
 }
 
-// cos and sin of position * base^(-2i/dims), evaluated in double and kept in fp32: one table per distinct
+double RotationSpec::frequency(int pair) const {
+  const double f = std::pow(base, -2.0 * pair / dims);
+  if (!scaling) return f;
+  const double periods = scaling->original * f / (2 * M_PI);  // that fit into the original positions
+  if (periods > scaling->high) return f;
+  if (periods < scaling->low) return f / scaling->factor;
+  const double s = (periods - scaling->low) / (scaling->high - scaling->low);
+  return (1 - s) * f / scaling->factor + s * f;
+}
+
+// cos and sin of position * frequency, evaluated in double and kept in fp32: one table per distinct
 // rotation, for every position a request can have.
 nf_rotation StackModel::rotation(const RotationSpec& r) {
   nf_rotation out{nullptr, r.dims, r.interleaved ? 1 : 0};
   if (r.dims == 0) return out;
-  float*& table = rotation_tables_[{r.dims, r.base}];
+  std::vector<double> key{(double)r.dims, r.base};
+  if (r.scaling) key.insert(key.end(), {r.scaling->factor, r.scaling->low, r.scaling->high, r.scaling->original});
+  float*& table = rotation_tables_[key];
   if (!table) {
     const int half = r.dims / 2;
     std::vector<float> v((size_t)spec.max_positions * half * 2);
     for (int i = 0; i < half; ++i) {
-      const double f = std::pow(r.base, -2.0 * i / r.dims);
+      const double f = r.frequency(i);
       for (int p = 0; p < spec.max_positions; ++p) {
         v[((size_t)p * half + i) * 2] = (float)std::cos(p * f);
         v[((size_t)p * half + i) * 2 + 1] = (float)std::sin(p * f);
@@ -352,12 +402,12 @@ nf_kv_layout StackModel::expandedLayout(int layer) const {
   const LatentAttentionSpec& a = *spec.layers[layer].latent;
   const int dim = pad8(a.dim) + a.rot_dim, vdim = pad8(a.vdim);
   if (dtype != NF_BF16 || dim > 256 || vdim > 256) return nf_kv_layout{};
-  return nf_kv_layout{dtype, a.heads, a.heads, dim, vdim, (dim + 31) / 32 * 32, (vdim + 15) / 16 * 16, page_size};
+  return nf_kv_layout{dtype, a.heads, a.heads, dim, vdim, (dim + 31) / 32 * 32, (vdim + 15) / 16 * 16, page_size, 1};
 }
 
 nf_kv_layout StackModel::kvLayout(int layer) const {
   const AttentionSpec& a = *spec.layers[layer].attention;
-  return nf_kv_layout{dtype, a.heads, a.kv_heads, a.dim, a.vdim, (a.dim + 31) / 32 * 32, (a.vdim + 15) / 16 * 16, page_size};
+  return nf_kv_layout{dtype, a.heads, a.kv_heads, a.dim, a.vdim, (a.dim + 31) / 32 * 32, (a.vdim + 15) / 16 * 16, page_size, a.maps()};
 }
 
 StackModel::StackModel(const StackModelSpec& spec_, const HostTensors& tensors, nf_dtype dtype_, int kv_pages_, int page_size_,
@@ -368,14 +418,16 @@ StackModel::StackModel(const StackModelSpec& spec_, const HostTensors& tensors, 
   try {
     weights.embed = L.matrix({{"embed", spec.vocab}}, W);
     if (spec.learned_positions) weights.pos = L.matrix({{"pos", spec.max_positions}}, W);
-    weights.head = L.matrix({{"head", spec.vocab}}, W);
-    weights.final_norm = L.norm("final.norm", spec.norm);
+    weights.head = spec.tied_head ? weights.embed : L.matrix({{"head", spec.vocab}}, W);
+    // the logits' scale is one of the rows that the output projection reads
+    weights.final_norm = L.norm("final.norm", spec.norm, spec.logit_scale);
     if (spec.token_side > 0) weights.side_embed = L.matrix({{"side.embed", spec.vocab}}, spec.token_side * (int)spec.layers.size());
     const int n = (int)spec.layers.size();
     weights.layers.resize(n);
     kv_data.assign(n, nullptr);
     state.assign(n, nullptr);
     shift_state.assign(n, nullptr);
+    conv_state.assign(n, nullptr);
     for (int i = 0; i < n; ++i) {
       const LayerSpec& s = spec.layers[i];
       LayerWeights& w = weights.layers[i];
@@ -385,7 +437,8 @@ StackModel::StackModel(const StackModelSpec& spec_, const HostTensors& tensors, 
         const AttentionSpec& a = *s.attention;
         const std::string p = l + a.prefix;
         std::vector<int> at;
-        std::vector<Loader::Part> parts{{p + "q", a.heads * a.dim}, {p + "k", a.kv_heads * a.dim}, {p + "v", a.kv_heads * a.vdim}};
+        std::vector<Loader::Part> parts{
+            {p + "q", a.heads * a.maps() * a.dim}, {p + "k", a.kv_heads * a.maps() * a.dim}, {p + "v", a.kv_heads * a.vdim}};
         if (a.head_gate) parts.push_back({p + "g", a.heads});
         w.attention.qkv = L.matrix(parts, W, &at);
         if (a.head_gate) w.attention.g_col = at[3];
@@ -400,6 +453,12 @@ StackModel::StackModel(const StackModelSpec& spec_, const HostTensors& tensors, 
         }
         if (a.sink) w.attention.sink = L.vectors({p + "sink"}, {a.heads}, a.heads, a.heads);
         if (a.unit_sink) w.attention.sink = L.upload(std::vector<float>((size_t)a.heads, 0.f));
+        if (a.difference) w.attention.map_weight = L.map_weight(a, p);
+        if (a.conv_taps > 0) {
+          w.attention.conv = L.taps({{p + "q.conv", parts[0].rows}, {p + "k.conv", parts[1].rows}, {p + "v.conv", parts[2].rows}}, at,
+                                    a.conv_taps, w.attention.qkv.N);
+          conv_state[i] = allocate((size_t)state_slots * (a.conv_taps - 1) * w.attention.qkv.N * elementBytes());
+        }
         w.attention.rot = rotation(a.rot);
         out_parts.push_back({p + "o", a.heads * a.vdim});
         const nf_kv_layout kv = kvLayout(i);

@@ -15,10 +15,17 @@
 #include "mini_json.h"
 #include "nanoflow_kernels.h"
 
+// Wavelengths above original / low are `factor` times longer, those below original / high as they are, and in between
+// one goes over into the other.
+struct RotationScaling {
+  double factor = 1, low = 1, high = 4, original = 1;
+};
 struct RotationSpec {
   int dims = 0;
   double base = 1e4;
   bool interleaved = false;
+  std::optional<RotationScaling> scaling = {};
+  double frequency(int pair) const;
 };
 
 // q of position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1).
@@ -27,7 +34,8 @@ struct QueryTemperatureSpec {
   int every = 1;
 };
 
-// Softmax attention over a window with kept first positions.
+// Softmax attention over a window with kept first positions; with `difference` the difference of two attentions per head over
+// the same values, the second's weight being exp(lq1 . lk1) - exp(lq2 . lk2) + difference.
 struct AttentionSpec {
   std::string prefix;  // of its tensors
   int heads = 0, kv_heads = 0, dim = 0, vdim = 0;
@@ -38,6 +46,11 @@ struct AttentionSpec {
   bool sink = false;       // a score per head in the denominator, from a tensor
   bool unit_sink = false;  // the same with score 0
   bool head_gate = false;  // a head's output times the sigmoid of a projection of the input
+  double softcap = 0;      // bound of the scores, 0: none
+  int conv_taps = 0;       // short convolution of the projections over time, 0: none
+  std::optional<double> difference;
+  bool head_norm = false;  // a head's output divided by its root mean square
+  int maps() const { return difference ? 2 : 1; }
   RotationSpec rot;
   std::optional<QueryTemperatureSpec> q_temp;
   double out_scale = 1;
@@ -49,6 +62,7 @@ struct LatentAttentionSpec {
   std::string prefix;
   int heads = 0, dim = 0, rot_dim = 0, vdim = 0, kv_rank = 0;
   double scale = 1;
+  int window = 0;    // 0: everything before
   RotationSpec rot;  // of the rotated part
 };
 
@@ -71,11 +85,24 @@ struct MlpSpec {
   int ff = 0;
   nf_activation act = NF_ACT_SQUARED_RELU;
 };
-// Feed-forwards of which every token uses `top`; the router's last `identity` outputs stand for the input itself.
+// Feed-forwards of which every token uses `top`; the router's last `identity` outputs stand for the input itself.  A token
+// chooses from the keep_groups best of `groups` runs of outputs.  shared_ff > 0: one more feed-forward for every
+// token, times the sigmoid of a projection.  It is held as always() experts of expertFf() columns beside the others, each
+// a share of its columns: activations are taken column by column, so the shares' outputs add up to its own.
 struct MixtureSpec {
   int experts = 0, identity = 0, top = 0, ff = 0;
   double scale = 1;
   nf_activation act = NF_ACT_GELU;
+  int groups = 1, keep_groups = 1;
+  bool correction = true;  // of the scores, where the choice is made
+  int shared_ff = 0;
+  int outputs() const { return experts + identity; }
+  int always() const {
+    const int room = 64 - top < 1024 - experts ? 64 - top : 1024 - experts, shares = (shared_ff + ff - 1) / ff;
+    return shared_ff > 0 ? (shares < room ? shares : room) : 0;
+  }
+  int expertFf() const { return shared_ff > 0 && (shared_ff + always() - 1) / always() > ff ? (shared_ff + always() - 1) / always() : ff; }
+  int perToken() const { return top + always(); }
 };
 // A layer's mixer: attention, latent attention, a recurrence, or attention and a recurrence side by side on the same
 // input; its feed-forward: dense, a mixture, or none.
@@ -96,6 +123,10 @@ struct StackModelSpec {
   bool learned_positions = false;
   nf_norm_kind norm = NF_NORM_RMS;  // of the residual stream (layer norms have a bias)
   bool pre_norm = false;            // x += f(norm(x)); else x += norm(f(x))
+  double norm_offset = 0;           // added to the stored weights of the stream's norms
+  double residual_scale = 1;        // of what a sublayer adds
+  bool tied_head = false;           // the output projection is the embedding table
+  double logit_scale = 1;
   int token_side = 0;               // size of the token input at the end of every layer, 0: none
   std::vector<LayerSpec> layers;
   int ld() const { return (width + 7) / 8 * 8; }
@@ -106,7 +137,7 @@ struct StackModelSpec {
   }
   bool hasState() const {
     for (const auto& l : layers)
-      if (l.recurrence) return true;
+      if (l.recurrence || (l.attention && l.attention->conv_taps > 1)) return true;
     return false;
   }
 };
@@ -159,6 +190,8 @@ struct AttentionWeights {
   void* bias = nullptr;
   int q_col = 0, k_col = 0, v_col = 0, g_col = 0;
   float *q_norm = nullptr, *k_norm = nullptr, *sink = nullptr;
+  void* conv = nullptr;  // [taps][columns of qkv]
+  float map_weight = 0;
   nf_rotation rot{};
 };
 struct LatentAttentionWeights {
@@ -215,6 +248,7 @@ public:
   std::vector<void*> kv_data;       // kv_pages pages (nf_kv_layout, nf_latent_layout)
   std::vector<float*> state;        // [state_slots][heads][dim_pad][vdim_pad]
   std::vector<float*> shift_state;  // [state_slots][ld]
+  std::vector<void*> conv_state;    // [state_slots][taps - 1][columns of qkv]
   nf_kv_layout kvLayout(int layer) const;
   nf_latent_layout latentLayout(int layer) const;
   // of a latent layer's keys and values written out for all heads; page 0: heads too large for it, or fp32
@@ -224,7 +258,7 @@ public:
 private:
   struct Loader;
   std::vector<void*> owned_;
-  std::map<std::pair<int, double>, float*> rotation_tables_;
+  std::map<std::vector<double>, float*> rotation_tables_;
   void* allocate(size_t bytes);  // zeroed device memory that lives as long as the model
   nf_rotation rotation(const RotationSpec& r);
 };

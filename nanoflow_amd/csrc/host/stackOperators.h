@@ -67,7 +67,7 @@ struct StackLinear : public StackOperator {
       NF_KERNEL_CHECK(nf_gemm_nk_bias_bf16((const uint16_t*)a, (const uint16_t*)w.ptr, (const uint16_t*)bias, (uint16_t*)d, rows, w.N, w.K,
                                            workspace, workspace_bytes, stream));
     } else {
-      auto f = act == NF_ACT_SQUARED_RELU ? nf_gemm_nk_relu2_bf16 : act == NF_ACT_SILU ? nf_gemm_nk_silu_bf16 : nf_gemm_nk_bf16;
+      auto f = act == NF_ACT_SQUARED_RELU ? nf_gemm_nk_relu2_bf16 : act == NF_ACT_SILU ? nf_gemm_nk_silu_bf16 : act == NF_ACT_GELU ? nf_gemm_nk_gelu_bf16 : nf_gemm_nk_bf16;
       NF_KERNEL_CHECK(f((const uint16_t*)a, (const uint16_t*)w.ptr, (uint16_t*)d, rows, w.N, w.K, workspace, workspace_bytes,
                         stream));
     }
@@ -149,12 +149,11 @@ private:
 };
 
 struct StackRouter : public StackOperator {
-  const float *z = nullptr, *correction = nullptr;
-  int shares = 1, ld = 0, outputs = 0, experts = 0, top = 0;
-  float scale = 1;
+  nf_route_args args{};
   nf_routing routing{};
   void work() override {
-    NF_KERNEL_CHECK(nf_route(z, shares, ld, batch->rows, outputs, experts, top, correction, scale, &routing, stream));
+    args.rows = batch->rows;
+    NF_KERNEL_CHECK(nf_route(&args, &routing, stream));
   }
 };
 
@@ -230,7 +229,8 @@ struct StackLatentQueries : public StackOperator {
   }
 };
 
-// Per-head norm and rotation of projected rows, append to the paged cache (the counterpart of RoPEAppend).
+// Short convolution, per-head norm and rotation of projected rows, append to the paged cache (the counterpart of
+// RoPEAppend); the convolution's state.
 struct StackQKVAppend : public StackOperator {
   nf_kv_layout kv{};
   const void* proj = nullptr;
@@ -238,11 +238,16 @@ struct StackQKVAppend : public StackOperator {
   const AttentionWeights* w = nullptr;
   float eps = 0;
   std::optional<nf_query_temperature> q_temp;
+  int conv_taps = 0;
+  void* conv_state = nullptr;
   void *q_out = nullptr, *kv_data = nullptr;
   void work() override {
+    const nf_short_conv conv{conv_taps, w->conv, conv_state, batch->input_indptr, batch->state_slots};
     NF_KERNEL_CHECK(nf_qkv_append(&kv, proj, ld, w->q_col, w->k_col, w->v_col, w->q_norm, w->k_norm, eps, &w->rot,
-                                  q_temp ? &*q_temp : nullptr, q_out, kv_data, batch->kv_indptr, batch->kv_indices, batch->rev_input_indptr, batch->positions,
-                                  batch->rows, stream));
+                                  q_temp ? &*q_temp : nullptr, conv_taps > 0 ? &conv : nullptr, q_out, kv_data, batch->kv_indptr,
+                                  batch->kv_indices, batch->rev_input_indptr, batch->positions, batch->rows, stream));
+    if (conv_taps > 1 && batch->prefill > 0)
+      NF_KERNEL_CHECK(nf_conv_state(kv.dtype, proj, ld, &conv, batch->positions, batch->decode, batch->prefill, stream));
   }
 };
 

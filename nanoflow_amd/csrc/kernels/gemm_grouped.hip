@@ -100,7 +100,7 @@ int nf_gemm_grouped(const nf_grouped_gemm_args* args, nf_stream_t stream) {
   NF_REQUIRE(args, "%s: null pointer", who);
   const nf_grouped_gemm_args& a = *args;
   NF_REQUIRE(a.dtype == NF_F32 || a.dtype == NF_BF16, "%s: unknown dtype %d", who, a.dtype);
-  NF_REQUIRE(a.act == NF_ACT_NONE || a.act == NF_ACT_GELU, "%s: unknown activation %d", who, a.act);
+  NF_REQUIRE(a.act == NF_ACT_NONE || a.act == NF_ACT_GELU || a.act == NF_ACT_SQUARED_RELU, "%s: unknown activation %d", who, a.act);
   NF_REQUIRE(a.groups > 0 && a.M >= 0 && a.N > 0 && a.K > 0 && a.N % 8 == 0 && a.K % 8 == 0 && a.lda >= a.K && a.ldd >= a.N && a.lda % 8 == 0 &&
                  a.ldd % 8 == 0 && a.a_group % 8 == 0 && a.d_group % 8 == 0,
              "%s: bad shape: %d groups, M=%d N=%d K=%d, strides %d %d", who, a.groups, a.M, a.N, a.K, a.lda, a.ldd);
@@ -118,10 +118,13 @@ int nf_gemm_grouped(const nf_grouped_gemm_args* args, nf_stream_t stream) {
   hipStream_t s = (hipStream_t)stream;
   if (a.dtype == NF_F32) {
     const int tiles_n = (a.N + kF32Tile - 1) / kF32Tile;
-    auto kern = a.act == NF_ACT_GELU ? gemm_grouped_f32_kernel<NF_ACT_GELU> : gemm_grouped_f32_kernel<NF_ACT_NONE>;
+    auto kern = a.act == NF_ACT_GELU           ? gemm_grouped_f32_kernel<NF_ACT_GELU>
+                : a.act == NF_ACT_SQUARED_RELU ? gemm_grouped_f32_kernel<NF_ACT_SQUARED_RELU>
+                                               : gemm_grouped_f32_kernel<NF_ACT_NONE>;
     kern<<<grid_of(a, kF32Tile, tiles_n), 256, 0, s>>>(a, tiles_n);
     return check_launch(who);
   }
+  if (a.act == NF_ACT_SQUARED_RELU) return dispatch_grouped<BF16SquaredRelu>(a, tile_rows, s);
   return a.act == NF_ACT_GELU ? dispatch_grouped<BF16Gelu>(a, tile_rows, s) : dispatch_grouped<BF16>(a, tile_rows, s);
 }
 

@@ -1,6 +1,6 @@
-// Attention of the layer-stack pipeline: per-head norm + rotation + query temperature + append to the paged
-// cache, and attention over a window with kept first positions, a sink in the softmax and a gate per head, for any
-// head sizes.
+// Attention of the layer-stack pipeline: short convolution + per-head norm + rotation + query temperature + append
+// to the paged cache, and attention over a window with kept first positions, capped scores, a sink in the softmax and a
+// gate per head, for any head sizes; also the difference of two attentions of a head over the same values.
 //
 // bf16 (attn_window_kernel, v_mfma_f32_16x16x32_bf16): S^T = K . Q^T, then O^T = V^T . P^T, per
 // (request, kv head, up to 16 of its query heads).  The 16 MFMA columns carry (token, head) pairs.
@@ -9,6 +9,8 @@
 //     second product's operand without a permute; V is cached transposed (a value column's 16 positions
 //     of a page are contiguous), so its operand is one 16-byte load as well.  Neither goes through LDS.
 //   * Softmax weights keep 32 bits: P is multiplied as two bf16 terms, P = hi + lo.
+//   * Two maps of a head are two sets of columns beside each other, with keys of their own: a value fragment serves
+//     both, and their difference and its norm are taken in fp32 where the sums are.
 //   * Only the 32-key steps that hold a visible key are visited: those of the kept first positions,
 //     then those of the window.
 //   * decode: one token per request, the wavefronts of a workgroup take every n-th step and merge
@@ -29,12 +31,78 @@ constexpr int kPage = 16;
 constexpr int kMaxHeadDim = 256;
 
 __host__ __device__ inline size_t kv_page_elements(const nf_kv_layout& kv) {
-  return (size_t)kv.kv_heads * kv.page * (kv.k_pad + kv.v_pad);
+  return (size_t)kv.kv_heads * kv.page * (kv.maps * kv.k_pad + kv.v_pad);
 }
+__host__ __device__ inline size_t kv_value_offset(const nf_kv_layout& kv) { return (size_t)kv.kv_heads * kv.maps * kv.page * kv.k_pad; }
 
 // ---------------------------------------------------------------- norm, rotation, append
 __device__ __forceinline__ float temperature(const nf_query_temperature& q, int pos) {
   return q.every > 0 ? 1.f + q.coef * logf((float)((pos + 1) / q.every + 1)) : 1.f;
+}
+
+// A row of the projections as the short convolution sees it: rows before it, of the batch or of the request's slot.
+template <class T>
+struct ConvRow {
+  const T* proj = nullptr;  // this row
+  const T* weight = nullptr;
+  T* state = nullptr;       // of the request's slot
+  int taps = 0, ld = 0, pos = 0, before = 0;  // before: rows of the portion ahead of this one
+  bool single = false;      // the request's only row, which leaves the state as well
+
+  __device__ __forceinline__ ConvRow(const nf_short_conv& c, const T* proj_, int ld_, int t, int req, int pos_)
+      : proj(proj_ + (size_t)t * ld_), weight((const T*)c.weight), taps(c.taps), ld(ld_), pos(pos_) {
+    if (taps < 1) return;
+    const int first = c.input_indptr[req];
+    before = t - first;
+    single = c.input_indptr[req + 1] - first == 1;
+    if (taps > 1) state = (T*)c.state + (size_t)c.state_slots[req] * (taps - 1) * ld;
+  }
+  // its value j rows back, j in 1 .. min(taps - 1, pos)
+  __device__ __forceinline__ const T* back(int j) const { return j <= before ? proj - (size_t)j * ld : state + (size_t)((pos - j) % (taps - 1)) * ld; }
+  // columns c .. c + 3; `owner`: of the threads that ask for them, the one that keeps the state
+  __device__ __forceinline__ float4_t four(int c, bool owner) const {
+    const typename Act<T>::raw4 cur = Act<T>::load_raw4(proj + c);
+    if (taps < 1) return Act<T>::widen4(cur);
+    const int past = min(taps - 1, pos);
+    float4_t y{0.f, 0.f, 0.f, 0.f};
+    constexpr int kAhead = 3;
+    for (int j0 = 1; j0 <= past; j0 += kAhead) {
+      typename Act<T>::raw4 x[kAhead], w[kAhead];
+#pragma unroll
+      for (int u = 0; u < kAhead; ++u) {  // past the last tap: the last one's again, left out below
+        const int j = min(j0 + u, past);
+        x[u] = Act<T>::load_raw4(back(j) + c);
+        w[u] = Act<T>::load_raw4(weight + (size_t)(taps - 1 - j) * ld + c);
+      }
+#pragma unroll
+      for (int u = 0; u < kAhead; ++u)
+        if (j0 + u <= past) y += Act<T>::widen4(x[u]) * Act<T>::widen4(w[u]);
+    }
+    y += Act<T>::widen4(cur) * Act<T>::load4(weight + (size_t)(taps - 1) * ld + c);
+    if (owner && single && taps > 1) *reinterpret_cast<typename Act<T>::raw4*>(state + (size_t)(pos % (taps - 1)) * ld + c) = cur;
+    return y;
+  }
+  __device__ __forceinline__ float one(int c) const {  // asked for by the owner only
+    const T cur = proj[c];
+    if (taps < 1) return Act<T>::load(&cur);
+    float y = 0.f;
+    for (int j = 1; j <= min(taps - 1, pos); ++j) y += Act<T>::load(back(j) + c) * Act<T>::load(weight + (size_t)(taps - 1 - j) * ld + c);
+    y += Act<T>::load(&cur) * Act<T>::load(weight + (size_t)(taps - 1) * ld + c);
+    if (single && taps > 1) state[(size_t)(pos % (taps - 1)) * ld + c] = cur;
+    return y;
+  }
+};
+
+// The last rows of every request that brings more than one, as the state of its convolution.  Sixteen bytes a thread.
+template <class T>
+__global__ __launch_bounds__(256) void conv_state_kernel(const T* __restrict__ proj, int ld, nf_short_conv conv, const int32_t* __restrict__ positions,
+                                                         int req_begin) {
+  const int req = req_begin + blockIdx.x, first = conv.input_indptr[req], end = conv.input_indptr[req + 1];
+  const int c = (blockIdx.y * 256 + threadIdx.x) * (16 / (int)sizeof(T)), keep = conv.taps - 1;
+  if (end - first < 2 || c >= ld) return;
+  T* state = (T*)conv.state + (size_t)conv.state_slots[req] * keep * ld;
+  for (int t = max(first, end - keep); t < end; ++t)
+    *reinterpret_cast<u32x4*>(state + (size_t)((positions[first] + t - first) % keep) * ld + c) = *reinterpret_cast<const u32x4*>(proj + (size_t)t * ld + c);
 }
 
 // One wavefront per (row, head): query heads, then key heads, then value heads.
@@ -42,7 +110,7 @@ template <class T>
 __global__ __launch_bounds__(256) void qkv_append_kernel(nf_kv_layout kv, const T* __restrict__ proj, int ld, int q_col,
                                                          int k_col, int v_col, const float* __restrict__ q_norm,
                                                          const float* __restrict__ k_norm, float eps, nf_rotation rot,
-                                                         nf_query_temperature q_temp, T* __restrict__ q_out, T* __restrict__ kv_data,
+                                                         nf_query_temperature q_temp, nf_short_conv conv, T* __restrict__ q_out, T* __restrict__ kv_data,
                                                          const int32_t* __restrict__ kv_indptr,
                                                          const int32_t* __restrict__ kv_indices,
                                                          const int32_t* __restrict__ rev_input_indptr,
@@ -51,11 +119,12 @@ __global__ __launch_bounds__(256) void qkv_append_kernel(nf_kv_layout kv, const 
   const int t = blockIdx.x, lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int job = blockIdx.y * 4 + wave;
-  const int H = kv.heads, G = kv.kv_heads;
+  const int H = kv.heads * kv.maps, G = kv.kv_heads * kv.maps, VG = kv.kv_heads;
   const int pos = positions[t], req = rev_input_indptr[t];
+  const ConvRow<T> row(conv, proj, ld, t, req, pos);
   T* page = nullptr;
   int entry = 0;
-  if (job >= H && job < H + 2 * G) {
+  if (job >= H && job < H + G + VG) {
     page = kv_data + (size_t)kv_indices[kv_indptr[req] + pos / kPage] * kv_page_elements(kv);
     entry = pos % kPage;
   }
@@ -63,14 +132,14 @@ __global__ __launch_bounds__(256) void qkv_append_kernel(nf_kv_layout kv, const 
   if (is_qk) {
     const bool is_q = job < H;
     const int head = is_q ? job : job - H;
-    const T* src = proj + (size_t)t * ld + (is_q ? q_col : k_col) + (size_t)head * kv.dim;
+    const int col = (is_q ? q_col : k_col) + head * kv.dim;
     const float* w = is_q ? q_norm : k_norm;
     float v[kMaxHeadDim / 64];
     float sq = 0.f;
 #pragma unroll
     for (int i = 0; i < kMaxHeadDim / 64; ++i) {
       const int c = i * 64 + lane;
-      v[i] = c < kv.dim ? Act<T>::load(src + c) : 0.f;
+      v[i] = c < kv.dim ? row.one(col + c) : 0.f;
       sq += v[i] * v[i];
     }
     if (w) {
@@ -105,11 +174,10 @@ __global__ __launch_bounds__(256) void qkv_append_kernel(nf_kv_layout kv, const 
       }
       Act<T>::store(dst + c, y * temp);
     }
-  } else if (job < H + 2 * G) {
+  } else if (job < H + G + VG) {
     const int head = job - H - G;
-    const T* src = proj + (size_t)t * ld + v_col + (size_t)head * kv.vdim;
-    T* dst = page + (size_t)G * kPage * kv.k_pad + (size_t)head * kv.v_pad * kPage + entry;
-    for (int c = lane; c < kv.v_pad; c += 64) Act<T>::store(dst + (size_t)c * kPage, c < kv.vdim ? Act<T>::load(src + c) : 0.f);
+    T* dst = page + kv_value_offset(kv) + (size_t)head * kv.v_pad * kPage + entry;
+    for (int c = lane; c < kv.v_pad; c += 64) Act<T>::store(dst + (size_t)c * kPage, c < kv.vdim ? row.one(v_col + head * kv.vdim + c) : 0.f);
   }
 }
 
@@ -120,7 +188,7 @@ template <class T>
 __global__ __launch_bounds__(256) void qkv_append4_kernel(nf_kv_layout kv, const T* __restrict__ proj, int ld, int q_col,
                                                           int k_col, int v_col, const float* __restrict__ q_norm,
                                                           const float* __restrict__ k_norm, float eps, nf_rotation rot,
-                                                          nf_query_temperature q_temp, T* __restrict__ q_out, T* __restrict__ kv_data,
+                                                          nf_query_temperature q_temp, nf_short_conv conv, T* __restrict__ q_out, T* __restrict__ kv_data,
                                                           const int32_t* __restrict__ kv_indptr,
                                                           const int32_t* __restrict__ kv_indices,
                                                           const int32_t* __restrict__ rev_input_indptr,
@@ -128,23 +196,24 @@ __global__ __launch_bounds__(256) void qkv_append4_kernel(nf_kv_layout kv, const
   __shared__ __attribute__((aligned(16))) float buf[kMaxHeadDim * 17];
   __shared__ long long row_page[16];  // element offset of the row's page, and its entry
   __shared__ int row_entry[16];
-  const int H = kv.heads, G = kv.kv_heads, tid = threadIdx.x;
+  const int H = kv.heads * kv.maps, G = kv.kv_heads * kv.maps, VG = kv.kv_heads, tid = threadIdx.x;
   if ((int)blockIdx.x < qk_blocks) {
     constexpr int kVec = kMaxHeadDim / 64;
     const int job = blockIdx.x * 16 + (tid >> 4), l = tid & 15;
     const bool live = job < rows * (H + G);
     const int t = live ? job / (H + G) : 0, head = live ? job % (H + G) : 0;
     const bool is_q = head < H;
-    const T* src = proj + (size_t)t * ld + (is_q ? q_col + head * kv.dim : k_col + (head - H) * kv.dim);
+    const int col = is_q ? q_col + head * kv.dim : k_col + (head - H) * kv.dim;
     const float* w = is_q ? q_norm : k_norm;
     float* mine = buf + (tid >> 4) * kMaxHeadDim;
-    const int pos = positions[t], half = rot.dims / 2;
+    const int pos = positions[t], req = rev_input_indptr[t], half = rot.dims / 2;
+    const ConvRow<T> row(conv, proj, ld, t, req, pos);
     const float temp = is_q ? temperature(q_temp, pos) : 1.f;
     T* dst;
     if (is_q) {
       dst = q_out + ((size_t)t * H + head) * kv.k_pad;
     } else {
-      const int page = kv_indices[kv_indptr[rev_input_indptr[t]] + pos / kPage];
+      const int page = kv_indices[kv_indptr[req] + pos / kPage];
       dst = kv_data + (size_t)page * kv_page_elements(kv) + ((size_t)(head - H) * kPage + pos % kPage) * kv.k_pad;
     }
     float4_t v[kVec];
@@ -153,7 +222,7 @@ __global__ __launch_bounds__(256) void qkv_append4_kernel(nf_kv_layout kv, const
     for (int i = 0; i < kVec; ++i) {
       const int c = (i * 16 + l) * 4;
       v[i] = float4_t{0.f, 0.f, 0.f, 0.f};
-      if (c < kv.dim) v[i] = Act<T>::load4(src + c);
+      if (c < kv.dim) v[i] = row.four(col + c, live);
 #pragma unroll
       for (int e = 0; e < 4; ++e) sq += v[i][e] * v[i][e];
     }
@@ -198,22 +267,22 @@ __global__ __launch_bounds__(256) void qkv_append4_kernel(nf_kv_layout kv, const
     }
     return;
   }
-  const int block = blockIdx.x - qk_blocks, head = block % G, row0 = block / G * 16;
+  const int block = blockIdx.x - qk_blocks, head = block % VG, row0 = block / VG * 16;
   if (tid < 16) {
     const int t = min(row0 + tid, rows - 1), pos = positions[t];
     row_page[tid] = (long long)kv_indices[kv_indptr[rev_input_indptr[t]] + pos / kPage] * (long long)kv_page_elements(kv);
     row_entry[tid] = row0 + tid < rows ? pos % kPage : -1;
   }
-  const int r = tid >> 4;
-  const T* src = proj + (size_t)min(row0 + r, rows - 1) * ld + v_col + head * kv.vdim;
+  const int r = tid >> 4, t = min(row0 + r, rows - 1);
+  const ConvRow<T> row(conv, proj, ld, t, rev_input_indptr[t], positions[t]);
   for (int c = (tid & 15) * 4; c < kv.v_pad; c += 64) {
     float4_t v{0.f, 0.f, 0.f, 0.f};
-    if (c < kv.vdim) v = Act<T>::load4(src + c);
+    if (c < kv.vdim) v = row.four(v_col + head * kv.vdim + c, row0 + r < rows);
 #pragma unroll
     for (int e = 0; e < 4; ++e) buf[(c + e) * 17 + r] = v[e];
   }
   __syncthreads();
-  T* base = kv_data + (size_t)G * kPage * kv.k_pad + (size_t)head * kv.v_pad * kPage;
+  T* base = kv_data + kv_value_offset(kv) + (size_t)head * kv.v_pad * kPage;
   for (int e = tid; e < kv.v_pad * 4; e += 256) {
     const int c = e >> 2, r0 = (e & 3) * 4, en = row_entry[r0];
     const float* v = buf + c * 17 + r0;
@@ -255,6 +324,22 @@ __device__ __forceinline__ float head_factor(const nf_window_attention_args& a, 
   return a.gate ? a.out_scale * sigmoid<T>(Act<T>::load((const T*)a.gate + (size_t)row * a.gate_ld + h)) : a.out_scale;
 }
 
+// Scores brought within +-softcap, in the exponent's units (base 2): softcap * tanh(s * scale / softcap) * log2 e, with
+// tanh x = 1 - 2 / (1 + e^2x).  Without a cap they are left alone and `scale` is still to be applied.
+struct ScoreCap {
+  float before, limit, scale;
+  __device__ __forceinline__ explicit ScoreCap(const nf_window_attention_args& a) {
+    constexpr float log2e = 1.44269504088896340736f;
+    limit = a.softcap > 0.f ? a.softcap * log2e : 0.f;
+    before = a.softcap > 0.f ? 2.f * log2e * a.scale / a.softcap : 0.f;
+    scale = a.softcap > 0.f ? 1.f : a.scale * log2e;
+  }
+  __device__ __forceinline__ void apply(float4_t& s) const {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) s[r] = fmaf(-2.f * limit, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s[r] * before)), limit);
+  }
+};
+
 // ---------------------------------------------------------------- fp32
 template <class T>
 __global__ __launch_bounds__(64) void attn_rows_kernel(nf_window_attention_args a) {
@@ -264,69 +349,83 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(nf_window_attention_args 
   const int lane = threadIdx.x, t = a.row_begin + blockIdx.x, h = blockIdx.y;
   const int req = a.rev_input_indptr[t], p = a.positions[t];
   const int g = h / (kv.heads / kv.kv_heads);
-  const T* q = (const T*)a.q + ((size_t)t * kv.heads + h) * kv.k_pad;
-  for (int c = lane; c < kv.k_pad; c += 64) sq[c] = Act<T>::load(q + c);
-  __syncthreads();
   const T* pool = (const T*)a.kv_data;
   const size_t page_elems = kv_page_elements(kv);
   const int32_t* pages = a.kv_indices + a.kv_indptr[req];
-  float m = a.sink ? a.sink[h] : -1e30f;
-  float l = 0.f;  // this lane's part of the denominator
-  float o[kMaxHeadDim / 64] = {};
   const StepRange steps = visible_steps(p, p, a.window, a.keep_first, 64);
-  for (int i = 0; i < steps.total; ++i) {
-    const int base = steps.at(i) * 64, j = base + lane;
-    const bool see = sees(p, j, a.window, a.keep_first);
-    float s = -INFINITY;
-    if (see) {
-      const T* k = pool + (size_t)pages[j / kPage] * page_elems + ((size_t)g * kPage + j % kPage) * kv.k_pad;
-      float dot = 0.f;
-      for (int c = 0; c < kv.k_pad; c += 4) {
-        const float4_t kk = Act<T>::load4(k + c), qq = *reinterpret_cast<const float4_t*>(sq + c);
-        dot += kk[0] * qq[0] + kk[1] * qq[1] + kk[2] * qq[2] + kk[3] * qq[3];
+  float out_row[kMaxHeadDim / 64] = {};
+  for (int map = 0; map < kv.maps; ++map) {
+    const T* q = (const T*)a.q + (((size_t)t * kv.heads + h) * kv.maps + map) * kv.k_pad;
+    __syncthreads();
+    for (int c = lane; c < kv.k_pad; c += 64) sq[c] = Act<T>::load(q + c);
+    __syncthreads();
+    float m = a.sink ? a.sink[h] : -1e30f;
+    float l = 0.f;  // this lane's part of the denominator
+    float o[kMaxHeadDim / 64] = {};
+    for (int i = 0; i < steps.total; ++i) {
+      const int base = steps.at(i) * 64, j = base + lane;
+      const bool see = sees(p, j, a.window, a.keep_first);
+      float s = -INFINITY;
+      if (see) {
+        const T* k = pool + (size_t)pages[j / kPage] * page_elems + (((size_t)g * kv.maps + map) * kPage + j % kPage) * kv.k_pad;
+        float dot = 0.f;
+        for (int c = 0; c < kv.k_pad; c += 4) {
+          const float4_t kk = Act<T>::load4(k + c), qq = *reinterpret_cast<const float4_t*>(sq + c);
+          dot += kk[0] * qq[0] + kk[1] * qq[1] + kk[2] * qq[2] + kk[3] * qq[3];
+        }
+        s = dot * a.scale;
+        if (a.softcap > 0.f) s = a.softcap * tanhf(s / a.softcap);
       }
-      s = dot * a.scale;
-    }
-    float mx = s;
+      float mx = s;
 #pragma unroll
-    for (int d = 32; d > 0; d >>= 1) mx = fmaxf(mx, __shfl_xor(mx, d, 64));
-    const float m_new = fmaxf(m, mx), alpha = expf(m - m_new);
-    const float w = see ? expf(s - m_new) : 0.f;
-    m = m_new;
-    l = l * alpha + w;
-    __syncthreads();
-    sp[lane] = w;
-    __syncthreads();
+      for (int d = 32; d > 0; d >>= 1) mx = fmaxf(mx, __shfl_xor(mx, d, 64));
+      const float m_new = fmaxf(m, mx), alpha = expf(m - m_new);
+      const float w = see ? expf(s - m_new) : 0.f;
+      m = m_new;
+      l = l * alpha + w;
+      __syncthreads();
+      sp[lane] = w;
+      __syncthreads();
 #pragma unroll
-    for (int e = 0; e < kMaxHeadDim / 64; ++e) o[e] *= alpha;
-    const int n_pages = min(4, (p - base) / kPage + 1);
-    for (int b = 0; b < n_pages; ++b) {
-      const T* v = pool + (size_t)pages[base / kPage + b] * page_elems + (size_t)kv.kv_heads * kPage * kv.k_pad +
-                   (size_t)g * kv.v_pad * kPage;
+      for (int e = 0; e < kMaxHeadDim / 64; ++e) o[e] *= alpha;
+      const int n_pages = min(4, (p - base) / kPage + 1);
+      for (int b = 0; b < n_pages; ++b) {
+        const T* v = pool + (size_t)pages[base / kPage + b] * page_elems + kv_value_offset(kv) + (size_t)g * kv.v_pad * kPage;
 #pragma unroll
-      for (int e = 0; e < kMaxHeadDim / 64; ++e) {
-        const int c = e * 64 + lane;
-        if (c >= kv.v_pad) break;
+        for (int e = 0; e < kMaxHeadDim / 64; ++e) {
+          const int c = e * 64 + lane;
+          if (c >= kv.v_pad) break;
 #pragma unroll
-        for (int r = 0; r < kPage; r += 4) {
-          const float4_t vv = Act<T>::load4(v + (size_t)c * kPage + r);
+          for (int r = 0; r < kPage; r += 4) {
+            const float4_t vv = Act<T>::load4(v + (size_t)c * kPage + r);
 #pragma unroll
-          for (int x = 0; x < 4; ++x) {
-            const float wt = sp[b * kPage + r + x];
-            if (wt != 0.f) o[e] += wt * vv[x];  // an entry past the sequence may hold anything
+            for (int x = 0; x < 4; ++x) {
+              const float wt = sp[b * kPage + r + x];
+              if (wt != 0.f) o[e] += wt * vv[x];  // an entry past the sequence may hold anything
+            }
           }
         }
       }
     }
+    l = wave_sum(l);
+    if (a.sink) l += expf(a.sink[h] - m);
+    const float part = (map == 0 ? 1.f : -a.map_weight) / l;
+#pragma unroll
+    for (int e = 0; e < kMaxHeadDim / 64; ++e) out_row[e] += o[e] * part;
   }
-  l = wave_sum(l);
-  if (a.sink) l += expf(a.sink[h] - m);
-  const float inv = head_factor<T>(a, t, h) / l;
+  float factor = head_factor<T>(a, t, h);
+  if (a.head_norm) {
+    float sum = 0.f;
+#pragma unroll
+    for (int e = 0; e < kMaxHeadDim / 64; ++e)
+      if (e * 64 + lane < kv.vdim) sum += out_row[e] * out_row[e];
+    factor /= sqrtf(wave_sum(sum) / (float)kv.vdim + a.head_eps);
+  }
   T* out = (T*)a.out + (size_t)t * a.out_ld + a.out_col + (size_t)h * kv.vdim;
 #pragma unroll
   for (int e = 0; e < kMaxHeadDim / 64; ++e) {
     const int c = e * 64 + lane;
-    if (c < kv.vdim) Act<T>::store(out + c, o[e] * inv);
+    if (c < kv.vdim) Act<T>::store(out + c, out_row[e] * factor);
   }
 }
 
@@ -349,10 +448,41 @@ __device__ __forceinline__ u32x4 load_cache(const bf16_t* p) {
   }
 }
 
+// What the lanes of a column (those with the same l16) hold of its output in the end, from the sums of its maps; `o` and `l`
+// hold kMaps entries.  The value columns are i * 16 + g * 4 ..
+template <int kMaps, int VD>
+__device__ __forceinline__ void finish_column(const nf_window_attention_args& a, float4_t (*o)[VD], const float* m, const float* l, int row, int h, int g) {
+  float den = l[0], f = 1.f;
+  if (a.sink) {
+    const float snk = a.sink[h] * 1.44269504088896340736f, mm = fmaxf(m[0], snk);
+    f = __builtin_amdgcn_exp2f(m[0] - mm);
+    den = den * f + __builtin_amdgcn_exp2f(snk - mm);
+  }
+  float factor = head_factor<bf16_t>(a, row, h), first = f / den;
+  if constexpr (kMaps == 2) {
+    const float second = a.map_weight / l[1];
+#pragma unroll
+    for (int i = 0; i < VD; ++i) o[0][i] = o[0][i] * first - o[1][i] * second;
+    first = 1.f;
+  }
+  if (a.head_norm) {
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < VD; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (i * 16 + g * 4 + r < a.kv.vdim) sum += o[0][i][r] * o[0][i][r];
+    factor /= sqrtf(sum_over_lane_groups(sum) * first * first / (float)a.kv.vdim + a.head_eps);
+  }
+#pragma unroll
+  for (int i = 0; i < VD; ++i) o[0][i] *= first * factor;
+}
+
 // KD: 32-wide pieces of k_pad, VD: 16-wide pieces of v_pad (both upper bounds), NB: column blocks per
 // wavefront.  gs: query heads of a kv head in one workgroup (at most 16).
-template <int KD, int VD, int NB, bool kDecode>
-__global__ __launch_bounds__(512) void attn_window_kernel(nf_window_attention_args a, int gs, int chunks, int tile_tokens) {
+constexpr int window_threads(int kMaps, int VD) { return kMaps == 2 && VD > 8 ? 256 : 512; }
+template <int KD, int VD, int NB, int kMaps, bool kDecode>
+__global__ __launch_bounds__(window_threads(kMaps, VD)) void attn_window_kernel(nf_window_attention_args a, int gs, int chunks, int tile_tokens) {
   extern __shared__ __attribute__((aligned(16))) float merge_lds[];
   const nf_kv_layout kv = a.kv;
   const int lane = threadIdx.x & 63, l16 = lane & 15, g = lane >> 4;
@@ -388,9 +518,10 @@ __global__ __launch_bounds__(512) void attn_window_kernel(nf_window_attention_ar
     if (tok0 >= len) return;
   }
 
+  constexpr int NC = NB * kMaps;  // sets of columns: a block's maps side by side
   int pos[NB], row[NB];
   bool live[NB];
-  B8 qf[NB][KD];
+  B8 qf[NC][KD];
   const int kd = kv.k_pad / 32, vd = kv.v_pad / 16;
 #pragma unroll
   for (int n = 0; n < NB; ++n) {
@@ -398,9 +529,12 @@ __global__ __launch_bounds__(512) void attn_window_kernel(nf_window_attention_ar
     live[n] = (kDecode ? l16 < heads : l16 < tpb * gs && tok < len && hc < heads);
     row[n] = row0 + (live[n] ? tok : (kDecode ? 0 : tok0));
     pos[n] = a.positions[row[n]];
-    const bf16_t* q = (const bf16_t*)a.q + ((size_t)row[n] * kv.heads + kvh * group + h0 + (live[n] ? hc : 0)) * kv.k_pad + g * 8;
+    const bf16_t* q = (const bf16_t*)a.q + ((size_t)row[n] * kv.heads + kvh * group + h0 + (live[n] ? hc : 0)) * kMaps * kv.k_pad + g * 8;
 #pragma unroll
-    for (int j = 0; j < KD; ++j) qf[n][j].u = live[n] && j < kd ? *reinterpret_cast<const u32x4*>(q + j * 32) : u32x4{0, 0, 0, 0};
+    for (int x = 0; x < kMaps; ++x)
+#pragma unroll
+      for (int j = 0; j < KD; ++j)
+        qf[n * kMaps + x][j].u = live[n] && j < kd ? *reinterpret_cast<const u32x4*>(q + x * kv.k_pad + j * 32) : u32x4{0, 0, 0, 0};
   }
   const int p0 = a.positions[row0 + tok0];
   const int p1 = kDecode ? p0 : p0 + min(NB * tpb, len - tok0) - 1;
@@ -413,36 +547,38 @@ __global__ __launch_bounds__(512) void attn_window_kernel(nf_window_attention_ar
   // this lane's pieces inside a page: K rows of tile b (b = 0, 1), V column piece
   const int key = 8 * (l16 >> 2) + (l16 & 3);  // of tile 0 in the step; tile 1: + 4
   const int kpg = key >> 4;                    // its page of the step's two (tile 1's is the same)
-  const size_t k_off0 = ((size_t)kvh * kPage + (key & 15)) * kv.k_pad + g * 8;
-  const size_t k_off1 = k_off0 + (size_t)4 * kv.k_pad;
-  const size_t v_off = (size_t)kv.kv_heads * kPage * kv.k_pad + ((size_t)kvh * kv.v_pad + l16) * kPage + (g & 1) * 8;
+  const size_t k_off = ((size_t)kvh * kMaps * kPage + (key & 15)) * kv.k_pad + g * 8;
+  const size_t v_off = kv_value_offset(kv) + ((size_t)kvh * kv.v_pad + l16) * kPage + (g & 1) * 8;
   const int vpg = g >> 1;
 
-  float4_t o[NB][VD];
-  float m[NB], l[NB];
+  float4_t o[NC][VD];
+  float m[NC], l[NC];
 #pragma unroll
-  for (int n = 0; n < NB; ++n) {
+  for (int n = 0; n < NC; ++n) {
     m[n] = -1e30f;
     l[n] = 0.f;
 #pragma unroll
     for (int i = 0; i < VD; ++i) o[n][i] = float4_t{0.f, 0.f, 0.f, 0.f};
   }
-  const float scale2 = a.scale * 1.44269504088896340736f;
+  const ScoreCap cap(a);
+  const float scale2 = cap.scale;
 
   // page ids are read a step before the loads that need them
   auto page_id = [&](int it, int which) {
     const int idx = steps.at(it) * 2 + which;
     return pages[idx < last_page ? idx : last_page];  // past the last page the keys are no one's: read something mapped
   };
-  B8 kf[2][KD];
+  B8 kf[kMaps][2][KD];
   auto load_k = [&](int id) {
-    const bf16_t* k = pool + (size_t)id * page_elems;
+    const bf16_t* k = pool + (size_t)id * page_elems + k_off;
 #pragma unroll
-    for (int j = 0; j < KD; ++j)
-      if (j < kd) {
-        kf[0][j].u = load_cache<kDecode>(k + k_off0 + j * 32);
-        kf[1][j].u = load_cache<kDecode>(k + k_off1 + j * 32);
-      }
+    for (int x = 0; x < kMaps; ++x)
+#pragma unroll
+      for (int j = 0; j < KD; ++j)
+        if (j < kd) {
+          kf[x][0][j].u = load_cache<kDecode>(k + (size_t)(x * kPage) * kv.k_pad + j * 32);
+          kf[x][1][j].u = load_cache<kDecode>(k + (size_t)(x * kPage + 4) * kv.k_pad + j * 32);
+        }
   };
   const int first = kDecode ? wave : 0, stride = kDecode ? waves : 1;
   if (first >= steps.total && !kDecode) return;
@@ -460,28 +596,29 @@ __global__ __launch_bounds__(512) void attn_window_kernel(nf_window_attention_ar
       if (i < vd) vf[i].u = load_cache<kDecode>(v + (size_t)i * 16 * kPage);
     const int next_k_id = page_id(min(it + 2 * stride, final_it), kpg);
     v_id = page_id(min(it + stride, final_it), vpg);
-    float4_t s[NB][2];
+    float4_t s[NC][2];
 #pragma unroll
-    for (int n = 0; n < NB; ++n)
+    for (int n = 0; n < NC; ++n)
 #pragma unroll
       for (int b = 0; b < 2; ++b) {
         s[n][b] = float4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int j = 0; j < KD; ++j)
-          if (j < kd) s[n][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[b][j].b, qf[n][j].b, s[n][b], 0, 0, 0);
+          if (j < kd) s[n][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[n % kMaps][b][j].b, qf[n][j].b, s[n][b], 0, 0, 0);
+        if (cap.limit > 0.f) cap.apply(s[n][b]);
       }
     if (it + stride < steps.total) load_k(k_id);
     k_id = next_k_id;
     const bool whole = base + 31 <= p0 && (a.window <= 0 || p1 - base < a.window || base + 31 < a.keep_first);
 #pragma unroll
-    for (int n = 0; n < NB; ++n) {
+    for (int n = 0; n < NC; ++n) {
       const int j0 = base + 8 * g;
       float mx = -1e30f;
 #pragma unroll
       for (int b = 0; b < 2; ++b)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          if (!whole && !sees(pos[n], j0 + 4 * b + r, a.window, a.keep_first)) s[n][b][r] = -INFINITY;
+          if (!whole && !sees(pos[n / kMaps], j0 + 4 * b + r, a.window, a.keep_first)) s[n][b][r] = -INFINITY;
           mx = fmaxf(mx, s[n][b][r]);
         }
       mx = mx > -1e30f ? mx * scale2 : mx;
@@ -518,62 +655,76 @@ __global__ __launch_bounds__(512) void attn_window_kernel(nf_window_attention_ar
 
   bf16_t* out = (bf16_t*)a.out;
 #pragma unroll
-  for (int n = 0; n < NB; ++n) {
+  for (int n = 0; n < NC; ++n) {
     l[n] += __shfl_xor(l[n], 16, 64);
     l[n] += __shfl_xor(l[n], 32, 64);
   }
   if constexpr (kDecode) {
-    // merge the wavefronts: m and l of [wave][16 columns], O of [wave][heads][v_pad]
+    // merge the wavefronts: m and l of [wave][map][16 columns], O of [wave][map][heads][v_pad]
     float* sm = merge_lds;
-    float* sl = sm + waves * 16;
-    float* so = sl + waves * 16;
-    if (g == 0) {
-      sm[wave * 16 + l16] = m[0];
-      sl[wave * 16 + l16] = l[0];
-    }
-    if (l16 < heads)
+    float* sl = sm + waves * kMaps * 16;
+    float* so = sl + waves * kMaps * 16;
 #pragma unroll
-      for (int i = 0; i < VD; ++i)
-        if (i < vd) *reinterpret_cast<float4_t*>(so + ((size_t)wave * gs + l16) * kv.v_pad + i * 16 + g * 4) = o[0][i];
+    for (int x = 0; x < kMaps; ++x) {
+      if (g == 0) {
+        sm[(wave * kMaps + x) * 16 + l16] = m[x];
+        sl[(wave * kMaps + x) * 16 + l16] = l[x];
+      }
+      if (l16 < heads)
+#pragma unroll
+        for (int i = 0; i < VD; ++i)
+          if (i < vd) *reinterpret_cast<float4_t*>(so + ((size_t)(wave * kMaps + x) * gs + l16) * kv.v_pad + i * 16 + g * 4) = o[x][i];
+    }
     __syncthreads();
+    bf16_t* dst = out + (size_t)row0 * a.out_ld + a.out_col + (size_t)(kvh * group + h0) * kv.vdim;
     for (int e = threadIdx.x; e < heads * kv.vdim; e += blockDim.x) {
       const int hc = e / kv.vdim, c = e % kv.vdim;
       const int h = kvh * group + h0 + hc;
-      const float snk = a.sink ? a.sink[h] * 1.44269504088896340736f : -1e30f;
-      float mm = snk;
-      for (int w = 0; w < waves; ++w) mm = fmaxf(mm, sm[w * 16 + hc]);
-      float den = a.sink ? __builtin_amdgcn_exp2f(snk - mm) : 0.f, acc = 0.f;
-      for (int w = 0; w < waves; ++w) {
-        const float f = __builtin_amdgcn_exp2f(sm[w * 16 + hc] - mm);
-        den += sl[w * 16 + hc] * f;
-        acc += so[((size_t)w * gs + hc) * kv.v_pad + c] * f;
+      float v = 0.f;
+#pragma unroll
+      for (int x = 0; x < kMaps; ++x) {
+        const float snk = a.sink ? a.sink[h] * 1.44269504088896340736f : -1e30f;
+        float mm = snk;
+        for (int w = 0; w < waves; ++w) mm = fmaxf(mm, sm[(w * kMaps + x) * 16 + hc]);
+        float den = a.sink ? __builtin_amdgcn_exp2f(snk - mm) : 0.f, acc = 0.f;
+        for (int w = 0; w < waves; ++w) {
+          const float f = __builtin_amdgcn_exp2f(sm[(w * kMaps + x) * 16 + hc] - mm);
+          den += sl[(w * kMaps + x) * 16 + hc] * f;
+          acc += so[((size_t)(w * kMaps + x) * gs + hc) * kv.v_pad + c] * f;
+        }
+        v += acc * ((x == 0 ? 1.f : -a.map_weight) / den);
       }
-      Act<bf16_t>::store(out + (size_t)row0 * a.out_ld + a.out_col + (size_t)h * kv.vdim + c, acc * (head_factor<bf16_t>(a, row0, h) / den));
+      if (a.head_norm) so[(size_t)hc * kv.v_pad + c] = v;  // read by this thread alone until now
+      else Act<bf16_t>::store(dst + e, v * head_factor<bf16_t>(a, row0, h));
+    }
+    if (!a.head_norm) return;
+    __syncthreads();
+    for (int hc = wave; hc < heads; hc += waves) {
+      const float* v = so + (size_t)hc * kv.v_pad;
+      float sum = 0.f;
+      for (int c = lane; c < kv.vdim; c += 64) sum += v[c] * v[c];
+      const float f = head_factor<bf16_t>(a, row0, kvh * group + h0 + hc) / sqrtf(wave_sum(sum) / (float)kv.vdim + a.head_eps);
+      for (int c = lane; c < kv.vdim; c += 64) Act<bf16_t>::store(dst + hc * kv.vdim + c, v[c] * f);
     }
   } else {
 #pragma unroll
     for (int n = 0; n < NB; ++n) {
-      if (!live[n]) continue;
       const int h = kvh * group + h0 + l16 % gs;
-      float den = l[n], f = 1.f;
-      if (a.sink) {
-        const float snk = a.sink[h] * 1.44269504088896340736f, mm = fmaxf(m[n], snk);
-        f = __builtin_amdgcn_exp2f(m[n] - mm);
-        den = den * f + __builtin_amdgcn_exp2f(snk - mm);
-      }
-      const float inv = f * head_factor<bf16_t>(a, row[n], h) / den;
+      finish_column<kMaps, VD>(a, o + n * kMaps, m + n * kMaps, l + n * kMaps, row[n], live[n] ? h : kvh * group + h0, g);
+      if (!live[n]) continue;
       bf16_t* dst = out + (size_t)row[n] * a.out_ld + a.out_col + (size_t)h * kv.vdim;
       const bool vec = (kv.vdim | a.out_ld | a.out_col) % 4 == 0;
 #pragma unroll
       for (int i = 0; i < VD; ++i) {
         const int c = i * 16 + g * 4;
         if (i >= vd || c >= kv.vdim) continue;
+        const float4_t v = o[n * kMaps][i];
         if (vec) {
-          Act<bf16_t>::store4(dst + c, o[n][i] * inv);
+          Act<bf16_t>::store4(dst + c, v);
         } else {
 #pragma unroll
           for (int r = 0; r < 4; ++r)
-            if (c + r < kv.vdim) Act<bf16_t>::store(dst + c + r, o[n][i][r] * inv);
+            if (c + r < kv.vdim) Act<bf16_t>::store(dst + c + r, v[r]);
         }
       }
     }
@@ -585,18 +736,19 @@ __global__ __launch_bounds__(512) void attn_window_kernel(nf_window_attention_ar
 // 16-byte slots --; then V as it is cached, per page and value column 32 bytes, halves swapped where bit 3 of the column is
 // set, for the same reason.
 constexpr int kTileRing = 4;
-template <int KD, int VD>
+template <int KD, int VD, int kMaps>
 struct TileShape {
-  static constexpr int planes = KD / 2, k_bytes = planes * 4096, v_groups = VD / 2;  // groups of 32 value columns
+  static constexpr int planes = kMaps * KD / 2, k_bytes = planes * 4096, v_groups = VD / 2;  // groups of 32 value columns
   static constexpr int v_bytes = 2 * v_groups * 1024, slot = k_bytes + v_bytes;
   static constexpr int loads = planes + v_groups / 2;  // per wavefront and slot
 };
 
 // KD: k_pad / 32 (even), VD: v_pad / 16 (a multiple of 4), NB: column blocks per wavefront.  blockIdx.x: kv head and chunk of its
 // query heads -- so that the tiles of a head tend to share an XCD's L2 --, blockIdx.y: tile.
-template <int KD, int VD, int NB>
+template <int KD, int VD, int NB, int kMaps>
 __global__ __launch_bounds__(256, 2) void attn_tile_kernel(nf_window_attention_args a, int gs, int chunks, int tile_tokens, bool all_resident) {
-  using S = TileShape<KD, VD>;
+  using S = TileShape<KD, VD, kMaps>;
+  constexpr int NC = NB * kMaps;  // sets of columns: a block's maps side by side
   extern __shared__ __attribute__((aligned(1024))) uint8_t ring[];
   const uint32_t lds0 = (uint32_t)(uintptr_t)(__attribute__((address_space(3))) uint8_t*)ring;
   const nf_kv_layout kv = a.kv;
@@ -647,11 +799,11 @@ __global__ __launch_bounds__(256, 2) void attn_tile_kernel(nf_window_attention_a
     }
     const int page = __builtin_amdgcn_readlane(ids, it % 32 * 2 + (wave >> 1));
     const uint8_t* base = (const uint8_t*)a.kv_data + (size_t)page * page_bytes;
-    const rsrc_t kr = make_rsrc(base + (size_t)kvh * kPage * KD * 64, (size_t)kPage * KD * 64);
-    const rsrc_t vr = make_rsrc(base + ((size_t)kv.kv_heads * kPage * KD * 32 + (size_t)kvh * VD * 16 * kPage) * 2, (size_t)VD * 16 * kPage * 2);
+    const rsrc_t kr = make_rsrc(base + (size_t)kvh * kMaps * kPage * KD * 64, (size_t)kMaps * kPage * KD * 64);
+    const rsrc_t vr = make_rsrc(base + ((size_t)kv.kv_heads * kMaps * kPage * KD * 32 + (size_t)kvh * VD * 16 * kPage) * 2, (size_t)VD * 16 * kPage * 2);
     const uint32_t slot = __builtin_amdgcn_readfirstlane(lds0 + (uint32_t)(it % kTileRing) * S::slot);
 #pragma unroll
-    for (int pl = 0; pl < S::planes; ++pl) load16_to_lds(kr, k_off + pl * 128, slot + pl * 4096 + wave * 1024);
+    for (int pl = 0; pl < S::planes; ++pl) load16_to_lds(kr, k_off + pl / (KD / 2) * (kPage * KD * 64) + pl % (KD / 2) * 128, slot + pl * 4096 + wave * 1024);
 #pragma unroll
     for (int c = 0; c < S::v_groups; c += 2)
       load16_to_lds(vr, v_off + c * 1024, slot + S::k_bytes + ((wave >> 1) * S::v_groups + (wave & 1) + c) * 1024);
@@ -667,30 +819,31 @@ __global__ __launch_bounds__(256, 2) void attn_tile_kernel(nf_window_attention_a
   for (int it = 0; it < min(kTileRing - 1, steps.total); ++it) load_step(it);
   int pos[NB], row[NB];
   bool live[NB];
-  B8 qf[NB][KD];
+  B8 qf[NC][KD];
 #pragma unroll
   for (int n = 0; n < NB; ++n) {
     const int tok = tok0 + n * tpb + l16 / gs, hc = l16 % gs;
     live[n] = l16 < tpb * gs && tok < len && hc < heads;
     row[n] = row0 + (live[n] ? tok : first_tok);
     pos[n] = p0 - first_tok + (live[n] ? tok : first_tok);
-    const bf16_t* q = (const bf16_t*)a.q + ((size_t)row[n] * kv.heads + kvh * group + h0 + (live[n] ? hc : 0)) * (KD * 32) + g * 8;
+    const bf16_t* q = (const bf16_t*)a.q + ((size_t)row[n] * kv.heads + kvh * group + h0 + (live[n] ? hc : 0)) * (kMaps * KD * 32) + g * 8;
 #pragma unroll
-    for (int j = 0; j < KD; ++j) qf[n][j].u = *reinterpret_cast<const u32x4*>(q + j * 32);  // columns of no token: never stored
+    for (int j = 0; j < kMaps * KD; ++j) qf[n * kMaps + j / KD][j % KD].u = *reinterpret_cast<const u32x4*>(q + j * 32);  // columns of no token: never stored
   }
   // Everything has landed once, here: a wait for the queries inside the loop would be one for the steps in flight.
   __builtin_amdgcn_s_waitcnt(0x0F70);
 
-  float4_t o[NB][VD];
-  float m[NB], l[NB];
+  float4_t o[NC][VD];
+  float m[NC], l[NC];
 #pragma unroll
-  for (int n = 0; n < NB; ++n) {
+  for (int n = 0; n < NC; ++n) {
     m[n] = -1e30f;
     l[n] = 0.f;
 #pragma unroll
     for (int i = 0; i < VD; ++i) o[n][i] = float4_t{0.f, 0.f, 0.f, 0.f};
   }
-  const float scale2 = a.scale * 1.44269504088896340736f;
+  const ScoreCap cap(a);
+  const float scale2 = cap.scale;
   const int key = 8 * (l16 >> 2) + (l16 & 3);  // of score tile 0; tile 1: + 4
   uint32_t kx[2][2];                           // [score tile][chunk half of a plane]
 #pragma unroll
@@ -703,31 +856,38 @@ __global__ __launch_bounds__(256, 2) void attn_tile_kernel(nf_window_attention_a
   const uint32_t vx = (uint32_t)S::k_bytes + (uint32_t)(g >> 1) * (S::v_groups * 1024) + (uint32_t)l16 * 32u + (uint32_t)((g & 1) ^ (l16 >> 3)) * 16u;
 
   auto compute = [&](const uint8_t* slot, int base) {
-    float4_t s[NB][2];
+    float4_t s[NC][2];
 #pragma unroll
-    for (int n = 0; n < NB; ++n)
+    for (int n = 0; n < NC; ++n)
 #pragma unroll
       for (int b = 0; b < 2; ++b) s[n][b] = float4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int j = 0; j < KD; ++j)
+    for (int x = 0; x < kMaps; ++x)
 #pragma unroll
-      for (int b = 0; b < 2; ++b) {
-        B8 k;
-        k.u = *reinterpret_cast<const u32x4*>(slot + (j >> 1) * 4096 + kx[b][j & 1]);
+      for (int j = 0; j < KD; ++j)
 #pragma unroll
-        for (int n = 0; n < NB; ++n) s[n][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k.b, qf[n][j].b, s[n][b], 0, 0, 0);
-      }
+        for (int b = 0; b < 2; ++b) {
+          B8 k;
+          k.u = *reinterpret_cast<const u32x4*>(slot + (x * (KD / 2) + (j >> 1)) * 4096 + kx[b][j & 1]);
+#pragma unroll
+          for (int n = x; n < NC; n += kMaps) s[n][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k.b, qf[n][j].b, s[n][b], 0, 0, 0);
+        }
+    if (cap.limit > 0.f)
+#pragma unroll
+      for (int n = 0; n < NC; ++n)
+#pragma unroll
+        for (int b = 0; b < 2; ++b) cap.apply(s[n][b]);
     const bool whole = base + 31 <= w0 && (a.window <= 0 || w1 - base < a.window || base + 31 < a.keep_first);
-    B8 hi[NB], lo[NB];
+    B8 hi[NC], lo[NC];
 #pragma unroll
-    for (int n = 0; n < NB; ++n) {
+    for (int n = 0; n < NC; ++n) {
       float mx = -1e30f;
       if (!whole)
 #pragma unroll
         for (int b = 0; b < 2; ++b)
 #pragma unroll
           for (int r = 0; r < 4; ++r)
-            if (!sees(pos[n], base + 8 * g + 4 * b + r, a.window, a.keep_first)) s[n][b][r] = -INFINITY;
+            if (!sees(pos[n / kMaps], base + 8 * g + 4 * b + r, a.window, a.keep_first)) s[n][b][r] = -INFINITY;
 #pragma unroll
       for (int b = 0; b < 2; ++b)
 #pragma unroll
@@ -757,9 +917,9 @@ __global__ __launch_bounds__(256, 2) void attn_tile_kernel(nf_window_attention_a
       B8 v;
       v.u = *reinterpret_cast<const u32x4*>(slot + vx + i * 512);
 #pragma unroll
-      for (int n = 0; n < NB; ++n) o[n][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v.b, hi[n].b, o[n][i], 0, 0, 0);
+      for (int n = 0; n < NC; ++n) o[n][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v.b, hi[n].b, o[n][i], 0, 0, 0);
 #pragma unroll
-      for (int n = 0; n < NB; ++n) o[n][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v.b, lo[n].b, o[n][i], 0, 0, 0);
+      for (int n = 0; n < NC; ++n) o[n][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v.b, lo[n].b, o[n][i], 0, 0, 0);
     }
   };
 
@@ -775,41 +935,37 @@ __global__ __launch_bounds__(256, 2) void attn_tile_kernel(nf_window_attention_a
   bf16_t* out = (bf16_t*)a.out;
   const bool vec = (kv.vdim | a.out_ld | a.out_col) % 4 == 0;
 #pragma unroll
+  for (int n = 0; n < NC; ++n) l[n] = sum_over_lane_groups(l[n]);
+#pragma unroll
   for (int n = 0; n < NB; ++n) {
-    l[n] = sum_over_lane_groups(l[n]);
-    if (!live[n]) continue;
     const int h = kvh * group + h0 + l16 % gs;
-    float den = l[n], f = 1.f;
-    if (a.sink) {
-      const float snk = a.sink[h] * 1.44269504088896340736f, mm = fmaxf(m[n], snk);
-      f = __builtin_amdgcn_exp2f(m[n] - mm);
-      den = den * f + __builtin_amdgcn_exp2f(snk - mm);
-    }
-    const float inv = f * head_factor<bf16_t>(a, row[n], h) / den;
+    finish_column<kMaps, VD>(a, o + n * kMaps, m + n * kMaps, l + n * kMaps, row[n], live[n] ? h : kvh * group + h0, g);
+    if (!live[n]) continue;
     bf16_t* dst = out + (size_t)row[n] * a.out_ld + a.out_col + (size_t)h * kv.vdim;
 #pragma unroll
     for (int i = 0; i < VD; ++i) {
       const int c = i * 16 + g * 4;
       if (c >= kv.vdim) continue;
+      const float4_t v = o[n * kMaps][i];
       if (vec) {
-        Act<bf16_t>::store4(dst + c, o[n][i] * inv);
+        Act<bf16_t>::store4(dst + c, v);
       } else {
 #pragma unroll
         for (int r = 0; r < 4; ++r)
-          if (c + r < kv.vdim) Act<bf16_t>::store(dst + c + r, o[n][i][r] * inv);
+          if (c + r < kv.vdim) Act<bf16_t>::store(dst + c + r, v[r]);
       }
     }
   }
 }
 
-template <int KD, int VD>
+template <int KD, int VD, int kMaps = 1>
 static int launch_tile(const nf_window_attention_args& a, hipStream_t s) {
-  constexpr int NB = 2;
+  constexpr int NB = 2 / kMaps;
   const int group = a.kv.heads / a.kv.kv_heads;
   const int chunks = (group + 15) / 16, gs = (group + chunks - 1) / chunks;
   const int tile_tokens = 4 * NB * (16 / gs);
-  const size_t lds = (size_t)kTileRing * TileShape<KD, VD>::slot;
-  auto kern = attn_tile_kernel<KD, VD, NB>;
+  const size_t lds = (size_t)kTileRing * TileShape<KD, VD, kMaps>::slot;
+  auto kern = attn_tile_kernel<KD, VD, NB, kMaps>;
   static bool attr_set = false;  // benign race: the call is idempotent
   if (!attr_set) {
     const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
@@ -824,23 +980,23 @@ static int launch_tile(const nf_window_attention_args& a, hipStream_t s) {
   return check_launch("nf_window_attention (tiles)");
 }
 
-template <int KD, int VD>
+template <int KD, int VD, int kMaps = 1>
 static int launch_window(const nf_window_attention_args& a, hipStream_t s) {
   const int group = a.kv.heads / a.kv.kv_heads;
   // a kv head's query heads in chunks of at most 16, as equal as possible
   const int chunks = (group + 15) / 16, gs = (group + chunks - 1) / chunks;
   const unsigned gy = (unsigned)(a.kv.kv_heads * chunks);
   if (a.decode) {
-    auto lds_of = [&](int w) { return (size_t)w * (32 + (size_t)gs * a.kv.v_pad) * sizeof(float); };
-    int waves = (long long)a.req_num * gy >= 512 ? 4 : 8;
+    auto lds_of = [&](int w) { return (size_t)w * kMaps * (32 + (size_t)gs * a.kv.v_pad) * sizeof(float); };
+    int waves = (long long)a.req_num * gy >= 512 || window_threads(kMaps, VD) < 512 ? 4 : 8;
     while (waves > 1 && lds_of(waves) > 64 * 1024) waves /= 2;
-    attn_window_kernel<KD, VD, 1, true><<<dim3((unsigned)a.req_num, gy), waves * 64, lds_of(waves), s>>>(a, gs, chunks, 0);
+    attn_window_kernel<KD, VD, 1, kMaps, true><<<dim3((unsigned)a.req_num, gy), waves * 64, lds_of(waves), s>>>(a, gs, chunks, 0);
     return check_launch("nf_window_attention (decode)");
   }
-  constexpr int NB = KD <= 4 ? 2 : 1;
+  constexpr int NB = KD <= 4 && kMaps == 1 ? 2 : 1;
   const int tile_tokens = 4 * NB * (16 / gs);
   const unsigned tiles = (unsigned)(a.max_rows / tile_tokens + a.req_num);
-  attn_window_kernel<KD, VD, NB, false><<<dim3(tiles, gy), 256, 0, s>>>(a, gs, chunks, tile_tokens);
+  attn_window_kernel<KD, VD, NB, kMaps, false><<<dim3(tiles, gy), 256, 0, s>>>(a, gs, chunks, tile_tokens);
   return check_launch("nf_window_attention (prefill)");
 }
 
@@ -852,6 +1008,7 @@ static int check_layout(const char* who, const nf_kv_layout& kv) {
   NF_REQUIRE(kv.dtype == NF_F32 || kv.dtype == NF_BF16, "%s: unknown dtype %d", who, kv.dtype);
   NF_REQUIRE(kv.heads > 0 && kv.kv_heads > 0 && kv.heads % kv.kv_heads == 0, "%s: %d query heads over %d kv heads", who,
              kv.heads, kv.kv_heads);
+  NF_REQUIRE(kv.maps == 1 || kv.maps == 2, "%s: %d maps per head", who, kv.maps);
   NF_REQUIRE(kv.page == kPage && kv.dim > 0 && kv.vdim > 0 && kv.dim <= kMaxHeadDim && kv.vdim <= kMaxHeadDim &&
                  kv.k_pad == (kv.dim + 31) / 32 * 32 && kv.v_pad == (kv.vdim + 15) / 16 * 16,
              "%s: page %d, dim %d (pad %d), vdim %d (pad %d): pages of 16, head sizes up to %d", who, kv.page, kv.dim,
@@ -864,8 +1021,8 @@ extern "C" {
 size_t nf_kv_page_elements(const nf_kv_layout* kv) { return kv ? kv_page_elements(*kv) : 0; }
 
 int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, int k_col, int v_col, const float* q_norm,
-                  const float* k_norm, float eps, const nf_rotation* rot, const nf_query_temperature* q_temp, void* q_out, void* kv_data,
-                  const int32_t* kv_indptr, const int32_t* kv_indices, const int32_t* rev_input_indptr,
+                  const float* k_norm, float eps, const nf_rotation* rot, const nf_query_temperature* q_temp, const nf_short_conv* conv, void* q_out,
+                  void* kv_data, const int32_t* kv_indptr, const int32_t* kv_indices, const int32_t* rev_input_indptr,
                   const int32_t* positions, int rows, nf_stream_t stream) {
   const char* who = "nf_qkv_append";
   NF_REQUIRE(kv && rot, "%s: null pointer", who);
@@ -873,37 +1030,56 @@ int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, i
   if (rc) return rc;
   NF_REQUIRE(rot->dims >= 0 && rot->dims % 2 == 0 && rot->dims <= kv->dim && (rot->dims == 0 || rot->table),
              "%s: %d of %d dimensions rotated", who, rot->dims, kv->dim);
-  NF_REQUIRE(rows >= 0 && q_col >= 0 && k_col >= 0 && v_col >= 0 && q_col + kv->heads * kv->dim <= ld &&
-                 k_col + kv->kv_heads * kv->dim <= ld && v_col + kv->kv_heads * kv->vdim <= ld,
+  NF_REQUIRE(rows >= 0 && q_col >= 0 && k_col >= 0 && v_col >= 0 && q_col + kv->heads * kv->maps * kv->dim <= ld &&
+                 k_col + kv->kv_heads * kv->maps * kv->dim <= ld && v_col + kv->kv_heads * kv->vdim <= ld,
              "%s: columns %d %d %d do not fit rows of %d", who, q_col, k_col, v_col, ld);
   NF_REQUIRE(!q_temp || q_temp->every > 0, "%s: a query temperature with blocks of %d positions", who, q_temp ? q_temp->every : 0);
+  const nf_short_conv cv = conv ? *conv : nf_short_conv{};
+  NF_REQUIRE(!conv || (cv.taps >= 1 && cv.taps <= 64 && cv.weight && cv.input_indptr && (cv.taps == 1 || (cv.state && cv.state_slots))),
+             "%s: a convolution of %d taps (1..64) needs weights, a state and slots", who, cv.taps);
   const nf_query_temperature temp = q_temp ? *q_temp : nf_query_temperature{0.f, 0};
   if (rows == 0) return NF_OK;
   NF_REQUIRE(proj && q_out && kv_data && kv_indptr && kv_indices && rev_input_indptr && positions, "%s: null pointer", who);
   hipStream_t s = (hipStream_t)stream;
   const size_t four = 4 * (kv->dtype == NF_BF16 ? 2 : 4);
-  if ((kv->dim | kv->vdim | ld | q_col | k_col | v_col) % 4 == 0 && (uintptr_t)proj % four == 0 &&
-      rot->dims % (rot->interleaved ? 4 : 8) == 0 && (long long)rows * (kv->heads + kv->kv_heads) < (1ll << 31)) {
-    const int qk_blocks = (rows * (kv->heads + kv->kv_heads) + 15) / 16, blocks = qk_blocks + (rows + 15) / 16 * kv->kv_heads;
+  const long long qk_jobs = (long long)rows * (kv->heads + kv->kv_heads) * kv->maps;
+  if ((kv->dim | kv->vdim | ld | q_col | k_col | v_col) % 4 == 0 && ((uintptr_t)proj | (uintptr_t)cv.weight | (uintptr_t)cv.state) % four == 0 &&
+      rot->dims % (rot->interleaved ? 4 : 8) == 0 && qk_jobs < (1ll << 30)) {
+    const int qk_blocks = (int)((qk_jobs + 15) / 16), blocks = qk_blocks + (rows + 15) / 16 * kv->kv_heads;
     if (kv->dtype == NF_BF16)
       qkv_append4_kernel<bf16_t><<<blocks, 256, 0, s>>>(*kv, (const bf16_t*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps,
-                                                        *rot, temp, (bf16_t*)q_out, (bf16_t*)kv_data, kv_indptr, kv_indices,
+                                                        *rot, temp, cv, (bf16_t*)q_out, (bf16_t*)kv_data, kv_indptr, kv_indices,
                                                         rev_input_indptr, positions, rows, qk_blocks);
     else
       qkv_append4_kernel<float><<<blocks, 256, 0, s>>>(*kv, (const float*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps,
-                                                       *rot, temp, (float*)q_out, (float*)kv_data, kv_indptr, kv_indices,
+                                                       *rot, temp, cv, (float*)q_out, (float*)kv_data, kv_indptr, kv_indices,
                                                        rev_input_indptr, positions, rows, qk_blocks);
     return check_launch(who);
   }
-  const dim3 grid((unsigned)rows, (unsigned)((kv->heads + 2 * kv->kv_heads + 3) / 4));
+  const dim3 grid((unsigned)rows, (unsigned)(((kv->heads + kv->kv_heads) * kv->maps + kv->kv_heads + 3) / 4));
   if (kv->dtype == NF_BF16)
-    qkv_append_kernel<bf16_t><<<grid, 256, 0, s>>>(*kv, (const bf16_t*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot, temp,
+    qkv_append_kernel<bf16_t><<<grid, 256, 0, s>>>(*kv, (const bf16_t*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot, temp, cv,
                                                    (bf16_t*)q_out, (bf16_t*)kv_data, kv_indptr, kv_indices, rev_input_indptr,
                                                    positions);
   else
-    qkv_append_kernel<float><<<grid, 256, 0, s>>>(*kv, (const float*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot, temp,
+    qkv_append_kernel<float><<<grid, 256, 0, s>>>(*kv, (const float*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot, temp, cv,
                                                   (float*)q_out, (float*)kv_data, kv_indptr, kv_indices, rev_input_indptr,
                                                   positions);
+  return check_launch(who);
+}
+
+int nf_conv_state(int dtype, const void* proj, int ld, const nf_short_conv* conv, const int32_t* positions, int req_begin, int req_num,
+                  nf_stream_t stream) {
+  const char* who = "nf_conv_state";
+  NF_REQUIRE(dtype == NF_F32 || dtype == NF_BF16, "%s: unknown dtype %d", who, dtype);
+  NF_REQUIRE(conv && conv->taps >= 1 && conv->taps <= 64 && ld > 0 && ld % 8 == 0 && req_begin >= 0 && req_num >= 0, "%s: taps or rows", who);
+  if (req_num == 0 || conv->taps == 1) return NF_OK;
+  NF_REQUIRE(proj && positions && conv->state && conv->input_indptr && conv->state_slots, "%s: null pointer", who);
+  NF_REQUIRE(((uintptr_t)proj | (uintptr_t)conv->state) % 16 == 0, "%s: operands must be 16-byte aligned", who);
+  const int per = 256 * (dtype == NF_BF16 ? 8 : 4);
+  const dim3 grid((unsigned)req_num, (unsigned)((ld + per - 1) / per));
+  if (dtype == NF_BF16) conv_state_kernel<bf16_t><<<grid, 256, 0, (hipStream_t)stream>>>((const bf16_t*)proj, ld, *conv, positions, req_begin);
+  else conv_state_kernel<float><<<grid, 256, 0, (hipStream_t)stream>>>((const float*)proj, ld, *conv, positions, req_begin);
   return check_launch(who);
 }
 
@@ -919,6 +1095,8 @@ int nf_window_attention(const nf_window_attention_args* args, nf_stream_t stream
   NF_REQUIRE(a.out_col >= 0 && a.out_col + a.kv.heads * a.kv.vdim <= a.out_ld, "%s: output columns %d + %d of %d", who,
              a.out_col, a.kv.heads * a.kv.vdim, a.out_ld);
   NF_REQUIRE(!a.gate || a.gate_ld >= a.kv.heads, "%s: gate rows of %d for %d heads", who, a.gate_ld, a.kv.heads);
+  NF_REQUIRE(a.kv.maps == 1 || !a.sink, "%s: a sink with two maps", who);
+  NF_REQUIRE(a.softcap >= 0.f && (!a.head_norm || a.head_eps >= 0.f), "%s: cap %g, eps %g", who, a.softcap, a.head_eps);
   NF_REQUIRE(!a.decode || a.max_rows == a.req_num, "%s: %d decode requests with %d rows", who, a.req_num, a.max_rows);
   if (a.req_num == 0 || a.max_rows == 0) return NF_OK;
   NF_REQUIRE(a.q && a.out && a.kv_data && a.input_indptr && a.kv_indptr && a.kv_indices && a.rev_input_indptr && a.positions,
@@ -929,12 +1107,22 @@ int nf_window_attention(const nf_window_attention_args* args, nf_stream_t stream
     attn_rows_kernel<float><<<dim3((unsigned)a.max_rows, (unsigned)a.kv.heads), 64, 0, s>>>(a);
     return check_launch(who);
   }
-  if (!(a.scale > 0.f)) {  // the matrix kernel takes the maximum before it scales
+  const int kd = a.kv.k_pad / 32, vd = a.kv.v_pad / 16;
+  // the matrix kernel takes the maximum before it scales; keys of two maps beyond 128 columns do not fit its registers
+  if (!(a.scale > 0.f) || (a.kv.maps == 2 && kd > 4)) {
     attn_rows_kernel<bf16_t><<<dim3((unsigned)a.max_rows, (unsigned)a.kv.heads), 64, 0, s>>>(a);
     return check_launch(who);
   }
-  const int kd = a.kv.k_pad / 32, vd = a.kv.v_pad / 16;
-  if (!a.decode && (long long)a.max_rows + a.req_num <= 65535) {
+  const bool tiles = !a.decode && (long long)a.max_rows + a.req_num <= 65535;
+  if (a.kv.maps == 2) {
+    if (tiles && kd == 2 && vd == 4) return launch_tile<2, 4, 2>(a, s);
+    if (tiles && kd == 2 && vd == 8) return launch_tile<2, 8, 2>(a, s);
+    if (tiles && kd == 4 && vd == 8) return launch_tile<4, 8, 2>(a, s);
+    if (tiles && kd == 4 && vd == 16) return launch_tile<4, 16, 2>(a, s);
+    if (kd <= 2 && vd <= 8) return launch_window<2, 8, 2>(a, s);
+    return launch_window<4, 16, 2>(a, s);
+  }
+  if (tiles) {
     if (kd == 2 && vd == 4) return launch_tile<2, 4>(a, s);
     if (kd == 4 && vd == 8) return launch_tile<4, 8>(a, s);
     if (kd == 6 && vd == 8) return launch_tile<6, 8>(a, s);

@@ -172,6 +172,9 @@ __global__ __launch_bounds__(256) void latent_queries_kernel(nf_kv_layout kv, in
   }
 }
 
+// The first position that one at p sees.
+__device__ __forceinline__ int first_seen(int p, int window) { return window > 0 && p >= window ? p - window + 1 : 0; }
+
 // ---------------------------------------------------------------- fp32, any size
 template <class T, int NE>  // NE x 64 latent columns at most
 __global__ __launch_bounds__(64) void latent_rows_kernel(nf_latent_attention_args a) {
@@ -186,10 +189,11 @@ __global__ __launch_bounds__(64) void latent_rows_kernel(nf_latent_attention_arg
   const int32_t* pages = a.kv_indices + a.kv_indptr[req];
   auto row_of = [&](int j) { return (const T*)a.kv_data + ((size_t)pages[j / kLatentPage] * kLatentPage + j % kLatentPage) * lay.row_ld; };
   float m = -1e30f, l = 0.f, o[NE] = {};
-  for (int base = 0; base <= p; base += 64) {
+  for (int base = first_seen(p, a.window) / 64 * 64; base <= p; base += 64) {
     const int j = base + lane;
+    const bool see = j <= p && j >= first_seen(p, a.window);
     float s = -INFINITY;
-    if (j <= p) {
+    if (see) {
       const T* k = row_of(j);
       float dot = 0.f;
       for (int c = 0; c < lay.row_ld; c += 4) {
@@ -201,7 +205,7 @@ __global__ __launch_bounds__(64) void latent_rows_kernel(nf_latent_attention_arg
     float mx = s;
 #pragma unroll
     for (int d = 32; d > 0; d >>= 1) mx = fmaxf(mx, __shfl_xor(mx, d, 64));
-    const float m_new = fmaxf(m, mx), alpha = expf(m - m_new), w = j <= p ? expf(s - m_new) : 0.f;
+    const float m_new = fmaxf(m, mx), alpha = expf(m - m_new), w = see ? expf(s - m_new) : 0.f;
     m = m_new;
     l = l * alpha + w;
     __syncthreads();
@@ -282,8 +286,9 @@ __global__ __launch_bounds__(CBS * 128) void latent_mfma_kernel(nf_latent_attent
   const int p_low = pos0 + col0 / H, p_high = pos0 + min(col0 + columns - 1, total - 1) / H;
 
   const int kd = kExact ? KD : lay.row_ld / 32, vd = kExact ? VD : (lay.rank_pad + 15) / 16, planes = kExact ? KD / 2 : lay.row_ld / 64;
-  const int n_tiles = p_high / kTileKeys + 1, per = (n_tiles + p.splits - 1) / p.splits;
-  const int t0 = blockIdx.y * per, t1 = min(n_tiles, t0 + per);
+  const int first_tile = first_seen(p_low, a.window) / kTileKeys;  // tiles before it are out of every column's window
+  const int end_tile = p_high / kTileKeys + 1, per = (end_tile - first_tile + p.splits - 1) / p.splits;
+  const int t0 = first_tile + blockIdx.y * per, t1 = min(end_tile, t0 + per);
   const int32_t* pages = a.kv_indices + a.kv_indptr[req];
   const int last_page = p_high / kLatentPage;
   const size_t page_bytes = (size_t)kLatentPage * lay.row_ld * 2;
@@ -419,6 +424,10 @@ __global__ __launch_bounds__(CBS * 128) void latent_mfma_kernel(nf_latent_attent
 #pragma unroll
       for (int r = 0; r < 4; ++r)
         if (base + r > pos) s[r] = -INFINITY;
+    if (a.window > 0 && t * kTileKeys <= p_high - a.window)
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (base + r <= pos - a.window) s[r] = -INFINITY;
     float mx = fmaxf(fmaxf(s[0], s[1]), fmaxf(s[2], s[3]));
     mx = max_over_lane_groups(mx > -1e30f ? mx * scale2 : -1e30f);
     if (g == 0) sh.mx[kt][cb][l16] = mx;
@@ -603,7 +612,7 @@ static int check_expand(const char* who, const nf_latent_expand_args* a) {
   const int rc = check_latent(who, a->layout);
   if (rc) return rc;
   const nf_kv_layout& kv = a->kv;
-  NF_REQUIRE(kv.dtype == a->layout.dtype && kv.heads == a->layout.heads && kv.kv_heads == kv.heads && kv.page == kLatentPage && a->dim_pad > 0 &&
+  NF_REQUIRE(kv.dtype == a->layout.dtype && kv.maps == 1 && kv.heads == a->layout.heads && kv.kv_heads == kv.heads && kv.page == kLatentPage && a->dim_pad > 0 &&
                  a->dim_pad % 8 == 0 && kv.dim == a->dim_pad + a->layout.rot_dim && kv.dim <= 256 && kv.vdim > 0 && kv.vdim % 8 == 0 &&
                  kv.vdim <= 256 && kv.k_pad == (kv.dim + 31) / 32 * 32 && kv.v_pad == (kv.vdim + 15) / 16 * 16,
              "%s: %d heads of %d + %d and %d", who, kv.heads, a->dim_pad, a->layout.rot_dim, kv.vdim);

@@ -117,7 +117,7 @@ __global__ __launch_bounds__(kRowThreads) void residual_rows_kernel(nf_residual_
 #pragma unroll
   for (int i = 0; i < kVec; ++i) {
     const int c = (i * kRowThreads + threadIdx.x) * 4;
-    v[i] += xr[i];
+    v[i] = v[i] * a.y_scale + xr[i];
     if (c < ld) *reinterpret_cast<float4_t*>(a.x + row + c) = v[i];
   }
   if (!a.act) return;

@@ -30,7 +30,7 @@ SYMBOLS = [
     "nf_gemm_tile_menu", "nf_gemm_tiled_workspace_bytes", "nf_gemm_f16_tiled",
     "nf_rmsnorm_quantize_e4m3", "nf_gemm_f8q_f16", "nf_dual_swiglu_f8q_f16",
     "nf_gemm_nk_workspace_bytes_upto", "nf_gemm_nk_bf16", "nf_gemm_nk_relu2_bf16", "nf_gemm_nk_silu_bf16", "nf_gemm_nk_bias_bf16",
-    "nf_gemm_nk_f32", "nf_gemm_nk_sums_shares", "nf_gemm_nk_sums_bytes_upto", "nf_gemm_nk_sums_bf16", "nf_routing_max_tiles", "nf_route",
+    "nf_gemm_nk_f32", "nf_gemm_nk_sums_shares", "nf_gemm_nk_sums_bytes_upto", "nf_gemm_nk_sums_bf16", "nf_routing_max_tiles", "nf_route", "nf_conv_state", "nf_gemm_nk_gelu_bf16",
     "nf_grouped_tile_rows", "nf_gemm_grouped", "nf_norm_rows", "nf_residual_rows", "nf_token_gate_rows", "nf_gated_norm_rows",
     "nf_embed_rows", "nf_token_shift", "nf_tanh_rows", "nf_argmax_f32", "nf_kv_page_elements", "nf_qkv_append",
     "nf_window_attention", "nf_latent_layout_of", "nf_latent_append", "nf_latent_gather", "nf_latent_pack", "nf_latent_queries", "nf_latent_workspace_bytes", "nf_latent_attention",
@@ -44,12 +44,13 @@ class Rotation(C.Structure):
 
 
 class KVLayout(C.Structure):
-    _fields_ = [(n, C.c_int) for n in ("dtype", "heads", "kv_heads", "dim", "vdim", "k_pad", "v_pad", "page")]
+    _fields_ = [(n, C.c_int) for n in ("dtype", "heads", "kv_heads", "dim", "vdim", "k_pad", "v_pad", "page", "maps")]
 
 
 class WindowAttentionArgs(C.Structure):
     _fields_ = [("kv", KVLayout), ("window", C.c_int), ("keep_first", C.c_int), ("scale", C.c_float),
-                ("out_scale", C.c_float), ("sink", C.c_void_p), ("gate", C.c_void_p), ("gate_ld", C.c_int), ("q", C.c_void_p),
+                ("out_scale", C.c_float), ("softcap", C.c_float), ("map_weight", C.c_float), ("head_eps", C.c_float),
+                ("head_norm", C.c_int), ("sink", C.c_void_p), ("gate", C.c_void_p), ("gate_ld", C.c_int), ("q", C.c_void_p),
                 ("out", C.c_void_p), ("out_ld", C.c_int), ("out_col", C.c_int), ("kv_data", C.c_void_p)] + \
         [(n, C.c_void_p) for n in ("input_indptr", "kv_indptr", "kv_indices", "rev_input_indptr", "positions")] + \
         [(n, C.c_int) for n in ("req_begin", "req_num", "row_begin", "max_rows", "decode")]
@@ -57,6 +58,10 @@ class WindowAttentionArgs(C.Structure):
 
 class QueryTemperature(C.Structure):
     _fields_ = [("coef", C.c_float), ("every", C.c_int)]
+
+
+class ShortConv(C.Structure):
+    _fields_ = [("taps", C.c_int)] + [(n, C.c_void_p) for n in ("weight", "state", "input_indptr", "state_slots")]
 
 
 class LatentLayout(C.Structure):
@@ -70,7 +75,7 @@ class LatentExpandArgs(C.Structure):
 
 
 class LatentAttentionArgs(C.Structure):
-    _fields_ = [("layout", LatentLayout), ("scale", C.c_float), ("q", C.c_void_p), ("out", C.c_void_p), ("kv_data", C.c_void_p)] + \
+    _fields_ = [("layout", LatentLayout), ("window", C.c_int), ("scale", C.c_float), ("q", C.c_void_p), ("out", C.c_void_p), ("kv_data", C.c_void_p)] + \
         [(n, C.c_void_p) for n in ("input_indptr", "kv_indptr", "kv_indices", "rev_input_indptr", "positions")] + \
         [(n, C.c_int) for n in ("req_begin", "req_num", "row_begin", "max_rows", "decode")] + \
         [("workspace", C.c_void_p), ("workspace_bytes", C.c_size_t)]
@@ -85,6 +90,12 @@ class Routing(C.Structure):
         [("tile_rows", C.c_int)]
 
 
+class RouteArgs(C.Structure):
+    _fields_ = [("z", C.c_void_p)] + \
+        [(n, C.c_int) for n in ("shares", "ld", "rows", "outputs", "experts", "top", "always", "groups", "keep_groups")] + \
+        [("correction", C.c_void_p), ("scale", C.c_float)]
+
+
 class GroupedGemmArgs(C.Structure):
     _fields_ = [(n, C.c_int) for n in ("dtype", "act", "groups", "M", "N", "K")] + \
         [("a", C.c_void_p), ("lda", C.c_int), ("a_group", C.c_size_t), ("b", C.c_void_p), ("d", C.c_void_p), ("ldd", C.c_int),
@@ -94,7 +105,7 @@ class GroupedGemmArgs(C.Structure):
 class ResidualArgs(C.Structure):
     _fields_ = [(n, C.c_int) for n in ("rows", "width", "ld", "y_dtype", "shares")] + \
         [("y", C.c_void_p), ("routing", C.POINTER(Routing)), ("top", C.c_int), ("y_ld", C.c_int), ("identity", C.c_void_p),
-         ("y_norm", Norm), ("next", Norm), ("x", C.c_void_p), ("dtype", C.c_int), ("act", C.c_void_p)]
+         ("y_norm", Norm), ("next", Norm), ("y_scale", C.c_float), ("x", C.c_void_p), ("dtype", C.c_int), ("act", C.c_void_p)]
 
 
 class RecurrenceArgs(C.Structure):
@@ -190,7 +201,8 @@ def lib() -> C.CDLL:
         l.nf_gemm_nk_bias_bf16.argtypes = [vp, vp, vp, vp, i32, i32, i32, vp, sz, vp]
         l.nf_gemm_nk_f32.argtypes = [vp, vp, vp, vp, i32, i32, i32, i32, vp]
         l.nf_routing_max_tiles.argtypes = l.nf_grouped_tile_rows.argtypes = [i32] * 3
-        l.nf_route.argtypes = [vp] + [i32] * 6 + [vp, f32, vp, vp]
+        l.nf_route.argtypes = [vp, vp, vp]
+        l.nf_conv_state.argtypes = [i32, vp, i32, vp, vp, i32, i32, vp]
         l.nf_gemm_grouped.argtypes = l.nf_residual_rows.argtypes = l.nf_latent_attention.argtypes = [vp, vp]
         l.nf_norm_rows.argtypes = [i32, vp, vp, vp, vp, i32, i32, i32, vp]
         l.nf_token_gate_rows.argtypes = [i32, vp, i32, vp, vp, i32, i32, i32, vp, i32, i32, vp]
@@ -205,7 +217,7 @@ def lib() -> C.CDLL:
         l.nf_token_shift.argtypes = [i32, vp, vp, vp, vp, i32, vp, vp, vp, vp, i32, i32, vp]
         l.nf_tanh_rows.argtypes = [i32, vp, i32, vp, i32, i32, vp]
         l.nf_argmax_f32.argtypes = [vp, vp, i32, i32, i32, vp]
-        l.nf_qkv_append.argtypes = [C.POINTER(KVLayout), vp, i32, i32, i32, i32, vp, vp, f32, C.POINTER(Rotation), vp, vp, vp, vp,
+        l.nf_qkv_append.argtypes = [C.POINTER(KVLayout), vp, i32, i32, i32, i32, vp, vp, f32, C.POINTER(Rotation), vp, vp, vp, vp, vp,
                                     vp, vp, vp, i32, vp]
         l.nf_window_attention.argtypes = [C.POINTER(WindowAttentionArgs), vp]
         l.nf_linear_recurrence.argtypes = [C.POINTER(RecurrenceArgs), vp]
@@ -674,7 +686,7 @@ NORM_NONE, NORM_RMS, NORM_LAYER = 0, 1, 2
 
 
 def gemm_nk(a, b, squared_relu=False, workspace=None, act=None, bias=None):
-    """act(a . b^T + bias), b [N, K], in the type of a (bf16: an activation or a bias, not both; no GELU)."""
+    """act(a . b^T + bias), b [N, K], in the type of a (bf16: an activation or a bias, not both)."""
     act = act or (ACT_SQUARED_RELU if squared_relu else ACT_NONE)
     M, K = a.shape
     N = b.shape[0]
@@ -687,7 +699,8 @@ def gemm_nk(a, b, squared_relu=False, workspace=None, act=None, bias=None):
         if bias is not None:
             _call("nf_gemm_nk_bias_bf16", _p(a), _p(b), _p(bias), *tail)
         else:
-            name = {ACT_NONE: "nf_gemm_nk_bf16", ACT_SQUARED_RELU: "nf_gemm_nk_relu2_bf16", ACT_SILU: "nf_gemm_nk_silu_bf16"}[act]
+            name = {ACT_NONE: "nf_gemm_nk_bf16", ACT_SQUARED_RELU: "nf_gemm_nk_relu2_bf16", ACT_SILU: "nf_gemm_nk_silu_bf16",
+                    ACT_GELU: "nf_gemm_nk_gelu_bf16"}[act]
             _call(name, _p(a), _p(b), *tail)
     return d
 
@@ -717,20 +730,20 @@ def norm(kind, weight=None, bias=None, eps=0.0) -> Norm:
     return n
 
 
-def residual_rows(y, x, act, width, y_norm=None, next_norm=None):
-    """x += y_norm(y) in place; y [shares, T, ld] fp32 or [T, ld] bf16; act (or None) receives next_norm(x) in its type."""
+def residual_rows(y, x, act, width, y_norm=None, next_norm=None, y_scale=1.0):
+    """x += y_scale * y_norm(y) in place; y [shares, T, ld] fp32 or [T, ld] bf16; act (or None) receives next_norm(x) in its type."""
     shares = y.shape[0] if y.dim() == 3 else 1
     T, ld = x.shape
     a = ResidualArgs(rows=T, width=width, ld=ld, y_dtype=_dt(y), shares=shares, y=_p(y), y_norm=y_norm or Norm(), next=next_norm or Norm(),
-                     x=_p(x), dtype=_dt(act) if act is not None else F32, act=_p(act))
+                     y_scale=y_scale, x=_p(x), dtype=_dt(act) if act is not None else F32, act=_p(act))
     _call("nf_residual_rows", C.byref(a), _stream())
 
 
-def mixture_rows(y, routing, top, identity, x, act, width, next_norm=None):
-    """x += the weighted sum of every token's sorted rows of y [sorted, ld] and of identity [T, ld]."""
+def mixture_rows(y, routing, top, identity, x, act, width, next_norm=None, y_scale=1.0):
+    """x += y_scale * the weighted sum of every token's sorted rows of y [sorted, ld] and of identity [T, ld]."""
     T, ld = x.shape
     a = ResidualArgs(rows=T, width=width, ld=ld, y=_p(y), routing=C.pointer(routing), top=top, y_ld=y.shape[1], identity=_p(identity),
-                     next=next_norm or Norm(), x=_p(x), dtype=_dt(identity), act=_p(act))
+                     next=next_norm or Norm(), y_scale=y_scale, x=_p(x), dtype=_dt(identity), act=_p(act))
     _call("nf_residual_rows", C.byref(a), _stream())
 
 
@@ -761,16 +774,19 @@ def token_gate_rows(sums, tokens, table, col0, dim):
     return out
 
 
-def route(z, outputs, experts, top, correction, scale, tile_rows):
-    """(Routing, dict of its tensors) of router outputs z [shares, T, ld] fp32."""
+def route(z, outputs, experts, top, correction, scale, tile_rows, groups=1, keep_groups=1, always=0):
+    """(Routing, dict of its tensors) of router outputs z [shares, T, ld] fp32; always: experts of every token behind the chosen
+    ones, weighed by the column after the outputs."""
     shares, T, ld = z.shape
-    n = T * top
+    n, e = T * (top + always), experts + always
     i32 = lambda k: torch.full((k,), -7, dtype=torch.int32, device=z.device)
     t = {"choice": i32(n), "weight": torch.empty(n, dtype=torch.float32, device=z.device), "place": i32(n), "row_of": i32(n),
-         "offsets": i32(experts + 1), "tile_group": i32(lib().nf_routing_max_tiles(n, experts, tile_rows)), "n_tiles": i32(1)}
+         "offsets": i32(e + 1), "tile_group": i32(lib().nf_routing_max_tiles(n, e, tile_rows)), "n_tiles": i32(1)}
     t["tile_row"] = torch.empty_like(t["tile_group"])
     r = Routing(**{k: _p(v) for k, v in t.items()}, tile_rows=tile_rows)
-    _call("nf_route", _p(z), shares, ld, T, outputs, experts, top, _p(correction), scale, C.byref(r), _stream())
+    a = RouteArgs(z=_p(z), shares=shares, ld=ld, rows=T, outputs=outputs, experts=experts, top=top, always=always, groups=groups,
+                  keep_groups=keep_groups, correction=_p(correction), scale=scale)
+    _call("nf_route", C.byref(a), C.byref(r), _stream())
     return r, t
 
 
@@ -812,9 +828,9 @@ def argmax_f32(logits, cols=None):
     return out
 
 
-def kv_layout(dtype, heads, kv_heads, dim, vdim) -> KVLayout:
+def kv_layout(dtype, heads, kv_heads, dim, vdim, maps=1) -> KVLayout:
     return KVLayout(BF16 if dtype == torch.bfloat16 else F32, heads, kv_heads, dim, vdim, (dim + 31) // 32 * 32,
-                    (vdim + 15) // 16 * 16, 16)
+                    (vdim + 15) // 16 * 16, 16, maps)
 
 
 def kv_pool(layout: KVLayout, pages, device="cuda"):
@@ -827,22 +843,35 @@ def rotation(table=None, dims=0, interleaved=False) -> Rotation:
     return Rotation(_p(table) if table is not None else None, dims, int(interleaved))
 
 
-def qkv_append(layout, proj, cols, q_norm, k_norm, eps, rot, pool, kv_indptr, kv_indices, rev_input_indptr, positions, q_temp=None):
-    """Returns the normed, rotated queries [T, heads, k_pad]; keys and values go to the pool's pages."""
+def short_conv(weight, state, input_indptr, state_slots) -> ShortConv:
+    """weight [taps, columns], state [slots, taps - 1, columns] in the type of the projected rows."""
+    c = ShortConv(weight.shape[0], _p(weight), _p(state), _p(input_indptr), _p(state_slots))
+    c.tensors = (weight, state, input_indptr, state_slots)      # the struct holds addresses only
+    return c
+
+
+def qkv_append(layout, proj, cols, q_norm, k_norm, eps, rot, pool, kv_indptr, kv_indices, rev_input_indptr, positions, q_temp=None, conv=None):
+    """Returns the normed, rotated queries [T, heads * maps, k_pad]; keys and values go to the pool's pages, what a convolution
+    needs of these rows to its state."""
     T = proj.shape[0]
-    q = torch.empty((T, layout.heads, layout.k_pad), dtype=proj.dtype, device=proj.device)
+    q = torch.empty((T, layout.heads * layout.maps, layout.k_pad), dtype=proj.dtype, device=proj.device)
     _call("nf_qkv_append", C.byref(layout), _p(proj), proj.shape[1], *cols, _p(q_norm), _p(k_norm), eps, C.byref(rot),
-          C.byref(QueryTemperature(*q_temp)) if q_temp else None, _p(q), _p(pool), _p(kv_indptr), _p(kv_indices), _p(rev_input_indptr), _p(positions), T, _stream())
+          C.byref(QueryTemperature(*q_temp)) if q_temp else None, C.byref(conv) if conv else None, _p(q), _p(pool), _p(kv_indptr),
+          _p(kv_indices), _p(rev_input_indptr), _p(positions), T, _stream())
+    if conv:
+        _call("nf_conv_state", _dt(proj), _p(proj), proj.shape[1], C.byref(conv), _p(positions), 0, kv_indptr.numel() - 1, _stream())
     return q
 
 
-def window_attention(layout, q, pool, batch, *, window, keep_first, scale, sink=None, out_scale=1.0, decode=0, gate=None):
+def window_attention(layout, q, pool, batch, *, window, keep_first, scale, sink=None, out_scale=1.0, decode=0, gate=None, softcap=0.0,
+                     map_weight=0.0, head_eps=None):
     """batch: dict of device arrays input_indptr, kv_indptr, kv_indices, rev_input_indptr, positions; the first
     `decode` requests have one row each.  Returns [T, heads * vdim]."""
     T = q.shape[0]
     out = torch.zeros((T, layout.heads * layout.vdim), dtype=q.dtype, device=q.device)
     n_req = batch["input_indptr"].numel() - 1
-    a = WindowAttentionArgs(kv=layout, window=window, keep_first=keep_first, scale=scale, out_scale=out_scale, sink=_p(sink),
+    a = WindowAttentionArgs(kv=layout, window=window, keep_first=keep_first, scale=scale, out_scale=out_scale, softcap=softcap,
+                            map_weight=map_weight, head_norm=int(head_eps is not None), head_eps=head_eps or 0.0, sink=_p(sink),
                             gate=_p(gate), gate_ld=gate.shape[1] if gate is not None else 0, q=_p(q), out=_p(out), out_ld=out.shape[1], out_col=0, kv_data=_p(pool))
     for n in ("input_indptr", "kv_indptr", "kv_indices", "rev_input_indptr", "positions"):
         setattr(a, n, _p(batch[n]))
@@ -894,13 +923,13 @@ def latent_queries(kv, dim_pad, proj, q_col, rot_dim, rot, positions, row_begin,
     return q
 
 
-def latent_attention(layout, q, pool, batch, *, scale, decode=0, workspace=True):
+def latent_attention(layout, q, pool, batch, *, scale, decode=0, workspace=True, window=0):
     """q [T, heads, row_ld]; returns [T, heads, rank_pad]."""
     T = q.shape[0]
     out = torch.zeros((T, layout.heads, layout.rank_pad), dtype=q.dtype, device=q.device)
     n_req = batch["input_indptr"].numel() - 1
     ws = torch.empty((max(lib().nf_latent_workspace_bytes(C.byref(layout), T), 16),), dtype=torch.uint8, device=q.device) if workspace else None
-    a = LatentAttentionArgs(layout=layout, scale=scale, q=_p(q), out=_p(out), kv_data=_p(pool), workspace=_p(ws),
+    a = LatentAttentionArgs(layout=layout, window=window, scale=scale, q=_p(q), out=_p(out), kv_data=_p(pool), workspace=_p(ws),
                             workspace_bytes=ws.numel() if workspace else 0)
     for n in ("input_indptr", "kv_indptr", "kv_indices", "rev_input_indptr", "positions"):
         setattr(a, n, _p(batch[n]))

@@ -75,7 +75,41 @@ def _fipuzen_shapes(cfg: dict, rank: int) -> dict:
     return out
 
 
-ARCHITECTURES = {"Zovovik": _zovovik_shapes, "Fipuzen": _fipuzen_shapes}
+def _pudadra_shapes(cfg: dict, rank: int) -> dict:
+    W = cfg["width"]
+    out = {"embed": (cfg["vocab"], W), "final.norm": (W,)}
+    for i, layer in enumerate(cfg["layers"]):
+        l, x, m = f"l{i}.", f"l{i}.mix.", layer["mixer"]
+        out[l + "norm1"] = (W,)
+        if layer["type"] == "attention":
+            for s, n in (("q", 2 * m["heads"] * m["dim"]), ("k", 2 * m["kv_heads"] * m["dim"]), ("v", m["kv_heads"] * m["vdim"])):
+                out[x + s] = (n, W)
+                if m.get("conv"):
+                    out[x + s + ".conv"] = (n, m["conv"])
+            out.update({x + s: (m["dim"],) for s in ("lq1", "lk1", "lq2", "lk2")})
+        else:
+            H, R = m["heads"], m["kv_rank"]
+            out.update({x + "q": (H * (m["dim"] + m["rot_dim"]), W), x + "dkv": (R + m["rot_dim"], W), x + "dkv.norm": (R,),
+                        x + "uk": (H * m["dim"], R), x + "uv": (H * m["vdim"], R)})
+        out[x + "o"] = (W, m["heads"] * m["vdim"])
+        f, p = layer.get("mlp"), l + "mlp."
+        if not f:
+            continue
+        out[l + "norm2"] = (W,)
+        blocks = {"": f["ff"]} if f["kind"] == "dense" else {f"e{e}.": f["expert"]["ff"] for e in range(f["router"]["experts"])}
+        if f["kind"] != "dense":
+            out[p + "router"] = (f["router"]["experts"], W)
+            if f.get("shared"):
+                blocks["shared."] = f["shared"]["ff"]
+                out[p + "shared.sg"] = (1, W)
+        for b, n in blocks.items():
+            out.update({p + b + "up": (n, W), p + b + "down": (W, n)})
+    return out
+
+
+ARCHITECTURES = {"Zovovik": _zovovik_shapes, "Fipuzen": _fipuzen_shapes, "Pudadra": _pudadra_shapes}
+# designs whose norms of the residual stream are stored as the difference from one
+NORMS_AROUND_ZERO = ("Pudadra",)
 
 
 def tensor_shapes(cfg: dict, rank: int = 16) -> dict:
@@ -97,7 +131,7 @@ def bits_to_f32(b) -> np.ndarray:
 
 
 def random_tensors(cfg: dict, seed: int = 0, rank: int = 16) -> dict:
-    """name -> bfloat16 bit patterns: projections N(0, 1 / inputs), norms around 1, small biases, shifts in
+    """name -> bfloat16 bit patterns: projections N(0, 1 / inputs), norms around what stands for 1, small biases, shifts in
     [0, 1], token decays that keep a state for a few to a few thousand tokens."""
     rng = np.random.default_rng(seed)
     out, expert_blocks = {}, {}
@@ -112,7 +146,10 @@ def random_tensors(cfg: dict, seed: int = 0, rank: int = 16) -> dict:
         n = min(int(np.prod(shape)), 1 << 22)
         x = rng.standard_normal(n, dtype=np.float32)
         if "norm" in leaf:
-            x = 1.0 + 0.1 * x
+            around_zero = cfg["architecture"] in NORMS_AROUND_ZERO and ".mix." not in name
+            x = 0.1 * x if around_zero else 1.0 + 0.1 * x
+        elif leaf in ("lq1", "lk1", "lq2", "lk2"):
+            x *= 0.7 * shape[0] ** -0.25
         elif ".mu." in name:
             x = rng.random(n, dtype=np.float32)
         elif leaf == "w0":

@@ -53,6 +53,36 @@ def fipuzen(layers, width=104, vocab=211, side=20, eps=1e-5, mlp=None):
     return {"architecture": "Fipuzen", "width": width, "vocab": vocab, "token_side": {"dim": side}, "norm": {"eps": eps}, "layers": out}
 
 
+SCALING = {"factor": 6.0, "low": 1.0, "high": 3.0, "original": 300}
+
+
+def differential(heads=6, kv_heads=2, dim=24, vdim=40, window=21, rot=16, base=300.0, scaling=SCALING, scale=0.25, softcap=6.0, conv=3, diff=0.4):
+    return {"type": "attention", "mixer": {
+        "heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale, "softcap": softcap, "conv": conv, "diff": diff,
+        "mask": {"size": window}, "rot": {"dims": rot, "base": base, **({"scaling": scaling} if scaling else {})}}}
+
+
+def windowed_latent(window=37, **kw):
+    m = latent(**kw)
+    m["mixer"]["mask"] = {"size": window}
+    return m
+
+
+def dense(ff=88):
+    return {"kind": "dense", "ff": ff}
+
+
+def grouped_moe(experts=8, groups=4, keep=2, top=3, ff=40, shared=56):
+    m = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "groups": {"count": groups, "keep": keep}, "top": top}}
+    return {**m, "shared": {"ff": shared}} if shared else m
+
+
+def pudadra(layers, width=104, vocab=211, eps=1e-5, residual_mult=0.7, logit_scale=0.3):
+    """layers: (mixer, feed-forward or None)"""
+    return {"architecture": "Pudadra", "width": width, "vocab": vocab, "residual_mult": residual_mult, "logit_scale": logit_scale,
+            "norm": {"eps": eps}, "layers": [{**mixer, "mlp": f} for mixer, f in layers]}
+
+
 # sizes that are not multiples of 8, equal and unequal head counts, no feed-forward, a window of one, windows without kept tokens
 CONFIGS = {
     "mixed": config([retention(), parallel(), (retention(heads=1, dim=16, vdim=16, rot=16, decay=(0.9,)), None), parallel(
@@ -71,6 +101,21 @@ CONFIGS = {
                             attention(heads=2, kv_heads=1, dim=160, vdim=144), (latent(heads=40, dim=16, rot=8, vdim=16, kv_rank=520), None)], width=128),
     "one expert": fipuzen([attention(heads=1, kv_heads=1, dim=8, vdim=8), (lightning(heads=1, dim=16, vdim=16, decay=(0.8,)), moe(1, 0, 1, 8, 1.0)),
                            (latent(heads=1, dim=8, rot=2, vdim=8, kv_rank=8), moe(1, 6, 2, 24))], width=40, side=8),
+    "two maps": pudadra([(differential(), dense()), (windowed_latent(), grouped_moe()), (differential(heads=4, kv_heads=4, dim=32, vdim=16, window=70, rot=32,
+                                                                                                     conv=4), None),
+                         (windowed_latent(heads=2, dim=16, rot=16, vdim=32, kv_rank=64, window=20), dense(70)),
+                         (differential(heads=2, kv_heads=1, dim=16, vdim=48, scaling=None, softcap=None, conv=2), grouped_moe(6, 1, 1, 2, 24, None))]),
+    "odd maps": pudadra([(windowed_latent(heads=3, dim=10, rot=6, vdim=9, kv_rank=21, base=50.0, window=11), grouped_moe(9, 3, 1, 2, 18, 70)),
+                         (differential(heads=3, kv_heads=1, dim=18, vdim=10, window=7, rot=6, conv=5, diff=0.15), grouped_moe(7, 7, 4, 4, 30, 13)),
+                         (differential(heads=1, kv_heads=1, dim=7, vdim=5, window=300, rot=2, conv=1, softcap=0.9, scale=1.0), dense(33))],
+                        width=51, vocab=97, eps=1e-3, residual_mult=1.0, logit_scale=1.7),
+    "large maps": pudadra([(differential(heads=4, kv_heads=2, dim=64, vdim=128, window=60, rot=64, scale=0.125), grouped_moe(16, 4, 3, 5, 72, 72)),
+                           (differential(heads=5, kv_heads=1, dim=96, vdim=144, window=33, rot=96, scale=0.1, conv=6), None),
+                           (windowed_latent(heads=20, dim=32, rot=32, vdim=48, kv_rank=288, window=50), dense(160)),
+                           (differential(heads=2, kv_heads=2, dim=160, vdim=72, window=90, rot=80, scale=0.08), grouped_moe(4, 2, 2, 4, 64, 300))], width=128),
+    "window of one map": pudadra([(differential(heads=2, kv_heads=2, dim=8, vdim=8, window=1, rot=8, conv=2), grouped_moe(2, 2, 1, 1, 8, 8)),
+                                  (windowed_latent(heads=1, dim=8, rot=2, vdim=8, kv_rank=8, window=1), None),
+                                  (differential(heads=9, kv_heads=3, dim=16, vdim=32, window=16, rot=0, conv=9), dense(8))], width=40),
     "window of one": config([parallel(heads=20, kv_heads=1, dim=8, vdim=8, window=1, keep=0, rot=8, right_heads=2, right_dim=8)], width=64),
 }
 

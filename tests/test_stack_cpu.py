@@ -106,7 +106,63 @@ def test_identity_experts_return_their_input():
     np.testing.assert_allclose(y, h)
 
 
-@pytest.mark.parametrize("name", ["mixed", "five layers"])
+def test_a_short_convolution_is_a_causal_filter():
+    rng = np.random.default_rng(5)
+    u, w = rng.standard_normal((9, 3)), rng.standard_normal((3, 4))
+    for c in range(3):
+        np.testing.assert_allclose(S.short_conv(u, w)[:, c], np.convolve(u[:, c], w[c, ::-1])[:9], rtol=1e-9, atol=1e-12)
+
+
+def test_stretched_frequencies_meet_at_both_ends():
+    lengths = np.array([10.0, 99.999, 100.001, 200.0, 299.999, 300.001, 5000.0])       # of waves; 300 positions, low 1, high 3
+    f = 2 * np.pi / lengths
+    g = S.stretched_frequencies(f, 4.0, 1.0, 3.0, 300)
+    np.testing.assert_allclose(g[:2], f[:2])
+    np.testing.assert_allclose(g[5:], f[5:] / 4)
+    np.testing.assert_allclose(g[[2, 4]], [f[2], f[4] / 4], rtol=1e-4)
+    np.testing.assert_allclose(g[3], f[3] * (0.25 + 0.75 * 0.25))                       # 1.5 waves: a quarter of the way
+
+
+def test_rotation_by_angles_is_the_rotation_by_halves():
+    x, p = np.random.default_rng(6).standard_normal((7, 2, 11)), np.arange(7)
+    angles = p[:, None] * 50.0 ** (-2.0 * np.arange(4) / 8)
+    np.testing.assert_allclose(S.rotate_by(x, angles), S.rotate(x, p, 8, 50.0, False), rtol=1e-12)
+
+
+def test_capped_scores():
+    s = np.array([-1e6, -0.01, 0.0, 0.01, 1e6])
+    np.testing.assert_allclose(S.capped(s, 5.0), [-5.0, -0.01, 0.0, 0.01, 5.0], rtol=1e-5)
+    assert S.capped(s, None) is s
+
+
+def test_the_difference_of_two_maps():
+    """Without the second map it is plain attention, normed; with equal maps a shorter copy of it, which the norm takes back."""
+    rng = np.random.default_rng(7)
+    q, k, v = rng.standard_normal((8, 4, 2, 5)), rng.standard_normal((8, 2, 2, 5)), rng.standard_normal((8, 2, 3))
+    mask = S.window_mask(8, 4, 0)
+    plain = S.rms_norm(S.sink_attention(q[:, :, 0], k[:, :, 0], v, mask, 0.4, None), 0.0) * 0.7
+    np.testing.assert_allclose(S.differential_attention(q, k, v, mask, 0.4, None, 0.0, 0.3, 0.0), plain, rtol=1e-9)
+    q[:, :, 1], k[:, :, 1] = q[:, :, 0], k[:, :, 0]
+    np.testing.assert_allclose(S.differential_attention(q, k, v, mask, 0.4, None, 0.6, 0.3, 0.0), plain, rtol=1e-9)
+    assert S.map_weight([0.0], [3.0], [1.0], [0.0], 0.3) == 0.3
+
+
+def test_choice_is_made_in_the_best_groups():
+    s = np.array([[0.05, 0.30, 0.20, 0.19, 0.01, 0.25]])          # groups of two: best 0.30, 0.20, 0.25
+    assert S.grouped_choice(s, 3, 3, 2).tolist() == [[1, 5, 0]]
+    assert S.grouped_choice(s, 3, 3, 3).tolist() == S.grouped_choice(s, 3, 1, 1).tolist() == [[1, 5, 2]]
+    assert S.grouped_choice(s, 2, 3, 1).tolist() == [[1, 0]]
+
+
+def test_latent_window_leaves_out_what_is_behind_it():
+    rng = np.random.default_rng(8)
+    q, qr, lat, kr = rng.standard_normal((9, 2, 3)), rng.standard_normal((9, 2, 2)), rng.standard_normal((9, 4)), rng.standard_normal((9, 2))
+    uk, uv = rng.standard_normal((2, 3, 4)), rng.standard_normal((2, 5, 4))
+    o = S.latent_attention(q, qr, lat, kr, uk, uv, 0.4, S.window_mask(9, 3, 0))
+    np.testing.assert_allclose(o[8], S.latent_attention(q[6:], qr[6:], lat[6:], kr[6:], uk, uv, 0.4)[2], rtol=1e-9)
+
+
+@pytest.mark.parametrize("name", ["mixed", "five layers", "two maps", "odd maps"])
 def test_a_prefix_does_not_see_what_follows(name):
     cfg = cases.CONFIGS[name]
     _, t = cases.tensors(cfg)
@@ -140,7 +196,16 @@ def test_configurations_are_checked(tmp_path):
                (cases.fipuzen([(cases.latent(), cases.moe(top=9, experts=4, identity=2))]), "experts"),
                (cases.fipuzen([(cases.latent(), {"kind": "dense", "ff": 8})]), "feed-forward"),
                (cases.fipuzen([{"type": "retention", "mixer": {}}]), "unknown mixer"),
-               (cases.fipuzen([(cases.latent(), {**cases.moe(), "expert": {}})]), "ff")]
+               (cases.fipuzen([(cases.latent(), {**cases.moe(), "expert": {}})]), "ff"),
+               (cases.pudadra([(cases.differential(heads=5, kv_heads=2), None)]), "multiple"),
+               (cases.pudadra([(cases.differential(window=0), None)]), "mask"), (cases.pudadra([(cases.windowed_latent(window=0), None)]), "mask"),
+               (cases.pudadra([(cases.differential(window=2.5), None)]), "integer"), (cases.pudadra([(cases.differential(conv=65), None)]), "taps"),
+               (cases.pudadra([(cases.differential(rot=26), None)]), "rotated"), (cases.pudadra([(cases.differential(softcap=-1.0), None)]), "bound"),
+               (cases.pudadra([(cases.differential(scaling={"factor": 2.0, "low": 3.0, "high": 3.0, "original": 9}), None)]), "scaling"),
+               (cases.pudadra([(cases.differential(), cases.grouped_moe(8, 3, 1, 1))]), "groups"),
+               (cases.pudadra([(cases.differential(), cases.grouped_moe(8, 4, 1, 3))]), "groups"),
+               (cases.pudadra([(cases.differential(), {"kind": "nosuch"})]), "feed-forward"),
+               ({k: v for k, v in cases.CONFIGS["two maps"].items() if k != "residual_mult"}, "residual_mult")]
         for cfg, word in bad:
             with pytest.raises(P.NanoflowPipelineError, match=word):
                 _set(tmp_path, cfg)
@@ -172,7 +237,7 @@ def test_pipeline_file_names_a_stack_model(tmp_path):
 
 
 @pytest.mark.parametrize("name,some", [("mixed", ("embed", "l1.mix.left.sink", "l1.mix.right.u")),
-                                       ("five layers", ("side.embed", "l0.mix.q.b", "l2.mlp.e1.down", "l2.mlp.correction"))])
+                                       ("two maps", ("embed", "l0.mix.q.conv", "l4.mix.lq2", "l1.mlp.shared.sg")), ("five layers", ("side.embed", "l0.mix.q.b", "l2.mlp.e1.down", "l2.mlp.correction"))])
 def test_safetensors_of_random_tensors_reads_back(tmp_path, name, some):
     from safetensors import safe_open
     cfg = cases.CONFIGS[name]
@@ -240,14 +305,23 @@ def test_argument_errors_without_a_gpu():
     l = K.lib()
     a = K.RecurrenceArgs(dtype=K.BF16, kind=7, heads=1, dim=8, vdim=8)
     assert l.nf_linear_recurrence(ctypes.byref(a), None) == -1 and b"kind" in l.nf_last_error()
-    w = K.WindowAttentionArgs(kv=K.KVLayout(K.BF16, 4, 3, 8, 8, 32, 16, 16))
+    w = K.WindowAttentionArgs(kv=K.KVLayout(K.BF16, 4, 3, 8, 8, 32, 16, 16, 1))
     assert l.nf_window_attention(ctypes.byref(w), None) == -1 and b"kv heads" in l.nf_last_error()
     assert l.nf_gemm_nk_bf16(None, None, None, 4, 12, 64, None, 0, None) == -1
     r = K.ResidualArgs(rows=4, width=8, ld=8, y_dtype=K.F32, shares=17)
     assert l.nf_residual_rows(ctypes.byref(r), None) == -1 and b"17 shares" in l.nf_last_error()
     r = K.ResidualArgs(rows=4, width=8, ld=8, y_dtype=K.F32, shares=1, next=K.Norm(kind=9))
     assert l.nf_residual_rows(ctypes.byref(r), None) == -1 and b"norm 9" in l.nf_last_error()
-    assert l.nf_route(None, 1, 8, 4, 8, 6, 9, None, 1.0, ctypes.byref(K.Routing(tile_rows=64)), None) == -1      # 9 of 8 outputs
+    w.kv = K.KVLayout(K.BF16, 4, 2, 8, 8, 32, 16, 16, 3)
+    assert l.nf_window_attention(ctypes.byref(w), None) == -1 and b"3 maps" in l.nf_last_error()
+    conv = K.ShortConv(taps=65)
+    assert l.nf_conv_state(K.BF16, None, 8, ctypes.byref(conv), None, 0, 1, None) == -1 and b"taps" in l.nf_last_error()
+    route = lambda **kw: l.nf_route(ctypes.byref(K.RouteArgs(**{**dict(shares=1, ld=16, rows=4, outputs=8, experts=6, top=2, scale=1.0), **kw})),
+                                    ctypes.byref(K.Routing(tile_rows=64)), None)
+    assert route(top=9) == -1 and b"top 9" in l.nf_last_error()                                   # of 8 outputs
+    assert route(groups=3, keep_groups=1) == -1 and b"groups" in l.nf_last_error()                # that do not divide them
+    assert route(groups=4, keep_groups=1, top=3) == -1 and b"top 3" in l.nf_last_error()          # of a group of two
+    assert route(ld=8, always=1) == -1 and b"ld=8" in l.nf_last_error()                           # no room for its gate
     g = K.GroupedGemmArgs(dtype=K.BF16, act=K.ACT_SILU, groups=2, M=4, N=8, K=8, lda=8, ldd=8)
     assert l.nf_gemm_grouped(ctypes.byref(g), None) == -1 and b"activation" in l.nf_last_error()
     g = K.GroupedGemmArgs(dtype=K.BF16, groups=2, M=4, N=8, K=8, lda=8, ldd=4)

@@ -43,8 +43,24 @@ def fipuzen_config(width, ff):
     return {"architecture": "Fipuzen", "width": width, "vocab": VOCAB, "token_side": {"dim": 256}, "norm": {"eps": 1e-5}, "layers": layers}
 
 
+def pudadra_config(width, ff):
+    """(attention, attention, latent attention, attention), all over the last 512 tokens: two maps of 64 over values of 128 (4 query
+    heads per kv head, convolutions of 4 taps), latents of 512 + 64 rotated; first a dense feed-forward of `ff`, then 32 experts
+    of a quarter of it in 8 groups, of which a token uses 4 out of 4 groups, and a shared one."""
+    n, window = width // 128, {"size": 512}
+    attention = {"heads": n, "kv_heads": n // 4, "dim": 64, "vdim": 128, "scale": 64 ** -0.5, "softcap": 30.0, "conv": 4, "diff": 0.4, "mask": window,
+                 "rot": {"dims": 64, "base": 5e5, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    latent = {"heads": n, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5, "mask": window, "rot": {"dims": 64, "base": 1e4}}
+    moe = {"kind": "moe", "expert": {"ff": ff // 4}, "shared": {"ff": ff // 4},
+           "router": {"experts": 32, "groups": {"count": 8, "keep": 4}, "top": 4}}
+    layers = [("attention", attention, {"kind": "dense", "ff": ff}), ("attention", attention, moe), ("latent_attention", latent, moe),
+              ("attention", attention, moe)]
+    return {"architecture": "Pudadra", "width": width, "vocab": VOCAB, "residual_mult": 0.5, "logit_scale": 0.5, "norm": {"eps": 1e-5},
+            "layers": [{"type": t, "mixer": m, "mlp": f} for t, m, f in layers]}
+
+
 # side -> configuration of a layer-stack model; "llama" is the other kind
-DESIGNS = {"stack": stack_config, "fipuzen": fipuzen_config}
+DESIGNS = {"stack": stack_config, "fipuzen": fipuzen_config, "pudadra": pudadra_config}
 SIZES = {"2048": (2048, 8192), "4096": (4096, 14336)}
 
 

@@ -61,14 +61,14 @@ def window_mask(T, size, keep_first):
     return (j <= i) & ((i - j < size) | (j < keep_first))
 
 
-def sink_attention(q, k, v, mask, scale, sink):
+def sink_attention(q, k, v, mask, scale, sink, cap=None):
     """q [T, H, d], k [T, G, d], v [T, G, e], sink [H] (or None): softmax whose denominator also
     holds exp(sink)."""
     T, H, _ = q.shape
     per = H // k.shape[1]
     out = np.empty((T, H, v.shape[-1]))
     for h in range(H):
-        s = np.where(mask, (q[:, h] @ k[:, h // per].T) * scale, -np.inf)
+        s = np.where(mask, capped((q[:, h] @ k[:, h // per].T) * scale, cap), -np.inf)
         m = s.max(axis=1, keepdims=True)
         if sink is not None:
             m = np.maximum(m, f64(sink)[h])

@@ -200,7 +200,7 @@ def test_gate_per_head(heads, kv_heads, dim, vdim):
 
 # ---------------------------------------------------------------- latent attention
 
-def latent_case(dtype, heads, rank, rot, b, n_decode, seed=0, mark=None, scale=None, workspace=True):
+def latent_case(dtype, heads, rank, rot, b, n_decode, seed=0, mark=None, scale=None, workspace=True, window=0):
     """Histories and the batch through append and attention; the plain result for the batch's rows.  mark: (request, query
     position, key position): that key is made to stand out for that query."""
     rng = np.random.default_rng(seed)
@@ -239,14 +239,14 @@ def latent_case(dtype, heads, rank, rot, b, n_decode, seed=0, mark=None, scale=N
     lens = np.diff(b.input_indptr)
     q = append(b, [full[r][len(full[r]) - n:] for r, n in enumerate(lens)], [queries[r][len(full[r]) - n:] for r, n in enumerate(lens)])
     assert not host(q[:, :, layout.rank_pad + rot:]).any()
-    got = K.latent_attention(layout, q, pool, device_batch(b), scale=scale, decode=n_decode, workspace=workspace)
+    got = K.latent_attention(layout, q, pool, device_batch(b), scale=scale, decode=n_decode, workspace=workspace, window=window)
     want = []
     for r, n in enumerate(lens):
         qr, lat, kr = plain[r]
         T = len(lat)
         qq = np.concatenate([rounded(queries[r], dtype), qr], -1)
         keys = np.concatenate([lat, kr], -1)
-        o = S.sink_attention(qq, keys[:, None], lat[:, None], S.window_mask(T, T + 1, 0), scale, None)
+        o = S.sink_attention(qq, keys[:, None], lat[:, None], S.window_mask(T, window or T + 1, 0), scale, None)
         want.append(o[T - n:])
     assert not host(got[:, :, rank:]).any()
     return got[:, :, :rank].contiguous(), np.concatenate(want)

@@ -186,7 +186,7 @@ def test_norm_rotation_and_append(heads, kv_heads, dim, vdim, rot_dims, interlea
         assert not pk.transpose(0, 2, 1, 3)[~touched].any() and not pv.transpose(0, 3, 1, 2)[~touched].any()
 
 
-def attention_case(dtype, heads, kv_heads, dim, vdim, window, keep, b, n_decode, seed=0, mark=None, scale=None, out_scale=1.0, gate=None):
+def attention_case(dtype, heads, kv_heads, dim, vdim, window, keep, b, n_decode, seed=0, mark=None, scale=None, out_scale=1.0, gate=None, softcap=None):
     """Histories and the batch through append and attention; the plain result for the batch's rows.
     mark: list of (request, query position, key position): that key is made to stand out for that query."""
     rng = np.random.default_rng(seed)
@@ -206,7 +206,7 @@ def attention_case(dtype, heads, kv_heads, dim, vdim, window, keep, b, n_decode,
     rows = np.concatenate([full[r][b.kv_len[r] - n:] for r, n in enumerate(np.diff(b.input_indptr))])
     q = append(layout, b, dev(rows, dtype), pool)
     got = K.window_attention(layout, q, pool, device_batch(b), window=window, keep_first=keep, scale=scale, sink=dev(sink, F32),
-                             out_scale=out_scale, decode=n_decode, gate=None if gate is None else dev(gate, dtype))
+                             out_scale=out_scale, decode=n_decode, gate=None if gate is None else dev(gate, dtype), softcap=softcap or 0.0)
     want = []
     for r, n in enumerate(np.diff(b.input_indptr)):
         v = rounded(full[r], dtype)
@@ -214,7 +214,7 @@ def attention_case(dtype, heads, kv_heads, dim, vdim, window, keep, b, n_decode,
         cut = lambda at, m, d: v[:, at:at + m * d].reshape(T, m, d)
         mask = S.window_mask(T, window or 10 ** 9, keep)
         o = S.sink_attention(cut(0, heads, dim), cut(heads * dim, kv_heads, dim), cut((heads + kv_heads) * dim, kv_heads, vdim), mask,
-                             scale, sink.astype(np.float32))
+                             scale, sink.astype(np.float32), softcap)
         want.append(o[T - n:].reshape(n, -1))
     return got, np.concatenate(want) * out_scale
 

@@ -196,7 +196,7 @@ def lib() -> C.CDLL:
         l.nf_attention_paged_f16.argtypes = [vp] * 7 + [i32] * 8 + [vp, sz, vp]
         l.nf_keep_token_f16.argtypes = [vp, vp, vp, i32, i32, vp]
         l.nf_argmax_f16.argtypes = [vp, vp, vp, i32, i32, vp]
-        for name in ("nf_gemm_nk_bf16", "nf_gemm_nk_relu2_bf16", "nf_gemm_nk_silu_bf16"):
+        for name in ("nf_gemm_nk_bf16", "nf_gemm_nk_relu2_bf16", "nf_gemm_nk_silu_bf16", "nf_gemm_nk_gelu_bf16"):
             getattr(l, name).argtypes = [vp, vp, vp, i32, i32, i32, vp, sz, vp]
         l.nf_gemm_nk_bias_bf16.argtypes = [vp, vp, vp, vp, i32, i32, i32, vp, sz, vp]
         l.nf_gemm_nk_f32.argtypes = [vp, vp, vp, vp, i32, i32, i32, i32, vp]

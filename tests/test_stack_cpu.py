@@ -300,6 +300,13 @@ def test_without_slots_nothing_changes():
     f.close()
 
 
+def test_every_entry_point_has_declared_argument_types():
+    """Without them ctypes hands pointers over as 32-bit integers."""
+    from nanoflow_amd import kernels as K
+    without = {name for name in K.SYMBOLS if getattr(K.lib(), name).argtypes is None}
+    assert without <= {"nf_abi_version", "nf_last_error"}, without      # these take none
+
+
 def test_argument_errors_without_a_gpu():
     from nanoflow_amd import kernels as K
     l = K.lib()

@@ -22,6 +22,7 @@
 // fp32 (attn_rows_kernel): one wavefront per (row, head), every product in 32-bit.
 #include <algorithm>
 #include <cmath>
+#include <type_traits>
 
 #include "layer_common.h"
 
@@ -40,13 +41,23 @@ __device__ __forceinline__ float temperature(const nf_query_temperature& q, int 
   return q.every > 0 ? 1.f + q.coef * logf((float)((pos + 1) / q.every + 1)) : 1.f;
 }
 
+template <int N>
+using Int = std::integral_constant<int, N>;
+
+template <class T>
+struct ConvRow;
+template <int R, class T>
+__device__ __forceinline__ void four_of(const ConvRow<T>* row, int c, const bool* owner, float4_t* y);
+
 // A row of the projections as the short convolution sees it: rows before it, of the batch or of the request's slot.
 template <class T>
 struct ConvRow {
   const T* proj = nullptr;  // this row
   const T* weight = nullptr;
   T* state = nullptr;       // of the request's slot
-  int taps = 0, ld = 0, pos = 0, before = 0;  // before: rows of the portion ahead of this one
+  int taps = 0, ld = 0, pos = 0;
+  int before = 0;           // rows of the portion ahead of this one
+  int place = 0;            // of this row in the state, which is a ring of taps - 1 rows
   bool single = false;      // the request's only row, which leaves the state as well
 
   __device__ __forceinline__ ConvRow(const nf_short_conv& c, const T* proj_, int ld_, int t, int req, int pos_)
@@ -55,31 +66,19 @@ struct ConvRow {
     const int first = c.input_indptr[req];
     before = t - first;
     single = c.input_indptr[req + 1] - first == 1;
-    if (taps > 1) state = (T*)c.state + (size_t)c.state_slots[req] * (taps - 1) * ld;
-  }
-  // its value j rows back, j in 1 .. min(taps - 1, pos)
-  __device__ __forceinline__ const T* back(int j) const { return j <= before ? proj - (size_t)j * ld : state + (size_t)((pos - j) % (taps - 1)) * ld; }
-  // columns c .. c + 3; `owner`: of the threads that ask for them, the one that keeps the state
-  __device__ __forceinline__ float4_t four(int c, bool owner) const {
-    const typename Act<T>::raw4 cur = Act<T>::load_raw4(proj + c);
-    if (taps < 1) return Act<T>::widen4(cur);
-    const int past = min(taps - 1, pos);
-    float4_t y{0.f, 0.f, 0.f, 0.f};
-    constexpr int kAhead = 3;
-    for (int j0 = 1; j0 <= past; j0 += kAhead) {
-      typename Act<T>::raw4 x[kAhead], w[kAhead];
-#pragma unroll
-      for (int u = 0; u < kAhead; ++u) {  // past the last tap: the last one's again, left out below
-        const int j = min(j0 + u, past);
-        x[u] = Act<T>::load_raw4(back(j) + c);
-        w[u] = Act<T>::load_raw4(weight + (size_t)(taps - 1 - j) * ld + c);
-      }
-#pragma unroll
-      for (int u = 0; u < kAhead; ++u)
-        if (j0 + u <= past) y += Act<T>::widen4(x[u]) * Act<T>::widen4(w[u]);
+    if (taps > 1) {
+      state = (T*)c.state + (size_t)c.state_slots[req] * (taps - 1) * ld;
+      place = pos % (taps - 1);
     }
-    y += Act<T>::widen4(cur) * Act<T>::load4(weight + (size_t)(taps - 1) * ld + c);
-    if (owner && single && taps > 1) *reinterpret_cast<typename Act<T>::raw4*>(state + (size_t)(pos % (taps - 1)) * ld + c) = cur;
+  }
+  __device__ __forceinline__ ConvRow() {}
+  // its value j rows back, j in 0 .. min(taps - 1, pos)
+  __device__ __forceinline__ const T* back(int j) const {
+    return j <= before ? proj - (size_t)j * ld : state + (size_t)(place - j + (place < j ? taps - 1 : 0)) * ld;
+  }
+  __device__ __forceinline__ float4_t four(int c, bool owner) const {
+    float4_t y;
+    four_of<1>(this, c, &owner, &y);
     return y;
   }
   __device__ __forceinline__ float one(int c) const {  // asked for by the owner only
@@ -88,10 +87,75 @@ struct ConvRow {
     float y = 0.f;
     for (int j = 1; j <= min(taps - 1, pos); ++j) y += Act<T>::load(back(j) + c) * Act<T>::load(weight + (size_t)(taps - 1 - j) * ld + c);
     y += Act<T>::load(&cur) * Act<T>::load(weight + (size_t)(taps - 1) * ld + c);
-    if (single && taps > 1) state[(size_t)(pos % (taps - 1)) * ld + c] = cur;
+    if (single && taps > 1) state[(size_t)place * ld + c] = cur;
     return y;
   }
 };
+
+// Columns c .. c + 3 of R rows that follow each other, everything requested at once; owner[u]: of the threads that ask for
+// them, the one that keeps row u's state.
+template <int R, class T>
+__device__ __forceinline__ void four_of(const ConvRow<T>* row, int c, const bool* owner, float4_t* y) {
+  typedef typename Act<T>::raw4 raw4;
+  raw4 cur[R];
+#pragma unroll
+  for (int u = 0; u < R; ++u) cur[u] = Act<T>::load_raw4(row[u].proj + c);
+  const int taps = row[0].taps, ld = row[0].ld;
+  if (taps < 1) {
+#pragma unroll
+    for (int u = 0; u < R; ++u) y[u] = Act<T>::widen4(cur[u]);
+    return;
+  }
+  const float4_t zero{0.f, 0.f, 0.f, 0.f}, last = Act<T>::load4(row[0].weight + (size_t)(taps - 1) * ld + c);
+  auto weight = [&](int j) { return Act<T>::load_raw4(row[0].weight + (size_t)(taps - 1 - min(j, taps - 1)) * ld + c); };
+  // past the first token or the last tap: the furthest there is again, left out of the sums
+  auto before = [&](int u, int j) { return Act<T>::load_raw4(row[u].back(min(j, min(taps - 1, row[u].pos))) + c); };
+  constexpr int kAhead = 3;
+  if (R > 1 && taps <= kAhead + 1 && row[R - 1].before >= R - 1) {  // all of one portion: every row is read once
+    raw4 x[kAhead], w[kAhead];
+    float4_t at[R + kAhead], f[kAhead];  // at[kAhead + u]: row u
+#pragma unroll
+    for (int k = 0; k < kAhead; ++k) w[k] = weight(k + 1);
+#pragma unroll
+    for (int k = 0; k < kAhead; ++k) x[k] = before(0, k + 1);
+#pragma unroll
+    for (int k = 0; k < kAhead; ++k) {
+      at[kAhead - 1 - k] = k + 1 <= row[0].pos ? Act<T>::widen4(x[k]) : zero;
+      f[k] = k + 1 < taps ? Act<T>::widen4(w[k]) : zero;
+    }
+#pragma unroll
+    for (int u = 0; u < R; ++u) at[kAhead + u] = Act<T>::widen4(cur[u]);
+#pragma unroll
+    for (int u = 0; u < R; ++u) {
+      y[u] = zero;
+#pragma unroll
+      for (int k = 0; k < kAhead; ++k) y[u] += at[kAhead + u - 1 - k] * f[k];
+      y[u] += at[kAhead + u] * last;
+    }
+    return;  // rows of such a portion are not single
+  }
+#pragma unroll
+  for (int u = 0; u < R; ++u) y[u] = zero;
+  for (int j0 = 1; j0 < taps; j0 += kAhead) {
+    raw4 x[R][kAhead], w[kAhead];
+#pragma unroll
+    for (int k = 0; k < kAhead; ++k) w[k] = weight(j0 + k);
+#pragma unroll
+    for (int u = 0; u < R; ++u)
+#pragma unroll
+      for (int k = 0; k < kAhead; ++k) x[u][k] = before(u, j0 + k);
+#pragma unroll
+    for (int u = 0; u < R; ++u)
+#pragma unroll
+      for (int k = 0; k < kAhead; ++k)
+        if (j0 + k <= min(taps - 1, row[u].pos)) y[u] += Act<T>::widen4(x[u][k]) * Act<T>::widen4(w[k]);
+  }
+#pragma unroll
+  for (int u = 0; u < R; ++u) {
+    y[u] += Act<T>::widen4(cur[u]) * last;
+    if (owner[u] && row[u].single && taps > 1) *reinterpret_cast<raw4*>(row[u].state + (size_t)row[u].place * ld + c) = cur[u];
+  }
+}
 
 // The last rows of every request that brings more than one, as the state of its convolution.  Sixteen bytes a thread.
 template <class T>
@@ -181,93 +245,118 @@ __global__ __launch_bounds__(256) void qkv_append_kernel(nf_kv_layout kv, const 
   }
 }
 
-// The same for sizes and columns that are multiples of four, which is what models have: a (row, query or key head) is
-// 16 lanes with 16-byte groups; values are turned through LDS, 16 rows of a head at a time, so that the
-// transposed cache is written four positions at once where four rows are an aligned run of one page.
-template <class T>
-__global__ __launch_bounds__(256) void qkv_append4_kernel(nf_kv_layout kv, const T* __restrict__ proj, int ld, int q_col,
+// The same for sizes and columns that are multiples of four, which is what models have.  A workgroup takes R rows of 16
+// heads, 16 lanes a head, kVec groups of four elements a lane, so that everything about a row is the same in all its
+// lanes.  Of many rows, values are turned through LDS, 16 rows of a head at a time, so that the transposed cache is
+// written four positions at once where four rows are an aligned run of one page; of few (value_blocks = 0) value heads
+// are taken like the others.
+template <class T, int kVec, int R>
+__global__ __launch_bounds__(256, kVec <= 2 ? 8 : 5) void qkv_append4_kernel(nf_kv_layout kv, const T* __restrict__ proj, int ld, int q_col,
                                                           int k_col, int v_col, const float* __restrict__ q_norm,
                                                           const float* __restrict__ k_norm, float eps, nf_rotation rot,
                                                           nf_query_temperature q_temp, nf_short_conv conv, T* __restrict__ q_out, T* __restrict__ kv_data,
                                                           const int32_t* __restrict__ kv_indptr,
                                                           const int32_t* __restrict__ kv_indices,
                                                           const int32_t* __restrict__ rev_input_indptr,
-                                                          const int32_t* __restrict__ positions, int rows, int qk_blocks) {
+                                                          const int32_t* __restrict__ positions, int rows, int value_blocks) {
   __shared__ __attribute__((aligned(16))) float buf[kMaxHeadDim * 17];
-  __shared__ long long row_page[16];  // element offset of the row's page, and its entry
-  __shared__ int row_entry[16];
   const int H = kv.heads * kv.maps, G = kv.kv_heads * kv.maps, VG = kv.kv_heads, tid = threadIdx.x;
-  if ((int)blockIdx.x < qk_blocks) {
-    constexpr int kVec = kMaxHeadDim / 64;
-    const int job = blockIdx.x * 16 + (tid >> 4), l = tid & 15;
-    const bool live = job < rows * (H + G);
-    const int t = live ? job / (H + G) : 0, head = live ? job % (H + G) : 0;
-    const bool is_q = head < H;
-    const int col = is_q ? q_col + head * kv.dim : k_col + (head - H) * kv.dim;
-    const float* w = is_q ? q_norm : k_norm;
-    float* mine = buf + (tid >> 4) * kMaxHeadDim;
-    const int pos = positions[t], req = rev_input_indptr[t], half = rot.dims / 2;
-    const ConvRow<T> row(conv, proj, ld, t, req, pos);
-    const float temp = is_q ? temperature(q_temp, pos) : 1.f;
-    T* dst;
-    if (is_q) {
-      dst = q_out + ((size_t)t * H + head) * kv.k_pad;
-    } else {
-      const int page = kv_indices[kv_indptr[req] + pos / kPage];
-      dst = kv_data + (size_t)page * kv_page_elements(kv) + ((size_t)(head - H) * kPage + pos % kPage) * kv.k_pad;
+  if ((int)blockIdx.x >= value_blocks) {
+    const int jobs = H + G + (value_blocks > 0 ? 0 : VG), head_blocks = (jobs + 15) / 16, block = blockIdx.x - value_blocks;
+    const int t0 = block / head_blocks * R, l = tid & 15, job = block % head_blocks * 16 + (tid >> 4);
+    const bool live = job < jobs;
+    const int head = live ? job : 0;
+    const bool is_q = head < H, is_v = head >= H + G;
+    const int dim = is_v ? kv.vdim : kv.dim;
+    const int col = is_q ? q_col + head * dim : is_v ? v_col + (head - H - G) * dim : k_col + (head - H) * dim;
+    const float* w = is_q ? q_norm : is_v ? nullptr : k_norm;
+    float* mine = buf + (tid >> 4) * (kVec * 64);
+    const int half = is_v ? 0 : rot.dims / 2;
+    ConvRow<T> row[R];
+    T* dst[R];
+    bool keep[R];
+#pragma unroll
+    for (int u = 0; u < R; ++u) {
+      const int t = min(t0 + u, rows - 1), pos = positions[t], req = rev_input_indptr[t];
+      row[u] = ConvRow<T>(conv, proj, ld, t, req, pos);
+      keep[u] = live && t0 + u < rows;
+      T* page = kv_data + (size_t)kv_indices[kv_indptr[req] + pos / kPage] * kv_page_elements(kv);
+      dst[u] = is_q   ? q_out + ((size_t)t * H + head) * kv.k_pad
+               : is_v ? page + kv_value_offset(kv) + (size_t)(head - H - G) * kv.v_pad * kPage + pos % kPage
+                      : page + ((size_t)(head - H) * kPage + pos % kPage) * kv.k_pad;
     }
-    float4_t v[kVec];
-    float sq = 0.f;
+    float4_t v[kVec][R];
 #pragma unroll
     for (int i = 0; i < kVec; ++i) {
       const int c = (i * 16 + l) * 4;
-      v[i] = float4_t{0.f, 0.f, 0.f, 0.f};
-      if (c < kv.dim) v[i] = row.four(col + c, live);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) sq += v[i][e] * v[i][e];
+      for (int u = 0; u < R; ++u) v[i][u] = float4_t{0.f, 0.f, 0.f, 0.f};
+      if (c < dim) four_of<R>(row, col + c, keep, v[i]);
     }
-    if (w) {
+    if (q_norm || k_norm) {  // asked by the whole workgroup: the sums are over lanes
 #pragma unroll
-      for (int m = 8; m > 0; m >>= 1) sq += __shfl_xor(sq, m, 64);
-      const float inv = 1.f / sqrtf(sq / (float)kv.dim + eps);
+      for (int u = 0; u < R; ++u) {
+        float sq = 0.f;
+#pragma unroll
+        for (int i = 0; i < kVec; ++i)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) sq += v[i][u][e] * v[i][u][e];
+#pragma unroll
+        for (int m = 8; m > 0; m >>= 1) sq += __shfl_xor(sq, m, 64);
+        const float inv = 1.f / sqrtf(sq / (float)dim + eps);
+        if (w)
+#pragma unroll
+          for (int i = 0; i < kVec; ++i) {
+            const int c = (i * 16 + l) * 4;
+            if (c < dim) v[i][u] = v[i][u] * inv * *reinterpret_cast<const float4_t*>(w + c);
+          }
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < R; ++u) {
+      const float temp = is_q ? temperature(q_temp, row[u].pos) : 1.f;
+      const float* tab = rot.table + (size_t)row[u].pos * half * 2;
+      if (!rot.interleaved) {  // a lane's partners are in its own wavefront
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+        __builtin_amdgcn_wave_barrier();
+#pragma unroll
+        for (int i = 0; i < kVec; ++i) *reinterpret_cast<float4_t*>(mine + (i * 16 + l) * 4) = v[i][u];
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+        __builtin_amdgcn_wave_barrier();
+      }
 #pragma unroll
       for (int i = 0; i < kVec; ++i) {
         const int c = (i * 16 + l) * 4;
-        if (c < kv.dim) v[i] = v[i] * inv * *reinterpret_cast<const float4_t*>(w + c);
-      }
-    }
-    if (!rot.interleaved)
+        const float4_t x = v[i][u];
+        float4_t y = x;
+        if (c < 2 * half) {
+          if (rot.interleaved) {
+            const float4_t cs = *reinterpret_cast<const float4_t*>(tab + c);  // cos, sin of pair c / 2, then of the next
+            y = float4_t{x[0] * cs[0] - x[1] * cs[1], x[1] * cs[0] + x[0] * cs[1], x[2] * cs[2] - x[3] * cs[3], x[3] * cs[2] + x[2] * cs[3]};
+          } else {
+            const bool first = c < half;
+            const int f = first ? c : c - half;
+            const float4_t other = *reinterpret_cast<const float4_t*>(mine + (first ? c + half : f));
+            const float4_t a = *reinterpret_cast<const float4_t*>(tab + 2 * f), b = *reinterpret_cast<const float4_t*>(tab + 2 * f + 4);
+            const float4_t cs{a[0], a[2], b[0], b[2]}, sn{a[1], a[3], b[1], b[3]};
+            y = first ? x * cs - other * sn : x * cs + other * sn;
+          }
+        }
+        y = y * temp;
+        if (is_v) {
+          if (keep[u] && c < kv.v_pad)
 #pragma unroll
-      for (int i = 0; i < kVec; ++i) {
-        const int c = (i * 16 + l) * 4;
-        if (c < 2 * half) *reinterpret_cast<float4_t*>(mine + c) = v[i];
-      }
-    __syncthreads();
-#pragma unroll
-    for (int i = 0; i < kVec; ++i) {
-      const int c = (i * 16 + l) * 4;
-      if (c >= kv.k_pad || !live) continue;
-      float4_t y = v[i];
-      if (c < 2 * half) {
-        const float* tab = rot.table + (size_t)pos * half * 2;
-        if (rot.interleaved) {
-          const float4_t cs = *reinterpret_cast<const float4_t*>(tab + c);  // cos, sin of pair c / 2, then of the next
-          y = float4_t{v[i][0] * cs[0] - v[i][1] * cs[1], v[i][1] * cs[0] + v[i][0] * cs[1], v[i][2] * cs[2] - v[i][3] * cs[3],
-                       v[i][3] * cs[2] + v[i][2] * cs[3]};
-        } else {
-          const bool first = c < half;
-          const int f = first ? c : c - half;
-          const float4_t other = *reinterpret_cast<const float4_t*>(mine + (first ? c + half : f));
-          const float4_t t0 = *reinterpret_cast<const float4_t*>(tab + 2 * f), t1 = *reinterpret_cast<const float4_t*>(tab + 2 * f + 4);
-          const float4_t cs{t0[0], t0[2], t1[0], t1[2]}, sn{t0[1], t0[3], t1[1], t1[3]};
-          y = first ? v[i] * cs - other * sn : v[i] * cs + other * sn;
+            for (int e = 0; e < 4; ++e) Act<T>::store(dst[u] + (size_t)(c + e) * kPage, y[e]);
+        } else if (keep[u] && c < kv.k_pad) {
+          Act<T>::store4(dst[u] + c, y);
         }
       }
-      Act<T>::store4(dst + c, y * temp);
     }
     return;
   }
-  const int block = blockIdx.x - qk_blocks, head = block % VG, row0 = block / VG * 16;
+  __shared__ long long row_page[16];  // element offset of the row's page, and its entry
+  __shared__ int row_entry[16];
+  const int head = blockIdx.x % VG, row0 = blockIdx.x / VG * 16;
   if (tid < 16) {
     const int t = min(row0 + tid, rows - 1), pos = positions[t];
     row_page[tid] = (long long)kv_indices[kv_indptr[rev_input_indptr[t]] + pos / kPage] * (long long)kv_page_elements(kv);
@@ -1042,19 +1131,27 @@ int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, i
   NF_REQUIRE(proj && q_out && kv_data && kv_indptr && kv_indices && rev_input_indptr && positions, "%s: null pointer", who);
   hipStream_t s = (hipStream_t)stream;
   const size_t four = 4 * (kv->dtype == NF_BF16 ? 2 : 4);
-  const long long qk_jobs = (long long)rows * (kv->heads + kv->kv_heads) * kv->maps;
-  if ((kv->dim | kv->vdim | ld | q_col | k_col | v_col) % 4 == 0 && ((uintptr_t)proj | (uintptr_t)cv.weight | (uintptr_t)cv.state) % four == 0 &&
-      rot->dims % (rot->interleaved ? 4 : 8) == 0 && qk_jobs < (1ll << 30)) {
-    const int qk_blocks = (int)((qk_jobs + 15) / 16), blocks = qk_blocks + (rows + 15) / 16 * kv->kv_heads;
-    if (kv->dtype == NF_BF16)
-      qkv_append4_kernel<bf16_t><<<blocks, 256, 0, s>>>(*kv, (const bf16_t*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps,
-                                                        *rot, temp, cv, (bf16_t*)q_out, (bf16_t*)kv_data, kv_indptr, kv_indices,
-                                                        rev_input_indptr, positions, rows, qk_blocks);
-    else
-      qkv_append4_kernel<float><<<blocks, 256, 0, s>>>(*kv, (const float*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps,
-                                                       *rot, temp, cv, (float*)q_out, (float*)kv_data, kv_indptr, kv_indices,
-                                                       rev_input_indptr, positions, rows, qk_blocks);
-    return check_launch(who);
+  const uintptr_t places = (uintptr_t)proj | (uintptr_t)cv.weight | (uintptr_t)cv.state | (uintptr_t)q_out | (uintptr_t)kv_data;
+  const int sizes = kv->dim | kv->vdim | ld | q_col | k_col | v_col, turned = rot->interleaved ? rot->dims : rot->dims / 2;
+  if (sizes % 4 == 0 && places % four == 0 && turned % 4 == 0 && rows < (1 << 20)) {
+    const bool few = rows < 1024;
+    auto go = [&](auto type, auto vec, auto run) {
+      using T = decltype(type);
+      constexpr int kRun = decltype(run)::value;
+      const int value_blocks = few ? 0 : (rows + 15) / 16 * kv->kv_heads;
+      const int jobs = (kv->heads + kv->kv_heads) * kv->maps + (few ? kv->kv_heads : 0);
+      const int blocks = value_blocks + (rows + kRun - 1) / kRun * ((jobs + 15) / 16);
+      qkv_append4_kernel<T, decltype(vec)::value, kRun><<<(unsigned)blocks, 256, 0, s>>>(
+          *kv, (const T*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot, temp, cv, (T*)q_out, (T*)kv_data, kv_indptr, kv_indices,
+          rev_input_indptr, positions, rows, value_blocks);
+      return check_launch(who);
+    };
+    auto sized = [&](auto type, auto run) {
+      const int widest = few ? std::max(kv->k_pad, kv->v_pad) : kv->k_pad;
+      return widest <= 64 ? go(type, Int<1>{}, run) : widest <= 128 ? go(type, Int<2>{}, run) : go(type, Int<4>{}, run);
+    };
+    if (kv->dtype == NF_F32) return sized(float{}, Int<1>{});
+    return few ? sized(bf16_t{}, Int<1>{}) : sized(bf16_t{}, Int<2>{});
   }
   const dim3 grid((unsigned)rows, (unsigned)(((kv->heads + kv->kv_heads) * kv->maps + kv->kv_heads + 3) / 4));
   if (kv->dtype == NF_BF16)

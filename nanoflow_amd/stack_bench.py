@@ -74,15 +74,21 @@ def _sub_prefill(b, first, count, length, vocab, seed):
 
 
 def _time(run, steps, warmup):
+    """Milliseconds per iteration: `steps` of them in up to five blocks, the median block (the runtime pauses once in a while for
+    tens of milliseconds, which is not the model's)."""
     import torch
     for _ in range(warmup):
         run()
-    torch.cuda.synchronize()
-    t0 = time.perf_counter()
-    for _ in range(steps):
-        run()
-    torch.cuda.synchronize()
-    return (time.perf_counter() - t0) / steps * 1e3
+    per_block, times = max(steps // 5, 1), []
+    for first in range(0, steps, per_block):
+        n = min(per_block, steps - first)
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        for _ in range(n):
+            run()
+        torch.cuda.synchronize()
+        times.append((time.perf_counter() - t0) / n * 1e3)
+    return float(np.median(times))
 
 
 def _cases():

@@ -73,6 +73,57 @@ def test_convolution_rotation_and_append_in_portions(heads, kv_heads, dim, vdim,
             assert (host(state)[slot] == 77.0).all()                         # no one else's slot is touched
 
 
+@pytest.mark.parametrize("heads,kv_heads,dim,vdim,maps,rot,taps", [(4, 2, 64, 128, 2, 64, 4), (3, 1, 24, 40, 2, 16, 3), (2, 1, 100, 72, 1, 48, 6),
+                                                                   (1, 1, 160, 256, 2, 32, 2), (2, 2, 16, 16, 1, 8, 0)])
+def test_many_rows_are_the_rows_of_small_portions(heads, kv_heads, dim, vdim, maps, rot, taps):
+    """More than a thousand rows of unequal requests at a time, single tokens between them, against the same a few tokens at a time: the
+    same bits, whatever rows a workgroup has beside each other."""
+    rng = np.random.default_rng(taps)
+    qn, kn = heads * maps * dim, kv_heads * maps * dim
+    ld, lengths = (qn + kn + kv_heads * vdim + 7) // 8 * 8, [701, 2, 333, 1, 47, 515, 5]
+    n, cuts = len(lengths), [[120, 1, 333, 0, 46, 515, 2], [581, 1, 0, 1, 1, 0, 3]]      # 1017 rows in the first, few in the second
+    cuts = [[a + (9 if r == 0 else 0) for r, a in enumerate(cuts[0])], [a - (9 if r == 0 else 0) for r, a in enumerate(cuts[1])]]
+    assert sum(cuts[0]) >= 1024 and (np.array(cuts).sum(0) == lengths).all()
+    full = [rng.standard_normal((t, ld)) for t in lengths]
+    w, table = rng.standard_normal((max(taps, 1), ld)), table_of(800, rot, 50.0)
+    pages = np.split(rng.permutation(sum(-(-t // 16) for t in lengths)), np.cumsum([-(-t // 16) for t in lengths])[:-1])
+
+    def run(dtype, steps):
+        layout = K.kv_layout(dtype, heads, kv_heads, dim, vdim, maps)
+        state = torch.full((n, max(taps - 1, 1), ld), 77.0, dtype=dtype, device="cuda")
+        pool, at, queries = K.kv_pool(layout, sum(map(len, pages))), [0] * n, [[] for _ in range(n)]
+        for counts in steps:
+            live = [r for r in range(n) if counts[r]]
+            b = synth.make_batch([], [(at[r], counts[r]) for r in live], vocab=10, seed=0)
+            b.kv_indices = np.concatenate([pages[r][:used] for r, used in zip(live, np.diff(b.kv_indptr))]).astype(np.int32)
+            d, slots = device_batch(b), dev(np.array(live, np.int32))
+            conv = K.short_conv(dev(w, dtype), state, d["input_indptr"], slots) if taps else None
+            proj = dev(np.concatenate([full[r][at[r]:at[r] + counts[r]] for r in live]), dtype)
+            q = host(K.qkv_append(layout, proj, (0, qn, qn + kn), None, None, 1e-5, K.rotation(table, rot), pool, d["kv_indptr"], d["kv_indices"],
+                                  d["rev_input_indptr"], d["positions"], conv=conv))
+            for i, r in enumerate(live):
+                queries[r].append(q[b.input_indptr[i]:b.input_indptr[i + 1]])
+                at[r] += counts[r]
+        return [np.concatenate(q) for q in queries], host(pool)
+
+    pieces = []
+    left = list(lengths)
+    while any(left):
+        pieces.append([min(t, 3 + (7 * r + 5 * len(pieces)) % 90) for r, t in enumerate(left)])
+        left = [a - c for a, c in zip(left, pieces[-1])]
+    assert max(map(sum, pieces)) < 1024
+    for dtype in DTYPES:
+        many, few = run(dtype, cuts), run(dtype, pieces)
+        for a, b in zip(many[0], few[0]):
+            assert np.array_equal(a, b)
+        assert np.array_equal(many[1], few[1])
+        r = 0
+        y = rounded(full[r], dtype)[:, :qn]
+        if taps:
+            y = S.short_conv(y, rounded(w.T[:qn], dtype))
+        close(many[0][r][:, :, :dim], S.rotate(y.reshape(lengths[r], -1, dim), np.arange(lengths[r]), rot, 50.0, False), dtype)
+
+
 # ---------------------------------------------------------------- two maps, capped scores
 
 def maps_case(dtype, heads, kv_heads, dim, vdim, window, b, n_decode, seed=0, mark=None, scale=None, cap=5.0, weight=0.45, eps=1e-5, diff=0.3):

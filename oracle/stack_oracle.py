@@ -4,7 +4,9 @@ with data-dependent decay, two mixers side by side.  Fipuzen: attention with a u
 and a gate per head, latent attention, lightning attention, a mixture of experts with identity experts, token
 inputs to every layer.  Pudadra: differential attention over a window on convolved projections with capped
 scores, latent attention over a window, experts in groups of which some are left out, a gated shared
-expert.  Test infrastructure only: one function per mechanism, whole sequences at once, nothing
+expert.  Desalix: attention in chunks with normed, turned values and a sink, norms on both sides of a sublayer
+with one number each, layer scales, a run of layers passed several times, clamped gated experts whose input is
+weighed.  Test infrastructure only: one function per mechanism, whole sequences at once, nothing
 shared with the product path.
 
 A model is (config, tensors): the parsed config.json and a dict name -> numpy array (any float type).
@@ -409,12 +411,92 @@ def pudadra_forward(cfg, t, tokens, want_layers=False):
     return (logits, np.stack(layers)) if want_layers else logits
 
 
+# ---------------------------------------------------------------- Desalix
+
+def chunk_mask(T, size):
+    """[T, T] bool: a position sees those before it in its own run of `size` positions (None: all before it)."""
+    i, j = np.arange(T)[:, None], np.arange(T)[None, :]
+    return (j <= i) & ((i // size == j // size) if size else True)
+
+
+def turn_values(v, positions, base, back=False):
+    """v [T, heads, e]: all dimensions turned by the position, or back by it."""
+    e = v.shape[-1]
+    angles = f64(positions)[:, None] * f64(base) ** (-2.0 * np.arange(e // 2) / e)
+    return rotate_by(v, -angles if back else angles)
+
+
+def chunked_attention_mixer(t, pre, m, eps, h, positions):
+    T, H, G = h.shape[0], m["heads"], m["kv_heads"]
+    rot = m["rot"]
+    q = rms_norm(linear(t, pre + "q", h).reshape(T, H, m["dim"]), eps, t[pre + "q.norm"])
+    k = rms_norm(linear(t, pre + "k", h).reshape(T, G, m["dim"]), eps, t[pre + "k.norm"])
+    v = rms_norm(linear(t, pre + "v", h).reshape(T, G, m["vdim"]), eps)
+    q, k = (rotate(x, positions, rot["dims"], rot["base"], False) for x in (q, k))
+    o = sink_attention(q, k, turn_values(v, positions, rot["base"]), chunk_mask(T, (m.get("mask") or {}).get("size")), m["scale"], t[pre + "sink"])
+    return linear(t, pre + "o", turn_values(o, positions, rot["base"], back=True).reshape(T, -1))
+
+
+def clamped_expert(t, pre, limit, h):
+    """Gate and up bounded by `limit` (the gate from above only), the gate's sigmoid at 1.702 times itself, one added to up."""
+    g = np.minimum(linear(t, pre + "gate", h), limit)
+    u = np.clip(linear(t, pre + "up", h), -limit, limit)
+    return linear(t, pre + "down", g * sigmoid(1.702 * g) * (u + 1.0))
+
+
+def sigmoid_choice(z, top):
+    """(chosen [T, top], scores [T, top]): every output's own sigmoid, the largest of them as they are."""
+    s = sigmoid(z)
+    chosen = np.argsort(-s, axis=-1, kind="stable")[:, :top]
+    return chosen, np.take_along_axis(s, chosen, axis=-1)
+
+
+def input_weighted_mixture(t, pre, m, h):
+    chosen, weights = sigmoid_choice(linear(t, pre + "router", h), m["router"]["top"])
+    y = clamped_expert(t, pre + "shared.", m["shared"]["limit"], h) if m.get("shared") else np.zeros_like(h)
+    for token in range(h.shape[0]):
+        for e, w in zip(chosen[token], weights[token]):
+            y[token] += clamped_expert(t, f"{pre}e{e}.", m["expert"]["limit"], w * h[token])
+    return y
+
+
+def layer_runs(layers, loop):
+    """(layer, number of the pass that starts with it or None), in the order they are run."""
+    start, stop, times = (loop["start"], loop["stop"], loop["times"]) if loop else (0, 0, 0)
+    runs = [(i, None) for i in range(start)]
+    for p in range(times):
+        runs += [(i, p if i == start else None) for i in range(start, stop)]
+    return runs + [(i, None) for i in range(stop, layers)]
+
+
+def desalix_forward(cfg, t, tokens, want_layers=False):
+    tokens = np.asarray(tokens)
+    positions, eps = np.arange(len(tokens)), cfg["norm"]["eps"]
+    norm = lambda x, name: rms_norm(x, eps) * float(f64(t[name]).reshape(()))
+    embedded = f64(t["embed"])[tokens] * cfg["embedding"]["scale"]
+    x, layers = embedded, []
+    for i, enters in layer_runs(len(cfg["layers"]), cfg.get("loop")):
+        layer, pre = cfg["layers"][i], f"l{i}."
+        if enters is not None:
+            x = x + (embedded if enters > 0 else 0.0) + f64(t["loop.step"])[enters]
+        y = chunked_attention_mixer(t, pre + "mix.", layer["mixer"], eps, norm(x, pre + "norm1"), positions)
+        x = x + norm(y, pre + "norm1b") * f64(t[pre + "ls1"])
+        if layer.get("mlp"):
+            y = input_weighted_mixture(t, pre + "mlp.", layer["mlp"], norm(x, pre + "norm2"))
+            x = x + norm(y, pre + "norm2b") * f64(t[pre + "ls2"])
+        layers.append(x)
+    logits = linear(t, "head", norm(x, "final.norm"))
+    return (logits, np.stack(layers)) if want_layers else logits
+
+
 def forward(cfg, t, tokens, want_layers=False):
     """Logits [T, vocab] of a whole sequence (and the residual stream after every layer)."""
     if cfg["architecture"] == "Fipuzen":
         return fipuzen_forward(cfg, t, tokens, want_layers)
     if cfg["architecture"] == "Pudadra":
         return pudadra_forward(cfg, t, tokens, want_layers)
+    if cfg["architecture"] == "Desalix":
+        return desalix_forward(cfg, t, tokens, want_layers)
     tokens = np.asarray(tokens)
     positions = np.arange(len(tokens))
     eps = cfg["norm"]["eps"]

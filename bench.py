@@ -589,7 +589,8 @@ def run_stack(args):
     head = sizes[-1]["cases"]["prefill 2 x 1024"][side]
     layers = {"zovovik": "Zovovik layers (2 x [retention, parallel])",
               "fipuzen": "Fipuzen layers (attention, latent attention, lightning, attention; 5 of 32 experts and 8 identity experts)",
-              "pudadra": "Pudadra layers (attention, attention, latent attention, attention; dense, then 4 of 32 experts and a shared one)"}
+              "pudadra": "Pudadra layers (attention, attention, latent attention, attention; dense, then 4 of 32 experts and a shared one)",
+              "desalix": "Desalix layers (3 x attention in chunks, the middle one passed twice; 4 of 32 gated experts and a shared one)"}
     return {"metric": "tokens/s/GPU", "value": head["tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps,
             "warmup": warmup, "ms_per_step": head["ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
             "dtype": "bf16", "data": "synthetic", "sizes": sizes,
@@ -604,7 +605,7 @@ def main():
     ap.add_argument("--steps", type=int, default=None, help="timed steps (default: offline 256, iteration 5)")
     ap.add_argument("--warmup", type=int, default=None, help="untimed steps (default: offline 8, iteration 2)")
     ap.add_argument("--workload", default="offline", choices=["offline", "iteration", "stack"])
-    ap.add_argument("--design", default="zovovik", choices=["zovovik", "fipuzen", "pudadra"], help="stack workload: the layer-stack model")
+    ap.add_argument("--design", default="zovovik", choices=["zovovik", "fipuzen", "pudadra", "desalix"], help="stack workload: the layer-stack model")
     ap.add_argument("--shape", default="8b", choices=["8b", "70b"],
                     help="8b: the Llama-3-8B shape the headline metric is quoted on; 70b: the Llama-3-70B shape\n"
                          "(80 layers, hidden 8192, 64 Q / 8 KV heads, FFN 28672) resident on the one GPU")

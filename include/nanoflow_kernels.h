@@ -299,7 +299,7 @@ NF_API int nf_argmax_f16(const uint16_t* logits, uint16_t* max_vals, int32_t* ar
  * tables, recurrent state and whatever enters a recurrence besides projections are fp32.  Rows are
  * padded to `ld` elements (a multiple of 8); the columns past the true width are zero and stay zero. */
 enum nf_dtype { NF_F32 = 0, NF_BF16 = 1 };
-enum nf_activation { NF_ACT_NONE = 0, NF_ACT_SQUARED_RELU = 1, NF_ACT_SILU = 2, NF_ACT_GELU = 3 /* with erf */ };
+enum nf_activation { NF_ACT_NONE = 0, NF_ACT_SQUARED_RELU = 1, NF_ACT_SILU = 2, NF_ACT_GELU = 3 /* with erf */, NF_ACT_GATED = 4 /* of pairs of columns */ };
 
 /* D [M,N] = act(A [M,K] . B^T + bias), B [N,K] (k contiguous), bias [N] in the operands' type.  bf16: K % 8 == 0,
  * N % 8 == 0, fp32 sums, launches of at most 320 rows may be split over K through `workspace`
@@ -338,27 +338,39 @@ typedef struct nf_routing {
   int32_t* tile_row;   /*   nf_routing_max_tiles(rows * top, experts, tile_rows) of them                            */
   int32_t* n_tiles;
   int tile_rows;       /* rows of an m tile (nf_grouped_tile_rows) */
+  float* row_weight;   /* [rows * top] weight of a sorted row; null: not wanted */
 } nf_routing;
 NF_API int nf_routing_max_tiles(int sorted_rows, int experts, int tile_rows);
-/* Scores s = softmax of the router's outputs (the sum of `shares` fp32 [rows, ld] slices, `outputs` of the columns);
+/* Scores s = softmax of the router's outputs (the sum of `shares` fp32 [rows, ld] slices, `outputs` of the columns), or
+ * (NF_SCORES_SIGMOID) the sigmoid of each;
  * the `top` largest of s + correction (null: none) are chosen (the smaller index where two are equal), their weights are
  * s * scale.  Outputs from `experts` on are identity experts.  groups > 1: the outputs are that many equal runs of
  * neighbours, of which only the keep_groups with the largest entries are open to choice.  always > 0: behind its
  * choices every token has that many more experts, experts .. experts + always - 1 of the grouped product, each with weight
- * sigmoid(z[outputs]).  A row of the routing's arrays is then top + always long and offsets one of experts + always.
+ * sigmoid(z[outputs]), or (always_plain) 1.  A row of the routing's arrays is then top + always long and offsets one of experts + always.
  * outputs <= 1024, experts + always <= 1024, top + always <= 64. */
+enum nf_route_scores { NF_SCORES_SOFTMAX = 0, NF_SCORES_SIGMOID = 1 };
 typedef struct nf_route_args {
   const float* z;
   int shares, ld, rows, outputs, experts, top, always, groups, keep_groups;
   const float* correction;
   float scale;
+  int scores, always_plain;
 } nf_route_args;
 NF_API int nf_route(const nf_route_args* args, const nf_routing* routing, nf_stream_t stream);
 
 /* Grouped product D_g = act(A_g . B_g^T), B [groups][N][K]; N, K and all strides multiples of 8.
  * routing.n_tiles null: every group has M rows, at a + g * a_group and d + g * d_group (elements).
  * Else the groups are the routing's experts: D holds sorted rows, A too, or (gather) the tokens themselves, M of
- * them; max_rows bounds the number of sorted rows.  act: NF_ACT_NONE, NF_ACT_GELU or NF_ACT_SQUARED_RELU. */
+ * them; max_rows bounds the number of sorted rows.  act: NF_ACT_NONE, NF_ACT_GELU, NF_ACT_SQUARED_RELU or NF_ACT_GATED.
+ * weigh != 0: a sorted row of the product is multiplied by its routing.row_weight ahead of the activation.
+ * NF_ACT_GATED: columns 2c and 2c + 1 of the product are a gate g and an up u, limited by limits[group] (null: not):
+ * with g' = min(g, limit) and u' = clamp(u, -limit, limit), column c of D, N / 2 wide, is
+ * g' * sigmoid(slope * g') * (u' + shift); ldd a multiple of 4. */
+typedef struct nf_gated_act {
+  float slope, shift;
+  const float* limits;
+} nf_gated_act;
 typedef struct nf_grouped_gemm_args {
   int dtype, act, groups, M, N, K;
   const void* a;
@@ -370,6 +382,8 @@ typedef struct nf_grouped_gemm_args {
   size_t d_group;
   nf_routing routing;
   int gather, max_rows;
+  int weigh;
+  nf_gated_act gated;
 } nf_grouped_gemm_args;
 NF_API int nf_grouped_tile_rows(int dtype, int rows, int groups);
 NF_API int nf_gemm_grouped(const nf_grouped_gemm_args* args, nf_stream_t stream);
@@ -387,7 +401,9 @@ NF_API int nf_norm_rows(int dtype, const float* x, const int32_t* row_index, con
                         int ld, nf_stream_t stream);
 /* The end of a sublayer:  x += y_scale * y_norm(y),  act = next(x) in `dtype` (null: not written).  y is the sum of `shares` fp32
  * [rows, ld] slices (y_dtype NF_F32) or one bf16 [rows, ld]; or, with routing not null, a mixture's output: the weighted sum
- * over a token's `top` choices of sorted rows of y (row stride y_ld, `dtype`) and of `identity` [rows, ld] (`dtype`). */
+ * over a token's `top` choices of sorted rows of y (row stride y_ld, `dtype`; routing->weight null: all weights 1) and of `identity`
+ * [rows, ld] (`dtype`; null where there are no identity experts).  y null: nothing is added.  Then, ahead of next: x += add, one row of
+ * ld elements (null: none), and x += table_scale * table[tokens[t]], rows of ld elements in `dtype` (null: none). */
 typedef struct nf_residual_args {
   int rows, width, ld;
   int y_dtype, shares;
@@ -400,6 +416,10 @@ typedef struct nf_residual_args {
   float* x;
   int dtype;
   void* act;
+  const float* add;
+  const void* table;
+  const int32_t* tokens;
+  float table_scale;
 } nf_residual_args;
 NF_API int nf_residual_rows(const nf_residual_args* args, nf_stream_t stream);
 /* out [rows, cols] = gelu(sum of `shares` fp32 [rows, cols] slices) (the tanh form) * table[tokens[t]][col0 + c] for
@@ -410,10 +430,10 @@ NF_API int nf_token_gate_rows(int dtype, const float* sums, int shares, const in
 NF_API int nf_gated_norm_rows(int dtype, void* o, int o_ld, const void* g, int g_ld, const float* weight, int rows, int width,
                               float eps, nf_stream_t stream);
 
-/* x [rows, ld] fp32 = embed[tokens[t]] + pos[positions[t]] (pos may be null); act = x in `dtype` (null: not
+/* x [rows, ld] fp32 = scale * embed[tokens[t]] + pos[positions[t]] (pos may be null); act = x in `dtype` (null: not
  * written).  Tables have `ld` columns in `dtype`. */
 NF_API int nf_embed_rows(int dtype, const int32_t* tokens, const int32_t* positions, const void* embed, const void* pos,
-                         float* x, void* act, int rows, int ld, nf_stream_t stream);
+                         float scale, float* x, void* act, int rows, int ld, nf_stream_t stream);
 /* Token shift: with p the row before a row of x in its request (the request's slot of shift_state
  * [slots, ld] for the first row of a portion, zeros at position 0),
  *   out[s][t] = x[t] + (p - x[t]) * mu[s],  s < n_mix; out [n_mix][rows][ld] in `dtype`, mu [n_mix][ld]. */
@@ -446,11 +466,16 @@ NF_API size_t nf_kv_page_elements(const nf_kv_layout* kv);
 /* Projected rows (q | k | v at the given columns of `proj`, row stride ld) -> per-head RMS norm of q and k
  * (weights may be null), rotation, q scaled by nothing -> q_out [rows][heads][maps][k_pad]; k and v appended to the
  * cache at the row's position.  q_temp (may be null): q of position p is multiplied by
- * 1 + coef * ln(floor((p + 1) / every) + 1) as well. */
+ * 1 + coef * ln(floor((p + 1) / every) + 1) as well.  values (may be null): a head's values are divided by their root mean square
+ * (norm != 0, eps inside the root) and turned like the rest, pairs side by side (rot.interleaved). */
 typedef struct nf_query_temperature {
   float coef;
   int every;
 } nf_query_temperature;
+typedef struct nf_value_form {
+  int norm;
+  nf_rotation rot;
+} nf_value_form;
 /* Short causal convolution over time, each column of the projected rows by itself (conv null: none), ahead of norm and
  * rotation:  y_t = sum_j weight[j] * proj_(t - taps + 1 + j), zeros before position 0.  weight [taps][ld] and state
  * [slots][taps - 1][ld] have the rows' type and columns; position p lies in row p % (taps - 1) of its request's slot.
@@ -466,23 +491,27 @@ NF_API int nf_conv_state(int dtype, const void* proj, int ld, const nf_short_con
                          int req_num, nf_stream_t stream);
 NF_API int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, int k_col, int v_col,
                          const float* q_norm, const float* k_norm, float eps, const nf_rotation* rot,
-                         const nf_query_temperature* q_temp, const nf_short_conv* conv, void* q_out, void* kv_data, const int32_t* kv_indptr, const int32_t* kv_indices,
+                         const nf_query_temperature* q_temp, const nf_value_form* values, const nf_short_conv* conv, void* q_out, void* kv_data,
+                         const int32_t* kv_indptr, const int32_t* kv_indices,
                          const int32_t* rev_input_indptr, const int32_t* positions, int rows, nf_stream_t stream);
 
 /* Attention over the cache.  A row at position p sees position j iff j <= p and (p - j < window or
- * j < keep_first); window <= 0: all of j <= p.  Scores are q.k * scale, brought within
+ * j < keep_first); window <= 0: all of j <= p.  chunk > 0: of those only the j (or j < keep_first) with floor(j / chunk) =
+ * floor(p / chunk).  Scores are q.k * scale, brought within
  * +-softcap by softcap * tanh(score / softcap) where softcap > 0; sink (may be null): exp(sink[h]) is
  * added to the denominator.  Output: heads concatenated at column out_col of out (row stride out_ld),
  * multiplied by out_scale and, with gate not null, by sigmoid(gate[row][head]) (row stride gate_ld, the layout's
  * type).  Two maps: a head's output is that of its first less map_weight times that of its second (no sinks).  head_norm
- * != 0: divided by its root mean square (head_eps inside the root) ahead of out_scale.  Rows of requests [req_begin, req_begin + req_num) of the batch are computed;
+ * != 0: divided by its root mean square (head_eps inside the root) ahead of out_scale.  out_rot (dims 0: none, else all of vdim, pairs side
+ * by side): a head's output at position p is turned by -p.  Rows of requests [req_begin, req_begin + req_num) of the batch are computed;
  * max_rows bounds their number of rows.  decode != 0: every one of those requests has exactly one row. */
 typedef struct nf_window_attention_args {
   nf_kv_layout kv;
-  int window, keep_first;
+  int window, keep_first, chunk;
   float scale, out_scale, softcap, map_weight, head_eps;
   int head_norm;
   const float* sink;
+  nf_rotation out_rot;
   const void* gate;
   int gate_ld;
   const void* q;

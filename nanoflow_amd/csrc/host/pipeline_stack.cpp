@@ -103,7 +103,7 @@ LayerStackPipeline::Buffers LayerStackPipeline::plan(const StackModel& m, int T,
       const MixtureSpec& x = *s.mixture;
       top = std::max(top, (size_t)x.perToken());
       experts = std::max(experts, (size_t)(x.experts + x.always()));
-      expert_ff = std::max(expert_ff, (size_t)x.perToken() * w.up.N);
+      expert_ff = std::max(expert_ff, (size_t)x.perToken() * w.down.K);
       tiles = std::max(tiles, (size_t)nf_routing_max_tiles(T * x.perToken(), x.experts + x.always(), 64));
       b.router_sums_bytes = std::max(b.router_sums_bytes, sums(T, w.router, kSumsMaxShares));
     }
@@ -146,7 +146,7 @@ LayerStackPipeline::Buffers LayerStackPipeline::plan(const StackModel& m, int T,
     b.latent_page_ids = (int32_t*)arena.allocBytes((size_t)m.kv_pages * 4);
   }
   for (int32_t** p : {&b.routing.choice, &b.routing.place, &b.routing.row_of}) *p = (int32_t*)arena.allocBytes(T * top * 4);
-  b.routing.weight = (float*)arena.allocBytes(T * top * 4);
+  for (float** p : {&b.routing.weight, &b.routing.row_weight}) *p = (float*)arena.allocBytes(T * top * 4);
   b.routing.offsets = (int32_t*)arena.allocBytes((experts + 1) * 4);
   b.routing.tile_group = (int32_t*)arena.allocBytes(tiles * 4);
   b.routing.tile_row = (int32_t*)arena.allocBytes(tiles * 4);
@@ -192,7 +192,7 @@ void LayerStackPipeline::config(vortexConfigData* config_data_) {
   layer_outputs = nullptr;
   const StackModelSpec& spec = model->spec;
   const int ld = spec.ld();
-  if (keep_layers) HIP_CHECK(hipMalloc(&layer_outputs, spec.layers.size() * (size_t)T * ld * sizeof(float)));
+  if (keep_layers) HIP_CHECK(hipMalloc(&layer_outputs, model->runs.size() * (size_t)T * ld * sizeof(float)));
 
   for (StackOperator* op : std::initializer_list<StackOperator*>{&embedding, &linear, &firstNorm, &residualAdd, &grouped, &router,
                                                                  &tokenGate, &gatedNorm, &latentAppend, &latentAttention, &latentExpand, &latentQueries, &tokenShift,
@@ -212,6 +212,7 @@ void LayerStackPipeline::config(vortexConfigData* config_data_) {
   // where a norm comes first the rows themselves are not read, and in fp32 they are x
   embedding.act = model->dtype == NF_BF16 && !spec.pre_norm ? buf.act : nullptr;
   embedding.ld = ld;
+  embedding.scale = (float)spec.embedding_scale;
   firstNorm.x = buf.x;
   firstNorm.norm = model->weights.layers[0].norm1;
   firstNorm.out = buf.act;
@@ -266,7 +267,7 @@ void LayerStackPipeline::setProfiling(int level) {
   profile_gemms = level > 1;
   const unsigned stride = profileStride();
   timings.layer_stride = (int)stride;
-  const size_t n = model->spec.layers.size();
+  const size_t n = model->runs.size();
   attention.enableProfiling(profiling ? n : 0, stride);
   latentAttention.enableProfiling(profiling ? n : 0, stride);
   linear.enableProfiling(profile_gemms ? 10 * n + 1 : 0, 1);
@@ -290,26 +291,50 @@ void LayerStackPipeline::update(vortexUpdateData* u) {
   output_data.sampled_tokens = batch.logit_rows;
 }
 
-LayerStackPipeline::Next LayerStackPipeline::afterLayer(int layer) const {
-  if (layer + 1 == (int)model->spec.layers.size()) return {};  // the last norm takes the rows that are wanted
-  if (model->spec.pre_norm) return {true, model->weights.layers[layer + 1].norm1};
-  return {true, {}};
+// What the first sublayer of a run reads, and what comes ahead of it.
+LayerStackPipeline::Next LayerStackPipeline::beforeRun(int run) const {
+  const LayerRun& r = model->runs[run];
+  Next n{true, {}, r.enters};
+  if (model->spec.pre_norm) n.norm = model->weights.layers[r.layer].norm1;
+  return n;
 }
 
-LayerStackPipeline::Next LayerStackPipeline::afterFeedForward(int layer) const {
-  return model->spec.token_side > 0 ? Next{true, {}} : afterLayer(layer);
+LayerStackPipeline::Next LayerStackPipeline::afterLayer(int run) const {
+  if (run + 1 == (int)model->runs.size()) return {};  // the last norm takes the rows that are wanted
+  // the stream as a layer leaves it is copied out before anything else is added
+  if (layer_outputs && model->runs[run + 1].enters >= 0) return {};
+  return beforeRun(run + 1);
 }
 
-LayerStackPipeline::Next LayerStackPipeline::afterMixer(int layer) const {
-  if (!model->spec.layers[layer].hasFeedForward()) return afterFeedForward(layer);
+LayerStackPipeline::Next LayerStackPipeline::afterFeedForward(int run) const {
+  return model->spec.token_side > 0 ? Next{true, {}} : afterLayer(run);
+}
+
+LayerStackPipeline::Next LayerStackPipeline::afterMixer(int run) const {
+  const int layer = model->runs[run].layer;
+  if (!model->spec.layers[layer].hasFeedForward()) return afterFeedForward(run);
   return model->spec.pre_norm ? Next{true, model->weights.layers[layer].norm2} : Next{true, {}};
 }
 
 void LayerStackPipeline::setNext(const Next& next) {
+  nf_residual_args& r = residualAdd.args;
+  r.add = next.enters >= 0 ? model->weights.loop_step + (size_t)next.enters * model->spec.ld() : nullptr;
+  r.table = next.enters > 0 ? model->weights.embed.ptr : nullptr;
+  r.table_scale = (float)model->spec.embedding_scale;
   residualAdd.args.next = next.norm;
   // in fp32 the residual stream is its own plain form
   const bool written = next.wanted && (next.norm.kind != NF_NORM_NONE || model->dtype == NF_BF16);
   residualAdd.args.act = written ? buf.act : nullptr;
+}
+
+// What comes ahead of a run that no sublayer's end has left.
+void LayerStackPipeline::enterRun(int run) {
+  nf_residual_args& r = residualAdd.args;
+  r.y = nullptr;
+  r.routing = nullptr;
+  r.y_norm = nf_norm{};
+  setNext(beforeRun(run));
+  residualAdd.run();
 }
 
 // Projection back to the residual width, norm, residual add, what the next sublayer reads.
@@ -334,7 +359,8 @@ void LayerStackPipeline::sublayerOut(const void* a, const DeviceMatrix& w, const
 }
 
 // Router, the chosen experts' feed-forwards, their weighted sum added to the residual stream.
-void LayerStackPipeline::mixtureOut(int layer) {
+void LayerStackPipeline::mixtureOut(int run) {
+  const int layer = model->runs[run].layer;
   const MixtureSpec& s = *model->spec.layers[layer].mixture;
   const LayerWeights& w = model->weights.layers[layer];
   const int T = batch.rows, experts = s.experts + s.always(), slots = T * s.perToken(), ld = model->spec.ld();
@@ -352,26 +378,36 @@ void LayerStackPipeline::mixtureOut(int layer) {
   z.keep_groups = s.keep_groups;
   z.correction = w.correction;
   z.scale = (float)s.scale;
+  z.scores = s.scores;
+  z.always_plain = !s.shared_gate;
   router.routing = buf.routing;
+  if (!s.weigh_input) router.routing.row_weight = nullptr;
   router.routing.tile_rows = nf_grouped_tile_rows(model->dtype, slots, experts);
   router.run();
-  grouped.experts(h, ld, w.up, buf.expert_ff, w.up.N, experts, router.routing, true, slots, s.act);
+  const int ff = w.down.K;
+  grouped.experts(h, ld, w.up, buf.expert_ff, ff, experts, router.routing, true, slots, s.gated ? NF_ACT_GATED : s.act);
+  grouped.args.weigh = s.weigh_input;
+  if (s.gated) grouped.args.gated = nf_gated_act{(float)s.gated->slope, (float)s.gated->shift, w.limits};
   grouped.run();
-  grouped.experts(buf.expert_ff, w.up.N, w.down, buf.expert_out, ld, experts, router.routing, false, slots, NF_ACT_NONE);
+  grouped.experts(buf.expert_ff, ff, w.down, buf.expert_out, ld, experts, router.routing, false, slots, NF_ACT_NONE);
   grouped.run();
   nf_residual_args& r = residualAdd.args;
-  r.routing = &router.routing;
+  nf_routing places = router.routing;
+  if (s.weigh_input) places.weight = nullptr;  // it has been in the experts' inputs
+  r.routing = &places;
   r.y = buf.expert_out;
   r.y_ld = ld;
   r.top = s.perToken();
-  r.identity = h;
-  r.y_norm = model->spec.pre_norm ? nf_norm{} : w.norm2;
-  setNext(afterFeedForward(layer));
+  r.identity = s.identity > 0 ? h : nullptr;
+  r.y_norm = w.out_norm2;
+  setNext(afterFeedForward(run));
   residualAdd.run();
+  r.routing = nullptr;
 }
 
 // The layer's input for the tokens themselves.
-void LayerStackPipeline::tokenSide(int layer) {
+void LayerStackPipeline::tokenSide(int run) {
+  const int layer = model->runs[run].layer;
   const LayerWeights& w = model->weights.layers[layer];
   linear.setSums(plain(), w.side_gate, buf.side_sums, buf.side_sums_bytes, batch.rows, kSumsMaxShares).run();
   tokenGate.sums = buf.side_sums;
@@ -383,7 +419,7 @@ void LayerStackPipeline::tokenSide(int layer) {
   tokenGate.out = buf.side;
   tokenGate.cols = w.side_gate.N;
   tokenGate.run();
-  sublayerOut(buf.side, w.side_proj, w.side_norm, afterLayer(layer));
+  sublayerOut(buf.side, w.side_proj, w.side_norm, afterLayer(run));
 }
 
 // Pages of keys and values to write out for the prompts of a layer with latent attention; 0: attend over the latents.  Counted in
@@ -409,7 +445,8 @@ int LayerStackPipeline::expandPages(int layer) const {
   return saved > tokens * product ? pages : 0;
 }
 
-void LayerStackPipeline::latentBranch(int layer) {
+void LayerStackPipeline::latentBranch(int run) {
+  const int layer = model->runs[run].layer;
   const LatentAttentionSpec& s = *model->spec.layers[layer].latent;
   const LayerWeights& lw = model->weights.layers[layer];
   const LatentAttentionWeights& w = lw.latent;
@@ -419,7 +456,7 @@ void LayerStackPipeline::latentBranch(int layer) {
   latentAppend.proj = buf.attn_proj;
   latentAppend.w = &w;
   latentAppend.q = buf.q;
-  latentAppend.kv_data = model->kv_data[layer];
+  latentAppend.kv_data = model->kv_data[run];
   // rows that attend over the latents: all of them, or the decode rows
   const int pages = expandPages(layer), rows = pages > 0 ? batch.decode : batch.rows;
   latentAppend.q_rows = rows;
@@ -429,7 +466,7 @@ void LayerStackPipeline::latentBranch(int layer) {
     x.layout = l;
     x.kv = model->expandedLayout(layer);
     x.dim_pad = w.dim_pad;
-    x.kv_data = model->kv_data[layer];
+    x.kv_data = model->kv_data[run];
     x.kv_indptr = batch.kv_indptr;
     x.kv_indices = batch.kv_indices;
     x.req_begin = batch.decode;
@@ -477,7 +514,7 @@ void LayerStackPipeline::latentBranch(int layer) {
   a.scale = (float)s.scale;
   a.q = buf.q;
   a.out = buf.latent;
-  a.kv_data = model->kv_data[layer];
+  a.kv_data = model->kv_data[run];
   a.workspace = buf.latent_ws;
   a.workspace_bytes = buf.latent_ws_bytes;
   latentAttention.prompts = pages == 0;
@@ -486,7 +523,8 @@ void LayerStackPipeline::latentBranch(int layer) {
   grouped.run();
 }
 
-void LayerStackPipeline::attentionBranch(int layer, hipStream_t s) {
+void LayerStackPipeline::attentionBranch(int run, hipStream_t s) {
+  const int layer = model->runs[run].layer;
   const AttentionSpec& a = *model->spec.layers[layer].attention;
   const LayerWeights& w = model->weights.layers[layer];
   linear_side.setStream(s);
@@ -499,15 +537,18 @@ void LayerStackPipeline::attentionBranch(int layer, hipStream_t s) {
   qkvAppend.w = &w.attention;
   qkvAppend.q_temp.reset();
   if (a.q_temp) qkvAppend.q_temp = nf_query_temperature{(float)a.q_temp->coef, a.q_temp->every};
+  qkvAppend.value_norm = a.value_norm;
   qkvAppend.conv_taps = a.conv_taps;
-  qkvAppend.conv_state = model->conv_state[layer];
+  qkvAppend.conv_state = model->conv_state[run];
   qkvAppend.q_out = buf.q;
-  qkvAppend.kv_data = model->kv_data[layer];
+  qkvAppend.kv_data = model->kv_data[run];
   qkvAppend.run();
   nf_window_attention_args& g = attention.args;
   g.kv = qkvAppend.kv;
   g.window = a.window;
   g.keep_first = a.keep_first;
+  g.chunk = a.chunk;
+  g.out_rot = w.attention.value_rot;
   g.scale = (float)a.scale;
   g.out_scale = (float)a.out_scale;
   g.softcap = (float)a.softcap;
@@ -521,11 +562,12 @@ void LayerStackPipeline::attentionBranch(int layer, hipStream_t s) {
   g.out = buf.heads;
   g.out_ld = w.out.K;
   g.out_col = 0;
-  g.kv_data = model->kv_data[layer];
+  g.kv_data = model->kv_data[run];
   attention.run();
 }
 
-void LayerStackPipeline::recurrenceBranch(int layer) {
+void LayerStackPipeline::recurrenceBranch(int run) {
+  const int layer = model->runs[run].layer;
   const LayerSpec& spec = model->spec.layers[layer];
   const RecurrenceSpec& r = *spec.recurrence;
   const LayerWeights& lw = model->weights.layers[layer];
@@ -556,7 +598,7 @@ void LayerStackPipeline::recurrenceBranch(int layer) {
     a.k_scale = (float)r.k_scale;
     a.log2_decay = w.log2_decay;
   } else {
-    tokenShift.shift_state = model->shift_state[layer];
+    tokenShift.shift_state = model->shift_state[run];
     tokenShift.mu = w.mu;
     tokenShift.run();
     auto mixed = [&](int s) { return (const void*)((const uint8_t*)buf.mix + (size_t)s * T * tokenShift.ld * es); };
@@ -584,12 +626,12 @@ void LayerStackPipeline::recurrenceBranch(int layer) {
     a.u = w.u;
     a.norm_weight = w.norm;
     a.shift_x = buf.x;
-    a.shift_state = model->shift_state[layer];
+    a.shift_state = model->shift_state[run];
     a.shift_ld = tokenShift.ld;
   }
   a.eps = (float)model->spec.eps;
   a.out_scale = (float)r.out_scale;
-  a.state = model->state[layer];
+  a.state = model->state[run];
   a.out = buf.heads;
   a.out_ld = lw.out.K;
   a.out_col = spec.attention ? spec.attention->heads * spec.attention->vdim : 0;
@@ -610,39 +652,42 @@ void LayerStackPipeline::recurrenceBranch(int layer) {
   }
 }
 
-void LayerStackPipeline::enqueueMixer(int layer) {
+void LayerStackPipeline::enqueueMixer(int run) {
+  const int layer = model->runs[run].layer;
   const LayerSpec& s = model->spec.layers[layer];
   const bool both = s.attention && s.recurrence;
   if (both) {  // two mixers that read the same rows and write different columns
     HIP_CHECK(hipEventRecord(fork, stream_all));
     HIP_CHECK(hipStreamWaitEvent(stream_side, fork, 0));
-    attentionBranch(layer, stream_side);
+    attentionBranch(run, stream_side);
     HIP_CHECK(hipEventRecord(join, stream_side));
   } else if (s.attention) {
-    attentionBranch(layer, stream_all);
+    attentionBranch(run, stream_all);
   }
-  if (s.latent) latentBranch(layer);
-  if (s.recurrence) recurrenceBranch(layer);
+  if (s.latent) latentBranch(run);
+  if (s.recurrence) recurrenceBranch(run);
   if (both) HIP_CHECK(hipStreamWaitEvent(stream_all, join, 0));
   const LayerWeights& w = model->weights.layers[layer];
-  sublayerOut(buf.heads, w.out, model->spec.pre_norm ? nf_norm{} : w.norm1, afterMixer(layer));
+  sublayerOut(buf.heads, w.out, w.out_norm1, afterMixer(run));
 }
 
 void LayerStackPipeline::enqueueIteration() {
   const StackModelSpec& spec = model->spec;
   embedding.run();
-  if (spec.pre_norm) firstNorm.run();
-  for (int i = 0; i < (int)spec.layers.size(); ++i) {
-    enqueueMixer(i);
-    const LayerWeights& w = model->weights.layers[i];
-    if (spec.layers[i].mlp) {
-      linear.set(sublayerInput(), w.up, buf.ff, batch.rows, spec.layers[i].mlp->act).run();
-      sublayerOut(buf.ff, w.down, spec.pre_norm ? nf_norm{} : w.norm2, afterFeedForward(i));
+  if (spec.pre_norm && model->runs[0].enters < 0) firstNorm.run();
+  for (int run = 0; run < (int)model->runs.size(); ++run) {
+    const LayerSpec& layer = spec.layers[model->runs[run].layer];
+    const LayerWeights& w = model->weights.layers[model->runs[run].layer];
+    if (model->runs[run].enters >= 0 && (run == 0 || layer_outputs)) enterRun(run);
+    enqueueMixer(run);
+    if (layer.mlp) {
+      linear.set(sublayerInput(), w.up, buf.ff, batch.rows, layer.mlp->act).run();
+      sublayerOut(buf.ff, w.down, w.out_norm2, afterFeedForward(run));
     }
-    if (spec.layers[i].mixture) mixtureOut(i);
-    if (spec.token_side > 0) tokenSide(i);
+    if (layer.mixture) mixtureOut(run);
+    if (spec.token_side > 0) tokenSide(run);
     if (layer_outputs)
-      HIP_CHECK(hipMemcpyAsync(layer_outputs + (size_t)i * config_data.global_batch_size * spec.ld(), buf.x,
+      HIP_CHECK(hipMemcpyAsync(layer_outputs + (size_t)run * config_data.global_batch_size * spec.ld(), buf.x,
                                (size_t)batch.rows * spec.ld() * sizeof(float), hipMemcpyDeviceToDevice, stream_all));
   }
   if (batch.logit_rows == 0) return;
@@ -655,8 +700,8 @@ vortexOutputData LayerStackPipeline::run() {
   HIP_CHECK(hipEventRecord(events[EventManager::GEMM_TIMING_START], stream_all));
   std::vector<int> sig = baseSignature();
   sig.push_back(batch.logit_rows);
-  for (int i = 0; i < (int)model->spec.layers.size(); ++i)
-    if (model->spec.layers[i].latent) sig.push_back(expandPages(i));
+  for (const LayerRun& r : model->runs)
+    if (model->spec.layers[r.layer].latent) sig.push_back(expandPages(r.layer));
   if (layer_outputs) {
     ++graph_eager;
     enqueueIteration();

@@ -27,7 +27,7 @@ public:
   int logitLd() const { return model->weights.head.N; }
   int vocab() const { return model->spec.vocab; }
   // The residual stream [rows][ld]; with keepLayers(true) before config(), also after every layer
-  // ([layers][max rows][ld]; eager iterations only).
+  // run of a layer ([runs][max rows][ld]; eager iterations only).
   const float* residual() const { return buf.x; }
   const float* layerOutputs() const { return layer_outputs; }
   int rows() const { return batch.rows; }
@@ -66,26 +66,30 @@ private:
   };
   static Buffers plan(const StackModel& m, int T, AllocationManager<half>& arena);
   void enqueueIteration();
-  void enqueueMixer(int layer);
+  // run: of a layer, in the model's order of runs
+  void enqueueMixer(int run);
   // What the row operator at the end of a sublayer leaves for the next one.
   struct Next {
     bool wanted = false;
-    nf_norm norm{};  // NF_NORM_NONE: x as it is
+    nf_norm norm{};   // NF_NORM_NONE: x as it is
+    int enters = -1;  // the pass over looped layers that it starts
   };
-  Next afterMixer(int layer) const;
-  Next afterFeedForward(int layer) const;
-  Next afterLayer(int layer) const;
+  Next beforeRun(int run) const;
+  Next afterMixer(int run) const;
+  Next afterFeedForward(int run) const;
+  Next afterLayer(int run) const;
+  void enterRun(int run);
   void setNext(const Next& next);
   // the residual stream as a sublayer reads it without a norm
   const void* plain() const { return model->dtype == NF_BF16 ? buf.act : buf.x; }
   const void* sublayerInput() const { return model->spec.pre_norm ? buf.act : plain(); }
   void sublayerOut(const void* a, const DeviceMatrix& w, const nf_norm& y_norm, const Next& next);
-  void mixtureOut(int layer);
-  void tokenSide(int layer);
+  void mixtureOut(int run);
+  void tokenSide(int run);
   int expandPages(int layer) const;
-  void latentBranch(int layer);
-  void attentionBranch(int layer, hipStream_t s);
-  void recurrenceBranch(int layer);
+  void latentBranch(int run);
+  void attentionBranch(int run, hipStream_t s);
+  void recurrenceBranch(int run);
 
   StackModel* model;
   Buffers buf;

@@ -798,7 +798,7 @@ int pllm_stack_layer_output(int layer, float* out, int* rows, int* width) {
   if (!p || g_running || !rows || !width || !p->layerOutputs())
     return fail(NF_PLLM_ERR_STATE, "pllm_stack_layer_output: no kept layers");
   const StackModelSpec& s = ActiveStackModel->spec;
-  if (layer < 0 || layer >= (int)s.layers.size()) return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_stack_layer_output: layer %d", layer);
+  if (layer < 0 || layer >= (int)s.runs().size()) return fail(NF_PLLM_ERR_INVALID_ARGUMENT, "pllm_stack_layer_output: layer %d", layer);
   *rows = p->rows();
   *width = s.width;
   if (out && *rows > 0)

@@ -32,6 +32,11 @@ StackModelSpec parseStackModel(const mini_json::Value& config) {
   require(s.width > 0 && s.vocab > 0 && s.max_positions >= 0 && !s.layers.empty(), "width, vocab and layers must be positive");
   require(s.max_positions > 0 || !s.learned_positions, "max_positions must be positive");
   require(s.token_side >= 0, "the token input's size");
+  require(!s.post_norm || s.pre_norm, "norms on both sides of a sublayer");
+  require(!s.layer_scale || s.post_norm || !s.pre_norm, "a scale per column goes with a norm of the sublayer's output");
+  require(!s.loop || (s.loop->start >= 0 && s.loop->start < s.loop->stop && s.loop->stop <= (int)s.layers.size() && s.loop->times > 0 &&
+                      (long long)(s.loop->stop - s.loop->start) * s.loop->times <= 100000),
+          "loop.start < loop.stop among the layers, loop.times at least 1");
   for (size_t i = 0; i < s.layers.size(); ++i) {
     const LayerSpec& l = s.layers[i];
     const std::string at = "layer " + std::to_string(i) + ": ";
@@ -48,7 +53,10 @@ StackModelSpec parseStackModel(const mini_json::Value& config) {
       require(a.heads > 0 && a.kv_heads > 0 && a.heads % a.kv_heads == 0, at + "query heads must be a multiple of the kv heads");
       require(a.dim > 0 && a.dim <= 256 && a.vdim > 0 && a.vdim <= 256, at + "attention head sizes must be in 1..256");
       rotation(a.rot, a.dim);
-      require(a.window >= 0 && a.keep_first >= 0, at + "window");
+      require(a.window >= 0 && a.keep_first >= 0 && a.chunk >= 0, at + "window");
+      rotation(a.value_rot, a.vdim);
+      require(!a.value_rot.scaling && (a.value_rot.dims == 0 || a.value_rot.dims == a.vdim), at + "rotated values");
+      require(a.value_rot.dims == 0 || (a.conv_taps == 0 && !a.bias), at + "rotated values of a biased or convolved projection");
       require(!a.q_temp || a.q_temp->every > 0, at + "query temperature");
       require(!a.sink || !a.unit_sink, at + "two sinks");
       require(!a.difference || (!a.sink && !a.unit_sink), at + "a sink in a difference of attentions");
@@ -76,6 +84,8 @@ StackModelSpec parseStackModel(const mini_json::Value& config) {
       require(m.ff > 0, at + "feed-forward width");
       require(m.experts > 0 && m.identity >= 0 && m.experts + m.identity <= 1024, at + "1..1024 experts, the identity experts among them");
       require(m.top > 0 && m.top <= m.experts + m.identity && m.top <= 64, at + "a token uses 1..64 of the experts");
+      require(!m.weigh_input || m.identity == 0, at + "identity experts with a weighed input");
+      require(!m.gated || (m.gated->limit >= 0 && m.gated->shared_limit >= 0), at + "limit of the experts");
       require(m.groups > 0 && m.outputs() % m.groups == 0 && m.keep_groups > 0 && m.keep_groups <= m.groups &&
                   m.top <= m.outputs() / m.groups * m.keep_groups,
               at + "equal groups of experts, the kept ones with room for the choice");
@@ -83,6 +93,16 @@ StackModelSpec parseStackModel(const mini_json::Value& config) {
     }
   }
   return s;
+}
+
+std::vector<LayerRun> StackModelSpec::runs() const {
+  std::vector<LayerRun> r;
+  const LoopSpec l = loop ? *loop : LoopSpec{0, 0, 0};
+  for (int i = 0; i < l.start; ++i) r.push_back({i, -1});
+  for (int t = 0; t < l.times; ++t)
+    for (int i = l.start; i < l.stop; ++i) r.push_back({i, i == l.start ? t : -1});
+  for (int i = l.stop; i < (int)layers.size(); ++i) r.push_back({i, -1});
+  return r;
 }
 
 // ---------------------------------------------------------------- safetensors
@@ -184,9 +204,17 @@ struct StackModel::Loader {
     return it->second;
   }
   // rows of several [n_i][k] tensors, one below the other
+  // halves > 0: in groups of `halves` rows (columns of an output projection), row c of a group's first half and row
+  // c of its second are laid beside each other -- pairs of a rotation by halves, for operators that turn neighbours
   struct Part {
     std::string name;
     int rows;
+    int halves = 0;
+    int place(int i) const {
+      if (halves == 0) return i;
+      const int c = i % halves, half = halves / 2;
+      return i - c + (c < half ? 2 * c : 2 * (c - half) + 1);
+    }
   };
   void put(uint8_t* dst, float f) {
     if (m.dtype == NF_BF16) {
@@ -226,7 +254,9 @@ struct StackModel::Loader {
     int at = 0;
     for (const auto& p : parts) {
       if (first_row) first_row->push_back(at);
-      put_rows(get(p.name, {p.rows, cols}), p.rows, cols, at, 0, K);
+      const HostTensor& t = get(p.name, {p.rows, cols});
+      if (p.halves == 0) put_rows(t, p.rows, cols, at, 0, K);
+      else for (int r = 0; r < p.rows; ++r) put_block(t, cols, r, 1, 0, cols, at + p.place(r), 0, K);
       at += p.rows;
     }
     return finish(N, K);
@@ -239,7 +269,9 @@ struct StackModel::Loader {
     start(N, K);
     int at = 0;
     for (const auto& p : parts) {
-      put_rows(get(p.name, {rows, p.rows}), rows, p.rows, 0, at, K);
+      const HostTensor& t = get(p.name, {rows, p.rows});
+      if (p.halves == 0) put_rows(t, rows, p.rows, 0, at, K);
+      else for (int c = 0; c < p.rows; ++c) put_block(t, p.rows, 0, rows, c, 1, 0, at + p.place(c), K);
       at += p.rows;
     }
     return finish(N, K);
@@ -250,8 +282,17 @@ struct StackModel::Loader {
     for (size_t i = 0; i < parts.size(); ++i) put_rows(get(parts[i].name, {parts[i].rows}), 1, parts[i].rows, 0, at[i], N);
     return finish(1, N).ptr;
   }
-  nf_norm norm(const std::string& name, nf_norm_kind kind, double scale = 1) {
+  // `columns`: a tensor that multiplies the weights column by column
+  nf_norm norm(const std::string& name, nf_norm_kind kind, double scale = 1, const std::string& columns = "") {
     const int W = m.spec.width, ld = m.spec.ld();
+    if (m.spec.scalar_norms || !columns.empty()) {
+      std::vector<float> v((size_t)ld, 0.f);
+      const HostTensor& w = m.spec.scalar_norms ? get(name, {}) : get(name, {W});
+      const HostTensor* by = columns.empty() ? nullptr : &get(columns, {W});
+      for (int c = 0; c < W; ++c)
+        v[c] = (float)((element(w, m.spec.scalar_norms ? 0 : c) + m.spec.norm_offset) * scale * (by ? element(*by, c) : 1.0));
+      return nf_norm{kind, upload(v), kind == NF_NORM_LAYER ? vectors({name + ".b"}, {W}, W, ld) : nullptr, (float)m.spec.eps};
+    }
     return nf_norm{kind, vectors({name}, {W}, W, ld, m.spec.norm_offset, scale), kind == NF_NORM_LAYER ? vectors({name + ".b"}, {W}, W, ld) : nullptr, (float)m.spec.eps};
   }
 
@@ -297,18 +338,31 @@ struct StackModel::Loader {
   void mixture(const MixtureSpec& s, const std::string& p, LayerWeights& w) {
     const int W = m.spec.width, columns = s.expertFf(), ff = pad8(columns), K = pad8(W), all = s.experts + s.always();
     auto share = [&](int j) { return std::max(0, std::min(columns, s.shared_ff - j * columns)); };  // of the shared expert's columns
-    start((size_t)all * ff, K);
-    for (int e = 0; e < s.experts; ++e) put_rows(get(p + "e" + std::to_string(e) + ".up", {s.ff, W}), s.ff, W, e * ff, 0, K);
-    for (int j = 0; j < s.always(); ++j) put_block(get(p + "shared.up", {s.shared_ff, W}), W, j * columns, share(j), 0, W, (s.experts + j) * ff, 0, K);
-    w.up = finish(ff, K);
+    // gate and up: a column's two rows beside each other
+    const std::vector<std::string> first = s.gated ? std::vector<std::string>{"gate", "up"} : std::vector<std::string>{"up"};
+    const int n = (int)first.size();
+    start((size_t)all * n * ff, K);
+    for (int i = 0; i < n; ++i) {
+      auto rows = [&](const HostTensor& t, int from, int count, int expert) {
+        for (int r = 0; r < count; ++r) put_block(t, W, from + r, 1, 0, W, (expert * ff + r) * n + i, 0, K);
+      };
+      for (int e = 0; e < s.experts; ++e) rows(get(p + "e" + std::to_string(e) + "." + first[i], {s.ff, W}), 0, s.ff, e);
+      for (int j = 0; j < s.always(); ++j) rows(get(p + "shared." + first[i], {s.shared_ff, W}), j * columns, share(j), s.experts + j);
+    }
+    w.up = finish(n * ff, K);
     start((size_t)all * K, ff);
     for (int e = 0; e < s.experts; ++e) put_rows(get(p + "e" + std::to_string(e) + ".down", {W, s.ff}), W, s.ff, e * K, 0, ff);
     for (int j = 0; j < s.always(); ++j)
       put_block(get(p + "shared.down", {W, s.shared_ff}), s.shared_ff, 0, W, j * columns, share(j), (s.experts + j) * K, 0, ff);
     w.down = finish(K, ff);
     std::vector<Part> router{{p + "router", s.outputs()}};
-    if (s.always() > 0) router.push_back({p + "shared.sg", 1});
+    if (s.always() > 0 && s.shared_gate) router.push_back({p + "shared.sg", 1});
     w.router = matrix(router, W);
+    if (s.gated) {
+      std::vector<float> limits((size_t)all, (float)s.gated->limit);
+      for (int j = 0; j < s.always(); ++j) limits[s.experts + j] = (float)s.gated->shared_limit;
+      w.limits = upload(limits);
+    }
     if (s.correction) w.correction = vectors({p + "correction"}, {s.outputs()}, s.outputs(), s.outputs());
   }
   // weights [channels][taps] of convolutions on the columns from at[i] on -> [taps][N] in the activations' type
@@ -410,9 +464,13 @@ nf_kv_layout StackModel::kvLayout(int layer) const {
   return nf_kv_layout{dtype, a.heads, a.kv_heads, a.dim, a.vdim, (a.dim + 31) / 32 * 32, (a.vdim + 15) / 16 * 16, page_size, a.maps()};
 }
 
+// Values that are turned by halves are kept with their pairs side by side: the value projection's rows and the output
+// projection's columns are laid out for it.
+static int halves_of_values(const AttentionSpec& a) { return a.value_rot.dims > 0 && !a.value_rot.interleaved ? a.vdim : 0; }
+
 StackModel::StackModel(const StackModelSpec& spec_, const HostTensors& tensors, nf_dtype dtype_, int kv_pages_, int page_size_,
                        int state_slots_)
-    : spec(spec_), dtype(dtype_), kv_pages(kv_pages_), page_size(page_size_), state_slots(state_slots_) {
+    : spec(spec_), dtype(dtype_), kv_pages(kv_pages_), page_size(page_size_), state_slots(state_slots_), runs(spec_.runs()) {
   const int W = spec.width, ld = spec.ld();
   Loader L{*this, tensors, {}};
   try {
@@ -424,10 +482,17 @@ StackModel::StackModel(const StackModelSpec& spec_, const HostTensors& tensors, 
     if (spec.token_side > 0) weights.side_embed = L.matrix({{"side.embed", spec.vocab}}, spec.token_side * (int)spec.layers.size());
     const int n = (int)spec.layers.size();
     weights.layers.resize(n);
-    kv_data.assign(n, nullptr);
-    state.assign(n, nullptr);
-    shift_state.assign(n, nullptr);
-    conv_state.assign(n, nullptr);
+    if (spec.loop) {
+      const HostTensor& steps = L.get("loop.step", {spec.loop->times, W});
+      std::vector<float> v((size_t)spec.loop->times * ld, 0.f);
+      for (int t = 0; t < spec.loop->times; ++t)
+        for (int c = 0; c < W; ++c) v[(size_t)t * ld + c] = element(steps, (size_t)t * W + c);
+      weights.loop_step = L.upload(v);
+    }
+    kv_data.assign(runs.size(), nullptr);
+    state.assign(runs.size(), nullptr);
+    shift_state.assign(runs.size(), nullptr);
+    conv_state.assign(runs.size(), nullptr);
     for (int i = 0; i < n; ++i) {
       const LayerSpec& s = spec.layers[i];
       LayerWeights& w = weights.layers[i];
@@ -438,7 +503,7 @@ StackModel::StackModel(const StackModelSpec& spec_, const HostTensors& tensors, 
         const std::string p = l + a.prefix;
         std::vector<int> at;
         std::vector<Loader::Part> parts{
-            {p + "q", a.heads * a.maps() * a.dim}, {p + "k", a.kv_heads * a.maps() * a.dim}, {p + "v", a.kv_heads * a.vdim}};
+            {p + "q", a.heads * a.maps() * a.dim}, {p + "k", a.kv_heads * a.maps() * a.dim}, {p + "v", a.kv_heads * a.vdim, halves_of_values(a)}};
         if (a.head_gate) parts.push_back({p + "g", a.heads});
         w.attention.qkv = L.matrix(parts, W, &at);
         if (a.head_gate) w.attention.g_col = at[3];
@@ -457,12 +522,12 @@ StackModel::StackModel(const StackModelSpec& spec_, const HostTensors& tensors, 
         if (a.conv_taps > 0) {
           w.attention.conv = L.taps({{p + "q.conv", parts[0].rows}, {p + "k.conv", parts[1].rows}, {p + "v.conv", parts[2].rows}}, at,
                                     a.conv_taps, w.attention.qkv.N);
-          conv_state[i] = allocate((size_t)state_slots * (a.conv_taps - 1) * w.attention.qkv.N * elementBytes());
         }
         w.attention.rot = rotation(a.rot);
-        out_parts.push_back({p + "o", a.heads * a.vdim});
-        const nf_kv_layout kv = kvLayout(i);
-        kv_data[i] = allocate((size_t)kv_pages * nf_kv_page_elements(&kv) * elementBytes());
+        RotationSpec turned = a.value_rot;
+        turned.interleaved = true;
+        w.attention.value_rot = rotation(turned);
+        out_parts.push_back({p + "o", a.heads * a.vdim, halves_of_values(a)});
       }
       if (s.recurrence) {
         const RecurrenceSpec& r = *s.recurrence;
@@ -498,20 +563,18 @@ StackModel::StackModel(const StackModelSpec& spec_, const HostTensors& tensors, 
           w.recurrence.u = L.vectors({p + "u"}, {r.heads, r.dim}, qk, qk);
           w.recurrence.norm = L.vectors({p + "norm"}, {vg}, vg, vg);
           w.recurrence.mu = L.vectors({p + "mu.r", p + "mu.k", p + "mu.v", p + "mu.g", p + "mu.w"}, {W}, W, ld);
-          shift_state[i] = static_cast<float*>(allocate((size_t)state_slots * ld * sizeof(float)));
         }
         out_parts.push_back({p + "o", vg});
-        state[i] = static_cast<float*>(
-            allocate((size_t)state_slots * r.heads * nf_recurrence_state_elements(r.dim, r.vdim) * sizeof(float)));
       }
-      if (s.latent) {
-        L.latent(*s.latent, l + s.latent->prefix, w);
-        kv_data[i] = allocate((size_t)kv_pages * page_size * latentLayout(i).row_ld * elementBytes());
-      } else {
-        w.out = L.columns(out_parts, W);
-      }
-      w.norm1 = L.norm(l + "norm1", spec.norm);
-      if (s.hasFeedForward()) w.norm2 = L.norm(l + "norm2", spec.norm);
+      if (s.latent) L.latent(*s.latent, l + s.latent->prefix, w);
+      else w.out = L.columns(out_parts, W);
+      auto norms = [&](const std::string& name, const std::string& scale, nf_norm& in, nf_norm& out) {
+        const std::string columns = spec.layer_scale ? l + scale : "";
+        if (spec.pre_norm) in = L.norm(l + name, spec.norm);
+        if (!spec.pre_norm || spec.post_norm) out = L.norm(l + name + (spec.pre_norm ? "b" : ""), spec.norm, 1, columns);
+      };
+      norms("norm1", "ls1", w.norm1, w.out_norm1);
+      if (s.hasFeedForward()) norms("norm2", "ls2", w.norm2, w.out_norm2);
       if (s.mlp) {
         w.up = L.matrix({{l + "mlp.up", s.mlp->ff}}, W);
         w.down = L.matrix({{l + "mlp.down", W}}, s.mlp->ff);
@@ -521,6 +584,23 @@ StackModel::StackModel(const StackModelSpec& spec_, const HostTensors& tensors, 
         w.side_gate = L.matrix({{l + "side.gate", spec.token_side}}, W);
         w.side_proj = L.matrix({{l + "side.proj", W}}, spec.token_side);
         w.side_norm = L.norm(l + "side.norm", NF_NORM_RMS);
+      }
+    }
+    for (size_t r = 0; r < runs.size(); ++r) {  // caches and states
+      const int i = runs[r].layer;
+      const LayerSpec& s = spec.layers[i];
+      if (s.attention) {
+        const nf_kv_layout kv = kvLayout(i);
+        kv_data[r] = allocate((size_t)kv_pages * nf_kv_page_elements(&kv) * elementBytes());
+        if (s.attention->conv_taps > 0)
+          conv_state[r] = allocate((size_t)state_slots * (s.attention->conv_taps - 1) * weights.layers[i].attention.qkv.N * elementBytes());
+      }
+      if (s.latent) kv_data[r] = allocate((size_t)kv_pages * page_size * latentLayout(i).row_ld * elementBytes());
+      if (s.recurrence) {
+        state[r] = static_cast<float*>(allocate((size_t)state_slots * s.recurrence->heads *
+                                                nf_recurrence_state_elements(s.recurrence->dim, s.recurrence->vdim) * sizeof(float)));
+        if (s.recurrence->kind == NF_RECURRENCE_TOKEN_DECAY)
+          shift_state[r] = static_cast<float*>(allocate((size_t)state_slots * ld * sizeof(float)));
       }
     }
   } catch (...) {

@@ -41,6 +41,7 @@ struct AttentionSpec {
   int heads = 0, kv_heads = 0, dim = 0, vdim = 0;
   double scale = 1;
   int window = 0, keep_first = 0;  // window 0: everything before
+  int chunk = 0;                   // positions see their own run of this many only, counted from 0; 0: all of one
   bool qk_norm = false;
   bool bias = false;       // of q, k and v
   bool sink = false;       // a score per head in the denominator, from a tensor
@@ -52,6 +53,8 @@ struct AttentionSpec {
   bool head_norm = false;  // a head's output divided by its root mean square
   int maps() const { return difference ? 2 : 1; }
   RotationSpec rot;
+  bool value_norm = false;  // a value divided by its root mean square
+  RotationSpec value_rot;   // of the values by their positions; a head's output is turned back by the query's
   std::optional<QueryTemperatureSpec> q_temp;
   double out_scale = 1;
 };
@@ -89,13 +92,21 @@ struct MlpSpec {
 // chooses from the keep_groups best of `groups` runs of outputs.  shared_ff > 0: one more feed-forward for every
 // token, times the sigmoid of a projection.  It is held as always() experts of expertFf() columns beside the others, each
 // a share of its columns: activations are taken column by column, so the shares' outputs add up to its own.
+// With `gated` an expert has gate and up projections (nf_gated_act), each bounded by the expert's limit.
 struct MixtureSpec {
   int experts = 0, identity = 0, top = 0, ff = 0;
   double scale = 1;
   nf_activation act = NF_ACT_GELU;
   int groups = 1, keep_groups = 1;
   bool correction = true;  // of the scores, where the choice is made
+  nf_route_scores scores = NF_SCORES_SOFTMAX;
+  bool weigh_input = false;  // a choice's weight multiplies the expert's input, not its output
   int shared_ff = 0;
+  bool shared_gate = true;   // false: the shared feed-forward is added as it is
+  struct Gated {
+    double slope = 1, shift = 0, limit = 0, shared_limit = 0;
+  };
+  std::optional<Gated> gated;
   int outputs() const { return experts + identity; }
   int always() const {
     const int room = 64 - top < 1024 - experts ? 64 - top : 1024 - experts, shares = (shared_ff + ff - 1) / ff;
@@ -114,6 +125,15 @@ struct LayerSpec {
   std::optional<MixtureSpec> mixture;
   bool hasFeedForward() const { return mlp || mixture; }
 };
+// Layers [start, stop) run `times` times in a row, each pass with caches and states of its own.  Ahead of a pass its row of the
+// tensor loop.step is added to the stream, and ahead of every pass but the first the embedding output as well.
+struct LoopSpec {
+  int start = 0, stop = 0, times = 1;
+};
+// One run of a layer; enters: the pass that starts with it, -1: none.
+struct LayerRun {
+  int layer = 0, enters = -1;
+};
 
 struct StackModelSpec {
   std::string architecture;
@@ -123,12 +143,18 @@ struct StackModelSpec {
   bool learned_positions = false;
   nf_norm_kind norm = NF_NORM_RMS;  // of the residual stream (layer norms have a bias)
   bool pre_norm = false;            // x += f(norm(x)); else x += norm(f(x))
+  bool post_norm = false;           // with pre_norm: x += normb(f(norm(x)))
+  bool scalar_norms = false;        // the stream's norms have one weight for all columns
+  bool layer_scale = false;         // what a sublayer adds is multiplied column by column, after its norm
+  double embedding_scale = 1;
   double norm_offset = 0;           // added to the stored weights of the stream's norms
   double residual_scale = 1;        // of what a sublayer adds
   bool tied_head = false;           // the output projection is the embedding table
   double logit_scale = 1;
   int token_side = 0;               // size of the token input at the end of every layer, 0: none
   std::vector<LayerSpec> layers;
+  std::optional<LoopSpec> loop;
+  std::vector<LayerRun> runs() const;
   int ld() const { return (width + 7) / 8 * 8; }
   bool hasAttention() const {
     for (const auto& l : layers)
@@ -192,7 +218,7 @@ struct AttentionWeights {
   float *q_norm = nullptr, *k_norm = nullptr, *sink = nullptr;
   void* conv = nullptr;  // [taps][columns of qkv]
   float map_weight = 0;
-  nf_rotation rot{};
+  nf_rotation rot{}, value_rot{};  // value_rot: pairs side by side, whatever the design's layout
 };
 struct LatentAttentionWeights {
   DeviceMatrix proj;  // q unrotated [heads][dim_pad] | q rotated [heads][rot_dim] | latent | rotated key part
@@ -220,12 +246,15 @@ struct LayerWeights {
   DeviceMatrix up, down;               // of a mixture: per expert, one below the other
   DeviceMatrix router;
   float* correction = nullptr;
-  nf_norm norm1{}, norm2{};
+  nf_norm norm1{}, norm2{};            // pre_norm: of the sublayers' inputs
+  nf_norm out_norm1{}, out_norm2{};    // of their outputs
+  float* limits = nullptr;             // of a gated mixture's experts
   DeviceMatrix side_gate, side_proj;
   nf_norm side_norm{};
 };
 struct StackWeights {
   DeviceMatrix embed, pos, head, side_embed;
+  float* loop_step = nullptr;  // [times][ld]
   nf_norm final_norm{};
   std::vector<LayerWeights> layers;
 };
@@ -243,8 +272,9 @@ public:
   const StackModelSpec spec;
   const nf_dtype dtype;
   const int kv_pages, page_size, state_slots;
+  const std::vector<LayerRun> runs;
   StackWeights weights;
-  // per layer; null where the layer has none
+  // per run of a layer; null where the layer has none
   std::vector<void*> kv_data;       // kv_pages pages (nf_kv_layout, nf_latent_layout)
   std::vector<float*> state;        // [state_slots][heads][dim_pad][vdim_pad]
   std::vector<float*> shift_state;  // [state_slots][ld]

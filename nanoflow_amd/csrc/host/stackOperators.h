@@ -79,8 +79,9 @@ struct StackEmbedding : public StackOperator {
   float* x = nullptr;
   void* act = nullptr;
   int ld = 0;
+  float scale = 1;
   void work() override {
-    NF_KERNEL_CHECK(nf_embed_rows(dtype, batch->tokens, batch->positions, w->embed.ptr, w->pos.ptr, x, act, batch->rows, ld, stream));
+    NF_KERNEL_CHECK(nf_embed_rows(dtype, batch->tokens, batch->positions, w->embed.ptr, w->pos.ptr, scale, x, act, batch->rows, ld, stream));
   }
 };
 
@@ -93,14 +94,15 @@ struct StackNorm : public StackOperator {
   void work() override { NF_KERNEL_CHECK(nf_norm_rows(dtype, x, nullptr, &norm, out, batch->rows, width, ld, stream)); }
 };
 
-// The end of a sublayer: its output, normed or put together from experts, added to the residual stream, and what the next
-// sublayer reads.
+// The end of a sublayer: its output, normed or put together from experts, added to the residual stream, what a pass over
+// layers starts with, and what the next sublayer reads.
 struct StackResidual : public StackOperator {
   nf_residual_args args{};
   void work() override {
     nf_residual_args a = args;
     a.rows = batch->rows;
     a.dtype = dtype;
+    a.tokens = batch->tokens;
     NF_KERNEL_CHECK(nf_residual_rows(&a, stream));
   }
 };
@@ -238,13 +240,15 @@ struct StackQKVAppend : public StackOperator {
   const AttentionWeights* w = nullptr;
   float eps = 0;
   std::optional<nf_query_temperature> q_temp;
+  bool value_norm = false;
   int conv_taps = 0;
   void* conv_state = nullptr;
   void *q_out = nullptr, *kv_data = nullptr;
   void work() override {
+    const nf_value_form values{value_norm, w->value_rot};
     const nf_short_conv conv{conv_taps, w->conv, conv_state, batch->input_indptr, batch->state_slots};
     NF_KERNEL_CHECK(nf_qkv_append(&kv, proj, ld, w->q_col, w->k_col, w->v_col, w->q_norm, w->k_norm, eps, &w->rot,
-                                  q_temp ? &*q_temp : nullptr, conv_taps > 0 ? &conv : nullptr, q_out, kv_data, batch->kv_indptr,
+                                  q_temp ? &*q_temp : nullptr, &values, conv_taps > 0 ? &conv : nullptr, q_out, kv_data, batch->kv_indptr,
                                   batch->kv_indices, batch->rev_input_indptr, batch->positions, batch->rows, stream));
     if (conv_taps > 1 && batch->prefill > 0)
       NF_KERNEL_CHECK(nf_conv_state(kv.dtype, proj, ld, &conv, batch->positions, batch->decode, batch->prefill, stream));

@@ -24,11 +24,19 @@ __device__ __forceinline__ float f32_activation(float v) {
   }
 }
 
+// What becomes of a row of the product before it is stored: multiplied by row_scale[m] (null: not); with NF_ACT_GATED the
+// columns are pairs of a gate and an up (nf_gated_act) and D has half as many.
+struct RowEpilogue {
+  const float* row_scale = nullptr;
+  float slope = 1.f, shift = 0.f, limit = INFINITY;
+};
+
 // The tile at (m0, n0).  Row m of A is row a_rows[m] where a_rows is not null.
 template <int kAct>
 __device__ __forceinline__ void gemm_f32_tile(const float* __restrict__ A, const float* __restrict__ B, const float* __restrict__ bias,
                                               float* __restrict__ D, int M, int N, int K, int lda, int ldb, int ldd,
-                                              const int32_t* __restrict__ a_rows, int m0, int n0) {
+                                              const int32_t* __restrict__ a_rows, int m0, int n0,
+                                              const RowEpilogue& ep = {}) {
   __shared__ __attribute__((aligned(16))) float sa[kF32Tile * kF32Pitch], sb[kF32Tile * kF32Pitch];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int wm = (wave >> 1) * 32, wn = (wave & 1) * 32, l16 = lane & 15, lq = lane >> 4;
@@ -70,6 +78,16 @@ __device__ __forceinline__ void gemm_f32_tile(const float* __restrict__ A, const
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int m = m0 + wm + i * 16 + lq * 4 + r, n = n0 + wn + j * 16 + l16;
+        if (kAct == NF_ACT_GATED || ep.row_scale) {
+          const float v = acc[i][j][r] * (ep.row_scale && m < M ? ep.row_scale[m] : 1.f);
+          if constexpr (kAct == NF_ACT_GATED) {
+            const float up = fminf(fmaxf(__shfl_xor(v, 1, 64), -ep.limit), ep.limit), gate = fminf(v, ep.limit);
+            if (m < M && n < N && n % 2 == 0) D[(size_t)m * ldd + n / 2] = gate / (1.f + expf(-ep.slope * gate)) * (up + ep.shift);
+          } else if (m < M && n < N) {
+            D[(size_t)m * ldd + n] = f32_activation<kAct>(v);
+          }
+          continue;
+        }
         if (m < M && n < N) D[(size_t)m * ldd + n] = f32_activation<kAct>(acc[i][j][r] + (bias ? bias[n] : 0.f));
       }
 }

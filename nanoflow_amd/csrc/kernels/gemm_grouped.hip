@@ -38,9 +38,16 @@ __global__ __launch_bounds__(WM * WN * 64) void gemm_grouped_kernel(nf_grouped_g
   const int32_t* rows = routed && a.gather ? a.routing.row_of + t.row0 : nullptr;
   const uint16_t* A = (const uint16_t*)a.a + (routed ? (rows ? 0 : t.row0 * a.lda) : (size_t)t.group * a.a_group);
   uint16_t* D = (uint16_t*)a.d + (routed ? t.row0 * a.ldd : (size_t)t.group * a.d_group);
+  GroupEpilogue ep;
+  if (routed && a.weigh) ep.row_scale = a.routing.row_weight + t.row0;
+  if constexpr (std::is_same_v<E, BF16Gated>) {
+    ep.slope = a.gated.slope;
+    ep.shift = a.gated.shift;
+    if (a.gated.limits) ep.limit = a.gated.limits[t.group];
+  }
   gemm_tile<E, BM, BN, WM, WN, false, true, false, true>(A, (const uint16_t*)a.b + (size_t)t.group * a.N * a.K, nullptr, nullptr, D,
                                                          t.rows, a.N, a.K, 1.f, 0.f, a.N, t.m_base, t.n_tile * BN, a.lda, a.K, a.ldd,
-                                                         rows, a.M);
+                                                         rows, a.M, ep);
 }
 
 template <int kAct>
@@ -51,8 +58,15 @@ __global__ __launch_bounds__(256) void gemm_grouped_f32_kernel(nf_grouped_gemm_a
   const int32_t* rows = routed && a.gather ? a.routing.row_of + t.row0 : nullptr;
   const float* A = (const float*)a.a + (routed ? (rows ? 0 : t.row0 * a.lda) : (size_t)t.group * a.a_group);
   float* D = (float*)a.d + (routed ? t.row0 * a.ldd : (size_t)t.group * a.d_group);
+  RowEpilogue ep;
+  if (routed && a.weigh) ep.row_scale = a.routing.row_weight + t.row0;
+  if constexpr (kAct == NF_ACT_GATED) {
+    ep.slope = a.gated.slope;
+    ep.shift = a.gated.shift;
+    if (a.gated.limits) ep.limit = a.gated.limits[t.group];
+  }
   gemm_f32_tile<kAct>(A, (const float*)a.b + (size_t)t.group * a.N * a.K, nullptr, D, t.rows, a.N, a.K, a.lda, a.K, a.ldd, rows, t.m_base,
-                      t.n_tile * kF32Tile);
+                      t.n_tile * kF32Tile, ep);
 }
 
 unsigned grid_of(const nf_grouped_gemm_args& a, int bm, int tiles_n) {
@@ -100,13 +114,14 @@ int nf_gemm_grouped(const nf_grouped_gemm_args* args, nf_stream_t stream) {
   NF_REQUIRE(args, "%s: null pointer", who);
   const nf_grouped_gemm_args& a = *args;
   NF_REQUIRE(a.dtype == NF_F32 || a.dtype == NF_BF16, "%s: unknown dtype %d", who, a.dtype);
-  NF_REQUIRE(a.act == NF_ACT_NONE || a.act == NF_ACT_GELU || a.act == NF_ACT_SQUARED_RELU, "%s: unknown activation %d", who, a.act);
-  NF_REQUIRE(a.groups > 0 && a.M >= 0 && a.N > 0 && a.K > 0 && a.N % 8 == 0 && a.K % 8 == 0 && a.lda >= a.K && a.ldd >= a.N && a.lda % 8 == 0 &&
+  NF_REQUIRE(a.act == NF_ACT_NONE || a.act == NF_ACT_GELU || a.act == NF_ACT_SQUARED_RELU || a.act == NF_ACT_GATED, "%s: unknown activation %d", who, a.act);
+  NF_REQUIRE(a.groups > 0 && a.M >= 0 && a.N > 0 && a.K > 0 && a.N % 8 == 0 && a.K % 8 == 0 && a.lda >= a.K && a.ldd >= (a.act == NF_ACT_GATED ? a.N / 2 : a.N) && a.lda % 8 == 0 &&
                  a.ldd % 8 == 0 && a.a_group % 8 == 0 && a.d_group % 8 == 0,
              "%s: bad shape: %d groups, M=%d N=%d K=%d, strides %d %d", who, a.groups, a.M, a.N, a.K, a.lda, a.ldd);
   const bool routed = a.routing.n_tiles != nullptr;
   NF_REQUIRE(!routed || (a.routing.tile_group && a.routing.tile_row && a.routing.offsets && a.max_rows >= 0 && (!a.gather || a.routing.row_of)),
              "%s: incomplete routing", who);
+  NF_REQUIRE(!a.weigh || (routed && a.routing.row_weight), "%s: no weights of the sorted rows", who);
   if (a.M == 0 || (routed && a.max_rows == 0)) return NF_OK;
   NF_REQUIRE(a.a && a.b && a.d, "%s: null pointer", who);
   NF_REQUIRE(((uintptr_t)a.a | (uintptr_t)a.b | (uintptr_t)a.d) % 16 == 0, "%s: operands must be 16-byte aligned", who);
@@ -120,11 +135,13 @@ int nf_gemm_grouped(const nf_grouped_gemm_args* args, nf_stream_t stream) {
     const int tiles_n = (a.N + kF32Tile - 1) / kF32Tile;
     auto kern = a.act == NF_ACT_GELU           ? gemm_grouped_f32_kernel<NF_ACT_GELU>
                 : a.act == NF_ACT_SQUARED_RELU ? gemm_grouped_f32_kernel<NF_ACT_SQUARED_RELU>
+                : a.act == NF_ACT_GATED        ? gemm_grouped_f32_kernel<NF_ACT_GATED>
                                                : gemm_grouped_f32_kernel<NF_ACT_NONE>;
     kern<<<grid_of(a, kF32Tile, tiles_n), 256, 0, s>>>(a, tiles_n);
     return check_launch(who);
   }
   if (a.act == NF_ACT_SQUARED_RELU) return dispatch_grouped<BF16SquaredRelu>(a, tile_rows, s);
+  if (a.act == NF_ACT_GATED) return dispatch_grouped<BF16Gated>(a, tile_rows, s);
   return a.act == NF_ACT_GELU ? dispatch_grouped<BF16Gelu>(a, tile_rows, s) : dispatch_grouped<BF16>(a, tile_rows, s);
 }
 

@@ -131,6 +131,20 @@ struct BF16SquaredRelu : BF16 {
   }
 };
 
+// Pairs of neighbouring columns, a gate and an up, made one (nf_gated_act); D has half the product's columns.  Grouped products.
+struct BF16Gated : BF16 {};
+
+// What a grouped product does with a row ahead of its activation, and the constants of BF16Gated.
+struct GroupEpilogue {
+  const float* row_scale = nullptr;  // of the group's rows; null: 1
+  float slope = 1.f, shift = 0.f, limit = INFINITY;
+  __device__ __forceinline__ float gated(float g, float u) const {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g * __builtin_amdgcn_rcpf(1.f + __expf(-slope * g)) * (u + shift);
+  }
+};
+
 // SiLU(g)*u on values already rounded to the storage type, as the reference's dual epilogue
 // computes it (in fp16 there).
 template <class E>
@@ -156,7 +170,8 @@ __device__ __forceinline__ void gemm_tile(
     const uint16_t* __restrict__ A, const uint16_t* __restrict__ B0,
     const uint16_t* __restrict__ B1, const uint16_t* C, uint16_t* D,
     int M, int N, int K, float alpha, float beta, const int ldc, const int m_base, const int n_base,
-    const int lda, const int group_ldb = 0, const int group_ldd = 0, const int32_t* a_rows = nullptr, const int a_total = 0) {
+    const int lda, const int group_ldb = 0, const int group_ldd = 0, const int32_t* a_rows = nullptr, const int a_total = 0,
+    const GroupEpilogue& group = {}) {
   static_assert(!kGroup || (kBCol && !kDual && !kPartial), "grouped products: plain, k-contiguous weights");
   const int ldb = kGroup ? group_ldb : lda, ldd = kGroup ? group_ldd : N;
   constexpr int NB = kDual ? 2 : 1;
@@ -616,14 +631,16 @@ __device__ __forceinline__ void gemm_tile(
     // out-of-range offset), so the pass has no branches and all its loads are in flight together.
     const int gm0 = m_base + wm * (BM / WM) + i * 32, gn0 = n_base + wn * CW;
     const int rows = M - gm0 < 32 ? M - gm0 : 32;
-    const int recs = rows > 0 ? ((rows - 1) * ldd + N) * 2 : 0;
+    constexpr bool kPairs = std::is_same_v<E, BF16Gated>;
+    static_assert(!kPairs || kGroup, "gate and up side by side: grouped products");
+    const int recs = rows > 0 ? ((rows - 1) * ldd + (kPairs ? N / 2 : N)) * 2 : 0;
     const size_t row0 = (size_t)(rows > 0 ? gm0 : 0) * ldd;
     const __amdgpu_buffer_rsrc_t d_rsrc = __builtin_amdgcn_make_buffer_rsrc(D + row0, 0, recs, 0x00020000);
     uint32_t off[ITER];
 #pragma unroll
     for (int it = 0; it < ITER; ++it) {
       const int c = it * 64 + lane, gn = gn0 + (c % CPR) * 4;
-      off[it] = gn < N ? (uint32_t)((c / CPR) * ldd + gn) * 2u : kOob;
+      off[it] = gn < N ? (uint32_t)((c / CPR) * ldd + (kPairs ? gn / 2 : gn)) * 2u : kOob;
     }
     u32v2_t cv[ITER];
     if constexpr (!kDual && !kPartial) {
@@ -671,6 +688,21 @@ __device__ __forceinline__ void gemm_tile(
     for (int it = 0; it < ITER; ++it) {
       const int c = it * 64 + lane;
       a4[it] = *reinterpret_cast<const float4_t*>(ep + (c / CPR) * ROWP + (c % CPR) * 16);
+    }
+    if constexpr (kGroup) {
+      if (group.row_scale) {
+#pragma unroll
+        for (int it = 0; it < ITER; ++it) {
+          const int r = (it * 64 + lane) / CPR;
+          a4[it] *= r < rows ? group.row_scale[gm0 + r] : 0.f;
+        }
+      }
+    }
+    if constexpr (kPairs) {
+#pragma unroll
+      for (int it = 0; it < ITER; ++it)
+        __builtin_amdgcn_raw_buffer_store_b32(E::pack2(group.gated(a4[it][0], a4[it][1]), group.gated(a4[it][2], a4[it][3])), d_rsrc, off[it], 0, 0);
+      continue;
     }
     auto store_group = [&](int it, float4_t v) {
       __builtin_amdgcn_raw_buffer_store_b64(u32v2_t{E::pack2(v[0], v[1]), E::pack2(v[2], v[3])}, d_rsrc, off[it], 0, 0);

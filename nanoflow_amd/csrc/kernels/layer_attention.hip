@@ -1,6 +1,6 @@
 // Attention of the layer-stack pipeline: short convolution + per-head norm + rotation + query temperature + append
-// to the paged cache, and attention over a window with kept first positions, capped scores, a sink in the softmax and a
-// gate per head, for any head sizes; also the difference of two attentions of a head over the same values.
+// to the paged cache, and attention over a window or a chunk with kept first positions, capped scores, a sink in the softmax,
+// outputs turned back and a gate per head, for any head sizes; also the difference of two attentions of a head over the same values.
 //
 // bf16 (attn_window_kernel, v_mfma_f32_16x16x32_bf16): S^T = K . Q^T, then O^T = V^T . P^T, per
 // (request, kv head, up to 16 of its query heads).  The 16 MFMA columns carry (token, head) pairs.
@@ -39,6 +39,26 @@ __host__ __device__ inline size_t kv_value_offset(const nf_kv_layout& kv) { retu
 // ---------------------------------------------------------------- norm, rotation, append
 __device__ __forceinline__ float temperature(const nf_query_temperature& q, int pos) {
   return q.every > 0 ? 1.f + q.coef * logf((float)((pos + 1) / q.every + 1)) : 1.f;
+}
+
+// Column c of a row whose columns 2m and 2m + 1 are turned by `way` (1 or -1) times the position; `other`: its pair's other one.
+__device__ __forceinline__ float turn_pair(float y, float other, const nf_rotation& rot, int pos, int c, float way) {
+  if (c >= rot.dims) return y;
+  const float* t = rot.table + (size_t)pos * rot.dims + (c & ~1);
+  return y * t[0] + (c & 1 ? way : -way) * other * t[1];
+}
+// The same of columns c .. c + 3, c a multiple of four.
+__device__ __forceinline__ float4_t turn_four(float4_t x, const nf_rotation& rot, int pos, int c, float way) {
+  typedef float f32x2_t __attribute__((ext_vector_type(2)));
+  if (c >= rot.dims) return x;
+  const float* t = rot.table + (size_t)pos * rot.dims + c;
+  const f32x2_t a = *reinterpret_cast<const f32x2_t*>(t), b = *reinterpret_cast<const f32x2_t*>(t + (c + 2 < rot.dims ? 2 : 0));
+  float4_t y{x[0] * a[0] - way * x[1] * a[1], x[1] * a[0] + way * x[0] * a[1], x[2], x[3]};
+  if (c + 2 < rot.dims) {
+    y[2] = x[2] * b[0] - way * x[3] * b[1];
+    y[3] = x[3] * b[0] + way * x[2] * b[1];
+  }
+  return y;
 }
 
 template <int N>
@@ -174,7 +194,7 @@ template <class T>
 __global__ __launch_bounds__(256) void qkv_append_kernel(nf_kv_layout kv, const T* __restrict__ proj, int ld, int q_col,
                                                          int k_col, int v_col, const float* __restrict__ q_norm,
                                                          const float* __restrict__ k_norm, float eps, nf_rotation rot,
-                                                         nf_query_temperature q_temp, nf_short_conv conv, T* __restrict__ q_out, T* __restrict__ kv_data,
+                                                         nf_query_temperature q_temp, nf_value_form vform, nf_short_conv conv, T* __restrict__ q_out, T* __restrict__ kv_data,
                                                          const int32_t* __restrict__ kv_indptr,
                                                          const int32_t* __restrict__ kv_indices,
                                                          const int32_t* __restrict__ rev_input_indptr,
@@ -241,7 +261,22 @@ __global__ __launch_bounds__(256) void qkv_append_kernel(nf_kv_layout kv, const 
   } else if (job < H + G + VG) {
     const int head = job - H - G;
     T* dst = page + kv_value_offset(kv) + (size_t)head * kv.v_pad * kPage + entry;
-    for (int c = lane; c < kv.v_pad; c += 64) Act<T>::store(dst + (size_t)c * kPage, c < kv.vdim ? row.one(v_col + head * kv.vdim + c) : 0.f);
+    float v[kMaxHeadDim / 64];
+    float sq = 0.f;
+#pragma unroll
+    for (int i = 0; i < kMaxHeadDim / 64; ++i) {
+      const int c = i * 64 + lane;
+      v[i] = c < kv.vdim ? row.one(v_col + head * kv.vdim + c) : 0.f;
+      sq += v[i] * v[i];
+    }
+    const float inv = vform.norm ? 1.f / sqrtf(wave_sum(sq) / (float)kv.vdim + eps) : 1.f;
+#pragma unroll
+    for (int i = 0; i < kMaxHeadDim / 64; ++i) {
+      const int c = i * 64 + lane;
+      float y = v[i] * inv;
+      if (vform.rot.dims > 0) y = turn_pair(y, __shfl_xor(y, 1, 64), vform.rot, pos, c, 1.f);
+      if (c < kv.v_pad) Act<T>::store(dst + (size_t)c * kPage, y);
+    }
   }
 }
 
@@ -254,7 +289,7 @@ template <class T, int kVec, int R>
 __global__ __launch_bounds__(256, kVec <= 2 ? 8 : 5) void qkv_append4_kernel(nf_kv_layout kv, const T* __restrict__ proj, int ld, int q_col,
                                                           int k_col, int v_col, const float* __restrict__ q_norm,
                                                           const float* __restrict__ k_norm, float eps, nf_rotation rot,
-                                                          nf_query_temperature q_temp, nf_short_conv conv, T* __restrict__ q_out, T* __restrict__ kv_data,
+                                                          nf_query_temperature q_temp, nf_value_form vform, nf_short_conv conv, T* __restrict__ q_out, T* __restrict__ kv_data,
                                                           const int32_t* __restrict__ kv_indptr,
                                                           const int32_t* __restrict__ kv_indices,
                                                           const int32_t* __restrict__ rev_input_indptr,
@@ -293,7 +328,7 @@ __global__ __launch_bounds__(256, kVec <= 2 ? 8 : 5) void qkv_append4_kernel(nf_
       for (int u = 0; u < R; ++u) v[i][u] = float4_t{0.f, 0.f, 0.f, 0.f};
       if (c < dim) four_of<R>(row, col + c, keep, v[i]);
     }
-    if (q_norm || k_norm) {  // asked by the whole workgroup: the sums are over lanes
+    if (q_norm || k_norm || vform.norm) {  // asked by the whole workgroup: the sums are over lanes
 #pragma unroll
       for (int u = 0; u < R; ++u) {
         float sq = 0.f;
@@ -304,12 +339,16 @@ __global__ __launch_bounds__(256, kVec <= 2 ? 8 : 5) void qkv_append4_kernel(nf_
 #pragma unroll
         for (int m = 8; m > 0; m >>= 1) sq += __shfl_xor(sq, m, 64);
         const float inv = 1.f / sqrtf(sq / (float)dim + eps);
-        if (w)
+        if (w) {
 #pragma unroll
           for (int i = 0; i < kVec; ++i) {
             const int c = (i * 16 + l) * 4;
             if (c < dim) v[i][u] = v[i][u] * inv * *reinterpret_cast<const float4_t*>(w + c);
           }
+        } else if (is_v && vform.norm) {
+#pragma unroll
+          for (int i = 0; i < kVec; ++i) v[i][u] *= inv;
+        }
       }
     }
 #pragma unroll
@@ -344,6 +383,7 @@ __global__ __launch_bounds__(256, kVec <= 2 ? 8 : 5) void qkv_append4_kernel(nf_
         }
         y = y * temp;
         if (is_v) {
+          if (vform.rot.dims > 0) y = turn_four(y, vform.rot, row[u].pos, c, 1.f);
           if (keep[u] && c < kv.v_pad)
 #pragma unroll
             for (int e = 0; e < 4; ++e) Act<T>::store(dst[u] + (size_t)(c + e) * kPage, y[e]);
@@ -364,9 +404,21 @@ __global__ __launch_bounds__(256, kVec <= 2 ? 8 : 5) void qkv_append4_kernel(nf_
   }
   const int r = tid >> 4, t = min(row0 + r, rows - 1);
   const ConvRow<T> row(conv, proj, ld, t, rev_input_indptr[t], positions[t]);
+  float inv = 1.f;
+  if (vform.norm) {  // the row's 16 lanes are of one wavefront; what they read here they read again below, from the cache
+    float sq = 0.f;
+    for (int c = (tid & 15) * 4; c < kv.vdim; c += 64) {
+      const float4_t v = row.four(v_col + head * kv.vdim + c, false);
+      sq += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+    }
+#pragma unroll
+    for (int m = 8; m > 0; m >>= 1) sq += __shfl_xor(sq, m, 64);
+    inv = 1.f / sqrtf(sq / (float)kv.vdim + eps);
+  }
   for (int c = (tid & 15) * 4; c < kv.v_pad; c += 64) {
     float4_t v{0.f, 0.f, 0.f, 0.f};
-    if (c < kv.vdim) v = row.four(v_col + head * kv.vdim + c, row0 + r < rows);
+    if (c < kv.vdim) v = row.four(v_col + head * kv.vdim + c, row0 + r < rows) * inv;
+    if (vform.rot.dims > 0) v = turn_four(v, vform.rot, row.pos, c, 1.f);
 #pragma unroll
     for (int e = 0; e < 4; ++e) buf[(c + e) * 17 + r] = v[e];
   }
@@ -391,21 +443,25 @@ struct StepRange {
   int head, skip_to, total;  // steps [0, head), then [skip_to, ...): `total` of both
   __device__ __forceinline__ int at(int i) const { return i < head ? i : skip_to + i - head; }
 };
+// The first position that one at p sees, the kept first ones aside; it does not fall as p grows.
+__device__ __forceinline__ int first_seen(const nf_window_attention_args& a, int p) {
+  const int lo = a.window > 0 ? p - a.window + 1 : 0;
+  return a.chunk > 0 ? max(lo, p - p % a.chunk) : lo;
+}
 // The steps of `width` keys in which a token at a position in [p0, p1] sees a key.
-__device__ __forceinline__ StepRange visible_steps(int p0, int p1, int window, int keep_first, int width) {
+__device__ __forceinline__ StepRange visible_steps(const nf_window_attention_args& a, int p0, int p1, int width) {
   const int end = p1 / width + 1;
-  if (window <= 0) return {0, 0, end};
-  const int kept = keep_first > p1 + 1 ? p1 + 1 : keep_first;
+  const int lo = first_seen(a, p0);
+  if (lo <= 0) return {0, 0, end};
+  const int kept = a.keep_first > p1 + 1 ? p1 + 1 : a.keep_first;
   const int head = (kept + width - 1) / width;
-  const int lo = p0 - window + 1;
   int skip_to = lo > 0 ? lo / width : 0;
   if (skip_to < head) skip_to = head;
   return {head, skip_to, head + (end > skip_to ? end - skip_to : 0)};
 }
 
-__device__ __forceinline__ bool sees(int p, int j, int window, int keep_first) {
-  return j <= p && (window <= 0 || p - j < window || j < keep_first);
-}
+// lo: first_seen of p
+__device__ __forceinline__ bool sees(int p, int lo, int j, int keep_first) { return j <= p && (j >= lo || j < keep_first); }
 
 // What a head's output is multiplied by in the end.
 template <class T>
@@ -441,7 +497,8 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(nf_window_attention_args 
   const T* pool = (const T*)a.kv_data;
   const size_t page_elems = kv_page_elements(kv);
   const int32_t* pages = a.kv_indices + a.kv_indptr[req];
-  const StepRange steps = visible_steps(p, p, a.window, a.keep_first, 64);
+  const StepRange steps = visible_steps(a, p, p, 64);
+  const int seen_from = first_seen(a, p);
   float out_row[kMaxHeadDim / 64] = {};
   for (int map = 0; map < kv.maps; ++map) {
     const T* q = (const T*)a.q + (((size_t)t * kv.heads + h) * kv.maps + map) * kv.k_pad;
@@ -453,7 +510,7 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(nf_window_attention_args 
     float o[kMaxHeadDim / 64] = {};
     for (int i = 0; i < steps.total; ++i) {
       const int base = steps.at(i) * 64, j = base + lane;
-      const bool see = sees(p, j, a.window, a.keep_first);
+      const bool see = sees(p, seen_from, j, a.keep_first);
       float s = -INFINITY;
       if (see) {
         const T* k = pool + (size_t)pages[j / kPage] * page_elems + (((size_t)g * kv.maps + map) * kPage + j % kPage) * kv.k_pad;
@@ -514,6 +571,7 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(nf_window_attention_args 
 #pragma unroll
   for (int e = 0; e < kMaxHeadDim / 64; ++e) {
     const int c = e * 64 + lane;
+    if (a.out_rot.dims > 0) out_row[e] = turn_pair(out_row[e], __shfl_xor(out_row[e], 1, 64), a.out_rot, p, c, -1.f);
     if (c < kv.vdim) Act<T>::store(out + c, out_row[e] * factor);
   }
 }
@@ -540,7 +598,7 @@ __device__ __forceinline__ u32x4 load_cache(const bf16_t* p) {
 // What the lanes of a column (those with the same l16) hold of its output in the end, from the sums of its maps; `o` and `l`
 // hold kMaps entries.  The value columns are i * 16 + g * 4 ..
 template <int kMaps, int VD>
-__device__ __forceinline__ void finish_column(const nf_window_attention_args& a, float4_t (*o)[VD], const float* m, const float* l, int row, int h, int g) {
+__device__ __forceinline__ void finish_column(const nf_window_attention_args& a, float4_t (*o)[VD], const float* m, const float* l, int row, int pos, int h, int g) {
   float den = l[0], f = 1.f;
   if (a.sink) {
     const float snk = a.sink[h] * 1.44269504088896340736f, mm = fmaxf(m[0], snk);
@@ -565,6 +623,9 @@ __device__ __forceinline__ void finish_column(const nf_window_attention_args& a,
   }
 #pragma unroll
   for (int i = 0; i < VD; ++i) o[0][i] *= first * factor;
+  if (a.out_rot.dims > 0)
+#pragma unroll
+    for (int i = 0; i < VD; ++i) o[0][i] = turn_four(o[0][i], a.out_rot, pos, i * 16 + g * 4, -1.f);
 }
 
 // KD: 32-wide pieces of k_pad, VD: 16-wide pieces of v_pad (both upper bounds), NB: column blocks per
@@ -608,7 +669,7 @@ __global__ __launch_bounds__(window_threads(kMaps, VD)) void attn_window_kernel(
   }
 
   constexpr int NC = NB * kMaps;  // sets of columns: a block's maps side by side
-  int pos[NB], row[NB];
+  int pos[NB], lo_key[NB], row[NB];
   bool live[NB];
   B8 qf[NC][KD];
   const int kd = kv.k_pad / 32, vd = kv.v_pad / 16;
@@ -618,6 +679,7 @@ __global__ __launch_bounds__(window_threads(kMaps, VD)) void attn_window_kernel(
     live[n] = (kDecode ? l16 < heads : l16 < tpb * gs && tok < len && hc < heads);
     row[n] = row0 + (live[n] ? tok : (kDecode ? 0 : tok0));
     pos[n] = a.positions[row[n]];
+    lo_key[n] = first_seen(a, pos[n]);
     const bf16_t* q = (const bf16_t*)a.q + ((size_t)row[n] * kv.heads + kvh * group + h0 + (live[n] ? hc : 0)) * kMaps * kv.k_pad + g * 8;
 #pragma unroll
     for (int x = 0; x < kMaps; ++x)
@@ -627,7 +689,8 @@ __global__ __launch_bounds__(window_threads(kMaps, VD)) void attn_window_kernel(
   }
   const int p0 = a.positions[row0 + tok0];
   const int p1 = kDecode ? p0 : p0 + min(NB * tpb, len - tok0) - 1;
-  const StepRange steps = visible_steps(p0, p1, a.window, a.keep_first, 32);
+  const StepRange steps = visible_steps(a, p0, p1, 32);
+  const int all_from = first_seen(a, p1);  // every token sees the keys from here to its own
 
   const size_t page_elems = kv_page_elements(kv);
   const int32_t* pages = a.kv_indices + a.kv_indptr[req];
@@ -698,7 +761,7 @@ __global__ __launch_bounds__(window_threads(kMaps, VD)) void attn_window_kernel(
       }
     if (it + stride < steps.total) load_k(k_id);
     k_id = next_k_id;
-    const bool whole = base + 31 <= p0 && (a.window <= 0 || p1 - base < a.window || base + 31 < a.keep_first);
+    const bool whole = base + 31 <= p0 && (base >= all_from || base + 31 < a.keep_first);
 #pragma unroll
     for (int n = 0; n < NC; ++n) {
       const int j0 = base + 8 * g;
@@ -707,7 +770,7 @@ __global__ __launch_bounds__(window_threads(kMaps, VD)) void attn_window_kernel(
       for (int b = 0; b < 2; ++b)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          if (!whole && !sees(pos[n / kMaps], j0 + 4 * b + r, a.window, a.keep_first)) s[n][b][r] = -INFINITY;
+          if (!whole && !sees(pos[n / kMaps], lo_key[n / kMaps], j0 + 4 * b + r, a.keep_first)) s[n][b][r] = -INFINITY;
           mx = fmaxf(mx, s[n][b][r]);
         }
       mx = mx > -1e30f ? mx * scale2 : mx;
@@ -783,6 +846,7 @@ __global__ __launch_bounds__(window_threads(kMaps, VD)) void attn_window_kernel(
         }
         v += acc * ((x == 0 ? 1.f : -a.map_weight) / den);
       }
+      if (a.out_rot.dims > 0) v = turn_pair(v, __shfl_xor(v, 1, 64), a.out_rot, p0, c, -1.f);  // heads of an even size: a pair's threads are neighbours
       if (a.head_norm) so[(size_t)hc * kv.v_pad + c] = v;  // read by this thread alone until now
       else Act<bf16_t>::store(dst + e, v * head_factor<bf16_t>(a, row0, h));
     }
@@ -799,7 +863,7 @@ __global__ __launch_bounds__(window_threads(kMaps, VD)) void attn_window_kernel(
 #pragma unroll
     for (int n = 0; n < NB; ++n) {
       const int h = kvh * group + h0 + l16 % gs;
-      finish_column<kMaps, VD>(a, o + n * kMaps, m + n * kMaps, l + n * kMaps, row[n], live[n] ? h : kvh * group + h0, g);
+      finish_column<kMaps, VD>(a, o + n * kMaps, m + n * kMaps, l + n * kMaps, row[n], pos[n], live[n] ? h : kvh * group + h0, g);
       if (!live[n]) continue;
       bf16_t* dst = out + (size_t)row[n] * a.out_ld + a.out_col + (size_t)h * kv.vdim;
       const bool vec = (kv.vdim | a.out_ld | a.out_col) % 4 == 0;
@@ -869,7 +933,8 @@ __global__ __launch_bounds__(256, 2) void attn_tile_kernel(nf_window_attention_a
   const int p0 = a.positions[row0] + first_tok, p1 = p0 + min(tile_tokens, len - first_tok) - 1;  // the workgroup's
   const int w0 = p0 + wave * NB * tpb, w1 = min(w0 + NB * tpb - 1, p1);                          // this wavefront's; none: w0 > w1
 
-  const StepRange steps = visible_steps(p0, p1, a.window, a.keep_first, 32);
+  const StepRange steps = visible_steps(a, p0, p1, 32);
+  const int all_from = first_seen(a, w1);  // every token of the wavefront sees the keys from here to its own
   const int32_t* pages = a.kv_indices + a.kv_indptr[req];
   const int last_page = p1 / kPage;
   const size_t page_bytes = kv_page_elements(kv) * 2;
@@ -906,7 +971,7 @@ __global__ __launch_bounds__(256, 2) void attn_tile_kernel(nf_window_attention_a
 
 #pragma unroll 1
   for (int it = 0; it < min(kTileRing - 1, steps.total); ++it) load_step(it);
-  int pos[NB], row[NB];
+  int pos[NB], lo_key[NB], row[NB];
   bool live[NB];
   B8 qf[NC][KD];
 #pragma unroll
@@ -915,6 +980,7 @@ __global__ __launch_bounds__(256, 2) void attn_tile_kernel(nf_window_attention_a
     live[n] = l16 < tpb * gs && tok < len && hc < heads;
     row[n] = row0 + (live[n] ? tok : first_tok);
     pos[n] = p0 - first_tok + (live[n] ? tok : first_tok);
+    lo_key[n] = first_seen(a, pos[n]);
     const bf16_t* q = (const bf16_t*)a.q + ((size_t)row[n] * kv.heads + kvh * group + h0 + (live[n] ? hc : 0)) * (kMaps * KD * 32) + g * 8;
 #pragma unroll
     for (int j = 0; j < kMaps * KD; ++j) qf[n * kMaps + j / KD][j % KD].u = *reinterpret_cast<const u32x4*>(q + j * 32);  // columns of no token: never stored
@@ -966,7 +1032,7 @@ __global__ __launch_bounds__(256, 2) void attn_tile_kernel(nf_window_attention_a
       for (int n = 0; n < NC; ++n)
 #pragma unroll
         for (int b = 0; b < 2; ++b) cap.apply(s[n][b]);
-    const bool whole = base + 31 <= w0 && (a.window <= 0 || w1 - base < a.window || base + 31 < a.keep_first);
+    const bool whole = base + 31 <= w0 && (base >= all_from || base + 31 < a.keep_first);
     B8 hi[NC], lo[NC];
 #pragma unroll
     for (int n = 0; n < NC; ++n) {
@@ -976,7 +1042,7 @@ __global__ __launch_bounds__(256, 2) void attn_tile_kernel(nf_window_attention_a
         for (int b = 0; b < 2; ++b)
 #pragma unroll
           for (int r = 0; r < 4; ++r)
-            if (!sees(pos[n / kMaps], base + 8 * g + 4 * b + r, a.window, a.keep_first)) s[n][b][r] = -INFINITY;
+            if (!sees(pos[n / kMaps], lo_key[n / kMaps], base + 8 * g + 4 * b + r, a.keep_first)) s[n][b][r] = -INFINITY;
 #pragma unroll
       for (int b = 0; b < 2; ++b)
 #pragma unroll
@@ -1028,7 +1094,7 @@ __global__ __launch_bounds__(256, 2) void attn_tile_kernel(nf_window_attention_a
 #pragma unroll
   for (int n = 0; n < NB; ++n) {
     const int h = kvh * group + h0 + l16 % gs;
-    finish_column<kMaps, VD>(a, o + n * kMaps, m + n * kMaps, l + n * kMaps, row[n], live[n] ? h : kvh * group + h0, g);
+    finish_column<kMaps, VD>(a, o + n * kMaps, m + n * kMaps, l + n * kMaps, row[n], pos[n], live[n] ? h : kvh * group + h0, g);
     if (!live[n]) continue;
     bf16_t* dst = out + (size_t)row[n] * a.out_ld + a.out_col + (size_t)h * kv.vdim;
 #pragma unroll
@@ -1110,8 +1176,8 @@ extern "C" {
 size_t nf_kv_page_elements(const nf_kv_layout* kv) { return kv ? kv_page_elements(*kv) : 0; }
 
 int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, int k_col, int v_col, const float* q_norm,
-                  const float* k_norm, float eps, const nf_rotation* rot, const nf_query_temperature* q_temp, const nf_short_conv* conv, void* q_out,
-                  void* kv_data, const int32_t* kv_indptr, const int32_t* kv_indices, const int32_t* rev_input_indptr,
+                  const float* k_norm, float eps, const nf_rotation* rot, const nf_query_temperature* q_temp, const nf_value_form* values,
+                  const nf_short_conv* conv, void* q_out, void* kv_data, const int32_t* kv_indptr, const int32_t* kv_indices, const int32_t* rev_input_indptr,
                   const int32_t* positions, int rows, nf_stream_t stream) {
   const char* who = "nf_qkv_append";
   NF_REQUIRE(kv && rot, "%s: null pointer", who);
@@ -1126,6 +1192,9 @@ int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, i
   const nf_short_conv cv = conv ? *conv : nf_short_conv{};
   NF_REQUIRE(!conv || (cv.taps >= 1 && cv.taps <= 64 && cv.weight && cv.input_indptr && (cv.taps == 1 || (cv.state && cv.state_slots))),
              "%s: a convolution of %d taps (1..64) needs weights, a state and slots", who, cv.taps);
+  const nf_value_form vf = values ? *values : nf_value_form{};
+  NF_REQUIRE(vf.rot.dims >= 0 && vf.rot.dims % 2 == 0 && vf.rot.dims <= kv->vdim && (vf.rot.dims == 0 || (vf.rot.table && vf.rot.interleaved)),
+             "%s: %d of %d value columns rotated, in pairs side by side", who, vf.rot.dims, kv->vdim);
   const nf_query_temperature temp = q_temp ? *q_temp : nf_query_temperature{0.f, 0};
   if (rows == 0) return NF_OK;
   NF_REQUIRE(proj && q_out && kv_data && kv_indptr && kv_indices && rev_input_indptr && positions, "%s: null pointer", who);
@@ -1142,7 +1211,7 @@ int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, i
       const int jobs = (kv->heads + kv->kv_heads) * kv->maps + (few ? kv->kv_heads : 0);
       const int blocks = value_blocks + (rows + kRun - 1) / kRun * ((jobs + 15) / 16);
       qkv_append4_kernel<T, decltype(vec)::value, kRun><<<(unsigned)blocks, 256, 0, s>>>(
-          *kv, (const T*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot, temp, cv, (T*)q_out, (T*)kv_data, kv_indptr, kv_indices,
+          *kv, (const T*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot, temp, vf, cv, (T*)q_out, (T*)kv_data, kv_indptr, kv_indices,
           rev_input_indptr, positions, rows, value_blocks);
       return check_launch(who);
     };
@@ -1155,11 +1224,11 @@ int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, i
   }
   const dim3 grid((unsigned)rows, (unsigned)(((kv->heads + kv->kv_heads) * kv->maps + kv->kv_heads + 3) / 4));
   if (kv->dtype == NF_BF16)
-    qkv_append_kernel<bf16_t><<<grid, 256, 0, s>>>(*kv, (const bf16_t*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot, temp, cv,
+    qkv_append_kernel<bf16_t><<<grid, 256, 0, s>>>(*kv, (const bf16_t*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot, temp, vf, cv,
                                                    (bf16_t*)q_out, (bf16_t*)kv_data, kv_indptr, kv_indices, rev_input_indptr,
                                                    positions);
   else
-    qkv_append_kernel<float><<<grid, 256, 0, s>>>(*kv, (const float*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot, temp, cv,
+    qkv_append_kernel<float><<<grid, 256, 0, s>>>(*kv, (const float*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot, temp, vf, cv,
                                                   (float*)q_out, (float*)kv_data, kv_indptr, kv_indices, rev_input_indptr,
                                                   positions);
   return check_launch(who);
@@ -1193,6 +1262,9 @@ int nf_window_attention(const nf_window_attention_args* args, nf_stream_t stream
              a.out_col, a.kv.heads * a.kv.vdim, a.out_ld);
   NF_REQUIRE(!a.gate || a.gate_ld >= a.kv.heads, "%s: gate rows of %d for %d heads", who, a.gate_ld, a.kv.heads);
   NF_REQUIRE(a.kv.maps == 1 || !a.sink, "%s: a sink with two maps", who);
+  NF_REQUIRE(a.out_rot.dims == 0 || (a.out_rot.dims == a.kv.vdim && a.kv.vdim % 2 == 0 && a.out_rot.table && a.out_rot.interleaved),
+             "%s: %d of %d output columns turned back, in pairs side by side", who, a.out_rot.dims, a.kv.vdim);
+  NF_REQUIRE(a.chunk >= 0, "%s: chunks of %d", who, a.chunk);
   NF_REQUIRE(a.softcap >= 0.f && (!a.head_norm || a.head_eps >= 0.f), "%s: cap %g, eps %g", who, a.softcap, a.head_eps);
   NF_REQUIRE(!a.decode || a.max_rows == a.req_num, "%s: %d decode requests with %d rows", who, a.req_num, a.max_rows);
   if (a.req_num == 0 || a.max_rows == 0) return NF_OK;

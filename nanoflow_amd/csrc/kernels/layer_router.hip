@@ -1,6 +1,6 @@
 // Routing of a mixture of experts: scores, choice, and the order of the chosen rows by expert.
 //
-// route_rows_kernel: one wavefront per token, its scores in registers (fp32 softmax over all outputs), groups of
+// route_rows_kernel: one wavefront per token, its scores in registers (fp32 softmax over all outputs, or a sigmoid of each), groups of
 //   outputs closed by the rank of their largest entry, the `top` largest taken one after the other, then the
 //   experts that every token has.
 // route_plan_kernel: one workgroup counts the rows of every expert, places them (an expert's rows consecutive)
@@ -44,10 +44,12 @@ __global__ __launch_bounds__(256) void route_rows_kernel(nf_route_args a, int32_
   float sum = 0.f;
 #pragma unroll
   for (int i = 0; i < kPer; ++i) {
-    s[i] = i * 64 + lane < outputs ? expf(s[i] - mx) : 0.f;
+    const bool is = i * 64 + lane < outputs;
+    if (a.scores == NF_SCORES_SIGMOID) s[i] = is ? 1.f / (1.f + expf(-s[i])) : 0.f;
+    else s[i] = is ? expf(s[i] - mx) : 0.f;
     sum += s[i];
   }
-  sum = wave_sum(sum);
+  sum = a.scores == NF_SCORES_SIGMOID ? 1.f : wave_sum(sum);
 #pragma unroll
   for (int i = 0; i < kPer; ++i) {
     const int o = i * 64 + lane;
@@ -110,9 +112,10 @@ __global__ __launch_bounds__(256) void route_rows_kernel(nf_route_args a, int32_
   }
   if (lane < a.always) {
     float g = 0.f;
-    for (int p = 0; p < shares; ++p) g += z[p * slice + outputs];
+    if (!a.always_plain)
+      for (int p = 0; p < shares; ++p) g += z[p * slice + outputs];
     choice[(size_t)t * per_token + a.top + lane] = outputs + lane;
-    weight[(size_t)t * per_token + a.top + lane] = 1.f / (1.f + expf(-g));
+    weight[(size_t)t * per_token + a.top + lane] = a.always_plain ? 1.f : 1.f / (1.f + expf(-g));
   }
 }
 
@@ -164,7 +167,10 @@ __global__ __launch_bounds__(1024) void route_plan_kernel(nf_routing r, int rows
     int at = -1;
     if (k >= top) at = first[routed + k - top] + t;
     else if (e < routed) at = atomicAdd(&first[e], 1);
-    if (at >= 0) r.row_of[at] = t;
+    if (at >= 0) {
+      r.row_of[at] = t;
+      if (r.row_weight) r.row_weight[at] = r.weight[i];
+    }
     r.place[i] = at;
   }
 }
@@ -191,9 +197,10 @@ int nf_route(const nf_route_args* args, const nf_routing* routing, nf_stream_t s
                                a.top <= a.outputs / a.groups * a.keep_groups),
              "%s: top %d of the outputs of %d of %d groups of %d", who, a.top, a.keep_groups, a.groups, a.outputs);
   const int per_token = a.top + a.always;
-  NF_REQUIRE(a.rows >= 0 && (long long)a.rows * per_token < (1ll << 31) && a.ld >= a.outputs + (a.always > 0) && a.shares >= 1 &&
+  NF_REQUIRE(a.rows >= 0 && (long long)a.rows * per_token < (1ll << 31) && a.ld >= a.outputs + (a.always > 0 && !a.always_plain) && a.shares >= 1 &&
                  a.shares <= kMaxShares && routing->tile_rows > 0,
              "%s: rows=%d ld=%d shares=%d tile_rows=%d", who, a.rows, a.ld, a.shares, routing->tile_rows);
+  NF_REQUIRE(a.scores == NF_SCORES_SOFTMAX || a.scores == NF_SCORES_SIGMOID, "%s: unknown scores %d", who, a.scores);
   if (a.rows == 0) return NF_OK;
   const nf_routing& r = *routing;
   NF_REQUIRE(a.z && r.choice && r.weight && r.place && r.row_of && r.offsets && r.tile_group && r.tile_row && r.n_tiles, "%s: null pointer", who);

@@ -1,5 +1,5 @@
 // Row operators of the layer-stack pipeline: embedding plus learned positions, the end of a sublayer (its output,
-// normed or put together from experts, added to the residual stream, and the next norm), gathered norms,
+// normed or put together from experts, added to the residual stream, what a pass over layers starts with, and the next norm), gathered norms,
 // gated norm, token shift, token gate, tanh, fp32 argmax.
 // HBM-bound; one workgroup per row (token shift: per 1024 columns of a row), 16-byte accesses, the row kept in registers between the
 // reduction and the write.  The residual stream is fp32.
@@ -13,13 +13,13 @@ constexpr int kMaxRowVec = 16;  // a row is at most 16 x 256 x 4 = 16384 columns
 template <class T>
 __global__ __launch_bounds__(kRowThreads) void embed_rows_kernel(const int32_t* __restrict__ tokens,
                                                                  const int32_t* __restrict__ positions,
-                                                                 const T* __restrict__ embed, const T* __restrict__ pos,
+                                                                 const T* __restrict__ embed, const T* __restrict__ pos, float scale,
                                                                  float* __restrict__ x, T* __restrict__ act, int ld) {
   const int t = blockIdx.x;
   const T* e = embed + (size_t)tokens[t] * ld;
   const T* p = pos ? pos + (size_t)positions[t] * ld : nullptr;
   for (int c = threadIdx.x * 4; c < ld; c += kRowThreads * 4) {
-    float4_t v = Act<T>::load4(e + c);
+    float4_t v = Act<T>::load4(e + c) * scale;
     if (p) v += Act<T>::load4(p + c);
     *reinterpret_cast<float4_t*>(x + (size_t)t * ld + c) = v;
     if (act) Act<T>::store4(act + (size_t)t * ld + c, v);
@@ -73,6 +73,7 @@ __global__ __launch_bounds__(kRowThreads) void residual_rows_kernel(nf_residual_
     if (c >= ld) continue;
     xr[i] = *reinterpret_cast<const float4_t*>(a.x + row + c);  // in flight together with the sublayer's output
     if constexpr (!kMixture) {
+      if (!y) continue;
       if constexpr (std::is_same_v<TY, float>) v[i] = sum_shares(y, slice, row + c, a.shares);
       else v[i] = Act<TY>::load4(y + row + c);
     }
@@ -81,13 +82,13 @@ __global__ __launch_bounds__(kRowThreads) void residual_rows_kernel(nf_residual_
     // the token's places and weights, one per lane (at most 64), then row after row by its number
     const int lane = threadIdx.x & 63;
     const int my_place = lane < a.top ? place[(size_t)t * a.top + lane] : -1;
-    const float my_weight = lane < a.top ? weight[(size_t)t * a.top + lane] : 0.f;
+    const float my_weight = lane >= a.top ? 0.f : weight ? weight[(size_t)t * a.top + lane] : 1.f;
     const float same = wave_sum(my_place < 0 ? my_weight : 0.f);  // of identity experts
     float4_t own[kVec];
 #pragma unroll
     for (int i = 0; i < kVec; ++i) {
       const int c = (i * kRowThreads + threadIdx.x) * 4;
-      own[i] = same != 0.f && c < ld ? Act<TY>::load4((const TY*)a.identity + row + c) : float4_t{0.f, 0.f, 0.f, 0.f};
+      own[i] = same != 0.f && c < ld && a.identity ? Act<TY>::load4((const TY*)a.identity + row + c) : float4_t{0.f, 0.f, 0.f, 0.f};
     }
     constexpr int kAhead = 4;
     for (int k0 = 0; k0 < a.top; k0 += kAhead) {
@@ -114,10 +115,13 @@ __global__ __launch_bounds__(kRowThreads) void residual_rows_kernel(nf_residual_
     for (int i = 0; i < kVec; ++i) v[i] += own[i] * same;
   }
   if (a.y_norm.kind != NF_NORM_NONE) norm_row<kVec>(v, a.y_norm, a.width, ld, scratch);
+  const T* e = a.table ? (const T*)a.table + (size_t)a.tokens[t] * ld : nullptr;
 #pragma unroll
   for (int i = 0; i < kVec; ++i) {
     const int c = (i * kRowThreads + threadIdx.x) * 4;
     v[i] = v[i] * a.y_scale + xr[i];
+    if (e && c < ld) v[i] += Act<T>::load4(e + c) * a.table_scale;
+    if (a.add && c < ld) v[i] += *reinterpret_cast<const float4_t*>(a.add + c);
     if (c < ld) *reinterpret_cast<float4_t*>(a.x + row + c) = v[i];
   }
   if (!a.act) return;
@@ -295,7 +299,7 @@ static int check_norm(const char* who, const nf_norm& n) {
 
 extern "C" {
 
-int nf_embed_rows(int dtype, const int32_t* tokens, const int32_t* positions, const void* embed, const void* pos, float* x,
+int nf_embed_rows(int dtype, const int32_t* tokens, const int32_t* positions, const void* embed, const void* pos, float scale, float* x,
                   void* act, int rows, int ld, nf_stream_t stream) {
   int rc = check_rows("nf_embed_rows", dtype, rows, 1, ld);
   if (rc) return rc;
@@ -303,10 +307,10 @@ int nf_embed_rows(int dtype, const int32_t* tokens, const int32_t* positions, co
   NF_REQUIRE(tokens && embed && x && (!pos || positions), "nf_embed_rows: null pointer");
   hipStream_t s = (hipStream_t)stream;
   if (dtype == NF_BF16)
-    embed_rows_kernel<bf16_t><<<rows, kRowThreads, 0, s>>>(tokens, positions, (const bf16_t*)embed, (const bf16_t*)pos, x,
+    embed_rows_kernel<bf16_t><<<rows, kRowThreads, 0, s>>>(tokens, positions, (const bf16_t*)embed, (const bf16_t*)pos, scale, x,
                                                            (bf16_t*)act, ld);
   else
-    embed_rows_kernel<float><<<rows, kRowThreads, 0, s>>>(tokens, positions, (const float*)embed, (const float*)pos, x,
+    embed_rows_kernel<float><<<rows, kRowThreads, 0, s>>>(tokens, positions, (const float*)embed, (const float*)pos, scale, x,
                                                           (float*)act, ld);
   return check_launch("nf_embed_rows");
 }
@@ -318,14 +322,14 @@ int nf_residual_rows(const nf_residual_args* args, nf_stream_t stream) {
   int rc = check_rows(who, a.dtype, a.rows, a.width, a.ld);
   if (rc || (rc = check_norm(who, a.y_norm)) || (rc = check_norm(who, a.next))) return rc;
   if (a.routing) {
-    NF_REQUIRE(a.top >= 1 && a.top <= 64 && a.y_ld >= a.ld && a.y_ld % 4 == 0 && a.routing->place && a.routing->weight && a.identity,
+    NF_REQUIRE(a.top >= 1 && a.top <= 64 && a.y_ld >= a.ld && a.y_ld % 4 == 0 && a.routing->place && (a.routing->weight || !a.identity),
                "%s: incomplete routing (top %d, stride %d)", who, a.top, a.y_ld);
-  } else {
+  } else if (a.y) {
     NF_REQUIRE((a.y_dtype == NF_F32 && a.shares >= 1 && a.shares <= kMaxShares) || (a.y_dtype == NF_BF16 && a.shares == 1),
                "%s: %d shares of dtype %d", who, a.shares, a.y_dtype);
   }
   if (a.rows == 0) return NF_OK;
-  NF_REQUIRE(a.y && a.x, "%s: null pointer", who);
+  NF_REQUIRE((a.y || (!a.routing && a.y_norm.kind == NF_NORM_NONE)) && a.x && (!a.table || a.tokens), "%s: null pointer", who);
   hipStream_t s = (hipStream_t)stream;
   return with_vec(a.ld, [&](auto v) {
     constexpr int V = decltype(v)::value;
@@ -335,7 +339,7 @@ int nf_residual_rows(const nf_residual_args* args, nf_stream_t stream) {
     };
     const bool b16 = a.dtype == NF_BF16;
     if (a.routing) return b16 ? go(residual_rows_kernel<bf16_t, bf16_t, V, true>) : go(residual_rows_kernel<float, float, V, true>);
-    if (a.y_dtype == NF_BF16) return b16 ? go(residual_rows_kernel<bf16_t, bf16_t, V, false>) : go(residual_rows_kernel<bf16_t, float, V, false>);
+    if (a.y && a.y_dtype == NF_BF16) return b16 ? go(residual_rows_kernel<bf16_t, bf16_t, V, false>) : go(residual_rows_kernel<bf16_t, float, V, false>);
     return b16 ? go(residual_rows_kernel<float, bf16_t, V, false>) : go(residual_rows_kernel<float, float, V, false>);
   });
 }

@@ -48,9 +48,9 @@ class KVLayout(C.Structure):
 
 
 class WindowAttentionArgs(C.Structure):
-    _fields_ = [("kv", KVLayout), ("window", C.c_int), ("keep_first", C.c_int), ("scale", C.c_float),
+    _fields_ = [("kv", KVLayout), ("window", C.c_int), ("keep_first", C.c_int), ("chunk", C.c_int), ("scale", C.c_float),
                 ("out_scale", C.c_float), ("softcap", C.c_float), ("map_weight", C.c_float), ("head_eps", C.c_float),
-                ("head_norm", C.c_int), ("sink", C.c_void_p), ("gate", C.c_void_p), ("gate_ld", C.c_int), ("q", C.c_void_p),
+                ("head_norm", C.c_int), ("sink", C.c_void_p), ("out_rot", Rotation), ("gate", C.c_void_p), ("gate_ld", C.c_int), ("q", C.c_void_p),
                 ("out", C.c_void_p), ("out_ld", C.c_int), ("out_col", C.c_int), ("kv_data", C.c_void_p)] + \
         [(n, C.c_void_p) for n in ("input_indptr", "kv_indptr", "kv_indices", "rev_input_indptr", "positions")] + \
         [(n, C.c_int) for n in ("req_begin", "req_num", "row_begin", "max_rows", "decode")]
@@ -58,6 +58,10 @@ class WindowAttentionArgs(C.Structure):
 
 class QueryTemperature(C.Structure):
     _fields_ = [("coef", C.c_float), ("every", C.c_int)]
+
+
+class ValueForm(C.Structure):
+    _fields_ = [("norm", C.c_int), ("rot", Rotation)]
 
 
 class ShortConv(C.Structure):
@@ -87,25 +91,31 @@ class Norm(C.Structure):
 
 class Routing(C.Structure):
     _fields_ = [(n, C.c_void_p) for n in ("choice", "weight", "place", "row_of", "offsets", "tile_group", "tile_row", "n_tiles")] + \
-        [("tile_rows", C.c_int)]
+        [("tile_rows", C.c_int), ("row_weight", C.c_void_p)]
 
 
 class RouteArgs(C.Structure):
     _fields_ = [("z", C.c_void_p)] + \
         [(n, C.c_int) for n in ("shares", "ld", "rows", "outputs", "experts", "top", "always", "groups", "keep_groups")] + \
-        [("correction", C.c_void_p), ("scale", C.c_float)]
+        [("correction", C.c_void_p), ("scale", C.c_float), ("scores", C.c_int), ("always_plain", C.c_int)]
+
+
+class GatedAct(C.Structure):
+    _fields_ = [("slope", C.c_float), ("shift", C.c_float), ("limits", C.c_void_p)]
 
 
 class GroupedGemmArgs(C.Structure):
     _fields_ = [(n, C.c_int) for n in ("dtype", "act", "groups", "M", "N", "K")] + \
         [("a", C.c_void_p), ("lda", C.c_int), ("a_group", C.c_size_t), ("b", C.c_void_p), ("d", C.c_void_p), ("ldd", C.c_int),
-         ("d_group", C.c_size_t), ("routing", Routing), ("gather", C.c_int), ("max_rows", C.c_int)]
+         ("d_group", C.c_size_t), ("routing", Routing), ("gather", C.c_int), ("max_rows", C.c_int), ("weigh", C.c_int),
+         ("gated", GatedAct)]
 
 
 class ResidualArgs(C.Structure):
     _fields_ = [(n, C.c_int) for n in ("rows", "width", "ld", "y_dtype", "shares")] + \
         [("y", C.c_void_p), ("routing", C.POINTER(Routing)), ("top", C.c_int), ("y_ld", C.c_int), ("identity", C.c_void_p),
-         ("y_norm", Norm), ("next", Norm), ("y_scale", C.c_float), ("x", C.c_void_p), ("dtype", C.c_int), ("act", C.c_void_p)]
+         ("y_norm", Norm), ("next", Norm), ("y_scale", C.c_float), ("x", C.c_void_p), ("dtype", C.c_int), ("act", C.c_void_p),
+         ("add", C.c_void_p), ("table", C.c_void_p), ("tokens", C.c_void_p), ("table_scale", C.c_float)]
 
 
 class RecurrenceArgs(C.Structure):
@@ -213,12 +223,12 @@ def lib() -> C.CDLL:
         l.nf_latent_append.argtypes = [vp, vp, i32, i32, i32, vp, f32] + [vp] * 7 + [i32, i32, vp]
         l.nf_gemm_nk_sums_shares.argtypes = [i32] * 4
         l.nf_gemm_nk_sums_bf16.argtypes = [vp, vp, vp, sz, i32, i32, i32, i32, vp]
-        l.nf_embed_rows.argtypes = [i32, vp, vp, vp, vp, vp, vp, i32, i32, vp]
+        l.nf_embed_rows.argtypes = [i32, vp, vp, vp, vp, f32, vp, vp, i32, i32, vp]
         l.nf_token_shift.argtypes = [i32, vp, vp, vp, vp, i32, vp, vp, vp, vp, i32, i32, vp]
         l.nf_tanh_rows.argtypes = [i32, vp, i32, vp, i32, i32, vp]
         l.nf_argmax_f32.argtypes = [vp, vp, i32, i32, i32, vp]
         l.nf_qkv_append.argtypes = [C.POINTER(KVLayout), vp, i32, i32, i32, i32, vp, vp, f32, C.POINTER(Rotation), vp, vp, vp, vp, vp,
-                                    vp, vp, vp, i32, vp]
+                                    vp, vp, vp, vp, i32, vp]
         l.nf_window_attention.argtypes = [C.POINTER(WindowAttentionArgs), vp]
         l.nf_linear_recurrence.argtypes = [C.POINTER(RecurrenceArgs), vp]
         size_calls = {"nf_kv_page_elements": [C.POINTER(KVLayout)], "nf_recurrence_state_elements": [i32, i32],
@@ -681,7 +691,8 @@ def _call(name, *args):
     _check(getattr(lib(), name)(*args), name)
 
 
-ACT_NONE, ACT_SQUARED_RELU, ACT_SILU, ACT_GELU = 0, 1, 2, 3
+ACT_NONE, ACT_SQUARED_RELU, ACT_SILU, ACT_GELU, ACT_GATED = 0, 1, 2, 3, 4
+SCORES_SOFTMAX, SCORES_SIGMOID = 0, 1
 NORM_NONE, NORM_RMS, NORM_LAYER = 0, 1, 2
 
 
@@ -715,12 +726,12 @@ def gemm_nk_sums(a, b, max_shares=1):
     return p
 
 
-def embed_rows(tokens, positions, embed, pos):
-    """(fp32 rows, rows in the tables' type)"""
+def embed_rows(tokens, positions, embed, pos, scale=1.0):
+    """(fp32 rows, rows in the tables' type); the embedding is multiplied by scale"""
     T, ld = tokens.numel(), embed.shape[1]
     x = torch.empty((T, ld), dtype=torch.float32, device=embed.device)
     act = torch.empty((T, ld), dtype=embed.dtype, device=embed.device)
-    _call("nf_embed_rows", _dt(embed), _p(tokens), _p(positions), _p(embed), _p(pos), _p(x), _p(act), T, ld, _stream())
+    _call("nf_embed_rows", _dt(embed), _p(tokens), _p(positions), _p(embed), _p(pos), scale, _p(x), _p(act), T, ld, _stream())
     return x, act
 
 
@@ -730,20 +741,26 @@ def norm(kind, weight=None, bias=None, eps=0.0) -> Norm:
     return n
 
 
-def residual_rows(y, x, act, width, y_norm=None, next_norm=None, y_scale=1.0):
-    """x += y_scale * y_norm(y) in place; y [shares, T, ld] fp32 or [T, ld] bf16; act (or None) receives next_norm(x) in its type."""
-    shares = y.shape[0] if y.dim() == 3 else 1
+def residual_rows(y, x, act, width, y_norm=None, next_norm=None, y_scale=1.0, add=None, table=None, tokens=None, table_scale=1.0):
+    """x += y_scale * y_norm(y) in place; y [shares, T, ld] fp32 or [T, ld] bf16 (or None); then x += add + table_scale * table[tokens];
+    act (or None) receives next_norm(x) in its type."""
+    shares = y.shape[0] if y is not None and y.dim() == 3 else 1
     T, ld = x.shape
-    a = ResidualArgs(rows=T, width=width, ld=ld, y_dtype=_dt(y), shares=shares, y=_p(y), y_norm=y_norm or Norm(), next=next_norm or Norm(),
-                     y_scale=y_scale, x=_p(x), dtype=_dt(act) if act is not None else F32, act=_p(act))
+    a = ResidualArgs(rows=T, width=width, ld=ld, y_dtype=F32 if y is None else _dt(y), shares=shares, y=_p(y), y_norm=y_norm or Norm(),
+                     next=next_norm or Norm(), y_scale=y_scale, x=_p(x), dtype=_dt(act) if act is not None else F32, act=_p(act), add=_p(add),
+                     table=_p(table), tokens=_p(tokens), table_scale=table_scale)
     _call("nf_residual_rows", C.byref(a), _stream())
 
 
-def mixture_rows(y, routing, top, identity, x, act, width, next_norm=None, y_scale=1.0):
-    """x += y_scale * the weighted sum of every token's sorted rows of y [sorted, ld] and of identity [T, ld]."""
+def mixture_rows(y, routing, top, identity, x, act, width, next_norm=None, y_scale=1.0, y_norm=None, plain=False):
+    """x += y_scale * y_norm of the weighted sum (plain: the sum) of every token's sorted rows of y [sorted, ld] and of identity
+    [T, ld] (or None)."""
     T, ld = x.shape
-    a = ResidualArgs(rows=T, width=width, ld=ld, y=_p(y), routing=C.pointer(routing), top=top, y_ld=y.shape[1], identity=_p(identity),
-                     next=next_norm or Norm(), y_scale=y_scale, x=_p(x), dtype=_dt(identity), act=_p(act))
+    if plain:
+        routing = Routing.from_buffer_copy(routing)
+        routing.weight = None
+    a = ResidualArgs(rows=T, y_norm=y_norm or Norm(), width=width, ld=ld, y=_p(y), routing=C.pointer(routing), top=top, y_ld=y.shape[1], identity=_p(identity),
+                     next=next_norm or Norm(), y_scale=y_scale, x=_p(x), dtype=_dt(y), act=_p(act))
     _call("nf_residual_rows", C.byref(a), _stream())
 
 
@@ -774,18 +791,19 @@ def token_gate_rows(sums, tokens, table, col0, dim):
     return out
 
 
-def route(z, outputs, experts, top, correction, scale, tile_rows, groups=1, keep_groups=1, always=0):
+def route(z, outputs, experts, top, correction, scale, tile_rows, groups=1, keep_groups=1, always=0, scores=SCORES_SOFTMAX, always_plain=False):
     """(Routing, dict of its tensors) of router outputs z [shares, T, ld] fp32; always: experts of every token behind the chosen
-    ones, weighed by the column after the outputs."""
+    ones, weighed by the column after the outputs (always_plain: by 1)."""
     shares, T, ld = z.shape
     n, e = T * (top + always), experts + always
     i32 = lambda k: torch.full((k,), -7, dtype=torch.int32, device=z.device)
     t = {"choice": i32(n), "weight": torch.empty(n, dtype=torch.float32, device=z.device), "place": i32(n), "row_of": i32(n),
-         "offsets": i32(e + 1), "tile_group": i32(lib().nf_routing_max_tiles(n, e, tile_rows)), "n_tiles": i32(1)}
+         "offsets": i32(e + 1), "tile_group": i32(lib().nf_routing_max_tiles(n, e, tile_rows)), "n_tiles": i32(1),
+         "row_weight": torch.full((n,), -7.0, dtype=torch.float32, device=z.device)}
     t["tile_row"] = torch.empty_like(t["tile_group"])
     r = Routing(**{k: _p(v) for k, v in t.items()}, tile_rows=tile_rows)
     a = RouteArgs(z=_p(z), shares=shares, ld=ld, rows=T, outputs=outputs, experts=experts, top=top, always=always, groups=groups,
-                  keep_groups=keep_groups, correction=_p(correction), scale=scale)
+                  keep_groups=keep_groups, correction=_p(correction), scale=scale, scores=scores, always_plain=int(always_plain))
     _call("nf_route", C.byref(a), C.byref(r), _stream())
     return r, t
 
@@ -799,11 +817,13 @@ def gemm_grouped_heads(a, b, d, a_group, d_group):
     return d
 
 
-def gemm_grouped_experts(a, b, d, routing, max_rows, gather, act=ACT_NONE):
-    """Sorted rows d = act(A . B_e^T): a holds tokens (gather) or sorted rows."""
+def gemm_grouped_experts(a, b, d, routing, max_rows, gather, act=ACT_NONE, weigh=False, gated=(1.0, 0.0, None)):
+    """Sorted rows d = act(A . B_e^T): a holds tokens (gather) or sorted rows.  weigh: the product's rows are multiplied by their
+    weights first; gated: slope, shift and limits per expert of ACT_GATED."""
     e, N, Kd = b.shape
     args = GroupedGemmArgs(dtype=_dt(a), act=act, groups=e, M=a.shape[0], N=N, K=Kd, a=_p(a), lda=a.shape[1], b=_p(b), d=_p(d),
-                           ldd=d.shape[1], routing=routing, gather=int(gather), max_rows=max_rows)
+                           ldd=d.shape[1], routing=routing, gather=int(gather), max_rows=max_rows, weigh=int(weigh),
+                           gated=GatedAct(gated[0], gated[1], _p(gated[2])))
     _call("nf_gemm_grouped", C.byref(args), _stream())
     return d
 
@@ -850,13 +870,15 @@ def short_conv(weight, state, input_indptr, state_slots) -> ShortConv:
     return c
 
 
-def qkv_append(layout, proj, cols, q_norm, k_norm, eps, rot, pool, kv_indptr, kv_indices, rev_input_indptr, positions, q_temp=None, conv=None):
+def qkv_append(layout, proj, cols, q_norm, k_norm, eps, rot, pool, kv_indptr, kv_indices, rev_input_indptr, positions, q_temp=None, conv=None,
+               value_norm=False, value_rot=None):
     """Returns the normed, rotated queries [T, heads * maps, k_pad]; keys and values go to the pool's pages, what a convolution
     needs of these rows to its state."""
     T = proj.shape[0]
     q = torch.empty((T, layout.heads * layout.maps, layout.k_pad), dtype=proj.dtype, device=proj.device)
     _call("nf_qkv_append", C.byref(layout), _p(proj), proj.shape[1], *cols, _p(q_norm), _p(k_norm), eps, C.byref(rot),
-          C.byref(QueryTemperature(*q_temp)) if q_temp else None, C.byref(conv) if conv else None, _p(q), _p(pool), _p(kv_indptr),
+          C.byref(QueryTemperature(*q_temp)) if q_temp else None,
+          C.byref(ValueForm(int(value_norm), value_rot or Rotation())) if value_norm or value_rot else None, C.byref(conv) if conv else None, _p(q), _p(pool), _p(kv_indptr),
           _p(kv_indices), _p(rev_input_indptr), _p(positions), T, _stream())
     if conv:
         _call("nf_conv_state", _dt(proj), _p(proj), proj.shape[1], C.byref(conv), _p(positions), 0, kv_indptr.numel() - 1, _stream())
@@ -864,13 +886,13 @@ def qkv_append(layout, proj, cols, q_norm, k_norm, eps, rot, pool, kv_indptr, kv
 
 
 def window_attention(layout, q, pool, batch, *, window, keep_first, scale, sink=None, out_scale=1.0, decode=0, gate=None, softcap=0.0,
-                     map_weight=0.0, head_eps=None):
+                     map_weight=0.0, head_eps=None, chunk=0, out_rot=None):
     """batch: dict of device arrays input_indptr, kv_indptr, kv_indices, rev_input_indptr, positions; the first
     `decode` requests have one row each.  Returns [T, heads * vdim]."""
     T = q.shape[0]
     out = torch.zeros((T, layout.heads * layout.vdim), dtype=q.dtype, device=q.device)
     n_req = batch["input_indptr"].numel() - 1
-    a = WindowAttentionArgs(kv=layout, window=window, keep_first=keep_first, scale=scale, out_scale=out_scale, softcap=softcap,
+    a = WindowAttentionArgs(kv=layout, window=window, keep_first=keep_first, chunk=chunk, out_rot=out_rot or Rotation(), scale=scale, out_scale=out_scale, softcap=softcap,
                             map_weight=map_weight, head_norm=int(head_eps is not None), head_eps=head_eps or 0.0, sink=_p(sink),
                             gate=_p(gate), gate_ld=gate.shape[1] if gate is not None else 0, q=_p(q), out=_p(out), out_ld=out.shape[1], out_col=0, kv_data=_p(pool))
     for n in ("input_indptr", "kv_indptr", "kv_indices", "rev_input_indptr", "positions"):

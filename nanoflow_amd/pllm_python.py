@@ -649,7 +649,7 @@ def stackInitTensors(tensors: dict, global_batch: int):
     kinds = {np.dtype(np.uint16): 0, np.dtype(np.float32): 1, np.dtype(np.int32): 2}
     keep, c = [], (_CHostTensor * len(tensors))()
     for i, (name, a) in enumerate(tensors.items()):
-        a = np.ascontiguousarray(a)
+        a = np.asarray(a, order="C")        # (a single number stays one)
         shape = (C.c_int64 * max(a.ndim, 1))(*a.shape)
         keep.extend([a, shape])
         c[i] = _CHostTensor(name.encode(), kinds[a.dtype], a.ndim, shape, a.ctypes.data)

@@ -59,8 +59,18 @@ def pudadra_config(width, ff):
             "layers": [{"type": t, "mixer": m, "mlp": f} for t, m, f in layers]}
 
 
+def desalix_config(width, ff):
+    """Three layers of attention in chunks of 1024 (heads of 128, 4 query heads per kv head), the middle one passed twice; 32 experts
+    of a quarter of `ff`, 4 of them per token, and a shared one."""
+    n, expert = width // 128, {"ff": ff // 4, "limit": 7.0}
+    attention = {"heads": n, "kv_heads": n // 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": 1024}, "rot": {"dims": 64, "base": 5e5}}
+    moe = {"kind": "moe", "expert": expert, "shared": expert, "router": {"experts": 32, "top": 4}}
+    return {"architecture": "Desalix", "width": width, "vocab": VOCAB, "embedding": {"scale": 8.0}, "norm": {"eps": 1e-5},
+            "loop": {"start": 1, "stop": 2, "times": 2}, "layers": [{"type": "attention", "mixer": attention, "mlp": moe}] * 3}
+
+
 # side -> configuration of a layer-stack model; "llama" is the other kind
-DESIGNS = {"stack": stack_config, "fipuzen": fipuzen_config, "pudadra": pudadra_config}
+DESIGNS = {"stack": stack_config, "fipuzen": fipuzen_config, "pudadra": pudadra_config, "desalix": desalix_config}
 SIZES = {"2048": (2048, 8192), "4096": (4096, 14336)}
 
 
@@ -111,7 +121,8 @@ def run_sizes(steps=20, warmup=4, sizes=tuple(SIZES), cases=None, sides=("stack"
         for side in sides:
             if side in DESIGNS:
                 cfg = DESIGNS[side](width, ff)
-                assert len(cfg["layers"]) == layers
+                loop = cfg.get("loop") or {"start": 0, "stop": 0, "times": 1}
+                assert len(cfg["layers"]) + (loop["times"] - 1) * (loop["stop"] - loop["start"]) == layers
                 e = engine.StackEngine(cfg, global_batch=2048, kv_pages=pages, state_slots=256, rank=64)
             else:
                 shape = synth.ModelShape(hidden=width, Hq=width // 128, Hkv=width // 512, d=128, ffn=ff, vocab=VOCAB, layers=layers)

@@ -107,7 +107,29 @@ def _pudadra_shapes(cfg: dict, rank: int) -> dict:
     return out
 
 
-ARCHITECTURES = {"Zovovik": _zovovik_shapes, "Fipuzen": _fipuzen_shapes, "Pudadra": _pudadra_shapes}
+def _desalix_shapes(cfg: dict, rank: int) -> dict:
+    W, V = cfg["width"], cfg["vocab"]
+    out = {"embed": (V, W), "head": (V, W), "final.norm": ()}
+    if cfg.get("loop"):
+        out["loop.step"] = (cfg["loop"]["times"], W)
+    for i, layer in enumerate(cfg["layers"]):
+        l, x, m = f"l{i}.", f"l{i}.mix.", layer["mixer"]
+        out.update({l + "norm1": (), l + "norm1b": (), l + "ls1": (W,)})
+        out.update({x + "q": (m["heads"] * m["dim"], W), x + "k": (m["kv_heads"] * m["dim"], W), x + "v": (m["kv_heads"] * m["vdim"], W),
+                    x + "q.norm": (m["dim"],), x + "k.norm": (m["dim"],), x + "sink": (m["heads"],), x + "o": (W, m["heads"] * m["vdim"])})
+        f, p = layer.get("mlp"), l + "mlp."
+        if not f:
+            continue
+        out.update({l + "norm2": (), l + "norm2b": (), l + "ls2": (W,), p + "router": (f["router"]["experts"], W)})
+        experts = {f"e{e}.": f["expert"]["ff"] for e in range(f["router"]["experts"])}
+        if f.get("shared"):
+            experts["shared."] = f["shared"]["ff"]
+        for e, n in experts.items():
+            out.update({p + e + "gate": (n, W), p + e + "up": (n, W), p + e + "down": (W, n)})
+    return out
+
+
+ARCHITECTURES = {"Zovovik": _zovovik_shapes, "Fipuzen": _fipuzen_shapes, "Pudadra": _pudadra_shapes, "Desalix": _desalix_shapes}
 # designs whose norms of the residual stream are stored as the difference from one
 NORMS_AROUND_ZERO = ("Pudadra",)
 
@@ -148,6 +170,8 @@ def random_tensors(cfg: dict, seed: int = 0, rank: int = 16) -> dict:
         if "norm" in leaf:
             around_zero = cfg["architecture"] in NORMS_AROUND_ZERO and ".mix." not in name
             x = 0.1 * x if around_zero else 1.0 + 0.1 * x
+        elif leaf in ("ls1", "ls2"):            # columns count differently, and either way
+            x = 0.3 * x + 0.5
         elif leaf in ("lq1", "lk1", "lq2", "lk2"):
             x *= 0.7 * shape[0] ** -0.25
         elif ".mu." in name:
@@ -160,7 +184,7 @@ def random_tensors(cfg: dict, seed: int = 0, rank: int = 16) -> dict:
             x = 0.2 * x
         elif leaf == "correction":
             x = 0.02 * x
-        elif name in ("embed", "pos", "side.embed"):
+        elif name in ("embed", "pos", "side.embed", "loop.step"):
             pass
         else:
             x *= shape[-1] ** -0.5

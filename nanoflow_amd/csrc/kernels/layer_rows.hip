@@ -324,7 +324,7 @@ int nf_residual_rows(const nf_residual_args* args, nf_stream_t stream) {
   if (a.routing) {
     NF_REQUIRE(a.top >= 1 && a.top <= 64 && a.y_ld >= a.ld && a.y_ld % 4 == 0 && a.routing->place && (a.routing->weight || !a.identity),
                "%s: incomplete routing (top %d, stride %d)", who, a.top, a.y_ld);
-  } else if (a.y) {
+  } else if (a.y || a.shares != 0) {
     NF_REQUIRE((a.y_dtype == NF_F32 && a.shares >= 1 && a.shares <= kMaxShares) || (a.y_dtype == NF_BF16 && a.shares == 1),
                "%s: %d shares of dtype %d", who, a.shares, a.y_dtype);
   }

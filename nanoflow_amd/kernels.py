@@ -860,7 +860,9 @@ def kv_pool(layout: KVLayout, pages, device="cuda"):
 
 def rotation(table=None, dims=0, interleaved=False) -> Rotation:
     """table: fp32 [positions, dims / 2, 2] of (cos, sin)."""
-    return Rotation(_p(table) if table is not None else None, dims, int(interleaved))
+    r = Rotation(_p(table) if table is not None else None, dims, int(interleaved))
+    r.tensors = (table,)            # the struct holds addresses only
+    return r
 
 
 def short_conv(weight, state, input_indptr, state_slots) -> ShortConv:

@@ -144,12 +144,12 @@ def tensor_shapes(cfg: dict, rank: int = 16) -> dict:
 
 def bf16_bits(a) -> np.ndarray:
     """float array -> bfloat16 bit patterns (uint16), round to nearest even."""
-    u = np.ascontiguousarray(a, dtype=np.float32).view(np.uint32)
-    return ((u + np.uint32(0x7fff) + ((u >> np.uint32(16)) & np.uint32(1))) >> np.uint32(16)).astype(np.uint16)
+    u = np.asarray(a, dtype=np.float32, order="C").view(np.uint32)
+    return np.asarray((u + np.uint32(0x7fff) + ((u >> np.uint32(16)) & np.uint32(1))) >> np.uint32(16), dtype=np.uint16)
 
 
 def bits_to_f32(b) -> np.ndarray:
-    return (b.astype(np.uint32) << np.uint32(16)).view(np.float32)
+    return np.asarray(b.astype(np.uint32) << np.uint32(16)).view(np.float32)
 
 
 def random_tensors(cfg: dict, seed: int = 0, rank: int = 16) -> dict:

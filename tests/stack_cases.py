@@ -83,6 +83,22 @@ def pudadra(layers, width=104, vocab=211, eps=1e-5, residual_mult=0.7, logit_sca
             "norm": {"eps": eps}, "layers": [{**mixer, "mlp": f} for mixer, f in layers]}
 
 
+def chunked(heads=6, kv_heads=2, dim=24, vdim=40, chunk=21, rot=16, base=300.0, scale=0.3):
+    return {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale,
+                                           "mask": chunk and {"size": chunk}, "rot": {"dims": rot, "base": base}}}
+
+
+def gated_moe(experts=6, top=2, ff=40, limit=0.6, shared=56, shared_limit=0.9):
+    m = {"kind": "moe", "expert": {"ff": ff, "limit": limit}, "router": {"experts": experts, "top": top}}
+    return {**m, "shared": {"ff": shared, "limit": shared_limit}} if shared else m
+
+
+def desalix(layers, loop=None, width=104, vocab=211, eps=1e-5, scale=1.7):
+    """layers: (mixer, feed-forward or None); loop: (start, stop, times)"""
+    return {"architecture": "Desalix", "width": width, "vocab": vocab, "embedding": {"scale": scale}, "norm": {"eps": eps},
+            "loop": loop and dict(zip(("start", "stop", "times"), loop)), "layers": [{**mixer, "mlp": f} for mixer, f in layers]}
+
+
 # sizes that are not multiples of 8, equal and unequal head counts, no feed-forward, a window of one, windows without kept tokens
 CONFIGS = {
     "mixed": config([retention(), parallel(), (retention(heads=1, dim=16, vdim=16, rot=16, decay=(0.9,)), None), parallel(
@@ -116,6 +132,19 @@ CONFIGS = {
     "window of one map": pudadra([(differential(heads=2, kv_heads=2, dim=8, vdim=8, window=1, rot=8, conv=2), grouped_moe(2, 2, 1, 1, 8, 8)),
                                   (windowed_latent(heads=1, dim=8, rot=2, vdim=8, kv_rank=8, window=1), None),
                                   (differential(heads=9, kv_heads=3, dim=16, vdim=32, window=16, rot=0, conv=9), dense(8))], width=40),
+    "chunks": desalix([(chunked(), gated_moe()), (chunked(heads=4, kv_heads=4, dim=32, vdim=16, chunk=50, rot=32), None), (chunked(chunk=16), gated_moe(4, 3, 24)),
+                       (chunked(heads=2, kv_heads=1, dim=16, vdim=48, chunk=35, base=90.0), gated_moe(5, 1, 64, 1.5, 20, 0.4))], loop=(1, 3, 3)),
+    "odd chunks": desalix([(chunked(heads=5, kv_heads=1, dim=18, vdim=10, chunk=7, rot=6), gated_moe(7, 4, 18, 0.3, 70, 2.0)),
+                           (chunked(heads=3, kv_heads=1, dim=9, vdim=6, chunk=40, rot=2, scale=0.8), None),
+                           (chunked(heads=2, kv_heads=2, dim=7, vdim=2, chunk=300, rot=0), gated_moe(3, 2, 13, 0.7, None))], loop=(0, 2, 2), width=51, vocab=97,
+                          eps=1e-3, scale=0.4),
+    "large chunks": desalix([(chunked(heads=4, kv_heads=2, dim=64, vdim=64, chunk=60, rot=64), gated_moe(16, 5, 72, 0.8, 72)),
+                             (chunked(heads=5, kv_heads=1, dim=128, vdim=128, chunk=33, rot=96, scale=0.1), gated_moe(4, 2, 64, 0.5, 300, 0.7)),
+                             (chunked(heads=20, kv_heads=1, dim=192, vdim=128, chunk=97, rot=128, scale=0.1), None),
+                             (chunked(heads=2, kv_heads=2, dim=160, vdim=144, chunk=64, rot=80), gated_moe(8, 8, 160, 1.0, 8))], loop=(2, 4, 2), width=128),
+    "chunk of one": desalix([(chunked(heads=2, kv_heads=2, dim=8, vdim=8, chunk=1, rot=8), gated_moe(1, 1, 8, 0.5, 8)),
+                             (chunked(heads=9, kv_heads=3, dim=16, vdim=32, chunk=None, rot=4), gated_moe(2, 1, 8, 0.5, None))], loop=(1, 2, 1), width=40),
+    "one chunk": desalix([(chunked(chunk=None), gated_moe(shared=None)), (chunked(heads=1, kv_heads=1, dim=8, vdim=8, chunk=128, rot=8), None)]),
     "window of one": config([parallel(heads=20, kv_heads=1, dim=8, vdim=8, window=1, keep=0, rot=8, right_heads=2, right_dim=8)], width=64),
 }
 

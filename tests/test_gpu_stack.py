@@ -80,7 +80,7 @@ def test_whole_prompts_and_every_layer(name, dtype):
     with make(name, dtype, keep_layers=True) as e:
         r = e.replay()
         got = r.step([("a", tok, range(len(tok)))], e.vocab)["a"]
-        for i in range(len(cfg["layers"])):
+        for i in range(len(layers)):
             check(P.stackLayerOutput(i), layers[i], dtype, f"layer {i}", chooses(name))
         check(got, want, dtype, "logits", chooses(name))
         r.close()
@@ -88,7 +88,7 @@ def test_whole_prompts_and_every_layer(name, dtype):
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("name", ["mixed", "odd", "wide heads", "five layers", "odd sizes", "large heads", "one expert", "two maps", "odd maps", "large maps",
-                                  "window of one map"])
+                                  "window of one map", "chunks", "odd chunks", "large chunks", "chunk of one", "one chunk"])
 def test_token_by_token_and_portions_agree_with_the_whole(name, dtype):
     (tok,), (want,) = sequences(name, [90])
     with make(name, dtype) as e:
@@ -106,7 +106,7 @@ def test_token_by_token_and_portions_agree_with_the_whole(name, dtype):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("name", ["mixed", "five layers", "two maps"])
+@pytest.mark.parametrize("name", ["mixed", "five layers", "two maps", "chunks"])
 def test_unequal_requests_beside_each_other_and_slots_used_again(name, dtype):
     """Portions beside single tokens, requests that pause, end and leave their pages and slots to others."""
     lengths = [140, 1, 33, 75, 64, 2, 110, 17, 48, 90]
@@ -142,7 +142,7 @@ def test_unequal_requests_beside_each_other_and_slots_used_again(name, dtype):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("name", ["mixed", "five layers", "two maps"])
+@pytest.mark.parametrize("name", ["mixed", "five layers", "two maps", "chunks"])
 def test_long_decoding(name, dtype):
     (tok,), (want,) = sequences(name, [330], seed=8)
     with make(name, dtype) as e:
@@ -156,7 +156,7 @@ def test_long_decoding(name, dtype):
         r.close()
 
 
-@pytest.mark.parametrize("name", ["mixed", "five layers", "two maps"])
+@pytest.mark.parametrize("name", ["mixed", "five layers", "two maps", "chunks"])
 def test_many_rows_and_only_some_logits(name):
     """A step of more rows than the small-batch paths take, logits of a few places only."""
     (tok,), (want,) = sequences(name, [580], seed=9)
@@ -199,7 +199,7 @@ def greedy(cfg, t, prompt, n):
     return seq[len(prompt):]
 
 
-@pytest.mark.parametrize("name", ["odd", "odd sizes", "five layers", "odd maps", "two maps"])
+@pytest.mark.parametrize("name", ["odd", "odd sizes", "five layers", "odd maps", "two maps", "odd chunks", "chunks"])
 def test_greedy_generation_through_the_scheduler(name):
     """The batch former and the serving loop (fp32: the sampled ids are the plain implementation's), eagerly and replayed from
     graphs; more requests than slots."""
@@ -226,7 +226,7 @@ def test_greedy_generation_through_the_scheduler(name):
             f.close()
 
 
-@pytest.mark.parametrize("name", ["mixed", "five layers", "two maps"])
+@pytest.mark.parametrize("name", ["mixed", "five layers", "two maps", "chunks"])
 def test_graph_replays_equal_eager_iterations(name):
     from nanoflow_amd import synth
     cfg, bits, _ = model(name)
@@ -253,7 +253,7 @@ def test_graph_replays_equal_eager_iterations(name):
         np.testing.assert_array_equal(run, logits[0][0])
 
 
-@pytest.mark.parametrize("name", ["mixed", "odd sizes", "two maps"])
+@pytest.mark.parametrize("name", ["mixed", "odd sizes", "two maps", "chunks"])
 def test_trace_program(name, tmp_path):
     """bin/trace_run on a model directory: steps on standard input, logits in files."""
     cfg, bits, _ = model(name)
@@ -276,7 +276,7 @@ def test_trace_program(name, tmp_path):
             check(np.fromfile(out / f"{i}.f32", "<f4").reshape(w.shape), w, dtype, f"step {i}", chooses(name))
 
 
-@pytest.mark.parametrize("name", ["odd", "odd sizes", "odd maps"])
+@pytest.mark.parametrize("name", ["odd", "odd sizes", "odd maps", "odd chunks"])
 def test_serve_command_line(name, tmp_path):
     cfg, bits, t = model(name)
     stack_models.save_model(str(tmp_path / "m"), cfg, bits)

@@ -162,7 +162,49 @@ def test_latent_window_leaves_out_what_is_behind_it():
     np.testing.assert_allclose(o[8], S.latent_attention(q[6:], qr[6:], lat[6:], kr[6:], uk, uv, 0.4)[2], rtol=1e-9)
 
 
-@pytest.mark.parametrize("name", ["mixed", "five layers", "two maps", "odd maps"])
+def test_chunk_mask_edges():
+    m = S.chunk_mask(30, 8)
+    assert m[15, 8] and not m[15, 7] and m[16, 16] and not m[16, 15] and not m[16, 17] and m[7, 0]
+    assert np.array_equal(S.chunk_mask(30, 1), np.eye(30, dtype=bool)) and np.array_equal(S.chunk_mask(9, None), np.tri(9, dtype=bool))
+
+
+def test_turned_values_come_back_turned_by_the_distance():
+    """A weighted sum of turned values, turned back at the query, is the sum of the values turned by key less query."""
+    rng = np.random.default_rng(9)
+    v, a = rng.standard_normal((6, 1, 8)), rng.random(6)
+    o = S.turn_values((a[:, None, None] * S.turn_values(v, np.arange(6), 40.0)).sum(0, keepdims=True), [5], 40.0, back=True)
+    want = sum(a[j] * S.turn_values(v[j:j + 1], [j - 5], 40.0) for j in range(6))
+    np.testing.assert_allclose(o, want, rtol=1e-12)
+    np.testing.assert_allclose(S.turn_values(v, np.arange(6), 40.0), S.rotate(v, np.arange(6), 8, 40.0, False), rtol=1e-12)
+
+
+def test_a_clamped_experts_bounds():
+    t = {"gate": np.array([[1.0], [1.0]]), "up": np.array([[1.0], [-1.0]]), "down": np.eye(2)}
+    sig = lambda z: 1 / (1 + np.exp(-z))
+    y = S.clamped_expert(t, "", 2.0, np.array([[1.0], [5.0], [-5.0]]))
+    np.testing.assert_allclose(y[0], [sig(1.702) * 2, 0], atol=1e-12)
+    np.testing.assert_allclose(y[1], [2 * sig(3.404) * 3, -2 * sig(3.404)])             # both bounded
+    np.testing.assert_allclose(y[2], [5 * sig(-8.51), -15 * sig(-8.51)])                # a gate is not bounded from below
+
+
+def test_weights_go_into_the_experts_and_are_not_shared_out():
+    rng = np.random.default_rng(10)
+    W, f = 5, 4
+    t = {f"m.e{e}.{s}": rng.standard_normal((W, f) if s == "down" else (f, W)) for e in range(3) for s in ("gate", "up", "down")}
+    t["m.router"] = np.zeros((3, W))
+    t["m.router"][:, 0] = [0.0, 2.0, 1.0]
+    h = np.ones((1, W))
+    y = S.input_weighted_mixture(t, "m.", {"router": {"top": 2}, "expert": {"limit": 0.5}}, h)
+    np.testing.assert_allclose(y, S.clamped_expert(t, "m.e1.", 0.5, h / (1 + np.exp(-2.0))) + S.clamped_expert(t, "m.e2.", 0.5, h / (1 + np.exp(-1.0))), rtol=1e-9)
+
+
+def test_order_of_looped_layers():
+    loop = {"start": 1, "stop": 3, "times": 2}
+    assert S.layer_runs(4, loop) == [(0, None), (1, 0), (2, None), (1, 1), (2, None), (3, None)]
+    assert S.layer_runs(2, None) == [(0, None), (1, None)] and S.layer_runs(1, {"start": 0, "stop": 1, "times": 3}) == [(0, 0), (0, 1), (0, 2)]
+
+
+@pytest.mark.parametrize("name", ["mixed", "five layers", "two maps", "odd maps", "chunks", "odd chunks"])
 def test_a_prefix_does_not_see_what_follows(name):
     cfg = cases.CONFIGS[name]
     _, t = cases.tensors(cfg)
@@ -205,7 +247,14 @@ def test_configurations_are_checked(tmp_path):
                (cases.pudadra([(cases.differential(), cases.grouped_moe(8, 3, 1, 1))]), "groups"),
                (cases.pudadra([(cases.differential(), cases.grouped_moe(8, 4, 1, 3))]), "groups"),
                (cases.pudadra([(cases.differential(), {"kind": "nosuch"})]), "feed-forward"),
-               ({k: v for k, v in cases.CONFIGS["two maps"].items() if k != "residual_mult"}, "residual_mult")]
+               ({k: v for k, v in cases.CONFIGS["two maps"].items() if k != "residual_mult"}, "residual_mult"),
+               (cases.desalix([(cases.chunked(heads=5, kv_heads=2), None)]), "multiple"), (cases.desalix([(cases.chunked(chunk=-3), None)]), "mask"),
+               (cases.desalix([(cases.chunked(chunk=2.5), None)]), "integer"), (cases.desalix([(cases.chunked(vdim=9), None)]), "rotated"),
+               (cases.desalix([(cases.chunked(rot=26), None)]), "rotated"), (cases.desalix([(cases.chunked(), cases.gated_moe(4, 5))]), "uses"),
+               (cases.desalix([(cases.chunked(), cases.gated_moe(limit=-1.0))]), "limit"), (cases.desalix([(cases.chunked(), cases.dense())]), "feed-forward"),
+               (cases.desalix([(cases.latent(), None)]), "unknown mixer"),
+               *((cases.desalix([(cases.chunked(), None)] * 2, loop=l), "loop") for l in ((0, 3, 2), (1, 1, 2), (-1, 1, 2), (0, 1, 0))),
+               ({k: v for k, v in cases.CONFIGS["chunks"].items() if k != "embedding"}, "embedding")]
         for cfg, word in bad:
             with pytest.raises(P.NanoflowPipelineError, match=word):
                 _set(tmp_path, cfg)
@@ -237,7 +286,7 @@ def test_pipeline_file_names_a_stack_model(tmp_path):
 
 
 @pytest.mark.parametrize("name,some", [("mixed", ("embed", "l1.mix.left.sink", "l1.mix.right.u")),
-                                       ("two maps", ("embed", "l0.mix.q.conv", "l4.mix.lq2", "l1.mlp.shared.sg")), ("five layers", ("side.embed", "l0.mix.q.b", "l2.mlp.e1.down", "l2.mlp.correction"))])
+                                       ("chunks", ("loop.step", "l0.norm1b", "final.norm", "l3.mlp.shared.gate")), ("two maps", ("embed", "l0.mix.q.conv", "l4.mix.lq2", "l1.mlp.shared.sg")), ("five layers", ("side.embed", "l0.mix.q.b", "l2.mlp.e1.down", "l2.mlp.correction"))])
 def test_safetensors_of_random_tensors_reads_back(tmp_path, name, some):
     from safetensors import safe_open
     cfg = cases.CONFIGS[name]
@@ -333,6 +382,11 @@ def test_argument_errors_without_a_gpu():
     assert l.nf_gemm_grouped(ctypes.byref(g), None) == -1 and b"activation" in l.nf_last_error()
     g = K.GroupedGemmArgs(dtype=K.BF16, groups=2, M=4, N=8, K=8, lda=8, ldd=4)
     assert l.nf_gemm_grouped(ctypes.byref(g), None) == -1 and b"strides" in l.nf_last_error()
+    g = K.GroupedGemmArgs(dtype=K.BF16, groups=2, M=4, N=8, K=8, lda=8, ldd=8, weigh=1)
+    assert l.nf_gemm_grouped(ctypes.byref(g), None) == -1 and b"weights" in l.nf_last_error()
+    w = K.WindowAttentionArgs(kv=K.KVLayout(K.BF16, 4, 2, 8, 8, 32, 16, 16, 1), out_ld=32, out_rot=K.Rotation(None, 8, 0))
+    assert l.nf_window_attention(ctypes.byref(w), None) == -1 and b"turned back" in l.nf_last_error()
+    assert route(scores=2) == -1 and b"scores" in l.nf_last_error()
     lay = K.LatentLayout()
     assert l.nf_latent_layout_of(K.BF16, 4, 20, 6, 16, ctypes.byref(lay)) == 0 and (lay.rank_pad, lay.row_ld) == (24, 64)
     assert l.nf_latent_layout_of(K.BF16, 4, 4000, 6, 16, ctypes.byref(lay)) == -1

@@ -285,7 +285,7 @@ __global__ __launch_bounds__(256) void qkv_append_kernel(nf_kv_layout kv, const 
 // lanes.  Of many rows, values are turned through LDS, 16 rows of a head at a time, so that the transposed cache is
 // written four positions at once where four rows are an aligned run of one page; of few (value_blocks = 0) value heads
 // are taken like the others.
-template <class T, int kVec, int R>
+template <class T, int kVec, int R, bool kConv>
 __global__ __launch_bounds__(256, kVec <= 2 ? 8 : 5) void qkv_append4_kernel(nf_kv_layout kv, const T* __restrict__ proj, int ld, int q_col,
                                                           int k_col, int v_col, const float* __restrict__ q_norm,
                                                           const float* __restrict__ k_norm, float eps, nf_rotation rot,
@@ -295,6 +295,7 @@ __global__ __launch_bounds__(256, kVec <= 2 ? 8 : 5) void qkv_append4_kernel(nf_
                                                           const int32_t* __restrict__ rev_input_indptr,
                                                           const int32_t* __restrict__ positions, int rows, int value_blocks) {
   __shared__ __attribute__((aligned(16))) float buf[kMaxHeadDim * 17];
+  if constexpr (!kConv) conv.taps = 0;  // its code is left out
   const int H = kv.heads * kv.maps, G = kv.kv_heads * kv.maps, VG = kv.kv_heads, tid = threadIdx.x;
   if ((int)blockIdx.x >= value_blocks) {
     const int jobs = H + G + (value_blocks > 0 ? 0 : VG), head_blocks = (jobs + 15) / 16, block = blockIdx.x - value_blocks;
@@ -1202,7 +1203,7 @@ int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, i
   const size_t four = 4 * (kv->dtype == NF_BF16 ? 2 : 4);
   const uintptr_t places = (uintptr_t)proj | (uintptr_t)cv.weight | (uintptr_t)cv.state | (uintptr_t)q_out | (uintptr_t)kv_data;
   const int sizes = kv->dim | kv->vdim | ld | q_col | k_col | v_col, turned = rot->interleaved ? rot->dims : rot->dims / 2;
-  if (sizes % 4 == 0 && places % four == 0 && turned % 4 == 0 && rows < (1 << 20)) {
+  if (sizes % 4 == 0 && places % four == 0 && (turned | vf.rot.dims) % 4 == 0 && rows < (1 << 20)) {
     const bool few = rows < 1024;
     auto go = [&](auto type, auto vec, auto run) {
       using T = decltype(type);
@@ -1210,10 +1211,12 @@ int nf_qkv_append(const nf_kv_layout* kv, const void* proj, int ld, int q_col, i
       const int value_blocks = few ? 0 : (rows + 15) / 16 * kv->kv_heads;
       const int jobs = (kv->heads + kv->kv_heads) * kv->maps + (few ? kv->kv_heads : 0);
       const int blocks = value_blocks + (rows + kRun - 1) / kRun * ((jobs + 15) / 16);
-      qkv_append4_kernel<T, decltype(vec)::value, kRun><<<(unsigned)blocks, 256, 0, s>>>(
-          *kv, (const T*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot, temp, vf, cv, (T*)q_out, (T*)kv_data, kv_indptr, kv_indices,
-          rev_input_indptr, positions, rows, value_blocks);
-      return check_launch(who);
+      auto launch = [&](auto kern) {
+        kern<<<(unsigned)blocks, 256, 0, s>>>(*kv, (const T*)proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, *rot, temp, vf, cv, (T*)q_out,
+                                              (T*)kv_data, kv_indptr, kv_indices, rev_input_indptr, positions, rows, value_blocks);
+        return check_launch(who);
+      };
+      return cv.taps > 0 ? launch(qkv_append4_kernel<T, decltype(vec)::value, kRun, true>) : launch(qkv_append4_kernel<T, decltype(vec)::value, kRun, false>);
     };
     auto sized = [&](auto type, auto run) {
       const int widest = few ? std::max(kv->k_pad, kv->v_pad) : kv->k_pad;

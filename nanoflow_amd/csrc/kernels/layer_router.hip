@@ -125,9 +125,16 @@ __global__ __launch_bounds__(1024) void route_plan_kernel(nf_routing r, int rows
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, routed = experts - always, per_token = top + always, n = rows * per_token;
   count[tid] = tid >= routed && tid < experts ? rows : 0;
   __syncthreads();
-  for (int i = tid; i < n; i += 1024) {
-    const int e = r.choice[i];
-    if (i % per_token < top && e < routed) atomicAdd(&count[e], 1);
+  constexpr int kAhead = 4;  // choices of a thread requested at once
+  for (int i0 = tid; i0 < n; i0 += kAhead * 1024) {
+    int e[kAhead];
+#pragma unroll
+    for (int k = 0; k < kAhead; ++k) e[k] = r.choice[min(i0 + k * 1024, n - 1)];
+#pragma unroll
+    for (int k = 0; k < kAhead; ++k) {
+      const int i = i0 + k * 1024;
+      if (i < n && i % per_token < top && e[k] < routed) atomicAdd(&count[e[k]], 1);
+    }
   }
   __syncthreads();
   // exclusive sums over the experts: rows, tiles
@@ -162,16 +169,27 @@ __global__ __launch_bounds__(1024) void route_plan_kernel(nf_routing r, int rows
     }
   }
   __syncthreads();
-  for (int i = tid; i < n; i += 1024) {
-    const int t = i / per_token, k = i % per_token, e = r.choice[i];
-    int at = -1;
-    if (k >= top) at = first[routed + k - top] + t;
-    else if (e < routed) at = atomicAdd(&first[e], 1);
-    if (at >= 0) {
-      r.row_of[at] = t;
-      if (r.row_weight) r.row_weight[at] = r.weight[i];
+  for (int i0 = tid; i0 < n; i0 += kAhead * 1024) {
+    int choice[kAhead];
+    float weight[kAhead];
+#pragma unroll
+    for (int x = 0; x < kAhead; ++x) {
+      choice[x] = r.choice[min(i0 + x * 1024, n - 1)];
+      weight[x] = r.weight[min(i0 + x * 1024, n - 1)];
     }
-    r.place[i] = at;
+#pragma unroll
+    for (int x = 0; x < kAhead; ++x) {
+      const int i = i0 + x * 1024, t = i / per_token, k = i % per_token, e = choice[x];
+      if (i >= n) break;
+      int at = -1;
+      if (k >= top) at = first[routed + k - top] + t;
+      else if (e < routed) at = atomicAdd(&first[e], 1);
+      if (at >= 0) {
+        r.row_of[at] = t;
+        if (r.row_weight) r.row_weight[at] = weight[x];
+      }
+      r.place[i] = at;
+    }
   }
 }
 

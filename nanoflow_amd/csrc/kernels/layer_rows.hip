@@ -8,6 +8,7 @@
 namespace nf {
 
 constexpr int kRowThreads = 256;
+constexpr int kFewRows = 512;
 constexpr int kMaxRowVec = 16;  // a row is at most 16 x 256 x 4 = 16384 columns
 
 template <class T>
@@ -26,9 +27,9 @@ __global__ __launch_bounds__(kRowThreads) void embed_rows_kernel(const int32_t* 
   }
 }
 
-// A row of up to kVec x 256 groups of four columns in registers, normed in place; columns from `width` on are zero before and
+// A row of up to kVec x kThreads groups of four columns in registers, normed in place; columns from `width` on are zero before and
 // after (the vectors are zero there).  `scratch`: 32 floats of LDS no one else uses.
-template <int kVec>
+template <int kVec, int kThreads = kRowThreads>
 __device__ __forceinline__ void norm_row(float4_t (&v)[kVec], const nf_norm& norm, int width, int ld, float* scratch) {
   const float inv_width = 1.f / (float)width;
   float mean = 0.f;
@@ -40,7 +41,7 @@ __device__ __forceinline__ void norm_row(float4_t (&v)[kVec], const nf_norm& nor
 #pragma unroll
     for (int i = 0; i < kVec; ++i)
 #pragma unroll
-      for (int e = 0; e < 4; ++e) v[i][e] = (i * kRowThreads + (int)threadIdx.x) * 4 + e < width ? v[i][e] - mean : 0.f;
+      for (int e = 0; e < 4; ++e) v[i][e] = (i * kThreads + (int)threadIdx.x) * 4 + e < width ? v[i][e] - mean : 0.f;
   }
   float sq = 0.f;
 #pragma unroll
@@ -50,16 +51,16 @@ __device__ __forceinline__ void norm_row(float4_t (&v)[kVec], const nf_norm& nor
   const float inv = 1.f / sqrtf(block_sum(sq, scratch + 16) * inv_width + norm.eps);
 #pragma unroll
   for (int i = 0; i < kVec; ++i) {
-    const int c = (i * kRowThreads + threadIdx.x) * 4;
+    const int c = (i * kThreads + threadIdx.x) * 4;
     if (c >= ld) continue;
     v[i] = v[i] * inv * *reinterpret_cast<const float4_t*>(norm.weight + c);
     if (norm.bias) v[i] += *reinterpret_cast<const float4_t*>(norm.bias + c);
   }
 }
 
-// kVec: 4-column groups per thread.  TY: float (summed over `shares` slices) or bf16_t; kMixture: TY rows of experts.
-template <class TY, class T, int kVec, bool kMixture>
-__global__ __launch_bounds__(kRowThreads) void residual_rows_kernel(nf_residual_args a, const int32_t* __restrict__ place,
+// kVec: 4-column groups per thread, kThreads: of the row, more where there are few rows.  TY: float (summed over `shares` slices) or bf16_t; kMixture: TY rows of experts.
+template <class TY, class T, int kVec, bool kMixture, int kThreads>
+__global__ __launch_bounds__(kThreads) void residual_rows_kernel(nf_residual_args a, const int32_t* __restrict__ place,
                                                                     const float* __restrict__ weight) {
   __shared__ float scratch[64];
   const int t = blockIdx.x, ld = a.ld;
@@ -68,7 +69,7 @@ __global__ __launch_bounds__(kRowThreads) void residual_rows_kernel(nf_residual_
   float4_t v[kVec], xr[kVec];
 #pragma unroll
   for (int i = 0; i < kVec; ++i) {
-    const int c = (i * kRowThreads + threadIdx.x) * 4;
+    const int c = (i * kThreads + threadIdx.x) * 4;
     v[i] = xr[i] = float4_t{0.f, 0.f, 0.f, 0.f};
     if (c >= ld) continue;
     xr[i] = *reinterpret_cast<const float4_t*>(a.x + row + c);  // in flight together with the sublayer's output
@@ -87,7 +88,7 @@ __global__ __launch_bounds__(kRowThreads) void residual_rows_kernel(nf_residual_
     float4_t own[kVec];
 #pragma unroll
     for (int i = 0; i < kVec; ++i) {
-      const int c = (i * kRowThreads + threadIdx.x) * 4;
+      const int c = (i * kThreads + threadIdx.x) * 4;
       own[i] = same != 0.f && c < ld && a.identity ? Act<TY>::load4((const TY*)a.identity + row + c) : float4_t{0.f, 0.f, 0.f, 0.f};
     }
     constexpr int kAhead = 4;
@@ -102,7 +103,7 @@ __global__ __launch_bounds__(kRowThreads) void residual_rows_kernel(nf_residual_
       }
 #pragma unroll
       for (int i = 0; i < kVec; ++i) {
-        const int c = (i * kRowThreads + threadIdx.x) * 4;
+        const int c = (i * kThreads + threadIdx.x) * 4;
         if (c >= ld) continue;
         float4_t e[kAhead];
 #pragma unroll
@@ -114,21 +115,21 @@ __global__ __launch_bounds__(kRowThreads) void residual_rows_kernel(nf_residual_
 #pragma unroll
     for (int i = 0; i < kVec; ++i) v[i] += own[i] * same;
   }
-  if (a.y_norm.kind != NF_NORM_NONE) norm_row<kVec>(v, a.y_norm, a.width, ld, scratch);
+  if (a.y_norm.kind != NF_NORM_NONE) norm_row<kVec, kThreads>(v, a.y_norm, a.width, ld, scratch);
   const T* e = a.table ? (const T*)a.table + (size_t)a.tokens[t] * ld : nullptr;
 #pragma unroll
   for (int i = 0; i < kVec; ++i) {
-    const int c = (i * kRowThreads + threadIdx.x) * 4;
+    const int c = (i * kThreads + threadIdx.x) * 4;
     v[i] = v[i] * a.y_scale + xr[i];
     if (e && c < ld) v[i] += Act<T>::load4(e + c) * a.table_scale;
     if (a.add && c < ld) v[i] += *reinterpret_cast<const float4_t*>(a.add + c);
     if (c < ld) *reinterpret_cast<float4_t*>(a.x + row + c) = v[i];
   }
   if (!a.act) return;
-  if (a.next.kind != NF_NORM_NONE) norm_row<kVec>(v, a.next, a.width, ld, scratch + 32);
+  if (a.next.kind != NF_NORM_NONE) norm_row<kVec, kThreads>(v, a.next, a.width, ld, scratch + 32);
 #pragma unroll
   for (int i = 0; i < kVec; ++i) {
-    const int c = (i * kRowThreads + threadIdx.x) * 4;
+    const int c = (i * kThreads + threadIdx.x) * 4;
     if (c < ld) Act<T>::store4((T*)a.act + row + c, v[i]);
   }
 }
@@ -331,17 +332,20 @@ int nf_residual_rows(const nf_residual_args* args, nf_stream_t stream) {
   if (a.rows == 0) return NF_OK;
   NF_REQUIRE((a.y || (!a.routing && a.y_norm.kind == NF_NORM_NONE)) && a.x && (!a.table || a.tokens), "%s: null pointer", who);
   hipStream_t s = (hipStream_t)stream;
-  return with_vec(a.ld, [&](auto v) {
-    constexpr int V = decltype(v)::value;
+  auto sized = [&](auto vec, auto threads) {
+    constexpr int V = decltype(vec)::value, N = decltype(threads)::value;
     auto go = [&](auto kern) {
-      kern<<<a.rows, kRowThreads, 0, s>>>(a, a.routing ? a.routing->place : nullptr, a.routing ? a.routing->weight : nullptr);
+      kern<<<a.rows, N, 0, s>>>(a, a.routing ? a.routing->place : nullptr, a.routing ? a.routing->weight : nullptr);
       return check_launch(who);
     };
     const bool b16 = a.dtype == NF_BF16;
-    if (a.routing) return b16 ? go(residual_rows_kernel<bf16_t, bf16_t, V, true>) : go(residual_rows_kernel<float, float, V, true>);
-    if (a.y && a.y_dtype == NF_BF16) return b16 ? go(residual_rows_kernel<bf16_t, bf16_t, V, false>) : go(residual_rows_kernel<bf16_t, float, V, false>);
-    return b16 ? go(residual_rows_kernel<float, bf16_t, V, false>) : go(residual_rows_kernel<float, float, V, false>);
-  });
+    if (a.routing) return b16 ? go(residual_rows_kernel<bf16_t, bf16_t, V, true, N>) : go(residual_rows_kernel<float, float, V, true, N>);
+    if (a.y && a.y_dtype == NF_BF16) return b16 ? go(residual_rows_kernel<bf16_t, bf16_t, V, false, N>) : go(residual_rows_kernel<bf16_t, float, V, false, N>);
+    return b16 ? go(residual_rows_kernel<float, bf16_t, V, false, N>) : go(residual_rows_kernel<float, float, V, false, N>);
+  };
+  // a row on more wavefronts where rows alone leave the CUs mostly empty, and where it is put together from many
+  if ((a.rows <= kFewRows || a.routing) && a.ld > 1024) return a.ld <= 4096 ? sized(ic<1>{}, ic<1024>{}) : a.ld <= 8192 ? sized(ic<2>{}, ic<1024>{}) : sized(ic<4>{}, ic<1024>{});
+  return with_vec(a.ld, [&](auto v) { return sized(v, ic<kRowThreads>{}); });
 }
 
 int nf_norm_rows(int dtype, const float* x, const int32_t* row_index, const nf_norm* norm, void* out, int n, int width, int ld,

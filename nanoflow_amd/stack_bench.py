@@ -60,10 +60,10 @@ def pudadra_config(width, ff):
 
 
 def desalix_config(width, ff):
-    """Three layers of attention in chunks of 1024 (heads of 128, 4 query heads per kv head), the middle one passed twice; 32 experts
+    """Three layers of attention in chunks of 1536 (heads of 128, 4 query heads per kv head), the middle one passed twice; 32 experts
     of a quarter of `ff`, 4 of them per token, and a shared one."""
     n, expert = width // 128, {"ff": ff // 4, "limit": 7.0}
-    attention = {"heads": n, "kv_heads": n // 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": 1024}, "rot": {"dims": 64, "base": 5e5}}
+    attention = {"heads": n, "kv_heads": n // 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": 1536}, "rot": {"dims": 64, "base": 5e5}}
     moe = {"kind": "moe", "expert": expert, "shared": expert, "router": {"experts": 32, "top": 4}}
     return {"architecture": "Desalix", "width": width, "vocab": VOCAB, "embedding": {"scale": 8.0}, "norm": {"eps": 1e-5},
             "loop": {"start": 1, "stop": 2, "times": 2}, "layers": [{"type": "attention", "mixer": attention, "mlp": moe}] * 3}

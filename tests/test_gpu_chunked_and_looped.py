@@ -116,7 +116,7 @@ def chunk_case(dtype, heads, kv_heads, dim, vdim, chunk, b, n_decode, seed=0, ma
     return got, want.reshape(len(want), -1)
 
 
-@pytest.mark.parametrize("heads,kv_heads,dim,vdim", [(4, 2, 64, 64), (6, 2, 32, 48), (5, 1, 18, 10), (20, 1, 128, 128), (3, 3, 192, 128), (2, 1, 160, 256), (6, 1, 96, 96),
+@pytest.mark.parametrize("heads,kv_heads,dim,vdim", [(4, 2, 64, 64), (6, 2, 32, 48), (5, 1, 18, 10), (20, 1, 128, 128), (3, 3, 192, 128), (2, 1, 160, 256), (7, 1, 96, 80),
                                                      (40, 2, 8, 2)])
 @pytest.mark.parametrize("chunk", [24, 1, 64, 0, 200, 37])
 def test_attention_in_chunks(heads, kv_heads, dim, vdim, chunk):
@@ -128,7 +128,7 @@ def test_attention_in_chunks(heads, kv_heads, dim, vdim, chunk):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("heads,kv_heads,dim,vdim", [(4, 2, 32, 32), (4, 1, 128, 128)])
-@pytest.mark.parametrize("chunk", [32, 40, 120])
+@pytest.mark.parametrize("chunk", [32, 40, 104])
 def test_a_key_at_the_chunks_edge(dtype, heads, kv_heads, dim, vdim, chunk):
     """Keys just inside and just outside the query's chunk, at the borders of pages and far back in it, for queries at either end of a chunk."""
     for query in (chunk - 1, chunk, chunk + 1, 2 * chunk - 1, 2 * chunk + 17):
@@ -264,8 +264,8 @@ def test_what_a_pass_starts_with(width, ld):
                 close(dx[:, :width], want, F32)
                 close(act[:, :width], S.rms_norm(want, eps, w), dtype)
                 assert not host(dx[:, width:]).any()
-        gx, _ = K.embed_rows(dev(tok), dev(tok), dtab, None, scale=12.0 / 7)
-        close(gx[:, :width], 12.0 / 7 * rounded(table, dtype)[tok], F32)
+        gx, _ = K.embed_rows(dev(tok), dev(tok), dtab, None, scale=1.7)
+        close(gx[:, :width], 1.7 * rounded(table, dtype)[tok], F32)
 
 
 # ---------------------------------------------------------------- whole models
